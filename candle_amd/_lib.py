@@ -1,5 +1,5 @@
 """ctypes binding of libcandle_hip_quant.so (the C ABI declared in include/candle_hip_quant.h and
-include/candle_hip_nn.h).
+include/candle_hip_nn.h) and of libcandle_hip_mixer.so (include/candle_hip_mixer.h, plus the glue of candle_hip_nn.h).
 
 The library must be built first (``python -m candle_amd.build`` or ``__graft_entry__.build()``);
 loading fails loudly when it is missing — there is no CPU or PyTorch fallback.
@@ -11,6 +11,7 @@ import os
 
 _HERE = os.path.dirname(os.path.abspath(__file__))
 LIB_PATH = os.path.join(_HERE, "libcandle_hip_quant.so")
+MIXER_LIB_PATH = os.path.join(_HERE, "libcandle_hip_mixer.so")
 
 _i64 = ctypes.c_int64
 _int = ctypes.c_int
@@ -75,6 +76,43 @@ SIGNATURES = {
     "cq_nn_argmax_embed": (_int, [_vp, _i64, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _i64, _i64, _vp, _vp]),
 }
 
+
+
+class MixHeads(ctypes.Structure):
+    """cq_mix_heads of include/candle_hip_mixer.h."""
+    _fields_ = [("norm_dev", _vp), ("cos_dev", _vp), ("sin_dev", _vp), ("dst_dev", _vp), ("src_off", _i64), ("dst_row_stride", _i64),
+                ("dst_head_stride", _i64), ("heads", ctypes.c_int32), ("dim", ctypes.c_int32), ("dim_pad", ctypes.c_int32),
+                ("rot_dims", ctypes.c_int32), ("by_position", ctypes.c_int32), ("ctx", ctypes.c_int32), ("factor", _f32),
+                ("reserved", ctypes.c_int32)]
+
+
+_heads = ctypes.POINTER(MixHeads)
+
+# include/candle_hip_mixer.h
+MIXER_SIGNATURES = {
+    "cq_dense_matmul_workspace_bytes": (_i64, [_int, _i64, _i64, _i64]),
+    "cq_dense_matmul": (_int, [_int, _vp, _i64, _vp, _i64, _vp, _i64, _vp, _i64, _int, _i64, _i64, _i64, _vp, _i64, _vp]),
+    "cq_dense_matvec": (_int, [_vp, _i64, _vp, _int, _vp, _f32, _i64, _vp, _vp, _int, _i64, _i64, _vp]),
+    "cq_mix_rms_norm_rows": (_int, [_vp, _i64, _vp, _vp, _i64, _vp, _vp, _i64, _i64, _i64, _f32, _vp]),
+    "cq_mix_poly_norm": (_int, [_vp, _i64, _vp, _vp, _i64, _i64, _i64, _f32, _vp]),
+    "cq_mix_tanh": (_int, [_vp, _i64, _vp, _i64, _i64, _i64, _vp]),
+    "cq_mix_pack_heads": (_int, [_vp, _i64, _heads, _int, _f32, _vp, _i64, _i64, _vp]),
+    "cq_mix_head_norm_gate": (_int, [_vp, _i64, _vp, _i64, _vp, _int, _f32, _vp, _i64, _i64, _i64, _i64, _f32, _vp]),
+    "cq_mix_talk_attention": (_int, [_vp, _vp, _vp, _vp, _f32, _i64, _i64, _f32, _vp, _i64, _i64, _i64, _i64, _i64, _i64, _i64, _i64, _i64, _vp]),
+    "cq_mix_talk_decode_workspace_bytes": (_i64, [_i64, _i64, _i64, _i64, _i64]),
+    "cq_mix_talk_decode": (_int, [_vp, _heads, _f32, _vp, _f32, _i64, _i64, _vp, _i64, _vp, _i64, _vp]),
+    "cq_mix_state_pad": (_i64, [_i64]),
+    "cq_mix_retention_workspace_bytes": (_i64, [_i64, _i64, _i64, _i64]),
+    "cq_mix_retention": (_int, [_vp, _vp, _vp, _i64, _vp, _vp, _vp, _i64, _i64, _i64, _i64, _i64, _i64, _vp, _i64, _vp]),
+    "cq_mix_talk_merge_retention_step": (_int, [_vp, _i64, _i64, _i64, _i64, _i64, _f32, _vp, _vp, _heads, _i64, _i64, _vp, _vp, _i64, _i64, _f32, _f32,
+                                                _vp, _vp, _i64, _vp]),
+    "cq_mix_delta_prep": (_int, [_vp, _i64, _i64, _i64, _i64, _vp, _i64, _vp, _vp, _vp, _i64, _i64, _i64, _vp]),
+    "cq_mix_delta_scan": (_int, [_vp, _vp, _i64, _vp, _vp, _i64, _i64, _i64, _i64, _vp]),
+    "cq_mix_delta_step": (_int, [_vp, _i64, _i64, _i64, _i64, _i64, _i64, _vp, _i64, _i64, _vp, _vp, _vp, _vp, _vp, _i64, _i64, _f32, _vp]),
+}
+# glue that the mixer library carries as well
+_MIXER_GLUE = ("cq_status_string", "cq_nn_embedding", "cq_nn_argmax")
+
 _lib = None
 
 
@@ -87,21 +125,36 @@ class CqError(RuntimeError):
         self.status = status
 
 
+def _load(path: str, signatures: dict) -> ctypes.CDLL:
+    if not os.path.exists(path):
+        raise ImportError(
+            f"{path} is missing: build the HIP extension first (python -m candle_amd.build). "
+            "There is no fallback path."
+        )
+    L = ctypes.CDLL(path)
+    for name, (res, args) in signatures.items():
+        fn = getattr(L, name)
+        fn.restype = res
+        fn.argtypes = args
+    return L
+
+
 def lib() -> ctypes.CDLL:
     global _lib
     if _lib is None:
-        if not os.path.exists(LIB_PATH):
-            raise ImportError(
-                f"{LIB_PATH} is missing: build the HIP extension first (python -m candle_amd.build). "
-                "There is no fallback path."
-            )
-        L = ctypes.CDLL(LIB_PATH)
-        for name, (res, args) in SIGNATURES.items():
-            fn = getattr(L, name)
-            fn.restype = res
-            fn.argtypes = args
-        _lib = L
+        _lib = _load(LIB_PATH, SIGNATURES)
     return _lib
+
+
+_mixer = None
+
+
+def mixer_lib() -> ctypes.CDLL:
+    """libcandle_hip_mixer.so: what models with bfloat16 weights and other sequence mixers run on, complete in itself."""
+    global _mixer
+    if _mixer is None:
+        _mixer = _load(MIXER_LIB_PATH, {**MIXER_SIGNATURES, **{n: SIGNATURES[n] for n in _MIXER_GLUE}})
+    return _mixer
 
 
 BENCH_LIB_PATH = os.path.join(_HERE, "libcq_bench.so")
@@ -123,7 +176,7 @@ def bench_lib():
 
 
 def status_string(status: int) -> str:
-    return lib().cq_status_string(status).decode()
+    return (_lib or _mixer or lib()).cq_status_string(status).decode()
 
 
 def check(fn: str, status: int) -> None:

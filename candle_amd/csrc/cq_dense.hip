@@ -1,0 +1,475 @@
+// Matrix products with unquantized bfloat16 weights: MFMA tiles for several activation rows (bf16 or f32 products, f32
+// accumulation), a weight-streaming matvec for one row with the norm / activation of the input as prologue and the
+// residual add as epilogue.  Activations and results are f32 in memory, like everywhere in this library; the bf16 product
+// rounds them on the way into LDS.
+#include "cq_device.h"
+#include "../../include/candle_hip_mixer.h"
+
+namespace {
+
+typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
+
+inline bool misaligned(const void *p, size_t a) { return (reinterpret_cast<uintptr_t>(p) & (a - 1)) != 0; }
+
+__device__ __forceinline__ float bf_lo(uint32_t v) { return __builtin_bit_cast(float, v << 16); }
+__device__ __forceinline__ float bf_hi(uint32_t v) { return __builtin_bit_cast(float, v & 0xffff0000u); }
+
+__device__ __forceinline__ bf16x8 round_bf16(const f32x4 &a, const f32x4 &b) {
+    bf16x8 r;
+#pragma unroll
+    for (int i = 0; i < 4; i++) {
+        r[i] = (__bf16)a[i];
+        r[4 + i] = (__bf16)b[i];
+    }
+    return r;
+}
+
+// where a tile's results go: the plane of a k split, or dst with the residual epilogue
+struct Out {
+    float *dst;
+    const float *add;
+    int64_t ldd, ld_add;
+    float *planes;          // != nullptr: [splits][m][n4]
+    int64_t n4;             // n rounded up to 4
+    int accumulate;
+};
+
+// four consecutive columns n .. n+3 of row m (n % 4 == 0)
+__device__ __forceinline__ void emit4(const Out &o, f32x4 v, int64_t m, int n, int64_t M, int N, int split) {
+    if (o.planes) {
+        *reinterpret_cast<f32x4 *>(o.planes + ((int64_t)split * M + m) * o.n4 + n) = v;
+        return;
+    }
+    float *d = o.dst + m * o.ldd + n;
+    const float *a = o.add ? o.add + m * o.ld_add + n : nullptr;
+    if (n + 4 <= N && ((reinterpret_cast<uintptr_t>(d) | reinterpret_cast<uintptr_t>(a)) & 15) == 0) {
+        if (o.accumulate) v += *reinterpret_cast<const f32x4 *>(d);
+        if (a) v += *reinterpret_cast<const f32x4 *>(a);
+        *reinterpret_cast<f32x4 *>(d) = v;
+        return;
+    }
+#pragma unroll
+    for (int i = 0; i < 4; i++)
+        if (n + i < N) d[i] = v[i] + (o.accumulate ? d[i] : 0.0f) + (a ? a[i] : 0.0f);
+}
+
+// Workgroups are dealt to the eight XCDs round-robin: give each XCD a contiguous run of tiles, so that the rows and columns
+// its workgroups share stay in its own L2.
+__device__ __forceinline__ int xcd_tile(int id, int total) {
+    const int q = total >> 3, r = total & 7, x = id & 7, i = id >> 3;
+    return x * q + min(x, r) + i;
+}
+
+// ---- bf16 tiles: BM activation rows x BN weight rows, k in steps of 64, LDS double-buffered -----------------------------
+// The weights are the A operand, so a lane ends with four consecutive output columns of one row.  LDS rows are 128 bytes in
+// eight 16-byte chunks, chunk c of row r at c ^ (r & 7).
+template <int BM, int BN, int WGM, int WGN>
+__global__ __launch_bounds__(256, 2) void dense_bf16_kernel(const uint16_t *__restrict__ w, int64_t ldw, const float *__restrict__ x, int64_t ldx, Out out,
+                                                         int64_t M, int N, int K, int tiles_m, int tiles_n, int k_split) {
+    constexpr int TM = BM / WGM / 16, TN = BN / WGN / 16, CA = BM * 8 / 256, CB = BN * 8 / 256;
+    __shared__ bf16x8 lds[2][(BM + BN) * 8];
+    const int tid = threadIdx.x, lane = tid & 63, wv = __builtin_amdgcn_readfirstlane(tid >> 6);
+    const int t = xcd_tile(blockIdx.x, tiles_m * tiles_n);
+    const int64_t m0 = (int64_t)(t % tiles_m) * BM;           // tiles that follow each other share the weight rows
+    const int n0 = (t / tiles_m) * BN;
+    const int k_lo = blockIdx.y * k_split, k_hi = min(K, k_lo + k_split);
+    const int wm = (wv / WGN) * (BM / WGM), wn = (wv % WGN) * (BN / WGN);
+
+    f32x4 ra[CA][2];
+    u32x4 rb[CB];
+    const float *xp[CA];
+    const uint16_t *wp[CB];
+#pragma unroll
+    for (int i = 0; i < CA; i++) {
+        const int c = tid + 256 * i;
+        xp[i] = x + min(m0 + (c >> 3), M - 1) * ldx + (c & 7) * 8;
+    }
+#pragma unroll
+    for (int i = 0; i < CB; i++) {
+        const int c = tid + 256 * i;
+        wp[i] = w + (int64_t)min(n0 + (c >> 3), N - 1) * ldw + (c & 7) * 8;
+    }
+    auto fetch = [&](int k) {
+#pragma unroll
+        for (int i = 0; i < CB; i++) rb[i] = *reinterpret_cast<const u32x4 *>(wp[i] + k);
+#pragma unroll
+        for (int i = 0; i < CA; i++) {
+            ra[i][0] = *reinterpret_cast<const f32x4 *>(xp[i] + k);
+            ra[i][1] = *reinterpret_cast<const f32x4 *>(xp[i] + k + 4);
+        }
+    };
+    auto stage = [&](int b) {
+#pragma unroll
+        for (int i = 0; i < CB; i++) {
+            const int c = tid + 256 * i, r = c >> 3;
+            lds[b][BM * 8 + r * 8 + ((c & 7) ^ (r & 7))] = __builtin_bit_cast(bf16x8, rb[i]);
+        }
+#pragma unroll
+        for (int i = 0; i < CA; i++) {
+            const int c = tid + 256 * i, r = c >> 3;
+            lds[b][r * 8 + ((c & 7) ^ (r & 7))] = round_bf16(ra[i][0], ra[i][1]);
+        }
+    };
+    f32x4 acc[TM][TN];
+#pragma unroll
+    for (int i = 0; i < TM; i++)
+#pragma unroll
+        for (int j = 0; j < TN; j++) acc[i][j] = f32x4{0.f, 0.f, 0.f, 0.f};
+
+    fetch(k_lo);
+    stage(0);
+    __syncthreads();
+    int cur = 0;
+    const int lr = lane & 15, lk = lane >> 4;
+    for (int k = k_lo; k < k_hi; k += 64) {
+        const bool more = k + 64 < k_hi;
+        if (more) fetch(k + 64);
+#pragma unroll
+        for (int s = 0; s < 2; s++) {
+            bf16x8 fa[TM], fb[TN];
+#pragma unroll
+            for (int i = 0; i < TM; i++) {
+                const int r = wm + 16 * i + lr;
+                fa[i] = lds[cur][r * 8 + ((4 * s + lk) ^ (r & 7))];
+            }
+#pragma unroll
+            for (int j = 0; j < TN; j++) {
+                const int r = wn + 16 * j + lr;
+                fb[j] = lds[cur][BM * 8 + r * 8 + ((4 * s + lk) ^ (r & 7))];
+            }
+#pragma unroll
+            for (int i = 0; i < TM; i++)
+#pragma unroll
+                for (int j = 0; j < TN; j++) acc[i][j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(fb[j], fa[i], acc[i][j], 0, 0, 0);
+        }
+        if (more) {
+            stage(cur ^ 1);
+            __syncthreads();
+            cur ^= 1;
+        }
+    }
+#pragma unroll
+    for (int i = 0; i < TM; i++) {
+        const int64_t m = m0 + wm + 16 * i + lr;
+        if (m >= M) continue;
+#pragma unroll
+        for (int j = 0; j < TN; j++) {
+            const int n = n0 + wn + 16 * j + 4 * lk;
+            if (n < N) emit4(out, acc[i][j], m, n, M, N, blockIdx.y);
+        }
+    }
+}
+
+// ---- f32 tiles: 64 x 64, k in steps of 32, weights widened on the way into LDS; a lane's float4 along k feeds four steps of
+// v_mfma_f32_16x16x4 (both operands use the same k order) ------------------------------------------------------------------
+constexpr int DF_ROW = 36;               // floats per LDS row: 32 + 4, 16 rows of a 16-byte read fall on distinct banks
+__global__ __launch_bounds__(256) void dense_f32_kernel(const uint16_t *__restrict__ w, int64_t ldw, const float *__restrict__ x, int64_t ldx, Out out,
+                                                        int64_t M, int N, int K, int tiles_m, int tiles_n, int k_split) {
+    __shared__ float lds[2][128 * DF_ROW];
+    const int tid = threadIdx.x, lane = tid & 63, wv = __builtin_amdgcn_readfirstlane(tid >> 6);
+    const int t = xcd_tile(blockIdx.x, tiles_m * tiles_n);
+    const int64_t m0 = (int64_t)(t % tiles_m) * 64;
+    const int n0 = (t / tiles_m) * 64;
+    const int k_lo = blockIdx.y * k_split, k_hi = min(K, k_lo + k_split);
+    const int wm = (wv >> 1) * 32, wn = (wv & 1) * 32;
+    f32x4 ra[2];
+    u32x4 rb;
+    const float *xp[2];
+#pragma unroll
+    for (int i = 0; i < 2; i++) {
+        const int c = tid + 256 * i;
+        xp[i] = x + min(m0 + (c >> 3), M - 1) * ldx + (c & 7) * 4;
+    }
+    const uint16_t *wp = w + (int64_t)min(n0 + (tid >> 2), N - 1) * ldw + (tid & 3) * 8;
+    auto fetch = [&](int k) {
+        rb = *reinterpret_cast<const u32x4 *>(wp + k);
+#pragma unroll
+        for (int i = 0; i < 2; i++) ra[i] = *reinterpret_cast<const f32x4 *>(xp[i] + k);
+    };
+    auto stage = [&](int b) {
+#pragma unroll
+        for (int i = 0; i < 2; i++) {
+            const int c = tid + 256 * i;
+            *reinterpret_cast<f32x4 *>(&lds[b][(c >> 3) * DF_ROW + (c & 7) * 4]) = ra[i];
+        }
+        float *d = &lds[b][(64 + (tid >> 2)) * DF_ROW + (tid & 3) * 8];
+        *reinterpret_cast<f32x4 *>(d) = f32x4{bf_lo(rb.x), bf_hi(rb.x), bf_lo(rb.y), bf_hi(rb.y)};
+        *reinterpret_cast<f32x4 *>(d + 4) = f32x4{bf_lo(rb.z), bf_hi(rb.z), bf_lo(rb.w), bf_hi(rb.w)};
+    };
+    f32x4 acc[2][2];
+#pragma unroll
+    for (int i = 0; i < 2; i++)
+#pragma unroll
+        for (int j = 0; j < 2; j++) acc[i][j] = f32x4{0.f, 0.f, 0.f, 0.f};
+    fetch(k_lo);
+    stage(0);
+    __syncthreads();
+    int cur = 0;
+    const int lr = lane & 15, lk = lane >> 4;
+    for (int k = k_lo; k < k_hi; k += 32) {
+        const bool more = k + 32 < k_hi;
+        if (more) fetch(k + 32);
+#pragma unroll
+        for (int s = 0; s < 2; s++) {
+            f32x4 fa[2], fb[2];
+#pragma unroll
+            for (int i = 0; i < 2; i++) {
+                fa[i] = *reinterpret_cast<const f32x4 *>(&lds[cur][(wm + 16 * i + lr) * DF_ROW + 16 * s + 4 * lk]);
+                fb[i] = *reinterpret_cast<const f32x4 *>(&lds[cur][(64 + wn + 16 * i + lr) * DF_ROW + 16 * s + 4 * lk]);
+            }
+#pragma unroll
+            for (int e = 0; e < 4; e++)
+#pragma unroll
+                for (int i = 0; i < 2; i++)
+#pragma unroll
+                    for (int j = 0; j < 2; j++) acc[i][j] = __builtin_amdgcn_mfma_f32_16x16x4f32(fb[j][e], fa[i][e], acc[i][j], 0, 0, 0);
+        }
+        if (more) {
+            stage(cur ^ 1);
+            __syncthreads();
+            cur ^= 1;
+        }
+    }
+#pragma unroll
+    for (int i = 0; i < 2; i++) {
+        const int64_t m = m0 + wm + 16 * i + lr;
+        if (m >= M) continue;
+#pragma unroll
+        for (int j = 0; j < 2; j++) {
+            const int n = n0 + wn + 16 * j + 4 * lk;
+            if (n < N) emit4(out, acc[i][j], m, n, M, N, blockIdx.y);
+        }
+    }
+}
+
+// the planes of a k split, added in order
+__global__ __launch_bounds__(256) void dense_planes_kernel(Out out, int64_t M, int N, int splits) {
+    const int64_t groups = out.n4 >> 2;
+    const int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x;
+    if (i >= M * groups) return;
+    const int64_t m = i / groups;
+    const int n = (int)(i - m * groups) * 4;
+    f32x4 v = *reinterpret_cast<const f32x4 *>(out.planes + m * out.n4 + n);
+    for (int s = 1; s < splits; s++) v += *reinterpret_cast<const f32x4 *>(out.planes + ((int64_t)s * M + m) * out.n4 + n);
+    Out o = out;
+    o.planes = nullptr;
+    emit4(o, v, m, n, M, N, 0);
+}
+
+struct Plan {
+    int bm, bn, tiles_m, tiles_n, splits, k_split;
+};
+
+Plan plan(int precision, int64_t m, int64_t n, int64_t k) {
+    Plan p;
+    auto tiles = [&](int bm, int bn) { return ((m + bm - 1) / bm) * ((n + bn - 1) / bn); };
+    if (precision == CQ_DENSE_F32) {
+        p.bm = p.bn = 64;
+    } else if (m > 64 && tiles(128, 128) >= 192) {
+        p.bm = p.bn = 128;
+    } else if (m > 32) {
+        p.bm = p.bn = 64;
+    } else {
+        p.bm = 32;
+        p.bn = 64;
+    }
+    p.tiles_m = (int)((m + p.bm - 1) / p.bm);
+    p.tiles_n = (int)((n + p.bn - 1) / p.bn);
+    // enough workgroups for two per CU, each with at least 256 of k
+    const int64_t t = (int64_t)p.tiles_m * p.tiles_n;
+    int64_t s = t >= 384 ? 1 : (512 + t - 1) / t;
+    s = s < k / 256 ? s : k / 256;
+    s = s < 1 ? 1 : (s > 16 ? 16 : s);
+    p.k_split = (int)((k / 64 + s - 1) / s) * 64;
+    p.splits = (int)((k + p.k_split - 1) / p.k_split);
+    return p;
+}
+
+// ---- one row --------------------------------------------------------------------------------------------------------------
+// 8 waves; a wave takes R weight rows at a time and walks them in blocks of 64 lanes x 8 elements x U, one block ahead; the
+// first block is requested before the prologue.  The input row sits in LDS as f32, zero beyond `dim` and up to a whole block.
+constexpr int MV_U = 2, MV_BLOCK = 512 * MV_U;
+
+__device__ __forceinline__ float block_sum_512(float v, float *red) {
+    v = wave_sum(v);
+    __syncthreads();
+    if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = v;
+    __syncthreads();
+    return ((red[0] + red[1]) + (red[2] + red[3])) + ((red[4] + red[5]) + (red[6] + red[7]));
+}
+
+template <int PRO, int R>
+__global__ __launch_bounds__(512) void dense_matvec_kernel(const uint16_t *__restrict__ w, int64_t ldw, const float *__restrict__ x,
+                                                           const float *__restrict__ vec, float eps, int dim, float *dst, const float *add, int accumulate,
+                                                           int n, int k) {
+    extern __shared__ __attribute__((aligned(16))) float xs[];           // k rounded up to MV_BLOCK
+    __shared__ float red[8];
+    const int tid = threadIdx.x, lane = tid & 63, wv = __builtin_amdgcn_readfirstlane(tid >> 6);
+    const int groups = (n + R - 1) / R, step = gridDim.x * 8;
+    const int kb_n = (k + MV_BLOCK - 1) / MV_BLOCK;
+    int g = blockIdx.x * 8 + wv;
+    u32x4 cur[R][MV_U], nxt[R][MV_U];
+    auto load = [&](int grp, int kb, u32x4 (&d)[R][MV_U]) {
+#pragma unroll
+        for (int r = 0; r < R; r++) {
+            const uint16_t *p = w + (int64_t)min(grp * R + r, n - 1) * ldw;
+#pragma unroll
+            for (int u = 0; u < MV_U; u++) d[r][u] = *reinterpret_cast<const u32x4 *>(p + min(kb * MV_BLOCK + u * 512 + lane * 8, k - 8));
+        }
+    };
+    if (g < groups) load(g, 0, cur);
+
+    const int k_all = kb_n * MV_BLOCK;
+    if (PRO == CQ_DENSE_PLAIN) {
+        for (int i = tid; i < k_all; i += 512) xs[i] = i < dim ? x[i] : 0.0f;
+    } else if (PRO == CQ_DENSE_NORM) {
+        float s = 0.0f;
+        for (int i = tid; i < k_all; i += 512) {
+            const float v = i < dim ? x[i] : 0.0f;
+            xs[i] = v;
+            s = fmaf(v, v, s);
+        }
+        const float m = sqrtf(block_sum_512(s, red) / (float)dim + eps);
+        for (int i = tid; i < dim; i += 512) xs[i] = xs[i] / m * vec[i];
+    } else {
+        float s2 = 0.0f, s4 = 0.0f, s6 = 0.0f;
+        for (int i = tid; i < k_all; i += 512) {
+            const float v = i < dim ? x[i] : 0.0f, q = v * v;
+            xs[i] = v;
+            s2 += q;
+            s4 = fmaf(q, q, s4);
+            s6 = fmaf(q * q, q, s6);
+        }
+        const float inv = 1.0f / (float)dim;
+        const float i1 = vec[0] / sqrtf(block_sum_512(s2, red) * inv + eps);
+        const float i2 = vec[1] / sqrtf(block_sum_512(s4, red) * inv + eps);
+        const float i3 = vec[2] / sqrtf(block_sum_512(s6, red) * inv + eps);
+        const float e = vec[3];
+        for (int i = tid; i < dim; i += 512) {
+            const float v = xs[i], q = v * v;
+            xs[i] = fmaf(i1, v, fmaf(i2, q, fmaf(i3, q * v, e)));
+        }
+    }
+    __syncthreads();
+
+    for (; g < groups; g += step) {
+        float acc[R];
+#pragma unroll
+        for (int r = 0; r < R; r++) acc[r] = 0.0f;
+        for (int kb = 0; kb < kb_n; kb++) {
+            const bool last = kb + 1 == kb_n;
+            const int ng = last ? g + step : g;
+            if (ng < groups) load(ng, last ? 0 : kb + 1, nxt);
+#pragma unroll
+            for (int u = 0; u < MV_U; u++) {
+                const f32x4 *xv = reinterpret_cast<const f32x4 *>(xs + kb * MV_BLOCK + u * 512 + lane * 8);
+                const f32x4 a = xv[0], b = xv[1];
+#pragma unroll
+                for (int r = 0; r < R; r++) {
+                    const u32x4 q = cur[r][u];
+                    acc[r] = fmaf(bf_lo(q.x), a.x, acc[r]);
+                    acc[r] = fmaf(bf_hi(q.x), a.y, acc[r]);
+                    acc[r] = fmaf(bf_lo(q.y), a.z, acc[r]);
+                    acc[r] = fmaf(bf_hi(q.y), a.w, acc[r]);
+                    acc[r] = fmaf(bf_lo(q.z), b.x, acc[r]);
+                    acc[r] = fmaf(bf_hi(q.z), b.y, acc[r]);
+                    acc[r] = fmaf(bf_lo(q.w), b.z, acc[r]);
+                    acc[r] = fmaf(bf_hi(q.w), b.w, acc[r]);
+                }
+            }
+#pragma unroll
+            for (int r = 0; r < R; r++)
+#pragma unroll
+                for (int u = 0; u < MV_U; u++) cur[r][u] = nxt[r][u];
+        }
+#pragma unroll
+        for (int r = 0; r < R; r++) {
+            const float s = wave_sum(acc[r]);
+            const int row = g * R + r;
+            if (lane == 0 && row < n) dst[row] = s + (accumulate ? dst[row] : 0.0f) + (add ? add[row] : 0.0f);
+        }
+    }
+}
+
+template <int PRO>
+int matvec_launch(const uint16_t *w, int64_t ldw, const float *x, const float *vec, float eps, int dim, float *dst, const float *add, int accumulate, int n,
+                  int k, hipStream_t s) {
+    const size_t lds = (size_t)((k + MV_BLOCK - 1) / MV_BLOCK) * MV_BLOCK * sizeof(float);
+    // rows per wave: as many as leave at least one group for every wave of 256 workgroups
+    const int r = n >= 8192 ? 4 : (n >= 4096 ? 2 : 1);
+    const int groups = (n + r - 1) / r;
+    const int blocks = (groups + 7) / 8 < 1024 ? (groups + 7) / 8 : 1024;
+#define CQ_MV(R_)                                                                                                                                    \
+    do {                                                                                                                                              \
+        if (lds > 64 * 1024) {                                                                                                                        \
+            const int e = (int)hipFuncSetAttribute(reinterpret_cast<const void *>(dense_matvec_kernel<PRO, R_>), hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024 - 64);        \
+            if (e) return e;                                                                                                                          \
+        }                                                                                                                                             \
+        hipLaunchKernelGGL((dense_matvec_kernel<PRO, R_>), dim3(blocks), dim3(512), lds, s, w, ldw, x, vec, eps, dim, dst, add, accumulate, n, k);    \
+    } while (0)
+    if (r == 4) CQ_MV(4);
+    else if (r == 2) CQ_MV(2);
+    else CQ_MV(1);
+#undef CQ_MV
+    return (int)hipGetLastError();
+}
+
+}  // namespace
+
+extern "C" {
+
+int64_t cq_dense_matmul_workspace_bytes(int precision, int64_t m, int64_t n, int64_t k) {
+    if (m <= 0 || n <= 0 || k <= 0 || k % 64) return 0;
+    const Plan p = plan(precision, m, n, k);
+    return p.splits > 1 ? (int64_t)p.splits * m * ((n + 3) / 4 * 4) * 4 : 0;
+}
+
+int cq_dense_matmul(int precision, const void *w_dev, int64_t ldw, const float *x_dev, int64_t ldx, float *dst_dev, int64_t ldd, const float *add_dev,
+                    int64_t ld_add, int accumulate, int64_t m, int64_t n, int64_t k, void *workspace_dev, int64_t workspace_bytes, void *stream) {
+    if (precision != CQ_DENSE_BF16 && precision != CQ_DENSE_F32) return CQ_ERR_DTYPE;
+    if (m < 0 || n < 0 || k <= 0 || k % 64 || ldw % 64 || ldw < k || ldx % 4 || ldx < k || ldd < n || (add_dev && ld_add < n)) return CQ_ERR_SHAPE;
+    if (m == 0 || n == 0) return CQ_OK;
+    if (!w_dev || !x_dev || !dst_dev) return CQ_ERR_NULL;
+    if (misaligned(w_dev, 16) || misaligned(x_dev, 16) || misaligned(dst_dev, 4) || misaligned(add_dev, 4) || misaligned(workspace_dev, 16)) return CQ_ERR_ALIGN;
+    if (m > (1 << 24) || n > (1 << 24) || k > (1 << 24)) return CQ_ERR_RANGE;
+    const Plan p = plan(precision, m, n, k);
+    if ((int64_t)p.tiles_m * p.tiles_n > 0x7fffffffLL) return CQ_ERR_RANGE;
+    if (p.splits > 1 && (!workspace_dev || workspace_bytes < cq_dense_matmul_workspace_bytes(precision, m, n, k))) return CQ_ERR_WORKSPACE;
+    Out o;
+    o.dst = dst_dev;
+    o.add = add_dev;
+    o.ldd = ldd;
+    o.ld_add = ld_add;
+    o.accumulate = accumulate;
+    o.planes = p.splits > 1 ? (float *)workspace_dev : nullptr;
+    o.n4 = (n + 3) / 4 * 4;
+    hipStream_t s = (hipStream_t)stream;
+    const dim3 grid((unsigned)(p.tiles_m * p.tiles_n), (unsigned)p.splits);
+    const uint16_t *w = (const uint16_t *)w_dev;
+#define CQ_DM(K_) hipLaunchKernelGGL(K_, grid, dim3(256), 0, s, w, ldw, x_dev, ldx, o, m, (int)n, (int)k, p.tiles_m, p.tiles_n, p.k_split)
+    if (precision == CQ_DENSE_F32) CQ_DM(dense_f32_kernel);
+    else if (p.bm == 128) CQ_DM((dense_bf16_kernel<128, 128, 2, 2>));
+    else if (p.bm == 64) CQ_DM((dense_bf16_kernel<64, 64, 2, 2>));
+    else CQ_DM((dense_bf16_kernel<32, 64, 1, 4>));
+#undef CQ_DM
+    if (p.splits > 1)
+        hipLaunchKernelGGL(dense_planes_kernel, dim3((unsigned)((m * (o.n4 / 4) + 255) / 256)), dim3(256), 0, s, o, m, (int)n, p.splits);
+    return (int)hipGetLastError();
+}
+
+int cq_dense_matvec(const void *w_dev, int64_t ldw, const float *x_dev, int prologue, const float *vec_dev, float eps, int64_t dim, float *dst_dev,
+                    const float *add_dev, int accumulate, int64_t n, int64_t k, void *stream) {
+    if (n < 0 || k <= 0 || k % 64 || ldw % 64 || ldw < k || dim <= 0 || dim > k) return CQ_ERR_SHAPE;
+    if (prologue < CQ_DENSE_PLAIN || prologue > CQ_DENSE_POLY) return CQ_ERR_DTYPE;
+    if (n == 0) return CQ_OK;
+    if (!w_dev || !x_dev || !dst_dev || (prologue != CQ_DENSE_PLAIN && !vec_dev)) return CQ_ERR_NULL;
+    if (misaligned(w_dev, 16) || misaligned(x_dev, 4) || misaligned(vec_dev, 4) || misaligned(dst_dev, 4) || misaligned(add_dev, 4)) return CQ_ERR_ALIGN;
+    if (k > CQ_DENSE_MATVEC_MAX_K || n > (1 << 24)) return CQ_ERR_RANGE;
+    const uint16_t *w = (const uint16_t *)w_dev;
+    hipStream_t s = (hipStream_t)stream;
+    if (prologue == CQ_DENSE_PLAIN) return matvec_launch<CQ_DENSE_PLAIN>(w, ldw, x_dev, vec_dev, eps, (int)dim, dst_dev, add_dev, accumulate, (int)n, (int)k, s);
+    if (prologue == CQ_DENSE_NORM) return matvec_launch<CQ_DENSE_NORM>(w, ldw, x_dev, vec_dev, eps, (int)dim, dst_dev, add_dev, accumulate, (int)n, (int)k, s);
+    return matvec_launch<CQ_DENSE_POLY>(w, ldw, x_dev, vec_dev, eps, (int)dim, dst_dev, add_dev, accumulate, (int)n, (int)k, s);
+}
+
+}  // extern "C"

@@ -141,6 +141,16 @@ __device__ __forceinline__ float wave_sum(float v) {
     return __builtin_bit_cast(float, __builtin_amdgcn_readlane(__builtin_bit_cast(int, v), 63));
 }
 
+__device__ __forceinline__ float row16_sum(float v) {      // sum over each aligned group of 16 lanes, in every lane
+#define CQ_ADD(ctrl) v += __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, v), ctrl, 0xf, 0xf, true))
+    CQ_ADD(CQ_DPP_QUAD_XOR1);
+    CQ_ADD(CQ_DPP_QUAD_XOR2);
+    CQ_ADD(CQ_DPP_ROW_HALF_MIRROR);
+    CQ_ADD(0x140);                                          // row_mirror
+#undef CQ_ADD
+    return v;
+}
+
 // wave64 maximum of any float, in every lane
 __device__ __forceinline__ float wave_max(float v) {
 #define CQ_MX(ctrl, rmask) v = fmaxf(v, __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(__builtin_bit_cast(int, v), __builtin_bit_cast(int, v), ctrl, rmask, 0xf, false)))

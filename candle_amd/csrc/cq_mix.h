@@ -1,0 +1,74 @@
+// Device helpers shared by the sequence-mixer kernels.
+#pragma once
+#include "cq_device.h"
+#include "../../include/candle_hip_mixer.h"
+
+inline bool mix_misaligned(const void *p, size_t a) { return (reinterpret_cast<uintptr_t>(p) & (a - 1)) != 0; }
+
+__device__ __forceinline__ float mix_sigmoid(float z) { return 1.0f / (1.0f + expf(-z)); }
+
+__device__ __forceinline__ f32x4 mfma4(float a, float b, f32x4 c) { return __builtin_amdgcn_mfma_f32_16x16x4f32(a, b, c, 0, 0, 0); }
+
+// 1 / root mean square of a head (one wave; lane takes dimensions lane, lane + 64, ...)
+__device__ __forceinline__ float head_inv_rms(const float *src, int dim, float eps, int lane) {
+    float s = 0.0f;
+    for (int d = lane; d < dim; d += 64) s = fmaf(src[d], src[d], s);
+    return 1.0f / sqrtf(wave_sum(s) / (float)dim + eps);
+}
+
+// Element d of a head after its norm (inv = 1 / rms, or 1 without a norm), rotation at position p and factor.
+__device__ __forceinline__ float head_value(const cq_mix_heads &g, const float *src, int d, float inv, int64_t p) {
+    auto val = [&](int i) { return g.norm_dev ? src[i] * inv * g.norm_dev[i] : src[i]; };
+    float v = val(d);
+    if (d < g.rot_dims) {
+        const int half = g.rot_dims >> 1;
+        const int i = d < half ? d : d - half;
+        const float c = g.cos_dev[p * half + i], s = g.sin_dev[p * half + i];
+        const float o = val(d < half ? d + half : i);
+        v = d < half ? v * c - o * s : v * c + o * s;
+    }
+    return v * g.factor;
+}
+
+// shapes and pointers of a group that a kernel will read (and write, unless `no_dst`)
+inline int mix_check_group(const cq_mix_heads &g, bool no_dst) {
+    if (g.heads <= 0 || g.dim <= 0 || g.src_off < 0 || g.rot_dims < 0 || g.rot_dims % 2 || g.rot_dims > g.dim) return CQ_ERR_SHAPE;
+    if (g.rot_dims && (!g.cos_dev || !g.sin_dev)) return CQ_ERR_NULL;
+    if (g.rot_dims && g.ctx <= 0) return CQ_ERR_SHAPE;
+    if (no_dst) return CQ_OK;
+    if (!g.dst_dev) return CQ_ERR_NULL;
+    if (g.dim_pad < g.dim || (g.by_position && g.ctx <= 0)) return CQ_ERR_SHAPE;
+    return CQ_OK;
+}
+
+// Keys that position p sees, in order: [0, keep) then [lo, p].
+struct Visible {
+    int keep, lo, n;
+};
+__host__ __device__ inline Visible visible_keys(int p, int window, int keep_first) {
+    Visible v;
+    v.lo = p >= window ? p - window + 1 : 0;
+    v.keep = keep_first < v.lo ? keep_first : v.lo;
+    v.n = v.keep + p - v.lo + 1;
+    return v;
+}
+
+// Split of a single token's visible keys over workgroups, and the record each leaves per head: acc[vdim], then m and l.
+__host__ __device__ inline int64_t talk_max_keys(int64_t window, int64_t keep_first, int64_t ctx) {
+    const int64_t n = keep_first > ctx - window ? ctx : window + keep_first;
+    return n < ctx ? n : ctx;
+}
+__host__ __device__ inline int talk_split_keys(int64_t max_keys) { return max_keys <= 4096 ? 16 : 64; }
+__host__ __device__ inline int talk_splits(int64_t max_keys) { return (int)((max_keys + talk_split_keys(max_keys) - 1) / talk_split_keys(max_keys)); }
+__host__ __device__ inline int talk_record(int vdim) { return (vdim + 3) / 4 * 4 + 4; }
+
+// max over each aligned group of 16 lanes, in every lane
+__device__ __forceinline__ float row16_max(float v) {
+#define CQ_MX(ctrl) v = fmaxf(v, __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, v), ctrl, 0xf, 0xf, true)))
+    CQ_MX(CQ_DPP_QUAD_XOR1);
+    CQ_MX(CQ_DPP_QUAD_XOR2);
+    CQ_MX(CQ_DPP_ROW_HALF_MIRROR);
+    CQ_MX(0x140);                                          // row_mirror
+#undef CQ_MX
+    return v;
+}

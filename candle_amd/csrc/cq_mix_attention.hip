@@ -1,0 +1,450 @@
+// Softmax attention whose scores are mixed across heads before the softmax, over a sliding window plus the first tokens of
+// the sequence.  Mixing couples the heads, so one workgroup holds the scores of all heads for its queries and keys.
+// f32 throughout (v_mfma_f32_16x16x4): scores, weights, caches.
+#include "cq_mix.h"
+
+namespace {
+
+// ---- several queries ------------------------------------------------------------------------------------------------------
+// Workgroup: 16 query rows x all heads, 8 waves, keys in tiles of KT, one pass with a running maximum.  Per tile:
+//   scores   wave w takes heads [w NHW, (w + 1) NHW): q k^T into LDS, [head][query][key]
+//   mixing   wave w takes queries 2 w and 2 w + 1 of every head: talk x scores on the matrix cores (heads are the contracted
+//            dimension), mask, running softmax in registers, weights back into the same LDS words, rescale factors to `alpha`
+//   values   wave w takes U units (head, 64 output columns): weights x V added to the outputs it holds in registers
+// blockIdx.y: units beyond 8 U (the scores are computed again there).
+// LDS strides: query rows of KT + 4 floats (16 rows x 4 keys of an operand read fall on 64 banks), head blocks of 16 rows + 16
+// (4 heads x 16 keys likewise).
+template <int NHW, bool SHARED_K, int U, int VS, int KT>
+__global__ __launch_bounds__(512) void talk_attention_kernel(const float *__restrict__ q, const float *__restrict__ k_cache, const float *__restrict__ v_cache,
+                                                             const float *__restrict__ talk, float scale, int window, int keep_first, float out_scale,
+                                                             float *__restrict__ out, int64_t out_stride, int pos, int rows, int H, int G, int dp, int vdim,
+                                                             int vp, int ctx) {
+    constexpr int NHT = NHW <= 2 ? 1 : NHW / 2, HP = 16 * NHT;           // heads padded to tiles of 16
+    constexpr int RS = KT + 4, HS = 16 * RS + 16, TS = HP + 4, KTL = KT / 16;
+    extern __shared__ __attribute__((aligned(16))) float smem[];
+    float *S = smem, *T = S + HP * HS, *alpha = T + HP * TS;
+    const int tid = threadIdx.x, lane = tid & 63, wv = __builtin_amdgcn_readfirstlane(tid >> 6), lr = lane & 15, lk = lane >> 4;
+    const int r0 = blockIdx.x * 16, nr = min(16, rows - r0);
+    const int p0 = pos + r0, last = p0 + nr - 1;                         // positions of the first and last query
+    const int R = H / G, nvc = (vp + 63) / 64;
+
+    for (int i = tid; i < HP * HP; i += 512) {
+        const int h = i / HP, g = i - h * HP;
+        T[h * TS + g] = h < H && g < H ? talk[h * H + g] * scale : 0.0f;
+    }
+    for (int i = tid; i < (HP - H) * HS; i += 512) S[H * HS + i] = 0.0f;
+
+    float m_run[2][NHT][4], l_run[2][NHT][4];
+#pragma unroll
+    for (int a = 0; a < 2; a++)
+#pragma unroll
+        for (int b = 0; b < NHT; b++)
+#pragma unroll
+            for (int e = 0; e < 4; e++) {
+                m_run[a][b][e] = -INFINITY;
+                l_run[a][b][e] = 0.0f;
+            }
+    f32x4 o[U][4];
+#pragma unroll
+    for (int u = 0; u < U; u++)
+#pragma unroll
+        for (int n = 0; n < 4; n++) o[u][n] = f32x4{0.f, 0.f, 0.f, 0.f};
+
+    const int h0 = wv * NHW;
+    const float *qrow = q + (int64_t)(r0 + min(lr, nr - 1)) * H * dp + 4 * lk;
+    const int u0 = ((int)blockIdx.y * 8 + wv) * U, n_units = H * nvc;
+
+    // tiles of the kept first tokens, then of the window
+    const int t_lo = max(0, p0 - window + 1) / KT, t_hi = last / KT;
+    const int n_keep = min((keep_first + KT - 1) / KT, t_lo);
+    for (int it = 0; it < n_keep + t_hi - t_lo + 1; it++) {
+        const int j0 = (it < n_keep ? it : t_lo + it - n_keep) * KT;
+        // ---- scores ----
+        if (h0 < H) {
+            f32x4 acc[NHW][KTL];
+#pragma unroll
+            for (int i = 0; i < NHW; i++)
+#pragma unroll
+                for (int t = 0; t < KTL; t++) acc[i][t] = f32x4{0.f, 0.f, 0.f, 0.f};
+            const float *krow[KTL];
+#pragma unroll
+            for (int t = 0; t < KTL; t++) krow[t] = k_cache + (int64_t)min(j0 + 16 * t + lr, last) * dp + 4 * lk;
+            const int64_t kv_stride = (int64_t)ctx * dp;
+            for (int c = 0; c < dp; c += 16) {
+                f32x4 kf[KTL], qf[NHW];
+                if (SHARED_K) {
+#pragma unroll
+                    for (int t = 0; t < KTL; t++) kf[t] = *reinterpret_cast<const f32x4 *>(krow[t] + (h0 / R) * kv_stride + c);
+                }
+#pragma unroll
+                for (int i = 0; i < NHW; i++) qf[i] = *reinterpret_cast<const f32x4 *>(qrow + min(h0 + i, H - 1) * dp + c);
+#pragma unroll
+                for (int i = 0; i < NHW; i++) {
+                    if (!SHARED_K) {
+#pragma unroll
+                        for (int t = 0; t < KTL; t++) kf[t] = *reinterpret_cast<const f32x4 *>(krow[t] + (min(h0 + i, H - 1) / R) * kv_stride + c);
+                    }
+#pragma unroll
+                    for (int e = 0; e < 4; e++)
+#pragma unroll
+                        for (int t = 0; t < KTL; t++) acc[i][t] = mfma4(qf[i][e], kf[t][e], acc[i][t]);
+                }
+            }
+#pragma unroll
+            for (int i = 0; i < NHW; i++)
+                if (h0 + i < H) {
+#pragma unroll
+                    for (int t = 0; t < KTL; t++)
+#pragma unroll
+                        for (int e = 0; e < 4; e++) S[(h0 + i) * HS + (4 * lk + e) * RS + 16 * t + lr] = acc[i][t][e];
+                }
+        }
+        __syncthreads();
+
+        // ---- mixing and softmax: queries 2 wv, 2 wv + 1, one after the other ----
+#pragma unroll
+        for (int a = 0; a < 2; a++) {
+            f32x4 acc[KTL][NHT];
+#pragma unroll
+            for (int t = 0; t < KTL; t++)
+#pragma unroll
+                for (int b = 0; b < NHT; b++) acc[t][b] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll 2
+            for (int s = 0; s < HP / 4; s++) {
+                float tf[NHT], sf[KTL];
+#pragma unroll
+                for (int b = 0; b < NHT; b++) tf[b] = T[(16 * b + lr) * TS + 4 * s + lk];
+#pragma unroll
+                for (int t = 0; t < KTL; t++) sf[t] = S[(4 * s + lk) * HS + (2 * wv + a) * RS + 16 * t + lr];
+#pragma unroll
+                for (int t = 0; t < KTL; t++)
+#pragma unroll
+                    for (int b = 0; b < NHT; b++) acc[t][b] = mfma4(tf[b], sf[t], acc[t][b]);
+            }
+            const int p = p0 + 2 * wv + a;
+            bool vis[KTL];
+#pragma unroll
+            for (int t = 0; t < KTL; t++) {
+                const int j = j0 + 16 * t + lr;
+                vis[t] = j <= p && (p - j < window || j < keep_first);
+            }
+#pragma unroll
+            for (int b = 0; b < NHT; b++)
+#pragma unroll
+                for (int e = 0; e < 4; e++) {
+                    float s[KTL], mx = -INFINITY, sum = 0.0f;
+#pragma unroll
+                    for (int t = 0; t < KTL; t++) {
+                        s[t] = vis[t] ? acc[t][b][e] : -INFINITY;
+                        mx = fmaxf(mx, s[t]);
+                    }
+                    const float m_old = m_run[a][b][e], m = fmaxf(m_old, row16_max(mx));
+                    const float al = m_old > -INFINITY ? __expf(m_old - m) : 0.0f;
+                    const int h = 16 * b + 4 * lk + e;
+#pragma unroll
+                    for (int t = 0; t < KTL; t++) {
+                        const float w = vis[t] ? __expf(s[t] - m) : 0.0f;
+                        sum += w;
+                        S[h * HS + (2 * wv + a) * RS + 16 * t + lr] = w;
+                    }
+                    m_run[a][b][e] = m;
+                    l_run[a][b][e] = l_run[a][b][e] * al + row16_sum(sum);
+                    if (lr == 0) alpha[h * 16 + 2 * wv + a] = al;
+                }
+        }
+        __syncthreads();
+
+        // ---- values ----
+#pragma unroll
+        for (int ub = 0; ub < U; ub += VS) {
+            if (u0 + ub < n_units) {
+                const int g = (u0 + ub) / (R * nvc), c = ((u0 + ub) / R) % nvc;
+#pragma unroll
+                for (int half = 0; half < KTL; half++) {
+                    float vf[4][4];
+#pragma unroll
+                    for (int s = 0; s < 4; s++) {
+                        const float *vr = v_cache + ((int64_t)g * ctx + min(j0 + 16 * half + 4 * s + lk, last)) * vp;
+#pragma unroll
+                        for (int n = 0; n < 4; n++) vf[s][n] = vr[min(64 * c + 16 * n + lr, vp - 1)];
+                    }
+#pragma unroll
+                    for (int v = 0; v < VS; v++) {
+                        const int u = ub + v;
+                        if (u0 + u < n_units) {
+                            const int h = g * R + (u0 + u) % R;
+                            if (half == 0) {
+                                const f32x4 al = *reinterpret_cast<const f32x4 *>(&alpha[h * 16 + 4 * lk]);
+#pragma unroll
+                                for (int n = 0; n < 4; n++) o[u][n] *= al;
+                            }
+#pragma unroll
+                            for (int s = 0; s < 4; s++) {
+                                const float w = S[h * HS + lr * RS + 16 * half + 4 * s + lk];
+#pragma unroll
+                                for (int n = 0; n < 4; n++) o[u][n] = mfma4(w, vf[s][n], o[u][n]);
+                            }
+                        }
+                    }
+                }
+            }
+        }
+        __syncthreads();
+    }
+#pragma unroll
+    for (int a = 0; a < 2; a++)
+#pragma unroll
+        for (int b = 0; b < NHT; b++)
+#pragma unroll
+            for (int e = 0; e < 4; e++)
+                if (lr == 0) alpha[(16 * b + 4 * lk + e) * 16 + 2 * wv + a] = l_run[a][b][e];
+    __syncthreads();
+#pragma unroll
+    for (int u = 0; u < U; u++) {
+        if (u0 + u >= n_units) continue;
+        const int g = (u0 + u) / (R * nvc), c = ((u0 + u) / R) % nvc, h = g * R + (u0 + u) % R;
+#pragma unroll
+        for (int n = 0; n < 4; n++) {
+            const int col = 64 * c + 16 * n + lr;
+            if (col >= vdim) continue;
+#pragma unroll
+            for (int e = 0; e < 4; e++) {
+                const int row = 4 * lk + e;
+                if (row < nr) out[(int64_t)(r0 + row) * out_stride + (int64_t)h * vdim + col] = out_scale * o[u][n][e] / alpha[h * 16 + row];
+            }
+        }
+    }
+}
+
+template <int NHW, bool SHARED_K, int U, int VS, int KT>
+int talk_launch(const float *q, const float *kc, const float *vc, const float *talk, float scale, int window, int keep, float out_scale, float *out,
+                int64_t out_stride, int pos, int rows, int H, int G, int dp, int vdim, int vp, int ctx, hipStream_t s) {
+    constexpr int HP = 16 * (NHW <= 2 ? 1 : NHW / 2);
+    constexpr size_t lds = (size_t)(HP * (16 * (KT + 4) + 16) + HP * (HP + 4) + HP * 16) * sizeof(float);
+    if (lds > 64 * 1024) {
+        const int e = (int)hipFuncSetAttribute(reinterpret_cast<const void *>(talk_attention_kernel<NHW, SHARED_K, U, VS, KT>),
+                                               hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+        if (e) return e;
+    }
+    const int units = H * ((vp + 63) / 64);
+    hipLaunchKernelGGL((talk_attention_kernel<NHW, SHARED_K, U, VS, KT>), dim3((rows + 15) / 16, (units + 8 * U - 1) / (8 * U)), dim3(512), lds, s, q, kc, vc,
+                       talk, scale, window, keep, out_scale, out, out_stride, pos, rows, H, G, dp, vdim, vp, ctx);
+    return (int)hipGetLastError();
+}
+
+// ---- one query --------------------------------------------------------------------------------------------------------------
+// Workgroup: KD of the visible keys x all heads, 8 waves.  It normalizes and rotates q itself; the workgroup that holds the
+// last visible key (the new token) first does the same for k and v and appends them to the caches.
+//   scores  16 lanes per (kv head, key), each key row read once for the heads that share it
+//   mixing  one thread per (head, key)
+//   values  one thread per (kv head, column), four heads at a time
+template <int NC, int KD>
+__global__ __launch_bounds__(512) void talk_decode_kernel(const float *__restrict__ row, cq_mix_heads gq, cq_mix_heads gk, cq_mix_heads gv, float eps,
+                                                          const float *__restrict__ talk, float scale, int window, int keep_first,
+                                                          const int32_t *__restrict__ pos_dev, int pos0, float *__restrict__ rec, int splits) {
+    extern __shared__ __attribute__((aligned(16))) float smem[];
+    const int H = gq.heads, G = gk.heads, R = H / G, dp = gk.dim_pad, vdim = gv.dim, ctx = gk.ctx;
+    constexpr int SS = KD + 1;
+    float *qs = smem, *sc = qs + H * dp, *mx = sc + H * SS;
+    const int tid = threadIdx.x, lane = tid & 63, wv = __builtin_amdgcn_readfirstlane(tid >> 6), sp = blockIdx.x;
+    const int p = pos0 + (pos_dev ? pos_dev[0] : 0);
+    const Visible vis = visible_keys(p, window, keep_first);
+    const int s0 = sp * KD, cnt = min(KD, vis.n - s0);
+    if (p >= ctx || cnt <= 0) return;                                // uniform: no key of this split is visible yet
+
+    for (int h = wv; h < H; h += 8) {
+        const float *s = row + gq.src_off + (int64_t)h * gq.dim;
+        const float inv = gq.norm_dev ? head_inv_rms(s, gq.dim, eps, lane) : 1.0f;
+        for (int d = lane; d < dp; d += 64) qs[h * dp + d] = d < gq.dim ? head_value(gq, s, d, inv, p) : 0.0f;
+    }
+    if (s0 + cnt == vis.n) {
+        for (int g = wv; g < 2 * G; g += 8) {
+            const cq_mix_heads &gr = g < G ? gk : gv;
+            const int hh = g < G ? g : g - G;
+            const float *s = row + gr.src_off + (int64_t)hh * gr.dim;
+            float *d = gr.dst_dev + hh * gr.dst_head_stride + (int64_t)p * gr.dst_row_stride;
+            const float inv = gr.norm_dev ? head_inv_rms(s, gr.dim, eps, lane) : 1.0f;
+            for (int i = lane; i < gr.dim_pad; i += 64) d[i] = i < gr.dim ? head_value(gr, s, i, inv, p) : 0.0f;
+        }
+        __threadfence_block();
+    }
+    __syncthreads();
+
+    auto key_of = [&](int j) {                                       // j-th key of the split, clamped to one that exists
+        const int s = s0 + min(j, cnt - 1);
+        return s < vis.keep ? s : vis.lo + s - vis.keep;
+    };
+    // ---- scores ----
+    {
+        constexpr int PB = 4;
+        const int sub = lane & 15, grp = wv * 4 + (lane >> 4), pairs = G * KD;
+        for (int b = grp; b < pairs; b += 32 * PB) {
+            f32x4 kd[PB][NC];
+#pragma unroll
+            for (int i = 0; i < PB; i++) {
+                const int pr = min(b + 32 * i, pairs - 1), g = pr / KD;
+                const float *kr = gk.dst_dev + g * gk.dst_head_stride + (int64_t)key_of(pr - g * KD) * gk.dst_row_stride;
+#pragma unroll
+                for (int c = 0; c < NC; c++) {
+                    const int d = 64 * c + 4 * sub;
+                    kd[i][c] = d < dp ? *reinterpret_cast<const f32x4 *>(kr + d) : f32x4{0.f, 0.f, 0.f, 0.f};
+                }
+            }
+#pragma unroll
+            for (int i = 0; i < PB; i++) {
+                const int pr = b + 32 * i, g = min(pr, pairs - 1) / KD;
+                for (int r = 0; r < R; r++) {
+                    const float *qh = qs + (g * R + r) * dp;
+                    float a = 0.0f;
+#pragma unroll
+                    for (int c = 0; c < NC; c++) {
+                        const int d = 64 * c + 4 * sub;
+                        const f32x4 qv = d < dp ? *reinterpret_cast<const f32x4 *>(qh + d) : f32x4{0.f, 0.f, 0.f, 0.f};
+                        a = fmaf(qv.x, kd[i][c].x, a);
+                        a = fmaf(qv.y, kd[i][c].y, a);
+                        a = fmaf(qv.z, kd[i][c].z, a);
+                        a = fmaf(qv.w, kd[i][c].w, a);
+                    }
+                    a = row16_sum(a);
+                    if (sub == 0 && pr < pairs) sc[(g * R + r) * SS + pr - g * KD] = a * scale;
+                }
+            }
+        }
+    }
+    __syncthreads();
+    // ---- mixing ----
+    for (int i = tid; i < H * KD; i += 512) {
+        const int h = i / KD, j = i - h * KD;
+        const float *t = talk + h * H;
+        float a0 = 0.0f, a1 = 0.0f;
+        int g = 0;
+        for (; g + 2 <= H; g += 2) {
+            a0 = fmaf(t[g], sc[g * SS + j], a0);
+            a1 = fmaf(t[g + 1], sc[(g + 1) * SS + j], a1);
+        }
+        if (g < H) a0 = fmaf(t[g], sc[g * SS + j], a0);
+        mx[h * SS + j] = j < cnt ? a0 + a1 : -INFINITY;
+    }
+    __syncthreads();
+    // ---- softmax of the split: 16 lanes per head ----
+    const int stride = talk_record(vdim);
+    for (int h = wv * 4 + (lane >> 4); h < (H + 3) / 4 * 4; h += 32) {
+        const int hh = min(h, H - 1);
+        float s[KD / 16], m = -INFINITY, l = 0.0f;
+#pragma unroll
+        for (int i = 0; i < KD / 16; i++) {
+            s[i] = mx[hh * SS + 16 * i + (lane & 15)];
+            m = fmaxf(m, s[i]);
+        }
+        m = row16_max(m);
+#pragma unroll
+        for (int i = 0; i < KD / 16; i++) {
+            s[i] = s[i] > -INFINITY ? __expf(s[i] - m) : 0.0f;
+            l += s[i];
+        }
+        l = row16_sum(l);
+        if (h < H) {
+#pragma unroll
+            for (int i = 0; i < KD / 16; i++) sc[h * SS + 16 * i + (lane & 15)] = s[i];
+            if ((lane & 15) == 0) {
+                float *r = rec + ((int64_t)h * splits + sp) * stride + stride - 4;
+                r[0] = m;
+                r[1] = l;
+            }
+        }
+    }
+    __syncthreads();
+    // ---- values ----
+    for (int i = tid; i < G * vdim; i += 512) {
+        const int g = i / vdim, e = i - g * vdim;
+        const float *vb = gv.dst_dev + g * gv.dst_head_stride + e;
+        for (int r = 0; r < R; r += 4) {
+            float a[4] = {0.f, 0.f, 0.f, 0.f};
+            for (int jb = 0; jb < KD; jb += 16) {
+                float vv[16];
+#pragma unroll
+                for (int j = 0; j < 16; j++) vv[j] = vb[(int64_t)key_of(jb + j) * gv.dst_row_stride];
+#pragma unroll
+                for (int j = 0; j < 16; j++)
+#pragma unroll
+                    for (int x = 0; x < 4; x++) a[x] = fmaf(sc[(g * R + min(r + x, R - 1)) * SS + jb + j], vv[j], a[x]);
+            }
+#pragma unroll
+            for (int x = 0; x < 4; x++)
+                if (r + x < R) rec[((int64_t)(g * R + r + x) * splits + sp) * stride + e] = a[x];
+        }
+    }
+}
+
+template <int NC, int KD>
+int talk_decode_launch(const float *row, const cq_mix_heads *g, float eps, const float *talk, float scale, int window, int keep, const int32_t *pos_dev, int pos,
+                       float *rec, int splits, hipStream_t s) {
+    const size_t lds = (size_t)g[0].heads * (g[1].dim_pad + 2 * (KD + 1)) * sizeof(float);
+    if (lds > 64 * 1024) {
+        const int e = (int)hipFuncSetAttribute(reinterpret_cast<const void *>(talk_decode_kernel<NC, KD>), hipFuncAttributeMaxDynamicSharedMemorySize,
+                                               160 * 1024);
+        if (e) return e;
+    }
+    hipLaunchKernelGGL((talk_decode_kernel<NC, KD>), dim3(splits), dim3(512), lds, s, row, g[0], g[1], g[2], eps, talk, scale, window, keep, pos_dev, pos, rec,
+                       splits);
+    return (int)hipGetLastError();
+}
+
+}  // namespace
+
+extern "C" {
+
+int cq_mix_talk_attention(const float *q_dev, const float *k_cache_dev, const float *v_cache_dev, const float *talk_dev, float scale, int64_t window,
+                          int64_t keep_first, float out_scale, float *out_dev, int64_t out_stride, int64_t pos, int64_t rows, int64_t n_head,
+                          int64_t n_kv_head, int64_t dim_pad, int64_t vdim, int64_t vdim_pad, int64_t ctx, void *stream) {
+    if (rows < 0 || pos < 0 || n_head <= 0 || n_kv_head <= 0 || n_head % n_kv_head || dim_pad <= 0 || dim_pad % 16 || vdim <= 0 || vdim_pad % 16 ||
+        vdim_pad < vdim || ctx <= 0 || window < 1 || keep_first < 0 || out_stride < n_head * vdim)
+        return CQ_ERR_SHAPE;
+    if (rows == 0) return CQ_OK;
+    if (!q_dev || !k_cache_dev || !v_cache_dev || !talk_dev || !out_dev) return CQ_ERR_NULL;
+    if (mix_misaligned(q_dev, 16) || mix_misaligned(k_cache_dev, 16) || mix_misaligned(v_cache_dev, 16)) return CQ_ERR_ALIGN;
+    if (pos + rows > ctx || ctx > (1 << 28) || n_head > CQ_MIX_MAX_HEADS || dim_pad > CQ_MIX_MAX_DIM || vdim_pad > CQ_MIX_MAX_DIM) return CQ_ERR_RANGE;
+    const int w = (int)(window < ctx ? window : ctx), keep = (int)(keep_first < ctx ? keep_first : ctx);
+    const int H = (int)n_head, G = (int)n_kv_head, R = H / G;
+    hipStream_t s = (hipStream_t)stream;
+#define CQ_TA(NHW_, SH_, U_, VS_, KT_)                                                                                                                \
+    talk_launch<NHW_, SH_, U_, VS_, KT_>(q_dev, k_cache_dev, v_cache_dev, talk_dev, scale, w, keep, out_scale, out_dev, out_stride, (int)pos, (int)rows, H, G, \
+                                         (int)dim_pad, (int)vdim, (int)vdim_pad, (int)ctx, s)
+    if (H <= 8) return R % 2 ? CQ_TA(1, true, 2, 1, 32) : CQ_TA(1, true, 2, 2, 32);
+    if (H <= 16) return R % 2 ? CQ_TA(2, false, 2, 1, 32) : CQ_TA(2, true, 2, 2, 32);
+    if (H <= 32) return R % 4 ? CQ_TA(4, false, 8, 1, 32) : CQ_TA(4, true, 8, 4, 32);
+    return R % 8 ? (R % 4 ? CQ_TA(8, false, 8, 1, 16) : CQ_TA(8, false, 8, 4, 16)) : CQ_TA(8, true, 8, 4, 16);
+#undef CQ_TA
+}
+
+int64_t cq_mix_talk_decode_workspace_bytes(int64_t n_head, int64_t vdim, int64_t window, int64_t keep_first, int64_t ctx) {
+    if (n_head <= 0 || vdim <= 0 || window < 1 || keep_first < 0 || ctx <= 0) return -1;
+    return n_head * talk_splits(talk_max_keys(window, keep_first, ctx)) * talk_record((int)vdim) * 4;
+}
+
+int cq_mix_talk_decode(const float *row_dev, const cq_mix_heads *qkv, float eps, const float *talk_dev, float scale, int64_t window, int64_t keep_first,
+                       const int32_t *pos_dev, int64_t pos, void *workspace_dev, int64_t workspace_bytes, void *stream) {
+    if (!row_dev || !qkv || !talk_dev || !workspace_dev) return CQ_ERR_NULL;
+    const cq_mix_heads &q = qkv[0], &k = qkv[1], &v = qkv[2];
+    for (int i = 0; i < 3; i++) {
+        const int e = mix_check_group(qkv[i], i == 0);
+        if (e) return e;
+    }
+    if (q.heads % k.heads || v.heads != k.heads || q.dim != k.dim || !k.by_position || !v.by_position || k.ctx != v.ctx || k.dim_pad % 16 || v.dim_pad % 16 ||
+        window < 1 || keep_first < 0 || pos < 0 || k.dst_row_stride % 4 || k.dst_head_stride % 4)
+        return CQ_ERR_SHAPE;
+    if (mix_misaligned(k.dst_dev, 16)) return CQ_ERR_ALIGN;
+    if (q.heads > CQ_MIX_MAX_HEADS || k.dim_pad > CQ_MIX_MAX_DIM || v.dim_pad > CQ_MIX_MAX_DIM || k.ctx > (1 << 28) || (!pos_dev && pos >= k.ctx)) return CQ_ERR_RANGE;
+    const int64_t n_max = talk_max_keys(window, keep_first, k.ctx);
+    if (workspace_bytes < cq_mix_talk_decode_workspace_bytes(q.heads, v.dim, window, keep_first, k.ctx)) return CQ_ERR_WORKSPACE;
+    const int w = (int)(window < k.ctx ? window : k.ctx), keep = (int)(keep_first < k.ctx ? keep_first : k.ctx), splits = talk_splits(n_max);
+    hipStream_t s = (hipStream_t)stream;
+#define CQ_TD(NC_, KD_) talk_decode_launch<NC_, KD_>(row_dev, qkv, eps, talk_dev, scale, w, keep, pos_dev, (int)pos, (float *)workspace_dev, splits, s)
+    const bool fine = talk_split_keys(n_max) == 16;
+    if (k.dim_pad <= 64) return fine ? CQ_TD(1, 16) : CQ_TD(1, 64);
+    if (k.dim_pad <= 128) return fine ? CQ_TD(2, 16) : CQ_TD(2, 64);
+    return fine ? CQ_TD(4, 16) : CQ_TD(4, 64);
+#undef CQ_TD
+}
+
+}  // extern "C"

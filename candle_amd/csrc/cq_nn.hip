@@ -146,16 +146,6 @@ constexpr int ATT_SPLIT = 128;
 constexpr int CQ_ATTN_MFMA_MIN = 64;         // query rows from which attn_mfma_kernel is used (head_dim 128)
 constexpr int CQ_ATTN_ROWS_MIN = 16;        // query rows from which a workgroup takes several rows (attn_rows_kernel)
 
-__device__ __forceinline__ float row16_sum(float v) {      // sum over each aligned group of 16 lanes, in every lane
-#define CQ_ADD(ctrl) v += __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, v), ctrl, 0xf, 0xf, true))
-    CQ_ADD(CQ_DPP_QUAD_XOR1);
-    CQ_ADD(CQ_DPP_QUAD_XOR2);
-    CQ_ADD(CQ_DPP_ROW_HALF_MIRROR);
-    CQ_ADD(0x140);                                          // row_mirror
-#undef CQ_ADD
-    return v;
-}
-
 template <int HD, int G>
 __global__ __launch_bounds__(256) void attn_kernel(const float *__restrict__ q, int64_t q_stride, const float *__restrict__ k_cache,
                                                    const float *__restrict__ v_cache, float *__restrict__ out, float *__restrict__ part,

@@ -17,13 +17,14 @@ from __future__ import annotations
 
 import dataclasses
 import math
-import time
-from typing import Dict, List, Optional, Sequence
+from typing import Dict, List, Optional
 
 import numpy as np
 import torch
 
 from . import _lib
+from .cache import SequenceCache
+from .generation import GreedyDecoder
 from .quantized import GgmlDType, QStorage, QTensor, _MATMUL_DTYPES
 
 
@@ -87,7 +88,7 @@ class LayerWeights:
         self.prefetch_span = 0       # bytes from attention_wo to the end of this layer's weights
 
 
-class ModelWeights:
+class ModelWeights(GreedyDecoder):
     """quantized_llama::ModelWeights for one GPU.  Build with ``random_init`` or ``from_blocks``."""
 
     def __init__(self, cfg: Config, device="cuda:0"):
@@ -151,22 +152,16 @@ class ModelWeights:
                 self.output = w
             else:
                 self.layers[li].w[name] = w
-        f32 = dict(dtype=torch.float32, device=self.device)
+        self.cache = SequenceCache(self.device)
         for lw in self.layers:
             w2 = lw.w["feed_forward_w2"]
             lw.prefetch_span = (w2.ptr + w2.nbytes - lw.w["attention_wo"].ptr) // 16 * 16
-            lw.k_cache = torch.zeros((cfg.n_kv_head, cfg.ctx, cfg.head_dim), **f32)
-            lw.v_cache = torch.zeros((cfg.n_kv_head, cfg.ctx, cfg.head_dim), **f32)
+            lw.k_cache, lw.v_cache = self.cache.add_kv(cfg.n_kv_head, cfg.ctx, cfg.head_dim, cfg.head_dim)
         cos, sin = precomput_freqs_cis(cfg.head_dim, cfg.rope_theta, cfg.ctx)
         self.cos = torch.from_numpy(cos).to(self.device)
         self.sin = torch.from_numpy(sin).to(self.device)
         self._alloc_activations(max_rows=1)
-        # device-side decode state for graph replay
-        self.token_dev = torch.zeros(1, dtype=torch.int32, device=self.device)
-        self.pos_dev = torch.zeros(1, dtype=torch.int32, device=self.device)
-        self.counter_dev = torch.zeros(1, dtype=torch.int32, device=self.device)
-        self.history_dev = torch.zeros(cfg.ctx, dtype=torch.int32, device=self.device)
-        self.argmax_ws = torch.zeros(1024, dtype=torch.uint8, device=self.device)      # CQ_NN_ARGMAX_WORKSPACE
+        self._init_greedy(cfg.ctx)         # device-side decode state for graph replay
         return plan
 
     def _alloc_activations(self, max_rows: int):
@@ -324,6 +319,7 @@ class ModelWeights:
 
     def clear_kv_cache(self):
         """quantized_llama.rs:558-566 — with a preallocated cache only the position matters."""
+        self.cache.reset()
         self.pos_dev.zero_()
 
     # ------------------------------------------------------------------------------------------ forward
@@ -573,15 +569,13 @@ class ModelWeights:
     def _argmax_dev(self, logits_ptr: int, embed: bool, sp) -> None:
         """Sampling::ArgMax into token_dev / history_dev, the position advanced; with `embed` the chosen token's embedding row
         and its partial sums of squares go to self.x / self.partials in the same launch."""
+        if not embed:
+            return super()._argmax_dev(logits_ptr, embed, sp)
         L, cfg = self.L, self.cfg
-        if embed:
-            _lib.check("cq_nn_argmax_embed", L.cq_nn_argmax_embed(logits_ptr, cfg.vocab, self.token_dev.data_ptr(), self.history_dev.data_ptr(),
-                                                                 self.counter_dev.data_ptr(), self.pos_dev.data_ptr(), self.argmax_ws.data_ptr(),
-                                                                 self.tok_embeddings.data_ptr(), self.x.data_ptr(), cfg.hidden, cfg.vocab,
-                                                                 self.partials.data_ptr(), sp))
-        else:
-            _lib.check("cq_nn_argmax", L.cq_nn_argmax(logits_ptr, cfg.vocab, self.token_dev.data_ptr(), self.history_dev.data_ptr(),
-                                                     self.counter_dev.data_ptr(), self.pos_dev.data_ptr(), self.argmax_ws.data_ptr(), sp))
+        _lib.check("cq_nn_argmax_embed", L.cq_nn_argmax_embed(logits_ptr, cfg.vocab, self.token_dev.data_ptr(), self.history_dev.data_ptr(),
+                                                             self.counter_dev.data_ptr(), self.pos_dev.data_ptr(), self.argmax_ws.data_ptr(),
+                                                             self.tok_embeddings.data_ptr(), self.x.data_ptr(), cfg.hidden, cfg.vocab,
+                                                             self.partials.data_ptr(), sp))
 
     def _decode_step_dev(self, max_kv_len: int, sp) -> None:
         """One greedy step driven entirely from device state: token_dev at position pos_dev -> next token_dev, pos_dev + 1.
@@ -590,65 +584,16 @@ class ModelWeights:
         self._enqueue(None if chain else self.token_dev.data_ptr(), 1, 0, self.pos_dev.data_ptr(), max_kv_len, sp)
         self._argmax_dev(self.logits.data_ptr(), chain, sp)
 
-    def generate_greedy(self, prompt: Sequence[int], n_new: int, use_graph: bool = True, max_kv: Optional[int] = None) -> dict:
-        """The loop of candle-examples/examples/quantized/main.rs:616-690 with temperature <= 0 (Sampling::ArgMax):
-        prefill the prompt in one forward, pick the arg-max token, then n_new - 1 single-token steps.
-        Returns the generated tokens and the wall-clock split prompt / decode, as the example prints them.
-        max_kv: the number of cache positions the captured step is laid out for (its attention split count follows from
-        it); by default exactly prompt + n_new, a server that captures one step for every request passes the context."""
-        cfg = self.cfg
-        prompt = [int(t) for t in prompt]
-        if len(prompt) + n_new > cfg.ctx:
-            raise ValueError("prompt + generated tokens exceed the context")
-        if max_kv is not None and not len(prompt) + n_new <= max_kv <= cfg.ctx:
-            raise ValueError("max_kv must cover prompt + generated tokens and fit the context")
-        dev = self.device
-        torch.cuda.synchronize(dev)
-        t0 = time.perf_counter()
-        logits = self.forward(torch.tensor([prompt], dtype=torch.int32, device=dev), 0)
-        stream = torch.cuda.current_stream(dev)
-        self.counter_dev.zero_()
-        self.pos_dev.fill_(len(prompt) - 1)       # argmax advances it to the position of the token it emits
-        steps = n_new - 1
-        if max_kv is None:
-            max_kv = len(prompt) + n_new
-        self._argmax_dev(logits.data_ptr(), steps > 0 and self._chain_embedding(max_kv), stream.cuda_stream)
-        torch.cuda.synchronize(dev)
-        t1 = time.perf_counter()
-        prompt_seconds = t1 - t0
-        if steps > 0:
-            if use_graph:
-                key = max_kv
-                if self._graph is None or self._graph_key != key:
-                    side = torch.cuda.Stream(device=dev)
-                    # capture must not disturb the live decode state: save and restore it around the warm-up run
-                    saved = (self.token_dev.clone(), self.pos_dev.clone(), self.counter_dev.clone(), self.x[:1].clone(), self.partials.clone())
-                    with torch.cuda.stream(side):
-                        self._decode_step_dev(max_kv, side.cuda_stream)
-                        side.synchronize()
-                        g = torch.cuda.CUDAGraph()
-                        with torch.cuda.graph(g, stream=side):
-                            self._decode_step_dev(max_kv, torch.cuda.current_stream(dev).cuda_stream)
-                    torch.cuda.synchronize(dev)
-                    self.token_dev.copy_(saved[0]); self.pos_dev.copy_(saved[1]); self.counter_dev.copy_(saved[2])
-                    self.x[:1].copy_(saved[3]); self.partials.copy_(saved[4])
-                    torch.cuda.synchronize(dev)
-                    self._graph, self._graph_key = g, key
-                t1 = time.perf_counter()
-                for _ in range(steps):
-                    self._graph.replay()
-            else:
-                for _ in range(steps):
-                    self._decode_step_dev(max_kv, stream.cuda_stream)
-        torch.cuda.synchronize(dev)
-        t2 = time.perf_counter()
-        if self.coop and self.coop_error():
-            # a cooperative launch gave up waiting for workgroups that were not running (a shared GPU): its tokens are invalid.
-            # The whole generation again through the chains of launches, which this model then keeps to.
-            import warnings
-            warnings.warn("a cooperative decode launch timed out; falling back to one launch per matvec")
-            self.coop = False
-            self._graph = None
-            return self.generate_greedy(prompt, n_new, use_graph)
-        tokens = self.history_dev[:n_new].cpu().tolist()
-        return {"tokens": tokens, "prompt_seconds": prompt_seconds, "decode_seconds": t2 - t1, "decode_steps": steps}
+    def _step_state(self):
+        return [self.token_dev, self.pos_dev, self.counter_dev, self.x[:1], self.partials]
+
+    def _steps_failed(self) -> bool:
+        if not (self.coop and self.coop_error()):
+            return False
+        # a cooperative launch gave up waiting for workgroups that were not running (a shared GPU): its tokens are invalid.
+        # The whole generation again through the chains of launches, which this model then keeps to.
+        import warnings
+        warnings.warn("a cooperative decode launch timed out; falling back to one launch per matvec")
+        self.coop = False
+        self._graph = None
+        return True

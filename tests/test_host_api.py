@@ -13,9 +13,9 @@ from candle_amd.quantized import GgmlDType, check_shape
 ROOT = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
 
 
-def declared_symbols():
+def declared_symbols(headers=("candle_hip_nn.h", "candle_hip_quant.h")):
     inc = os.path.join(ROOT, "include")
-    text = "".join(open(os.path.join(inc, f)).read() for f in sorted(os.listdir(inc)) if f.endswith(".h"))
+    text = "".join(open(os.path.join(inc, f)).read() for f in headers)
     text = re.sub(r"/\*.*?\*/", "", text, flags=re.S)
     return sorted(set(re.findall(r"\b(cq_[a-z0-9_]+)\s*\(", text)))
 
@@ -27,6 +27,15 @@ def test_library_exports_every_declared_symbol():
     for name in names:
         assert hasattr(L, name), f"{name} declared under include/ but not exported"
     assert set(names) == set(_lib.SIGNATURES), "ctypes signatures out of sync with the header"
+
+
+def test_mixer_library_exports_every_declared_symbol():
+    L = _lib.mixer_lib()
+    names = declared_symbols(("candle_hip_mixer.h",))
+    assert len(names) >= 15 and set(names) == set(_lib.MIXER_SIGNATURES)
+    for name in names + list(_lib._MIXER_GLUE):
+        assert hasattr(L, name), f"{name} declared in candle_hip_mixer.h but not exported"
+    assert sorted(os.listdir(os.path.join(ROOT, "include"))) == ["candle_hip_mixer.h", "candle_hip_nn.h", "candle_hip_quant.h"]
 
 
 def test_dtype_sizes_match_reference_and_oracle():
