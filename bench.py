@@ -40,6 +40,9 @@ The JSON line carries, besides the driver contract fields:
     python bench.py --workload decode8b [--steps 256] [--prompt 512]
                                    the 8B-shape Q4_K_M decoder: prompt and decode tok/s against the weight-streaming
                                    roofline (8 TB/s / weight bytes per token)
+    python bench.py --workload venizen [--steps 128] [--prompt 2048]
+                                   Venizen decoders at two sizes (random bf16 weights): prompt and decode tok/s, each beside
+                                   the Q4_K_M llama decoder of the same width, depth and feed-forward
 """
 import argparse
 import json
@@ -332,6 +335,63 @@ def decode8b(args):
     return out
 
 
+def venizen_config(width, vocab, ctx):
+    """Eight layer runs from six layers (two of them repeated once), heads of 128 / 64, a window of 1024."""
+    heads, ff = width // 128, width * 7 // 2
+    parallel = {"type": "parallel",
+                "mixer": {"left": {"heads": heads, "kv_heads": max(1, heads // 4), "dim": 128, "vdim": 128, "scale": 128 ** -0.5, "mask": {"size": 1024, "keep_first": 4},
+                                   "rot": {"base": 500000.0, "dims": 128}},
+                          "right": {"heads": heads // 2, "dim": 128, "vdim": 128, "rot": {"base": 10000.0, "dims": 128},
+                                    "decay": [1.0 - 2.0 ** -(5 + 5.0 * h / max(1, heads // 2 - 1)) for h in range(heads // 2)]},
+                          "left_scale": 1.0, "right_scale": 1.0},
+                "mlp": {"kind": "dense", "ff": ff}}
+    delta = {"type": "general_delta", "mixer": {"heads": width // 64, "dim": 64}, "mlp": None}
+    return {"vocab": vocab, "width": width, "norm": {"eps": 1e-5}, "layers": [parallel, delta, parallel, delta, parallel, delta],
+            "loop": {"start": 2, "stop": 4, "times": 2}}
+
+
+def venizen(args):
+    """Prompt and decode throughput of Venizen decoders at two widths, and of the Q4_K_M llama decoder of equal size."""
+    import torch
+
+    from candle_amd import quantized_llama as ql
+    from candle_amd import venizen as vz
+
+    n_new = args.steps if args.steps else 128
+    gen = torch.Generator()
+    gen.manual_seed(99)
+    ctx, vocab, records = args.prompt + n_new + 8, 32768, []
+    for width in (2048, 4096):
+        d = venizen_config(width, vocab, ctx)
+        cfg = vz.Config.from_dict(d, ctx)
+        prompt = torch.randint(0, vocab, (args.prompt,), generator=gen).tolist()
+        lcfg = ql.Config(n_layer=len(cfg.order), hidden=width, n_head=width // 128, n_kv_head=max(1, width // 512), head_dim=128, ffn=width * 7 // 2, vocab=vocab, ctx=ctx)
+        rec = {"width": width, "layer_runs": len(cfg.order), "ff": width * 7 // 2, "prompt": args.prompt}
+        for name, make in (("venizen_bf16", lambda: vz.Model.random_init(cfg, seed=7)), ("llama_q4_k_m", lambda: ql.ModelWeights.random_init(lcfg, seed=7))):
+            model = make()
+            model.generate_greedy(prompt, 8)
+            best = None
+            for _ in range(3):
+                r = model.generate_greedy(prompt, n_new, max_kv=ctx)
+                best = r if best is None or r["decode_seconds"] < best["decode_seconds"] else best
+                best["prompt_seconds"] = min(best["prompt_seconds"], r["prompt_seconds"])
+            tok_s, wbytes = best["decode_steps"] / best["decode_seconds"], model.weight_bytes_per_token()
+            rec[name] = {"prompt_tok_s": round(args.prompt / best["prompt_seconds"], 1), "decode_tok_s": round(tok_s, 1), "weight_bytes_per_token": wbytes,
+                         "decode_frac_of_weight_roofline": round(tok_s * wbytes / 1e9 / HBM_PEAK_GBPS, 4)}
+            if name == "venizen_bf16":
+                flop = 2.0 * sum(w.numel() for la in [model.layers[i] for i, _ in cfg.order]
+                                 for w in [x.w for x in la.mixer.denses() + (la.mlp.denses() if la.mlp else [])])
+                rec[name]["prompt_matmul_TFLOPs"] = round(flop * args.prompt / best["prompt_seconds"] / 1e12, 1)
+            del model
+            torch.cuda.empty_cache()
+        records.append(rec)
+    big = records[-1]["venizen_bf16"]
+    return {"metric": "Venizen decode tok/s (batch 1, greedy, width 4096)", "value": big["decode_tok_s"], "unit": "tok/s", "n_gpus": 1, "steps": n_new - 1, "warmup": 8,
+            "ms_per_step": round(1e3 / big["decode_tok_s"], 4), "higher_is_better": True, "scaling": "weak", "vs_baseline": None, "dtype": "bf16", "data": "synthetic",
+            "config": {"workload": "random-init weights, 8 layer runs, vocab %d, %d prompt tokens, then %d greedy steps from one HIP graph" % (vocab, args.prompt, n_new - 1)},
+            "results": records}
+
+
 def moe(args):
     """Qwen3-30B-A3B-shaped MoE layer stack (48 layers, 128 experts, top-8, hidden 2048, expert FFN 768, Q4_K,
     16 GB of expert weights, every layer with weights of its own): the three expert matmuls of each layer (gate, up on
@@ -492,9 +552,9 @@ def main():
     ap.add_argument("--gpus", type=int, default=1)
     ap.add_argument("--steps", type=int, default=None)
     ap.add_argument("--warmup", type=int, default=None)
-    ap.add_argument("--workload", choices=["decode", "prefill", "decode8b", "moe"], default="decode")
+    ap.add_argument("--workload", choices=["decode", "prefill", "decode8b", "moe", "venizen"], default="decode")
     ap.add_argument("--layers", type=int, default=32, help="--workload decode8b: number of decoder layers")
-    ap.add_argument("--prompt", type=int, default=512, help="--workload decode8b: prompt tokens")
+    ap.add_argument("--prompt", type=int, default=512, help="--workload decode8b / venizen: prompt tokens")
     ap.add_argument("--moe-tokens", default="1,16,256", help="--workload moe: token counts, comma separated")
     ap.add_argument("--moe-layers", type=int, default=48, help="--workload moe: layers, each with its own expert weights (340 MB per layer)")
     ap.add_argument("--wdtype", choices=sorted(WDTYPES), default="q4k",
@@ -515,6 +575,9 @@ def main():
         return
     if args.workload == "moe":
         print(json.dumps(moe(args)))
+        return
+    if args.workload == "venizen":
+        print(json.dumps(venizen(args)))
         return
     if args.steps is None:
         args.steps = 4000 if args.workload == "decode" else 50

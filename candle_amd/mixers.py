@@ -144,7 +144,7 @@ class TalkingAttention:
         if self.heads % self.kv_heads:
             raise ValueError("heads must be a multiple of kv_heads")
         self.scale = float(cfg["scale"])
-        mask = cfg["mask"]
+        mask = cfg.get("mask") or {"size": rt.ctx}   # no mask: every earlier key
         self.window, self.keep_first = int(mask["size"]), int(mask.get("keep_first", 0))
         self.rot = Rotation(rt, cfg.get("rot"))
         self.dp, self.vp = pad_to(self.dim, 16), pad_to(self.vdim, 16)
@@ -195,7 +195,8 @@ class Retention:
         if decay.shape != (self.heads,):
             raise ValueError("one decay per head")
         self.decay = rt.vector(torch.from_numpy(decay))
-        self.log2_decay = rt.vector(torch.from_numpy(np.log2(decay)))
+        with np.errstate(divide="ignore"):           # a decay of 0: finite, so that gamma^0 stays 1
+            self.log2_decay = rt.vector(torch.from_numpy(np.maximum(np.log2(decay), -1e30)))
         self.rot = Rotation(rt, cfg.get("rot"))
         self.dp = pad_to(self.dim, 16)
         self.projections = [get("q"), get("k"), get("v"), get("g")]

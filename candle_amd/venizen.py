@@ -8,7 +8,7 @@ from __future__ import annotations
 import dataclasses
 import json
 import os
-from typing import Callable, List, Optional, Sequence
+from typing import Callable, Dict, List, Optional, Sequence
 
 import torch
 
@@ -48,6 +48,31 @@ class Config:
             if layer.get("mlp") and layer["mlp"]["kind"] not in mixers.FEED_FORWARDS:
                 raise ValueError(f"layer {i}: unknown feed-forward {layer['mlp']['kind']!r}")
         return Config(vocab=int(d["vocab"]), width=int(d["width"]), eps=float(d["norm"]["eps"]), layers=layers, order=order, ctx=int(ctx))
+
+
+def tensor_shapes(cfg: Config) -> Dict[str, tuple]:
+    """{name: shape} of the checkpoint a configuration describes.  The rank of a delta mixer's decay is the tensors' own choice: a quarter of
+    its head size here, at least 16."""
+    w = cfg.width
+    out = {"embed": (cfg.vocab, w), "final.norm": (w,), "head": (cfg.vocab, w)}
+    for i, layer in enumerate(cfg.layers):
+        pre, m = f"l{i}.", layer["mixer"]
+        out[pre + "norm1"] = (w,)
+        if layer["type"] == "parallel":
+            a, r = m["left"], m["right"]
+            H, G, d, e = a["heads"], a["kv_heads"], a["dim"], a["vdim"]
+            out.update({pre + "mix.left." + n: s for n, s in (("q", (H * d, w)), ("k", (G * d, w)), ("v", (G * e, w)), ("q.norm", (d,)), ("k.norm", (d,)),
+                                                              ("talk", (H, H)), ("o", (w, H * e)))})
+            d, e = r["heads"] * r["dim"], r["heads"] * r["vdim"]
+            out.update({pre + "mix.right." + n: s for n, s in (("q", (d, w)), ("k", (d, w)), ("v", (e, w)), ("g", (e, w)), ("o", (w, e)))})
+        else:
+            d, rank = m["heads"] * m["dim"], max(16, m["dim"] // 4)
+            out.update({pre + "mix." + n: (d, w) for n in "rkvga"})
+            out.update({pre + "mix." + n: s for n, s in (("a.b", (d,)), ("w0", (d,)), ("norm", (d,)), ("w1", (rank, w)), ("w2", (d, rank)), ("o", (w, d)))})
+        if layer.get("mlp"):
+            ff = layer["mlp"]["ff"]
+            out.update({pre + "norm2": (w,), pre + "mlp.up": (ff, w), pre + "mlp.down": (w, ff), pre + "mlp.act": (4,)})
+    return out
 
 
 class Layer:
@@ -94,6 +119,23 @@ class Model(GreedyDecoder):
         with open(os.path.join(path, "config.json")) as f:
             cfg = Config.from_dict(json.load(f), ctx)
         return cls(cfg, SafetensorsFile(os.path.join(path, "model.safetensors")).tensor, device, dtype)
+
+    @classmethod
+    def random_init(cls, cfg: Config, seed: int = 0, device="cuda:0", dtype: str = "bfloat16") -> "Model":
+        """Random weights of the configured shapes, made on the device (benchmarks)."""
+        gen = torch.Generator(device=device)
+        gen.manual_seed(seed)
+        shapes = tensor_shapes(cfg)
+
+        def get(name: str) -> torch.Tensor:
+            shape = shapes[name]
+            if name.endswith("act"):
+                return torch.tensor([0.7, 0.2, 0.1, 0.0], device=device)
+            if len(shape) == 1:
+                return torch.ones(shape, device=device)
+            std = 1.0 if name == "embed" else shape[-1] ** -0.5
+            return (torch.randn(shape, generator=gen, device=device) * std).to(torch.bfloat16)
+        return cls(cfg, get, device, dtype)
 
     def denses(self) -> List[Dense]:
         out = [self.head]
