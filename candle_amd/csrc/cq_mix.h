@@ -16,23 +16,50 @@ __device__ __forceinline__ float head_inv_rms(const float *src, int dim, float e
     return 1.0f / sqrtf(wave_sum(s) / (float)dim + eps);
 }
 
-// Element d of a head after its norm (inv = 1 / rms, or 1 without a norm), rotation at position p and factor.
-__device__ __forceinline__ float head_value(const cq_mix_heads &g, const float *src, int d, float inv, int64_t p) {
-    auto val = [&](int i) { return g.norm_dev ? src[i] * inv * g.norm_dev[i] : src[i]; };
-    float v = val(d);
-    if (d < g.rot_dims) {
+// One head of a group in the registers of a wave (lane: dimensions lane + 64 e): everything it needs is requested by load(), so
+// that the norm's reduction is not followed by a second trip to memory.
+template <int NE>
+struct HeadRegs {
+    float v[NE], o[NE], wv[NE], wo[NE], c[NE], s[NE];
+
+    __device__ __forceinline__ void load(const cq_mix_heads &g, const float *src, int64_t p, int lane) {
         const int half = g.rot_dims >> 1;
-        const int i = d < half ? d : d - half;
-        const float c = g.cos_dev[p * half + i], s = g.sin_dev[p * half + i];
-        const float o = val(d < half ? d + half : i);
-        v = d < half ? v * c - o * s : v * c + o * s;
+#pragma unroll
+        for (int e = 0; e < NE; e++) {
+            const int d = lane + 64 * e;
+            const bool ok = d < g.dim, rot = d < g.rot_dims;
+            const int i = d < half ? d : d - half, other = d < half ? d + half : d - half;
+            v[e] = ok ? src[d] : 0.0f;
+            wv[e] = ok && g.norm_dev ? g.norm_dev[d] : 1.0f;
+            o[e] = rot ? src[other] : 0.0f;
+            wo[e] = rot && g.norm_dev ? g.norm_dev[other] : 1.0f;
+            c[e] = rot ? g.cos_dev[p * half + i] : 1.0f;
+            s[e] = rot ? g.sin_dev[p * half + i] : 0.0f;
+        }
     }
-    return v * g.factor;
-}
+    // the values after norm, rotation and factor, in place of v (zero beyond dim)
+    __device__ __forceinline__ void finish(const cq_mix_heads &g, float eps, int lane) {
+        float inv = 1.0f;
+        if (g.norm_dev) {
+            float q = 0.0f;
+#pragma unroll
+            for (int e = 0; e < NE; e++) q = fmaf(v[e], v[e], q);
+            inv = 1.0f / sqrtf(wave_sum(q) / (float)g.dim + eps);
+        }
+        const int half = g.rot_dims >> 1;
+#pragma unroll
+        for (int e = 0; e < NE; e++) {
+            const int d = lane + 64 * e;
+            const float a = v[e] * inv * wv[e], b = o[e] * inv * wo[e];
+            v[e] = (d < half ? a * c[e] - b * s[e] : a * c[e] + b * s[e]) * g.factor;
+        }
+    }
+};
 
 // shapes and pointers of a group that a kernel will read (and write, unless `no_dst`)
 inline int mix_check_group(const cq_mix_heads &g, bool no_dst) {
     if (g.heads <= 0 || g.dim <= 0 || g.src_off < 0 || g.rot_dims < 0 || g.rot_dims % 2 || g.rot_dims > g.dim) return CQ_ERR_SHAPE;
+    if (g.dim > CQ_MIX_MAX_DIM || g.dim_pad > CQ_MIX_MAX_DIM) return CQ_ERR_RANGE;
     if (g.rot_dims && (!g.cos_dev || !g.sin_dev)) return CQ_ERR_NULL;
     if (g.rot_dims && g.ctx <= 0) return CQ_ERR_SHAPE;
     if (no_dst) return CQ_OK;

@@ -5,45 +5,44 @@
 
 namespace {
 
+// A load from a wave-uniform base with a 32-bit byte offset: the address costs one register per lane.
+template <typename T> __device__ __forceinline__ T ld_at(const float *base, uint32_t bytes) {
+    return *reinterpret_cast<const T *>(reinterpret_cast<const char *>(base) + bytes);
+}
+
 // ---- several queries ------------------------------------------------------------------------------------------------------
-// Workgroup: 16 query rows x all heads, 8 waves, keys in tiles of KT, one pass with a running maximum.  Per tile:
+// Workgroup: 16 query rows x all heads, NW waves, keys in tiles of KT, one pass with a running maximum.  Per tile:
 //   scores   wave w takes heads [w NHW, (w + 1) NHW): q k^T into LDS, [head][query][key]
-//   mixing   wave w takes queries 2 w and 2 w + 1 of every head: talk x scores on the matrix cores (heads are the contracted
+//   mixing   wave w takes 16 / NW queries of every head: talk x scores on the matrix cores (heads are the contracted
 //            dimension), mask, running softmax in registers, weights back into the same LDS words, rescale factors to `alpha`
-//   values   wave w takes U units (head, 64 output columns): weights x V added to the outputs it holds in registers
-// blockIdx.y: units beyond 8 U (the scores are computed again there).
+//   values   wave w takes U units (head, 64 output columns): weights x V added to the outputs it holds in registers, V read once per VS units
+// blockIdx.y: units beyond NW U (the scores are computed again there).
 // LDS strides: query rows of KT + 4 floats (16 rows x 4 keys of an operand read fall on 64 banks), head blocks of 16 rows + 16
 // (4 heads x 16 keys likewise).
-template <int NHW, bool SHARED_K, int U, int VS, int KT>
-__global__ __launch_bounds__(512) void talk_attention_kernel(const float *__restrict__ q, const float *__restrict__ k_cache, const float *__restrict__ v_cache,
+template <int NW, int NHW, bool SHARED_K, int U, int VS, int KT>
+__global__ __launch_bounds__(64 * NW) void talk_attention_kernel(const float *__restrict__ q, const float *__restrict__ k_cache, const float *__restrict__ v_cache,
                                                              const float *__restrict__ talk, float scale, int window, int keep_first, float out_scale,
                                                              float *__restrict__ out, int64_t out_stride, int pos, int rows, int H, int G, int dp, int vdim,
                                                              int vp, int ctx) {
-    constexpr int NHT = NHW <= 2 ? 1 : NHW / 2, HP = 16 * NHT;           // heads padded to tiles of 16
+    constexpr int NHT = (NW * NHW + 15) / 16, HP = 16 * NHT, NT = 64 * NW, RW = 16 / NW;       // heads padded to tiles of 16; queries per wave
     constexpr int RS = KT + 4, HS = 16 * RS + 16, TS = HP + 4, KTL = KT / 16;
     extern __shared__ __attribute__((aligned(16))) float smem[];
-    float *S = smem, *T = S + HP * HS, *alpha = T + HP * TS;
+    float *S = smem, *T = S + HP * HS, *alpha = T + HP * TS, *m_run = alpha + HP * 16, *l_run = m_run + HP * 16;      // the last three: [head][query]
     const int tid = threadIdx.x, lane = tid & 63, wv = __builtin_amdgcn_readfirstlane(tid >> 6), lr = lane & 15, lk = lane >> 4;
     const int r0 = blockIdx.x * 16, nr = min(16, rows - r0);
     const int p0 = pos + r0, last = p0 + nr - 1;                         // positions of the first and last query
     const int R = H / G, nvc = (vp + 63) / 64;
 
-    for (int i = tid; i < HP * HP; i += 512) {
+    for (int i = tid; i < HP * HP; i += NT) {
         const int h = i / HP, g = i - h * HP;
         T[h * TS + g] = h < H && g < H ? talk[h * H + g] * scale : 0.0f;
     }
-    for (int i = tid; i < (HP - H) * HS; i += 512) S[H * HS + i] = 0.0f;
+    for (int i = tid; i < (HP - H) * HS; i += NT) S[H * HS + i] = 0.0f;
 
-    float m_run[2][NHT][4], l_run[2][NHT][4];
-#pragma unroll
-    for (int a = 0; a < 2; a++)
-#pragma unroll
-        for (int b = 0; b < NHT; b++)
-#pragma unroll
-            for (int e = 0; e < 4; e++) {
-                m_run[a][b][e] = -INFINITY;
-                l_run[a][b][e] = 0.0f;
-            }
+    for (int i = tid; i < HP * 16; i += NT) {
+        m_run[i] = -INFINITY;
+        l_run[i] = 0.0f;
+    }
     f32x4 o[U][4];
 #pragma unroll
     for (int u = 0; u < U; u++)
@@ -51,8 +50,9 @@ __global__ __launch_bounds__(512) void talk_attention_kernel(const float *__rest
         for (int n = 0; n < 4; n++) o[u][n] = f32x4{0.f, 0.f, 0.f, 0.f};
 
     const int h0 = wv * NHW;
-    const float *qrow = q + (int64_t)(r0 + min(lr, nr - 1)) * H * dp + 4 * lk;
-    const int u0 = ((int)blockIdx.y * 8 + wv) * U, n_units = H * nvc;
+    const float *qb = q + (int64_t)r0 * H * dp;
+    const uint32_t q_at = (min(lr, nr - 1) * H * dp + 4 * lk) * 4;
+    const int u0 = ((int)blockIdx.y * NW + wv) * U, n_units = H * nvc;
 
     // tiles of the kept first tokens, then of the window
     const int t_lo = max(0, p0 - window + 1) / KT, t_hi = last / KT;
@@ -66,23 +66,23 @@ __global__ __launch_bounds__(512) void talk_attention_kernel(const float *__rest
             for (int i = 0; i < NHW; i++)
 #pragma unroll
                 for (int t = 0; t < KTL; t++) acc[i][t] = f32x4{0.f, 0.f, 0.f, 0.f};
-            const float *krow[KTL];
+            uint32_t k_at[KTL];
 #pragma unroll
-            for (int t = 0; t < KTL; t++) krow[t] = k_cache + (int64_t)min(j0 + 16 * t + lr, last) * dp + 4 * lk;
+            for (int t = 0; t < KTL; t++) k_at[t] = (min(j0 + 16 * t + lr, last) * dp + 4 * lk) * 4u;
             const int64_t kv_stride = (int64_t)ctx * dp;
             for (int c = 0; c < dp; c += 16) {
                 f32x4 kf[KTL], qf[NHW];
                 if (SHARED_K) {
 #pragma unroll
-                    for (int t = 0; t < KTL; t++) kf[t] = *reinterpret_cast<const f32x4 *>(krow[t] + (h0 / R) * kv_stride + c);
+                    for (int t = 0; t < KTL; t++) kf[t] = ld_at<f32x4>(k_cache + (h0 / R) * kv_stride + c, k_at[t]);
                 }
 #pragma unroll
-                for (int i = 0; i < NHW; i++) qf[i] = *reinterpret_cast<const f32x4 *>(qrow + min(h0 + i, H - 1) * dp + c);
+                for (int i = 0; i < NHW; i++) qf[i] = ld_at<f32x4>(qb + min(h0 + i, H - 1) * dp + c, q_at);
 #pragma unroll
                 for (int i = 0; i < NHW; i++) {
                     if (!SHARED_K) {
 #pragma unroll
-                        for (int t = 0; t < KTL; t++) kf[t] = *reinterpret_cast<const f32x4 *>(krow[t] + (min(h0 + i, H - 1) / R) * kv_stride + c);
+                        for (int t = 0; t < KTL; t++) kf[t] = ld_at<f32x4>(k_cache + (min(h0 + i, H - 1) / R) * kv_stride + c, k_at[t]);
                     }
 #pragma unroll
                     for (int e = 0; e < 4; e++)
@@ -101,9 +101,9 @@ __global__ __launch_bounds__(512) void talk_attention_kernel(const float *__rest
         }
         __syncthreads();
 
-        // ---- mixing and softmax: queries 2 wv, 2 wv + 1, one after the other ----
+        // ---- mixing and softmax: queries RW wv .., one after the other ----
 #pragma unroll
-        for (int a = 0; a < 2; a++) {
+        for (int a = 0; a < RW; a++) {
             f32x4 acc[KTL][NHT];
 #pragma unroll
             for (int t = 0; t < KTL; t++)
@@ -115,13 +115,13 @@ __global__ __launch_bounds__(512) void talk_attention_kernel(const float *__rest
 #pragma unroll
                 for (int b = 0; b < NHT; b++) tf[b] = T[(16 * b + lr) * TS + 4 * s + lk];
 #pragma unroll
-                for (int t = 0; t < KTL; t++) sf[t] = S[(4 * s + lk) * HS + (2 * wv + a) * RS + 16 * t + lr];
+                for (int t = 0; t < KTL; t++) sf[t] = S[(4 * s + lk) * HS + (RW * wv + a) * RS + 16 * t + lr];
 #pragma unroll
                 for (int t = 0; t < KTL; t++)
 #pragma unroll
                     for (int b = 0; b < NHT; b++) acc[t][b] = mfma4(tf[b], sf[t], acc[t][b]);
             }
-            const int p = p0 + 2 * wv + a;
+            const int p = p0 + RW * wv + a;
             bool vis[KTL];
 #pragma unroll
             for (int t = 0; t < KTL; t++) {
@@ -138,52 +138,52 @@ __global__ __launch_bounds__(512) void talk_attention_kernel(const float *__rest
                         s[t] = vis[t] ? acc[t][b][e] : -INFINITY;
                         mx = fmaxf(mx, s[t]);
                     }
-                    const float m_old = m_run[a][b][e], m = fmaxf(m_old, row16_max(mx));
+                    const int h = 16 * b + 4 * lk + e, hr = h * 16 + RW * wv + a;
+                    const float m_old = m_run[hr], m = fmaxf(m_old, row16_max(mx));
                     const float al = m_old > -INFINITY ? __expf(m_old - m) : 0.0f;
-                    const int h = 16 * b + 4 * lk + e;
 #pragma unroll
                     for (int t = 0; t < KTL; t++) {
                         const float w = vis[t] ? __expf(s[t] - m) : 0.0f;
                         sum += w;
-                        S[h * HS + (2 * wv + a) * RS + 16 * t + lr] = w;
+                        S[h * HS + (RW * wv + a) * RS + 16 * t + lr] = w;
                     }
-                    m_run[a][b][e] = m;
-                    l_run[a][b][e] = l_run[a][b][e] * al + row16_sum(sum);
-                    if (lr == 0) alpha[h * 16 + 2 * wv + a] = al;
+                    sum = row16_sum(sum);
+                    m_run[hr] = m;                       // the same value from 16 lanes
+                    l_run[hr] = l_run[hr] * al + sum;
+                    alpha[hr] = al;
                 }
         }
         __syncthreads();
 
-        // ---- values ----
+        // ---- values (units beyond the last repeat it and are not stored) ----
+        if (u0 < n_units) {
 #pragma unroll
-        for (int ub = 0; ub < U; ub += VS) {
-            if (u0 + ub < n_units) {
-                const int g = (u0 + ub) / (R * nvc), c = ((u0 + ub) / R) % nvc;
+            for (int ub = 0; ub < U; ub += VS) {
+                const int uc = min(u0 + ub, n_units - VS);
+                const int g = uc / (R * nvc), c = (uc / R) % nvc, h0v = g * R + uc % R;
+                const float *vb = v_cache + (int64_t)g * ctx * vp + 64 * c;
 #pragma unroll
                 for (int half = 0; half < KTL; half++) {
                     float vf[4][4];
 #pragma unroll
                     for (int s = 0; s < 4; s++) {
-                        const float *vr = v_cache + ((int64_t)g * ctx + min(j0 + 16 * half + 4 * s + lk, last)) * vp;
+                        const uint32_t at = min(j0 + 16 * half + 4 * s + lk, last) * vp;
 #pragma unroll
-                        for (int n = 0; n < 4; n++) vf[s][n] = vr[min(64 * c + 16 * n + lr, vp - 1)];
+                        for (int n = 0; n < 4; n++) vf[s][n] = ld_at<float>(vb, (at + min(16 * n + lr, vp - 64 * c - 1)) * 4u);
                     }
 #pragma unroll
                     for (int v = 0; v < VS; v++) {
-                        const int u = ub + v;
-                        if (u0 + u < n_units) {
-                            const int h = g * R + (u0 + u) % R;
-                            if (half == 0) {
-                                const f32x4 al = *reinterpret_cast<const f32x4 *>(&alpha[h * 16 + 4 * lk]);
+                        const int u = ub + v, h = h0v + v;
+                        if (half == 0) {
+                            const f32x4 al = *reinterpret_cast<const f32x4 *>(&alpha[h * 16 + 4 * lk]);
 #pragma unroll
-                                for (int n = 0; n < 4; n++) o[u][n] *= al;
-                            }
+                            for (int n = 0; n < 4; n++) o[u][n] *= al;
+                        }
 #pragma unroll
-                            for (int s = 0; s < 4; s++) {
-                                const float w = S[h * HS + lr * RS + 16 * half + 4 * s + lk];
+                        for (int s = 0; s < 4; s++) {
+                            const float w = S[h * HS + lr * RS + 16 * half + 4 * s + lk];
 #pragma unroll
-                                for (int n = 0; n < 4; n++) o[u][n] = mfma4(w, vf[s][n], o[u][n]);
-                            }
+                            for (int n = 0; n < 4; n++) o[u][n] = mfma4(w, vf[s][n], o[u][n]);
                         }
                     }
                 }
@@ -191,14 +191,6 @@ __global__ __launch_bounds__(512) void talk_attention_kernel(const float *__rest
         }
         __syncthreads();
     }
-#pragma unroll
-    for (int a = 0; a < 2; a++)
-#pragma unroll
-        for (int b = 0; b < NHT; b++)
-#pragma unroll
-            for (int e = 0; e < 4; e++)
-                if (lr == 0) alpha[(16 * b + 4 * lk + e) * 16 + 2 * wv + a] = l_run[a][b][e];
-    __syncthreads();
 #pragma unroll
     for (int u = 0; u < U; u++) {
         if (u0 + u >= n_units) continue;
@@ -210,114 +202,142 @@ __global__ __launch_bounds__(512) void talk_attention_kernel(const float *__rest
 #pragma unroll
             for (int e = 0; e < 4; e++) {
                 const int row = 4 * lk + e;
-                if (row < nr) out[(int64_t)(r0 + row) * out_stride + (int64_t)h * vdim + col] = out_scale * o[u][n][e] / alpha[h * 16 + row];
+                if (row < nr) out[(int64_t)(r0 + row) * out_stride + (int64_t)h * vdim + col] = out_scale * o[u][n][e] / l_run[h * 16 + row];
             }
         }
     }
 }
 
-template <int NHW, bool SHARED_K, int U, int VS, int KT>
+template <int NW, int NHW, bool SHARED_K, int U, int VS, int KT>
 int talk_launch(const float *q, const float *kc, const float *vc, const float *talk, float scale, int window, int keep, float out_scale, float *out,
                 int64_t out_stride, int pos, int rows, int H, int G, int dp, int vdim, int vp, int ctx, hipStream_t s) {
-    constexpr int HP = 16 * (NHW <= 2 ? 1 : NHW / 2);
-    constexpr size_t lds = (size_t)(HP * (16 * (KT + 4) + 16) + HP * (HP + 4) + HP * 16) * sizeof(float);
+    constexpr int HP = (NW * NHW + 15) / 16 * 16;
+    constexpr size_t lds = (size_t)(HP * (16 * (KT + 4) + 16) + HP * (HP + 4) + 3 * HP * 16) * sizeof(float);
     if (lds > 64 * 1024) {
-        const int e = (int)hipFuncSetAttribute(reinterpret_cast<const void *>(talk_attention_kernel<NHW, SHARED_K, U, VS, KT>),
+        const int e = (int)hipFuncSetAttribute(reinterpret_cast<const void *>(talk_attention_kernel<NW, NHW, SHARED_K, U, VS, KT>),
                                                hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
         if (e) return e;
     }
     const int units = H * ((vp + 63) / 64);
-    hipLaunchKernelGGL((talk_attention_kernel<NHW, SHARED_K, U, VS, KT>), dim3((rows + 15) / 16, (units + 8 * U - 1) / (8 * U)), dim3(512), lds, s, q, kc, vc,
-                       talk, scale, window, keep, out_scale, out, out_stride, pos, rows, H, G, dp, vdim, vp, ctx);
+    hipLaunchKernelGGL((talk_attention_kernel<NW, NHW, SHARED_K, U, VS, KT>), dim3((rows + 15) / 16, (units + NW * U - 1) / (NW * U)), dim3(64 * NW), lds, s, q,
+                       kc, vc, talk, scale, window, keep, out_scale, out, out_stride, pos, rows, H, G, dp, vdim, vp, ctx);
     return (int)hipGetLastError();
 }
 
 // ---- one query --------------------------------------------------------------------------------------------------------------
-// Workgroup: KD of the visible keys x all heads, 8 waves.  It normalizes and rotates q itself; the workgroup that holds the
-// last visible key (the new token) first does the same for k and v and appends them to the caches.
+// Workgroup: KD of the visible keys x all heads, 16 waves.  The first K and V rows and the head mixing matrix are requested before
+// anything else; meanwhile the workgroup normalizes and rotates q itself.  The one that holds the last visible key (the new token) does
+// the same for k and v, appends them to the caches and uses its own copies.
 //   scores  16 lanes per (kv head, key), each key row read once for the heads that share it
 //   mixing  one thread per (head, key)
 //   values  one thread per (kv head, column), four heads at a time
 template <int NC, int KD>
-__global__ __launch_bounds__(512) void talk_decode_kernel(const float *__restrict__ row, cq_mix_heads gq, cq_mix_heads gk, cq_mix_heads gv, float eps,
-                                                          const float *__restrict__ talk, float scale, int window, int keep_first,
-                                                          const int32_t *__restrict__ pos_dev, int pos0, float *__restrict__ rec, int splits) {
+__global__ __launch_bounds__(1024) void talk_decode_kernel(const float *__restrict__ row, cq_mix_heads gq, cq_mix_heads gk, cq_mix_heads gv, float eps,
+                                                           const float *__restrict__ talk, float scale, int window, int keep_first,
+                                                           const int32_t *__restrict__ pos_dev, int pos0, float *__restrict__ rec, int splits) {
     extern __shared__ __attribute__((aligned(16))) float smem[];
-    const int H = gq.heads, G = gk.heads, R = H / G, dp = gk.dim_pad, vdim = gv.dim, ctx = gk.ctx;
-    constexpr int SS = KD + 1;
-    float *qs = smem, *sc = qs + H * dp, *mx = sc + H * SS;
+    const int H = gq.heads, G = gk.heads, R = H / G, dp = gk.dim_pad, vdim = gv.dim, vp = gv.dim_pad, ctx = gk.ctx;
+    constexpr int SS = KD + 1, PB = 2;
+    float *qs = smem, *kn = qs + H * dp, *vn = kn + G * dp, *T = vn + G * vp, *sc = T + H * H, *mx = sc + H * SS;
     const int tid = threadIdx.x, lane = tid & 63, wv = __builtin_amdgcn_readfirstlane(tid >> 6), sp = blockIdx.x;
     const int p = pos0 + (pos_dev ? pos_dev[0] : 0);
     const Visible vis = visible_keys(p, window, keep_first);
     const int s0 = sp * KD, cnt = min(KD, vis.n - s0);
     if (p >= ctx || cnt <= 0) return;                                // uniform: no key of this split is visible yet
-
-    for (int h = wv; h < H; h += 8) {
-        const float *s = row + gq.src_off + (int64_t)h * gq.dim;
-        const float inv = gq.norm_dev ? head_inv_rms(s, gq.dim, eps, lane) : 1.0f;
-        for (int d = lane; d < dp; d += 64) qs[h * dp + d] = d < gq.dim ? head_value(gq, s, d, inv, p) : 0.0f;
-    }
-    if (s0 + cnt == vis.n) {
-        for (int g = wv; g < 2 * G; g += 8) {
-            const cq_mix_heads &gr = g < G ? gk : gv;
-            const int hh = g < G ? g : g - G;
-            const float *s = row + gr.src_off + (int64_t)hh * gr.dim;
-            float *d = gr.dst_dev + hh * gr.dst_head_stride + (int64_t)p * gr.dst_row_stride;
-            const float inv = gr.norm_dev ? head_inv_rms(s, gr.dim, eps, lane) : 1.0f;
-            for (int i = lane; i < gr.dim_pad; i += 64) d[i] = i < gr.dim ? head_value(gr, s, i, inv, p) : 0.0f;
-        }
-        __threadfence_block();
-    }
-    __syncthreads();
-
+    const bool owner = s0 + cnt == vis.n;                            // key cnt - 1 is the new token
     auto key_of = [&](int j) {                                       // j-th key of the split, clamped to one that exists
         const int s = s0 + min(j, cnt - 1);
         return s < vis.keep ? s : vis.lo + s - vis.keep;
     };
-    // ---- scores ----
-    {
-        constexpr int PB = 4;
-        const int sub = lane & 15, grp = wv * 4 + (lane >> 4), pairs = G * KD;
-        for (int b = grp; b < pairs; b += 32 * PB) {
-            f32x4 kd[PB][NC];
+    const int sub = lane & 15, grp = wv * 4 + (lane >> 4), pairs = G * KD, items = G * vdim;
+    f32x4 kd[PB][NC];
+    float vv[16];
+    auto load_k = [&](int b) {
 #pragma unroll
-            for (int i = 0; i < PB; i++) {
-                const int pr = min(b + 32 * i, pairs - 1), g = pr / KD;
-                const float *kr = gk.dst_dev + g * gk.dst_head_stride + (int64_t)key_of(pr - g * KD) * gk.dst_row_stride;
+        for (int i = 0; i < PB; i++) {
+            const int pr = min(b + 64 * i, pairs - 1), g = pr / KD;
+            const float *kr = gk.dst_dev + g * gk.dst_head_stride + (int64_t)key_of(pr - g * KD) * gk.dst_row_stride;
+#pragma unroll
+            for (int c = 0; c < NC; c++) {
+                const int d = 64 * c + 4 * sub;
+                kd[i][c] = d < dp ? *reinterpret_cast<const f32x4 *>(kr + d) : f32x4{0.f, 0.f, 0.f, 0.f};
+            }
+        }
+    };
+    auto load_v = [&](int i, int jb) {
+        const int g = i / vdim;
+        const float *vb = gv.dst_dev + g * gv.dst_head_stride + (i - g * vdim);
+#pragma unroll
+        for (int j = 0; j < 16; j++) vv[j] = vb[(int64_t)key_of(jb + j) * gv.dst_row_stride];
+    };
+    load_k(grp);
+    load_v(min(tid, items - 1), 0);
+    for (int i = tid; i < H * H; i += 1024) T[i] = talk[i] * scale;
+    for (int h = wv; h < H; h += 32) {                                // two heads at a time
+        HeadRegs<NC> a, b;
+        const int h2 = min(h + 16, H - 1);
+        a.load(gq, row + gq.src_off + (int64_t)h * gq.dim, p, lane);
+        b.load(gq, row + gq.src_off + (int64_t)h2 * gq.dim, p, lane);
+        a.finish(gq, eps, lane);
+        b.finish(gq, eps, lane);
+#pragma unroll
+        for (int e = 0; e < NC; e++)
+            if (lane + 64 * e < dp) {
+                qs[h * dp + lane + 64 * e] = a.v[e];
+                if (h + 16 < H) qs[(h + 16) * dp + lane + 64 * e] = b.v[e];
+            }
+    }
+    if (owner) {
+        for (int x = wv; x < 2 * G; x += 16) {
+            const cq_mix_heads &gr = x < G ? gk : gv;
+            const int hh = x < G ? x : x - G;
+            float *dst = gr.dst_dev + hh * gr.dst_head_stride + (int64_t)p * gr.dst_row_stride, *own = (x < G ? kn : vn) + hh * gr.dim_pad;
+            HeadRegs<NC> a;
+            a.load(gr, row + gr.src_off + (int64_t)hh * gr.dim, p, lane);
+            a.finish(gr, eps, lane);
+#pragma unroll
+            for (int e = 0; e < NC; e++)
+                if (lane + 64 * e < gr.dim_pad) dst[lane + 64 * e] = own[lane + 64 * e] = a.v[e];
+        }
+    }
+    __syncthreads();
+
+    // ---- scores ----
+    for (int b = grp; b < pairs; b += 64 * PB) {
+        if (b != grp) load_k(b);
+#pragma unroll
+        for (int i = 0; i < PB; i++) {
+            const int pr = min(b + 64 * i, pairs - 1), g = pr / KD, j = pr - g * KD;
+            if (owner && j >= cnt - 1) {
+#pragma unroll
+                for (int c = 0; c < NC; c++)
+                    if (64 * c + 4 * sub < dp) kd[i][c] = *reinterpret_cast<const f32x4 *>(kn + g * dp + 64 * c + 4 * sub);
+            }
+            for (int r = 0; r < R; r++) {
+                const float *qh = qs + (g * R + r) * dp;
+                float a = 0.0f;
 #pragma unroll
                 for (int c = 0; c < NC; c++) {
                     const int d = 64 * c + 4 * sub;
-                    kd[i][c] = d < dp ? *reinterpret_cast<const f32x4 *>(kr + d) : f32x4{0.f, 0.f, 0.f, 0.f};
+                    const f32x4 qv = d < dp ? *reinterpret_cast<const f32x4 *>(qh + d) : f32x4{0.f, 0.f, 0.f, 0.f};
+                    a = fmaf(qv.x, kd[i][c].x, a);
+                    a = fmaf(qv.y, kd[i][c].y, a);
+                    a = fmaf(qv.z, kd[i][c].z, a);
+                    a = fmaf(qv.w, kd[i][c].w, a);
                 }
-            }
-#pragma unroll
-            for (int i = 0; i < PB; i++) {
-                const int pr = b + 32 * i, g = min(pr, pairs - 1) / KD;
-                for (int r = 0; r < R; r++) {
-                    const float *qh = qs + (g * R + r) * dp;
-                    float a = 0.0f;
-#pragma unroll
-                    for (int c = 0; c < NC; c++) {
-                        const int d = 64 * c + 4 * sub;
-                        const f32x4 qv = d < dp ? *reinterpret_cast<const f32x4 *>(qh + d) : f32x4{0.f, 0.f, 0.f, 0.f};
-                        a = fmaf(qv.x, kd[i][c].x, a);
-                        a = fmaf(qv.y, kd[i][c].y, a);
-                        a = fmaf(qv.z, kd[i][c].z, a);
-                        a = fmaf(qv.w, kd[i][c].w, a);
-                    }
-                    a = row16_sum(a);
-                    if (sub == 0 && pr < pairs) sc[(g * R + r) * SS + pr - g * KD] = a * scale;
-                }
+                a = row16_sum(a);
+                if (sub == 0) sc[(g * R + r) * SS + j] = a;
             }
         }
     }
     __syncthreads();
     // ---- mixing ----
-    for (int i = tid; i < H * KD; i += 512) {
+    for (int i = tid; i < H * KD; i += 1024) {
         const int h = i / KD, j = i - h * KD;
-        const float *t = talk + h * H;
+        const float *t = T + h * H;
         float a0 = 0.0f, a1 = 0.0f;
         int g = 0;
+#pragma unroll 4
         for (; g + 2 <= H; g += 2) {
             a0 = fmaf(t[g], sc[g * SS + j], a0);
             a1 = fmaf(t[g + 1], sc[(g + 1) * SS + j], a1);
@@ -328,12 +348,11 @@ __global__ __launch_bounds__(512) void talk_decode_kernel(const float *__restric
     __syncthreads();
     // ---- softmax of the split: 16 lanes per head ----
     const int stride = talk_record(vdim);
-    for (int h = wv * 4 + (lane >> 4); h < (H + 3) / 4 * 4; h += 32) {
-        const int hh = min(h, H - 1);
+    for (int h = grp; h < H; h += 64) {
         float s[KD / 16], m = -INFINITY, l = 0.0f;
 #pragma unroll
         for (int i = 0; i < KD / 16; i++) {
-            s[i] = mx[hh * SS + 16 * i + (lane & 15)];
+            s[i] = mx[h * SS + 16 * i + sub];
             m = fmaxf(m, s[i]);
         }
         m = row16_max(m);
@@ -341,29 +360,28 @@ __global__ __launch_bounds__(512) void talk_decode_kernel(const float *__restric
         for (int i = 0; i < KD / 16; i++) {
             s[i] = s[i] > -INFINITY ? __expf(s[i] - m) : 0.0f;
             l += s[i];
+            sc[h * SS + 16 * i + sub] = s[i];
         }
         l = row16_sum(l);
-        if (h < H) {
-#pragma unroll
-            for (int i = 0; i < KD / 16; i++) sc[h * SS + 16 * i + (lane & 15)] = s[i];
-            if ((lane & 15) == 0) {
-                float *r = rec + ((int64_t)h * splits + sp) * stride + stride - 4;
-                r[0] = m;
-                r[1] = l;
-            }
+        if (sub == 0) {
+            float *r = rec + ((int64_t)h * splits + sp) * stride + stride - 4;
+            r[0] = m;
+            r[1] = l;
         }
     }
     __syncthreads();
     // ---- values ----
-    for (int i = tid; i < G * vdim; i += 512) {
+    for (int i = tid; i < items; i += 1024) {
         const int g = i / vdim, e = i - g * vdim;
-        const float *vb = gv.dst_dev + g * gv.dst_head_stride + e;
         for (int r = 0; r < R; r += 4) {
             float a[4] = {0.f, 0.f, 0.f, 0.f};
             for (int jb = 0; jb < KD; jb += 16) {
-                float vv[16];
+                if (i != tid || jb > 0 || (KD > 16 && r > 0)) load_v(i, jb);
+                if (owner) {
+                    const float x = vn[g * vp + e];
 #pragma unroll
-                for (int j = 0; j < 16; j++) vv[j] = vb[(int64_t)key_of(jb + j) * gv.dst_row_stride];
+                    for (int j = 0; j < 16; j++) vv[j] = jb + j >= cnt - 1 ? x : vv[j];
+                }
 #pragma unroll
                 for (int j = 0; j < 16; j++)
 #pragma unroll
@@ -379,13 +397,15 @@ __global__ __launch_bounds__(512) void talk_decode_kernel(const float *__restric
 template <int NC, int KD>
 int talk_decode_launch(const float *row, const cq_mix_heads *g, float eps, const float *talk, float scale, int window, int keep, const int32_t *pos_dev, int pos,
                        float *rec, int splits, hipStream_t s) {
-    const size_t lds = (size_t)g[0].heads * (g[1].dim_pad + 2 * (KD + 1)) * sizeof(float);
+    const int H = g[0].heads, G = g[1].heads;
+    const size_t lds = (size_t)(H * (g[1].dim_pad + 2 * (KD + 1) + H) + G * (g[1].dim_pad + g[2].dim_pad)) * sizeof(float);
+    if (lds > 160 * 1024) return CQ_ERR_RANGE;
     if (lds > 64 * 1024) {
         const int e = (int)hipFuncSetAttribute(reinterpret_cast<const void *>(talk_decode_kernel<NC, KD>), hipFuncAttributeMaxDynamicSharedMemorySize,
                                                160 * 1024);
         if (e) return e;
     }
-    hipLaunchKernelGGL((talk_decode_kernel<NC, KD>), dim3(splits), dim3(512), lds, s, row, g[0], g[1], g[2], eps, talk, scale, window, keep, pos_dev, pos, rec,
+    hipLaunchKernelGGL((talk_decode_kernel<NC, KD>), dim3(splits), dim3(1024), lds, s, row, g[0], g[1], g[2], eps, talk, scale, window, keep, pos_dev, pos, rec,
                        splits);
     return (int)hipGetLastError();
 }
@@ -404,16 +424,17 @@ int cq_mix_talk_attention(const float *q_dev, const float *k_cache_dev, const fl
     if (!q_dev || !k_cache_dev || !v_cache_dev || !talk_dev || !out_dev) return CQ_ERR_NULL;
     if (mix_misaligned(q_dev, 16) || mix_misaligned(k_cache_dev, 16) || mix_misaligned(v_cache_dev, 16)) return CQ_ERR_ALIGN;
     if (pos + rows > ctx || ctx > (1 << 28) || n_head > CQ_MIX_MAX_HEADS || dim_pad > CQ_MIX_MAX_DIM || vdim_pad > CQ_MIX_MAX_DIM) return CQ_ERR_RANGE;
+    if (ctx * (dim_pad > vdim_pad ? dim_pad : vdim_pad) * 4 > 0x7fffffffLL) return CQ_ERR_RANGE;      // byte offsets inside a kv head are 32-bit
     const int w = (int)(window < ctx ? window : ctx), keep = (int)(keep_first < ctx ? keep_first : ctx);
     const int H = (int)n_head, G = (int)n_kv_head, R = H / G;
     hipStream_t s = (hipStream_t)stream;
-#define CQ_TA(NHW_, SH_, U_, VS_, KT_)                                                                                                                \
-    talk_launch<NHW_, SH_, U_, VS_, KT_>(q_dev, k_cache_dev, v_cache_dev, talk_dev, scale, w, keep, out_scale, out_dev, out_stride, (int)pos, (int)rows, H, G, \
-                                         (int)dim_pad, (int)vdim, (int)vdim_pad, (int)ctx, s)
-    if (H <= 8) return R % 2 ? CQ_TA(1, true, 2, 1, 32) : CQ_TA(1, true, 2, 2, 32);
-    if (H <= 16) return R % 2 ? CQ_TA(2, false, 2, 1, 32) : CQ_TA(2, true, 2, 2, 32);
-    if (H <= 32) return R % 4 ? CQ_TA(4, false, 8, 1, 32) : CQ_TA(4, true, 8, 4, 32);
-    return R % 8 ? (R % 4 ? CQ_TA(8, false, 8, 1, 16) : CQ_TA(8, false, 8, 4, 16)) : CQ_TA(8, true, 8, 4, 16);
+#define CQ_TA(NW_, NHW_, SH_, U_, VS_, KT_)                                                                                                            \
+    talk_launch<NW_, NHW_, SH_, U_, VS_, KT_>(q_dev, k_cache_dev, v_cache_dev, talk_dev, scale, w, keep, out_scale, out_dev, out_stride, (int)pos, (int)rows, \
+                                              H, G, (int)dim_pad, (int)vdim, (int)vdim_pad, (int)ctx, s)
+    if (H <= 8) return R % 2 ? CQ_TA(8, 1, true, 2, 1, 32) : CQ_TA(8, 1, true, 2, 2, 32);
+    if (H <= 16) return R % 2 ? CQ_TA(16, 1, true, 2, 1, 32) : CQ_TA(16, 1, true, 2, 2, 32);
+    if (H <= 32) return R % 2 ? CQ_TA(16, 2, false, 4, 1, 32) : (R % 4 ? CQ_TA(16, 2, true, 4, 2, 32) : CQ_TA(16, 2, true, 4, 4, 32));
+    return R % 4 ? CQ_TA(16, 4, false, 4, 1, 16) : CQ_TA(16, 4, true, 4, 4, 16);
 #undef CQ_TA
 }
 
@@ -441,8 +462,9 @@ int cq_mix_talk_decode(const float *row_dev, const cq_mix_heads *qkv, float eps,
     hipStream_t s = (hipStream_t)stream;
 #define CQ_TD(NC_, KD_) talk_decode_launch<NC_, KD_>(row_dev, qkv, eps, talk_dev, scale, w, keep, pos_dev, (int)pos, (float *)workspace_dev, splits, s)
     const bool fine = talk_split_keys(n_max) == 16;
-    if (k.dim_pad <= 64) return fine ? CQ_TD(1, 16) : CQ_TD(1, 64);
-    if (k.dim_pad <= 128) return fine ? CQ_TD(2, 16) : CQ_TD(2, 64);
+    const int widest = k.dim_pad > v.dim_pad ? k.dim_pad : v.dim_pad;
+    if (widest <= 64) return fine ? CQ_TD(1, 16) : CQ_TD(1, 64);
+    if (widest <= 128) return fine ? CQ_TD(2, 16) : CQ_TD(2, 64);
     return fine ? CQ_TD(4, 16) : CQ_TD(4, 64);
 #undef CQ_TD
 }

@@ -102,6 +102,7 @@ struct Groups {
 };
 
 // one wave per (row, head); heads of all groups numbered through
+template <int NE>
 __global__ __launch_bounds__(256) void pack_heads_kernel(const float *__restrict__ src, int64_t src_stride, Groups gs, int n_groups, int total_heads, float eps,
                                                          const int32_t *__restrict__ pos_dev, int64_t pos, int64_t rows) {
     const int lane = threadIdx.x & 63;
@@ -115,8 +116,12 @@ __global__ __launch_bounds__(256) void pack_heads_kernel(const float *__restrict
     if (g.ctx > 0 && p >= g.ctx) return;
     const float *s = src + r * src_stride + g.src_off + (int64_t)h * g.dim;
     float *d = g.dst_dev + h * g.dst_head_stride + (g.by_position ? p : r) * g.dst_row_stride;
-    const float inv = g.norm_dev ? head_inv_rms(s, g.dim, eps, lane) : 1.0f;
-    for (int i = lane; i < g.dim_pad; i += 64) d[i] = i < g.dim ? head_value(g, s, i, inv, p) : 0.0f;
+    HeadRegs<NE> x;
+    x.load(g, s, p, lane);
+    x.finish(g, eps, lane);
+#pragma unroll
+    for (int e = 0; e < NE; e++)
+        if (lane + 64 * e < g.dim_pad) d[lane + 64 * e] = x.v[e];
 }
 
 // one wave per (row, head)
@@ -188,6 +193,7 @@ int cq_mix_pack_heads(const float *src_dev, int64_t src_stride, const cq_mix_hea
     if (!src_dev || !groups) return CQ_ERR_NULL;
     Groups gs;
     int64_t total = 0;
+    int widest = 0;
     for (int i = 0; i < n_groups; i++) {
         const int e = mix_check_group(groups[i], false);
         if (e) return e;
@@ -195,10 +201,16 @@ int cq_mix_pack_heads(const float *src_dev, int64_t src_stride, const cq_mix_hea
         if (groups[i].ctx > 0 && !pos_dev && pos + rows > groups[i].ctx) return CQ_ERR_RANGE;
         gs.g[i] = groups[i];
         total += groups[i].heads;
+        widest = groups[i].dim_pad > widest ? groups[i].dim_pad : widest;
     }
     if (total > (1 << 20) || (rows * total + 3) / 4 > 0x7fffffffLL) return CQ_ERR_RANGE;
-    hipLaunchKernelGGL(pack_heads_kernel, dim3((unsigned)((rows * total + 3) / 4)), dim3(256), 0, (hipStream_t)stream, src_dev, src_stride, gs, n_groups,
-                       (int)total, eps, pos_dev, pos, rows);
+    const dim3 grid((unsigned)((rows * total + 3) / 4));
+    hipStream_t s = (hipStream_t)stream;
+#define CQ_PH(NE_) hipLaunchKernelGGL(pack_heads_kernel<NE_>, grid, dim3(256), 0, s, src_dev, src_stride, gs, n_groups, (int)total, eps, pos_dev, pos, rows)
+    if (widest <= 64) CQ_PH(1);
+    else if (widest <= 128) CQ_PH(2);
+    else CQ_PH(4);
+#undef CQ_PH
     return (int)hipGetLastError();
 }
 

@@ -10,7 +10,7 @@ namespace {
 // places in the chunk and S the state before it:
 //   o_i = gamma^(i+1) S^T q_i + sum_{j<=i} gamma^(i-j) (q_i . k_j) v_j,     S' = gamma^n S + sum_j gamma^(n-1-j) k_j v_j^T
 // A long call is cut into segments of whole chunks that run side by side: retention_segment_kernel leaves what each segment adds to the
-// state (Z), the segment's workgroup sums the Z of the segments before it, retention_state_kernel forms the final state.
+// state (Z), retention_prefix_kernel turns Z into the state before each segment and forms the final one.
 constexpr int RC = 64, RLD = 68;                     // chunk length; LDS row of 64 columns (16 rows x 4 fall on 64 banks)
 
 struct Retention {
@@ -75,7 +75,7 @@ __global__ __launch_bounds__(256) void retention_segment_kernel(Retention a) {
     }
 }
 
-__global__ __launch_bounds__(256) void retention_kernel(Retention a) {
+__global__ __launch_bounds__(256, 2) void retention_kernel(Retention a) {
     extern __shared__ __attribute__((aligned(16))) float smem[];
     float *S = smem, *A = S + a.dp * RLD;                 // state [dp][64], decayed q k^T [64][64]
     const int tid = threadIdx.x, lane = tid & 63, wv = __builtin_amdgcn_readfirstlane(tid >> 6), lr = lane & 15, lk = lane >> 4;
@@ -84,17 +84,13 @@ __global__ __launch_bounds__(256) void retention_kernel(Retention a) {
     const int seg0 = seg * a.seg_len, t_end = min(a.rows, seg0 + a.seg_len);
     float *state = a.state + (int64_t)h * a.vdim * a.sp;
 
-    const float g0 = exp2f(l2 * (float)seg0);
-    for (int i = tid; i < a.dp * 64; i += 256) {
-        const int col = i / a.dp, d = i - col * a.dp;      // rows of a column follow each other in memory
-        S[d * RLD + col] = 64 * vb + col < a.vdim ? g0 * state[(int64_t)(64 * vb + col) * a.sp + d] : 0.0f;
-    }
-    if (seg > 0) {
-        __syncthreads();
+    if (a.nseg > 1) {
+        const float *z = segment_z(a, h, vb, seg);
+        for (int i = tid; i < a.dp * 64; i += 256) S[(i >> 6) * RLD + (i & 63)] = z[i];
+    } else {
         for (int i = tid; i < a.dp * 64; i += 256) {
-            float s = 0.0f;
-            for (int x = 0; x < seg; x++) s = fmaf(exp2f(l2 * (float)(a.seg_len * (seg - 1 - x))), segment_z(a, h, vb, x)[i], s);
-            S[(i >> 6) * RLD + (i & 63)] += s;
+            const int col = i / a.dp, d = i - col * a.dp;      // rows of a column follow each other in memory
+            S[d * RLD + col] = 64 * vb + col < a.vdim ? state[(int64_t)(64 * vb + col) * a.sp + d] : 0.0f;
         }
     }
     __syncthreads();
@@ -178,17 +174,29 @@ __global__ __launch_bounds__(256) void retention_kernel(Retention a) {
         }
 }
 
-__global__ __launch_bounds__(256) void retention_state_kernel(Retention a) {
+__global__ __launch_bounds__(256) void retention_prefix_kernel(Retention a) {
     const int h = blockIdx.y;
-    const int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x;
-    if (i >= (int64_t)a.vdim * a.dp) return;
-    const int col = (int)(i / a.dp), d = (int)(i - (int64_t)col * a.dp);
-    const float l2 = a.log2_decay[h];
-    float *st = a.state + ((int64_t)h * a.vdim + col) * a.sp + d;
-    float s = exp2f(l2 * (float)a.rows) * st[0];
-    for (int x = 0; x < a.nseg; x++)
-        s = fmaf(exp2f(l2 * (float)(a.rows - min(a.rows, (x + 1) * a.seg_len))), segment_z(a, h, col >> 6, x)[d * 64 + (col & 63)], s);
-    st[0] = s;
+    const int i = blockIdx.x * 256 + threadIdx.x;             // element of the [nvb][dp][64] Z of a segment
+    if (i >= a.nvb * a.dp * 64) return;
+    const int vb = i / (a.dp * 64), in = i - vb * a.dp * 64, d = in >> 6, col = 64 * vb + (in & 63);
+    const float l2 = a.log2_decay[h], g = exp2f(l2 * (float)a.seg_len), g_last = exp2f(l2 * (float)(a.rows - (a.nseg - 1) * a.seg_len));
+    float *st = a.state + ((int64_t)h * a.vdim + min(col, a.vdim - 1)) * a.sp + d;
+    float *z = segment_z(a, h, vb, 0) + in;
+    const int64_t step = (int64_t)a.dp * 64;
+    float s = col < a.vdim ? st[0] : 0.0f;
+    constexpr int B = 8;                                      // the loads of eight segments before their chain
+    for (int x0 = 0; x0 < a.nseg; x0 += B) {
+        float v[B];
+#pragma unroll
+        for (int x = 0; x < B; x++) v[x] = z[min(x0 + x, a.nseg - 1) * step];
+#pragma unroll
+        for (int x = 0; x < B; x++)
+            if (x0 + x < a.nseg) {
+                z[(x0 + x) * step] = s;
+                s = fmaf(x0 + x == a.nseg - 1 ? g_last : g, s, v[x]);
+            }
+    }
+    if (col < a.vdim) st[0] = s;
 }
 
 void retention_plan(int64_t rows, int64_t heads, int64_t vdim, int *nseg, int *seg_len) {
@@ -213,17 +221,32 @@ struct StepArgs {
     int heads, vdim;
 };
 
+// The state columns of a wave are requested before q and k are worked out.
 template <int NR>
 __device__ __forceinline__ void retention_step(const StepArgs &a, int h, int p, float *sm) {
     const int tid = threadIdx.x, lane = tid & 63, wv = __builtin_amdgcn_readfirstlane(tid >> 6), sub = lane & 15, cg = lane >> 4;
-    float *qs = sm, *ks = qs + 64 * NR, *os = ks + 64 * NR;
+    constexpr int SP = 64 * NR;
+    float *qs = sm, *ks = qs + SP, *os = ks + SP;
     __shared__ float s_inv;
+    f32x4 s[NR];
+    float vj;
+    auto load = [&](int c0) {
+        const int col = min(c0 + cg, a.vdim - 1);
+        const float *st = a.state + ((int64_t)h * a.vdim + col) * SP + 4 * sub;
+#pragma unroll
+        for (int c = 0; c < NR; c++) s[c] = *reinterpret_cast<const f32x4 *>(st + 64 * c);
+        vj = a.row[a.v_off + (int64_t)h * a.vdim + col];
+    };
+    load(4 * wv);
     if (wv < 2) {
         const cq_mix_heads &g = wv == 0 ? a.gq : a.gk;
-        const float *s = a.row + g.src_off + (int64_t)h * g.dim;
-        const float inv = g.norm_dev ? head_inv_rms(s, g.dim, a.eps, lane) : 1.0f;
-        for (int d = lane; d < 64 * NR; d += 64) sm[wv * 64 * NR + d] = d < g.dim ? head_value(g, s, d, inv, p) : 0.0f;
+        HeadRegs<NR> x;
+        x.load(g, a.row + g.src_off + (int64_t)h * g.dim, p, lane);
+        x.finish(g, a.eps, lane);
+#pragma unroll
+        for (int e = 0; e < NR; e++) sm[wv * SP + lane + 64 * e] = x.v[e];
     }
+    const float dec = a.decay[h];
     __syncthreads();
     f32x4 qv[NR], kv[NR];
 #pragma unroll
@@ -231,15 +254,9 @@ __device__ __forceinline__ void retention_step(const StepArgs &a, int h, int p, 
         qv[c] = *reinterpret_cast<const f32x4 *>(qs + 64 * c + 4 * sub);
         kv[c] = *reinterpret_cast<const f32x4 *>(ks + 64 * c + 4 * sub);
     }
-    const float dec = a.decay[h];
-    for (int c0 = 4 * wv; c0 < a.vdim; c0 += 32) {
-        const int col = min(c0 + cg, a.vdim - 1);
-        float *st = a.state + ((int64_t)h * a.vdim + col) * (64 * NR) + 4 * sub;
-        const float vj = a.row[a.v_off + (int64_t)h * a.vdim + col];
-        f32x4 s[NR];
+    for (int c0 = 4 * wv; c0 < a.vdim; c0 += 64) {
+        if (c0 >= 64) load(c0);
         float o = 0.0f;
-#pragma unroll
-        for (int c = 0; c < NR; c++) s[c] = *reinterpret_cast<const f32x4 *>(st + 64 * c);
 #pragma unroll
         for (int c = 0; c < NR; c++)
 #pragma unroll
@@ -249,9 +266,10 @@ __device__ __forceinline__ void retention_step(const StepArgs &a, int h, int p, 
             }
         o = row16_sum(o);
         if (c0 + cg < a.vdim) {
+            float *st = a.state + ((int64_t)h * a.vdim + c0 + cg) * SP + 4 * sub;
 #pragma unroll
             for (int c = 0; c < NR; c++) *reinterpret_cast<f32x4 *>(st + 64 * c) = s[c];
-            if (sub == 0) os[col] = o;
+            if (sub == 0) os[c0 + cg] = o;
         }
     }
     __syncthreads();
@@ -260,7 +278,7 @@ __device__ __forceinline__ void retention_step(const StepArgs &a, int h, int p, 
         if (lane == 0) s_inv = inv;
     }
     __syncthreads();
-    for (int e = tid; e < a.vdim; e += 512) {
+    for (int e = tid; e < a.vdim; e += 1024) {
         const float g = a.row[a.g_off + (int64_t)h * a.vdim + e];
         a.ret_out[(int64_t)h * a.vdim + e] = a.ret_scale * os[e] * s_inv * (g * mix_sigmoid(g));
     }
@@ -268,9 +286,9 @@ __device__ __forceinline__ void retention_step(const StepArgs &a, int h, int p, 
 
 // Blocks [0, n_head): out of one attention head from its records; blocks behind them: one retention head each.
 template <int NR>
-__global__ __launch_bounds__(512) void talk_merge_retention_kernel(StepArgs a, const int32_t *__restrict__ pos_dev, int pos0) {
-    extern __shared__ __attribute__((aligned(16))) float sm[];          // max(splits + 512, 2 * 64 NR + vdim)
-    __shared__ float red[8];
+__global__ __launch_bounds__(1024) void talk_merge_retention_kernel(StepArgs a, const int32_t *__restrict__ pos_dev, int pos0) {
+    extern __shared__ __attribute__((aligned(16))) float sm[];          // max(splits + 1024, 2 * 64 NR + vdim)
+    __shared__ float red[16];
     const int tid = threadIdx.x, lane = tid & 63, wv = __builtin_amdgcn_readfirstlane(tid >> 6);
     const int p = pos0 + (pos_dev ? pos_dev[0] : 0);
     if (p >= a.ctx) return;
@@ -283,14 +301,16 @@ __global__ __launch_bounds__(512) void talk_merge_retention_kernel(StepArgs a, c
     const float *rec = a.rec + (int64_t)h * a.splits * stride;
     float *wt = sm, *part = sm + (n + 3) / 4 * 4;
     float m = -INFINITY;
-    for (int s = tid; s < n; s += 512) m = fmaxf(m, rec[(int64_t)s * stride + stride - 4]);
+    for (int s = tid; s < n; s += 1024) m = fmaxf(m, wt[s] = rec[(int64_t)s * stride + stride - 4]);
     m = wave_max(m);
     if (lane == 0) red[wv] = m;
     __syncthreads();
-    m = fmaxf(fmaxf(fmaxf(red[0], red[1]), fmaxf(red[2], red[3])), fmaxf(fmaxf(red[4], red[5]), fmaxf(red[6], red[7])));
+    m = red[0];
+#pragma unroll
+    for (int w = 1; w < 16; w++) m = fmaxf(m, red[w]);
     float l = 0.0f;
-    for (int s = tid; s < n; s += 512) {
-        const float w = __expf(rec[(int64_t)s * stride + stride - 4] - m);
+    for (int s = tid; s < n; s += 1024) {                    // the thread's own wt entries
+        const float w = __expf(wt[s] - m);
         wt[s] = w;
         l = fmaf(w, rec[(int64_t)s * stride + stride - 3], l);
     }
@@ -298,20 +318,22 @@ __global__ __launch_bounds__(512) void talk_merge_retention_kernel(StepArgs a, c
     __syncthreads();
     if (lane == 0) red[wv] = l;
     __syncthreads();
-    l = ((red[0] + red[1]) + (red[2] + red[3])) + ((red[4] + red[5]) + (red[6] + red[7]));
+    l = 0.0f;
+#pragma unroll
+    for (int w = 0; w < 16; w++) l += red[w];
     // 64 columns at a time, the waves share out the splits
     for (int e0 = 0; e0 < a.att_vdim; e0 += 64) {
         const int e = min(e0 + lane, a.att_vdim - 1);
         float acc = 0.0f;
 #pragma unroll 4
-        for (int s = wv; s < n; s += 8) acc = fmaf(wt[s], rec[(int64_t)s * stride + e], acc);
+        for (int s = wv; s < n; s += 16) acc = fmaf(wt[s], rec[(int64_t)s * stride + e], acc);
         __syncthreads();
         part[wv * 64 + lane] = acc;
         __syncthreads();
         if (wv == 0 && e0 + lane < a.att_vdim) {
             float t = 0.0f;
 #pragma unroll
-            for (int w = 0; w < 8; w++) t += part[w * 64 + lane];
+            for (int w = 0; w < 16; w++) t += part[w * 64 + lane];
             a.att_out[(int64_t)h * a.att_vdim + e0 + lane] = a.att_scale * t / l;
         }
     }
@@ -323,21 +345,21 @@ constexpr float DELTA_DECAY = 0.60653065971263342f;  // exp(-1/2)
 
 __device__ __forceinline__ float delta_decay(float wl, float w0) { return expf(-DELTA_DECAY * mix_sigmoid(wl + w0)); }
 
-// One head of a token as five vectors of `sp` floats: w | a u | u | k | r, zero beyond dim.  One wave.
+// One head of a token as four vectors of `sp` floats, w | a u | u | r, zero beyond dim, and |k| (k = |k| u).  One wave.
 template <typename WL>
-__device__ __forceinline__ void delta_pack(const float *r, const float *k, const float *al, WL wl, const float *w0, const float *ab, float *dst, int dim, int sp,
-                                           int lane) {
+__device__ __forceinline__ void delta_pack(const float *r, const float *k, const float *al, WL wl, const float *w0, const float *ab, float *dst, float *k_norm, int dim,
+                                           int sp, int lane) {
     float s = 0.0f;
     for (int d = lane; d < dim; d += 64) s = fmaf(k[d], k[d], s);
-    const float inv = 1.0f / sqrtf(wave_sum(s) + DELTA_UNIT_EPS);
+    const float norm = sqrtf(wave_sum(s) + DELTA_UNIT_EPS), inv = 1.0f / norm;
+    if (lane == 0) k_norm[0] = norm;
     for (int d = lane; d < sp; d += 64) {
         const bool ok = d < dim;
-        const float kd = ok ? k[d] : 0.0f, u = kd * inv;
+        const float u = ok ? k[d] * inv : 0.0f;
         dst[d] = ok ? delta_decay(wl(d), w0[d]) : 0.0f;
         dst[sp + d] = ok ? mix_sigmoid(al[d] + ab[d]) * u : 0.0f;
         dst[2 * sp + d] = u;
-        dst[3 * sp + d] = kd;
-        dst[4 * sp + d] = ok ? r[d] : 0.0f;
+        dst[3 * sp + d] = ok ? r[d] : 0.0f;
     }
 }
 
@@ -350,43 +372,59 @@ __global__ __launch_bounds__(256) void delta_prep_kernel(const float *__restrict
     const int64_t t = id / heads;
     const int64_t hd = (id - t * heads) * dim;
     const float *s = row + t * row_stride + hd, *w = wl + t * wl_stride + hd;
-    delta_pack(s + r_off, s + k_off, s + a_off, [&](int d) { return w[d]; }, w0 + hd, ab + hd, packed + id * 5 * sp, dim, sp, lane);
+    delta_pack(s + r_off, s + k_off, s + a_off, [&](int d) { return w[d]; }, w0 + hd, ab + hd, packed + id * 4 * sp, packed + rows * heads * 4 * sp + id, dim, sp, lane);
 }
 
-// One column step: s <- w s - b (u . s) + k v; returns this lane's part of r . s.  The 16 lanes of a column hold 4 NR rows each.
+// The rows of a column that a lane holds, and one token's vectors on them.
 template <int NR>
-__device__ __forceinline__ float delta_column(f32x4 (&s)[NR], const f32x4 (&w)[NR], const f32x4 (&b)[NR], const f32x4 (&u)[NR], const f32x4 (&k)[NR],
-                                              const f32x4 (&r)[NR], float v) {
+struct DeltaRows {
+    f32x4 w[NR], b[NR], u[NR], r[NR];
+    __device__ __forceinline__ void load(const float *vec, int sub) {
+#pragma unroll
+        for (int c = 0; c < NR; c++) {
+            const float *x = vec + 64 * c + 4 * sub;
+            w[c] = *reinterpret_cast<const f32x4 *>(x);
+            b[c] = *reinterpret_cast<const f32x4 *>(x + 64 * NR);
+            u[c] = *reinterpret_cast<const f32x4 *>(x + 2 * 64 * NR);
+            r[c] = *reinterpret_cast<const f32x4 *>(x + 3 * 64 * NR);
+        }
+    }
+};
+
+// One column step: s <- w s - b (u . s) + u v (v: the value times |k|); returns this lane's part of r . s.
+template <int NR>
+__device__ __forceinline__ float delta_column(f32x4 (&s)[NR], const DeltaRows<NR> &x, float v) {
     float x0 = 0.0f, x1 = 0.0f;
 #pragma unroll
     for (int c = 0; c < NR; c++) {
-        x0 = fmaf(u[c].x, s[c].x, x0);
-        x1 = fmaf(u[c].y, s[c].y, x1);
-        x0 = fmaf(u[c].z, s[c].z, x0);
-        x1 = fmaf(u[c].w, s[c].w, x1);
+        x0 = fmaf(x.u[c].x, s[c].x, x0);
+        x1 = fmaf(x.u[c].y, s[c].y, x1);
+        x0 = fmaf(x.u[c].z, s[c].z, x0);
+        x1 = fmaf(x.u[c].w, s[c].w, x1);
     }
     const float us = row16_sum(x0 + x1);
     float o0 = 0.0f, o1 = 0.0f;
 #pragma unroll
     for (int c = 0; c < NR; c++) {
 #pragma unroll
-        for (int e = 0; e < 4; e++) s[c][e] = fmaf(-b[c][e], us, fmaf(w[c][e], s[c][e], k[c][e] * v));
-        o0 = fmaf(r[c].x, s[c].x, o0);
-        o1 = fmaf(r[c].y, s[c].y, o1);
-        o0 = fmaf(r[c].z, s[c].z, o0);
-        o1 = fmaf(r[c].w, s[c].w, o1);
+        for (int e = 0; e < 4; e++) s[c][e] = fmaf(-x.b[c][e], us, fmaf(x.w[c][e], s[c][e], x.u[c][e] * v));
+        o0 = fmaf(x.r[c].x, s[c].x, o0);
+        o1 = fmaf(x.r[c].y, s[c].y, o1);
+        o0 = fmaf(x.r[c].z, s[c].z, o0);
+        o1 = fmaf(x.r[c].w, s[c].w, o1);
     }
     return o0 + o1;
 }
 
 // Token after token.  Workgroup: 16 value columns of one head, 4 waves x 4 columns; the packed vectors of TB tokens at a time go
-// through LDS (double-buffered: the next block's loads are in flight while this one runs), one token ahead into registers.
+// through LDS (double-buffered: the next block's loads are in flight while this one runs) and from there, one token ahead, into
+// registers.  The lanes' parts of r . s are collected for the block and summed 16 tokens at a time, off the chain of state updates.
 template <int NR, int TB>
 __global__ __launch_bounds__(256) void delta_scan_kernel(const float *__restrict__ packed, const float *__restrict__ v, int64_t v_stride,
                                                          float *__restrict__ state, float *__restrict__ out, int64_t out_stride, int rows, int heads, int dim,
                                                          int ncb) {
-    constexpr int SP = 64 * NR, VEC = 5 * SP, LOADS = TB * VEC / 4 / 256;
-    static_assert(TB * VEC % 1024 == 0, "whole float4 per thread");
+    constexpr int SP = 64 * NR, VEC = 4 * SP, LOADS = TB * VEC / 4 / 256;
+    static_assert(TB * VEC % 1024 == 0 && TB <= 16, "whole float4 per thread");
     extern __shared__ __attribute__((aligned(16))) float smem[];         // 2 x { packed [TB][VEC], v [TB][16] }
     const int tid = threadIdx.x, lane = tid & 63, wv = __builtin_amdgcn_readfirstlane(tid >> 6), sub = lane & 15, cg = lane >> 4;
     // workgroups of one head on one XCD (dealt round-robin): they read the same packed vectors
@@ -400,22 +438,28 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(const float *__restrict
     for (int c = 0; c < NR; c++) s[c] = *reinterpret_cast<const f32x4 *>(st + 64 * c);
     const int64_t tok = (int64_t)heads * VEC;
     const float *src = packed + (int64_t)h * VEC;
+    const float *knorm = packed + (int64_t)rows * tok + h;
     const float *vsrc = v + (int64_t)h * dim + min(16 * cb + (tid & 15), dim - 1);
+    float *dst = out + (int64_t)h * dim + col;
 
     f32x4 ld[LOADS];
-    float ldv = 0.0f;
+    float ldv = 0.0f, ldk = 0.0f;
     auto fetch = [&](int t0) {
 #pragma unroll
         for (int i = 0; i < LOADS; i++) {
             const int x = tid + 256 * i, t = min(t0 + x / (VEC / 4), rows - 1);
             ld[i] = *reinterpret_cast<const f32x4 *>(src + t * tok + 4 * (x % (VEC / 4)));
         }
-        if (tid < TB * 16) ldv = vsrc[(int64_t)min(t0 + (tid >> 4), rows - 1) * v_stride];
+        if (tid < TB * 16) {
+            const int64_t t = min(t0 + (tid >> 4), rows - 1);
+            ldv = vsrc[t * v_stride];
+            ldk = knorm[t * heads];
+        }
     };
-    auto stage = [&](float *dst) {
+    auto stage = [&](float *to) {
 #pragma unroll
-        for (int i = 0; i < LOADS; i++) *reinterpret_cast<f32x4 *>(dst + 4 * (tid + 256 * i)) = ld[i];
-        if (tid < TB * 16) dst[TB * VEC + tid] = ldv;
+        for (int i = 0; i < LOADS; i++) *reinterpret_cast<f32x4 *>(to + 4 * (tid + 256 * i)) = ld[i];
+        if (tid < TB * 16) to[TB * VEC + tid] = ldv * ldk;
     };
     constexpr int BUF = TB * VEC + TB * 16;
     fetch(0);
@@ -425,27 +469,36 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(const float *__restrict
     for (int t0 = 0; t0 < rows; t0 += TB) {
         const bool more = t0 + TB < rows;
         if (more) fetch(t0 + TB);
-        const float *b = smem + cur * BUF;
+        const float *b = smem + cur * BUF, *bv = b + TB * VEC + 4 * wv + cg;
         const int n = min(TB, rows - t0);
-        auto body = [&](int t) {
-            const float *x = b + t * VEC + 4 * sub;
-            f32x4 w[NR], a[NR], u[NR], k[NR], r[NR];
-#pragma unroll
-            for (int c = 0; c < NR; c++) {
-                w[c] = *reinterpret_cast<const f32x4 *>(x + 64 * c);
-                a[c] = *reinterpret_cast<const f32x4 *>(x + SP + 64 * c);
-                u[c] = *reinterpret_cast<const f32x4 *>(x + 2 * SP + 64 * c);
-                k[c] = *reinterpret_cast<const f32x4 *>(x + 3 * SP + 64 * c);
-                r[c] = *reinterpret_cast<const f32x4 *>(x + 4 * SP + 64 * c);
-            }
-            const float o = row16_sum(delta_column<NR>(s, w, a, u, k, r, b[TB * VEC + 16 * t + 4 * wv + cg]));
-            if (sub == 0 && col < dim) out[(int64_t)(t0 + t) * out_stride + (int64_t)h * dim + col] = o;
-        };
         if (n == TB) {
+            DeltaRows<NR> x[2];
+            float vx[2], o[TB];
+            x[0].load(b, sub);
+            vx[0] = bv[0];
 #pragma unroll
-            for (int t = 0; t < TB; t++) body(t);
+            for (int t = 0; t < TB; t++) {
+                if (t + 1 < TB) {
+                    x[(t + 1) & 1].load(b + (t + 1) * VEC, sub);
+                    vx[(t + 1) & 1] = bv[16 * (t + 1)];
+                }
+                o[t] = delta_column<NR>(s, x[t & 1], vx[t & 1]);
+            }
+            // lane `sub` ends with the sum of token t0 + sub
+            float mine = 0.0f;
+#pragma unroll
+            for (int t = 0; t < TB; t++) {
+                const float sum = row16_sum(o[t]);
+                mine = sub == t ? sum : mine;
+            }
+            if (sub < TB && col < dim) dst[(int64_t)(t0 + sub) * out_stride] = mine;
         } else {
-            for (int t = 0; t < n; t++) body(t);
+            for (int t = 0; t < n; t++) {
+                DeltaRows<NR> x;
+                x.load(b + t * VEC, sub);
+                const float o = row16_sum(delta_column<NR>(s, x, bv[16 * t]));
+                if (sub == 0 && col < dim) dst[(int64_t)(t0 + t) * out_stride] = o;
+            }
         }
         if (more) {
             stage(smem + (cur ^ 1) * BUF);
@@ -468,19 +521,29 @@ struct DeltaStep {
     float eps;
 };
 
-// one token, one head per workgroup
+// One token, one head per workgroup of 16 waves.  The first 64 state columns are requested before anything else.
 template <int NR>
-__global__ __launch_bounds__(512) void delta_step_kernel(DeltaStep a) {
+__global__ __launch_bounds__(1024) void delta_step_kernel(DeltaStep a) {
     constexpr int SP = 64 * NR;
     extern __shared__ __attribute__((aligned(16))) float low[];           // tanh of the rank values, zero up to ldw2
-    __shared__ __attribute__((aligned(16))) float vec[5 * SP], wl[SP], os[SP];
-    __shared__ float s_inv;
+    __shared__ __attribute__((aligned(16))) float vec[4 * SP], wl[SP], os[SP];
+    __shared__ float s_inv, k_norm;
     const int tid = threadIdx.x, lane = tid & 63, wv = __builtin_amdgcn_readfirstlane(tid >> 6), sub = lane & 15, cg = lane >> 4;
     const int h = blockIdx.x;
     const int64_t hd = (int64_t)h * a.dim;
-    for (int i = tid; i < a.ldw2; i += 512) low[i] = i < a.rank ? tanhf(a.row[a.low_off + i]) : 0.0f;
+    f32x4 s[NR];
+    float vj;
+    auto load = [&](int c0) {
+        const int col = min(c0 + cg, a.dim - 1);
+        const float *st = a.state + (hd + col) * SP + 4 * sub;
+#pragma unroll
+        for (int c = 0; c < NR; c++) s[c] = *reinterpret_cast<const f32x4 *>(st + 64 * c);
+        vj = a.row[a.v_off + hd + col];
+    };
+    load(4 * wv);
+    for (int i = tid; i < a.ldw2; i += 1024) low[i] = i < a.rank ? tanhf(a.row[a.low_off + i]) : 0.0f;
     __syncthreads();
-    for (int i0 = wv * 4; i0 < a.dim; i0 += 32) {
+    for (int i0 = wv * 4; i0 < a.dim; i0 += 64) {
         const uint16_t *w = a.w2 + (hd + min(i0 + cg, a.dim - 1)) * a.ldw2;
         float acc = 0.0f;
         for (int j = 4 * sub; j < a.ldw2; j += 64) {
@@ -496,31 +559,20 @@ __global__ __launch_bounds__(512) void delta_step_kernel(DeltaStep a) {
     }
     __syncthreads();
     if (wv == 0) {
-        const float *s = a.row + hd;
-        delta_pack(s + a.r_off, s + a.k_off, s + a.a_off, [&](int d) { return wl[d]; }, a.w0 + hd, a.ab + hd, vec, a.dim, SP, lane);
+        const float *x = a.row + hd;
+        delta_pack(x + a.r_off, x + a.k_off, x + a.a_off, [&](int d) { return wl[d]; }, a.w0 + hd, a.ab + hd, vec, &k_norm, a.dim, SP, lane);
     }
     __syncthreads();
-    f32x4 w[NR], b[NR], u[NR], k[NR], r[NR];
-#pragma unroll
-    for (int c = 0; c < NR; c++) {
-        const float *x = vec + 64 * c + 4 * sub;
-        w[c] = *reinterpret_cast<const f32x4 *>(x);
-        b[c] = *reinterpret_cast<const f32x4 *>(x + SP);
-        u[c] = *reinterpret_cast<const f32x4 *>(x + 2 * SP);
-        k[c] = *reinterpret_cast<const f32x4 *>(x + 3 * SP);
-        r[c] = *reinterpret_cast<const f32x4 *>(x + 4 * SP);
-    }
-    for (int c0 = 4 * wv; c0 < a.dim; c0 += 32) {
-        const int col = min(c0 + cg, a.dim - 1);
-        float *st = a.state + (hd + col) * SP + 4 * sub;
-        f32x4 s[NR];
-#pragma unroll
-        for (int c = 0; c < NR; c++) s[c] = *reinterpret_cast<const f32x4 *>(st + 64 * c);
-        const float o = row16_sum(delta_column<NR>(s, w, b, u, k, r, a.row[a.v_off + hd + col]));
+    DeltaRows<NR> x;
+    x.load(vec, sub);
+    for (int c0 = 4 * wv; c0 < a.dim; c0 += 64) {
+        if (c0 >= 64) load(c0);
+        const float o = row16_sum(delta_column<NR>(s, x, vj * k_norm));
         if (c0 + cg < a.dim) {
+            float *st = a.state + (hd + c0 + cg) * SP + 4 * sub;
 #pragma unroll
             for (int c = 0; c < NR; c++) *reinterpret_cast<f32x4 *>(st + 64 * c) = s[c];
-            if (sub == 0) os[col] = o;
+            if (sub == 0) os[c0 + cg] = o;
         }
     }
     __syncthreads();
@@ -529,7 +581,7 @@ __global__ __launch_bounds__(512) void delta_step_kernel(DeltaStep a) {
         if (lane == 0) s_inv = inv;
     }
     __syncthreads();
-    for (int e = tid; e < a.dim; e += 512) a.out[hd + e] = os[e] * s_inv * a.weight[hd + e] * mix_sigmoid(a.row[a.g_off + hd + e]);
+    for (int e = tid; e < a.dim; e += 1024) a.out[hd + e] = os[e] * s_inv * a.weight[hd + e] * mix_sigmoid(a.row[a.g_off + hd + e]);
 }
 
 }  // namespace
@@ -569,10 +621,11 @@ int cq_mix_retention(const float *q_dev, const float *k_dev, const float *v_dev,
         const int e = (int)hipFuncSetAttribute(reinterpret_cast<const void *>(retention_kernel), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
         if (e) return e;
     }
-    if (a.nseg > 1) hipLaunchKernelGGL(retention_segment_kernel, grid, dim3(256), 0, s, a);
+    if (a.nseg > 1) {
+        hipLaunchKernelGGL(retention_segment_kernel, grid, dim3(256), 0, s, a);
+        hipLaunchKernelGGL(retention_prefix_kernel, dim3((unsigned)((a.nvb * a.dp * 64 + 255) / 256), (unsigned)heads), dim3(256), 0, s, a);
+    }
     hipLaunchKernelGGL(retention_kernel, grid, dim3(256), lds, s, a);
-    if (a.nseg > 1)
-        hipLaunchKernelGGL(retention_state_kernel, dim3((unsigned)((vdim * dim_pad + 255) / 256), (unsigned)heads), dim3(256), 0, s, a);
     return (int)hipGetLastError();
 }
 
@@ -600,14 +653,14 @@ int cq_mix_talk_merge_retention_step(const void *workspace_dev, int64_t n_head, 
     a.att_out = att_out_dev; a.state = state_dev; a.ret_out = ret_out_dev; a.row = row_dev; a.decay = decay_dev;
     a.gq = qk[0]; a.gk = qk[1]; a.v_off = v_off; a.g_off = g_off; a.heads = (int)heads; a.vdim = (int)vdim;
     const int sp = (int)cq_mix_state_pad(qk[0].dim);
-    const int f0 = (a.splits + 3) / 4 * 4 + 512, f1 = 2 * sp + a.vdim;
+    const int f0 = (a.splits + 3) / 4 * 4 + 1024, f1 = 2 * sp + a.vdim;
     const size_t lds = (size_t)(f0 > f1 ? f0 : f1) * sizeof(float);
     if (lds > 64 * 1024) return CQ_ERR_RANGE;
     hipStream_t s = (hipStream_t)stream;
     const dim3 grid((unsigned)(n_head + heads));
-    if (sp == 64) hipLaunchKernelGGL(talk_merge_retention_kernel<1>, grid, dim3(512), lds, s, a, pos_dev, (int)pos);
-    else if (sp == 128) hipLaunchKernelGGL(talk_merge_retention_kernel<2>, grid, dim3(512), lds, s, a, pos_dev, (int)pos);
-    else hipLaunchKernelGGL(talk_merge_retention_kernel<4>, grid, dim3(512), lds, s, a, pos_dev, (int)pos);
+    if (sp == 64) hipLaunchKernelGGL(talk_merge_retention_kernel<1>, grid, dim3(1024), lds, s, a, pos_dev, (int)pos);
+    else if (sp == 128) hipLaunchKernelGGL(talk_merge_retention_kernel<2>, grid, dim3(1024), lds, s, a, pos_dev, (int)pos);
+    else hipLaunchKernelGGL(talk_merge_retention_kernel<4>, grid, dim3(1024), lds, s, a, pos_dev, (int)pos);
     return (int)hipGetLastError();
 }
 
@@ -636,7 +689,7 @@ int cq_mix_delta_scan(const float *packed_dev, const float *v_dev, int64_t v_str
     hipStream_t s = (hipStream_t)stream;
 #define CQ_DS(NR_, TB_)                                                                                                                                   \
     do {                                                                                                                                                   \
-        const size_t lds = (size_t)2 * (TB_ * 5 * 64 * NR_ + TB_ * 16) * sizeof(float);                                                                    \
+        const size_t lds = (size_t)2 * (TB_ * 4 * 64 * NR_ + TB_ * 16) * sizeof(float);                                                                    \
         if (lds > 64 * 1024) {                                                                                                                             \
             const int e = (int)hipFuncSetAttribute(reinterpret_cast<const void *>(delta_scan_kernel<NR_, TB_>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds); \
             if (e) return e;                                                                                                                               \
@@ -666,9 +719,9 @@ int cq_mix_delta_step(const float *row_dev, int64_t r_off, int64_t k_off, int64_
     const size_t lds = (size_t)ldw2 * sizeof(float);
     hipStream_t s = (hipStream_t)stream;
     const int sp = (int)cq_mix_state_pad(dim);
-    if (sp == 64) hipLaunchKernelGGL(delta_step_kernel<1>, dim3((unsigned)heads), dim3(512), lds, s, a);
-    else if (sp == 128) hipLaunchKernelGGL(delta_step_kernel<2>, dim3((unsigned)heads), dim3(512), lds, s, a);
-    else hipLaunchKernelGGL(delta_step_kernel<4>, dim3((unsigned)heads), dim3(512), lds, s, a);
+    if (sp == 64) hipLaunchKernelGGL(delta_step_kernel<1>, dim3((unsigned)heads), dim3(1024), lds, s, a);
+    else if (sp == 128) hipLaunchKernelGGL(delta_step_kernel<2>, dim3((unsigned)heads), dim3(1024), lds, s, a);
+    else hipLaunchKernelGGL(delta_step_kernel<4>, dim3((unsigned)heads), dim3(1024), lds, s, a);
     return (int)hipGetLastError();
 }
 

@@ -329,7 +329,7 @@ class GeneralDelta(Mixer):
         ldp, ldw, ldo = pad_to(self.w_in.n, 4), pad_to(w, 4), self.w_out.kp
         row = rt.scratch("projection", rows * ldp)
         low, wl = rt.scratch("delta_low", rows * self.w2.kp), rt.scratch("delta_decay", rows * ldw)
-        packed = rt.scratch("delta_packed", rows * self.heads * 5 * L.cq_mix_state_pad(self.dim))
+        packed = rt.scratch("delta_packed", rows * self.heads * (4 * L.cq_mix_state_pad(self.dim) + 1))
         raw, out = rt.scratch("mixer_raw", rows * w), rt.scratch("mixer_out", rows * ldo)
         self.w_in.rows(h, ldh, row, ldp, rows, sp)
         check("cq_mix_tanh", L.cq_mix_tanh(row + 4 * self.low_off, ldp, low, self.w2.kp, rows, self.rank, sp))

@@ -119,7 +119,8 @@ int cq_mix_talk_merge_retention_step(const void *workspace_dev, int64_t n_head, 
  * S <- diag(w) S - (a u)(u^T S) + k v^T (both terms read the old S), o = S^T r, u = k / sqrt(sum(k^2) + 1e-6),
  * w = exp(-exp(-1/2) sigmoid(wl + w0)), a = sigmoid(al + a_bias).  States [heads, dim, state_pad], column-major as above.
  * row_dev: projection rows with r, k, v, al at the given offsets (each heads * dim); wl [rows, heads * dim].
- * cq_mix_delta_prep packs w | a u | u | k | r per (row, head), state_pad floats each, for cq_mix_delta_scan, whose out is the raw o. */
+ * cq_mix_delta_prep packs w | a u | u | r per (row, head), state_pad floats each, and behind them the |k| = sqrt(sum(k^2) + 1e-6) of every
+ * (row, head), rows * heads * (4 state_pad + 1) floats in all, for cq_mix_delta_scan, whose out is the raw o. */
 int cq_mix_delta_prep(const float *row_dev, int64_t row_stride, int64_t r_off, int64_t k_off, int64_t a_off, const float *wl_dev, int64_t wl_stride,
                       const float *w0_dev, const float *a_bias_dev, float *packed_dev, int64_t rows, int64_t heads, int64_t dim, void *stream);
 int cq_mix_delta_scan(const float *packed_dev, const float *v_dev, int64_t v_stride, float *state_dev, float *out_dev, int64_t out_stride, int64_t rows,
