@@ -98,7 +98,8 @@ MIXER_SIGNATURES = {
     "cq_mix_tanh": (_int, [_vp, _i64, _vp, _i64, _i64, _i64, _vp]),
     "cq_mix_pack_heads": (_int, [_vp, _i64, _heads, _int, _f32, _vp, _i64, _i64, _vp]),
     "cq_mix_head_norm_gate": (_int, [_vp, _i64, _vp, _i64, _vp, _int, _f32, _vp, _i64, _i64, _i64, _i64, _f32, _vp]),
-    "cq_mix_talk_attention": (_int, [_vp, _vp, _vp, _vp, _f32, _i64, _i64, _f32, _vp, _i64, _i64, _i64, _i64, _i64, _i64, _i64, _i64, _i64, _vp]),
+    "cq_mix_talk_attention_workspace_bytes": (_i64, [_i64, _i64, _i64, _i64, _i64, _i64]),
+    "cq_mix_talk_attention": (_int, [_vp, _vp, _vp, _vp, _f32, _i64, _i64, _f32, _vp, _i64, _i64, _i64, _i64, _i64, _i64, _i64, _i64, _i64, _vp, _i64, _vp]),
     "cq_mix_talk_decode_workspace_bytes": (_i64, [_i64, _i64, _i64, _i64, _i64]),
     "cq_mix_talk_decode": (_int, [_vp, _heads, _f32, _vp, _f32, _i64, _i64, _vp, _i64, _vp, _i64, _vp]),
     "cq_mix_state_pad": (_i64, [_i64]),

@@ -16,14 +16,15 @@ template <typename T> __device__ __forceinline__ T ld_at(const float *base, uint
 //   mixing   wave w takes 16 / NW queries of every head: talk x scores on the matrix cores (heads are the contracted
 //            dimension), mask, running softmax in registers, weights back into the same LDS words, rescale factors to `alpha`
 //   values   wave w takes U units (head, 64 output columns): weights x V added to the outputs it holds in registers, V read once per VS units
-// blockIdx.y: units beyond NW U (the scores are computed again there).
+// blockIdx.y: units beyond NW U (the scores are computed again there).  blockIdx.z: split of the key tiles, for calls with too few
+// query rows to fill the chip; a split leaves unnormalized outputs with their maximum and sum, talk_combine_kernel merges them.
 // LDS strides: query rows of KT + 4 floats (16 rows x 4 keys of an operand read fall on 64 banks), head blocks of 16 rows + 16
 // (4 heads x 16 keys likewise).
 template <int NW, int NHW, bool SHARED_K, int U, int VS, int KT>
 __global__ __launch_bounds__(64 * NW) void talk_attention_kernel(const float *__restrict__ q, const float *__restrict__ k_cache, const float *__restrict__ v_cache,
                                                              const float *__restrict__ talk, float scale, int window, int keep_first, float out_scale,
-                                                             float *__restrict__ out, int64_t out_stride, int pos, int rows, int H, int G, int dp, int vdim,
-                                                             int vp, int ctx) {
+                                                             float *__restrict__ out, int64_t out_stride, float *__restrict__ part, int pos, int rows, int H, int G,
+                                                             int dp, int vdim, int vp, int ctx) {
     constexpr int NHT = (NW * NHW + 15) / 16, HP = 16 * NHT, NT = 64 * NW, RW = 16 / NW;       // heads padded to tiles of 16; queries per wave
     constexpr int RS = KT + 4, HS = 16 * RS + 16, TS = HP + 4, KTL = KT / 16;
     extern __shared__ __attribute__((aligned(16))) float smem[];
@@ -43,6 +44,7 @@ __global__ __launch_bounds__(64 * NW) void talk_attention_kernel(const float *__
         m_run[i] = -INFINITY;
         l_run[i] = 0.0f;
     }
+    __syncthreads();
     f32x4 o[U][4];
 #pragma unroll
     for (int u = 0; u < U; u++)
@@ -57,7 +59,8 @@ __global__ __launch_bounds__(64 * NW) void talk_attention_kernel(const float *__
     // tiles of the kept first tokens, then of the window
     const int t_lo = max(0, p0 - window + 1) / KT, t_hi = last / KT;
     const int n_keep = min((keep_first + KT - 1) / KT, t_lo);
-    for (int it = 0; it < n_keep + t_hi - t_lo + 1; it++) {
+    const int n_tiles = n_keep + t_hi - t_lo + 1, nz = gridDim.z, z = blockIdx.z;
+    for (int it = n_tiles * z / nz; it < n_tiles * (z + 1) / nz; it++) {
         const int j0 = (it < n_keep ? it : t_lo + it - n_keep) * KT;
         // ---- scores ----
         if (h0 < H) {
@@ -202,15 +205,60 @@ __global__ __launch_bounds__(64 * NW) void talk_attention_kernel(const float *__
 #pragma unroll
             for (int e = 0; e < 4; e++) {
                 const int row = 4 * lk + e;
-                if (row < nr) out[(int64_t)(r0 + row) * out_stride + (int64_t)h * vdim + col] = out_scale * o[u][n][e] / l_run[h * 16 + row];
+                if (row >= nr) continue;
+                if (nz == 1) out[(int64_t)(r0 + row) * out_stride + (int64_t)h * vdim + col] = out_scale * o[u][n][e] / l_run[h * 16 + row];
+                else part[((int64_t)(z * rows + r0 + row) * H + h) * vdim + col] = o[u][n][e];
             }
+        }
+    }
+    if (nz > 1 && blockIdx.y == 0) {
+        float *ml = part + (int64_t)nz * rows * H * vdim;                 // [split][row][head] of (m, l)
+        for (int i = tid; i < nr * H; i += NT) {
+            const int row = i / H, h = i - row * H;
+            float *x = ml + 2 * ((int64_t)(z * rows + r0 + row) * H + h);
+            x[0] = m_run[h * 16 + row];
+            x[1] = l_run[h * 16 + row];
         }
     }
 }
 
+// one wave per (row, head)
+__global__ __launch_bounds__(256) void talk_combine_kernel(const float *__restrict__ part, int nz, int64_t rows, int H, int vdim, float out_scale,
+                                                           float *__restrict__ out, int64_t out_stride) {
+    const int lane = threadIdx.x & 63;
+    const int64_t id = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6), n = rows * H;
+    if (id >= n) return;
+    const float *ml = part + nz * n * vdim + 2 * id;
+    float m = -INFINITY, l = 0.0f;
+    for (int z = 0; z < nz; z++) m = fmaxf(m, ml[2 * n * z]);
+    for (int z = 0; z < nz; z++) l = fmaf(ml[2 * n * z] > -INFINITY ? __expf(ml[2 * n * z] - m) : 0.0f, ml[2 * n * z + 1], l);
+    const int64_t r = id / H;
+    float *o = out + r * out_stride + (id - r * H) * vdim;
+    for (int e = lane; e < vdim; e += 64) {
+        float a = 0.0f;
+        for (int z = 0; z < nz; z++) {
+            const float w = ml[2 * n * z] > -INFINITY ? __expf(ml[2 * n * z] - m) : 0.0f;
+            a = fmaf(w, part[(n * z + id) * vdim + e], a);
+        }
+        o[e] = out_scale * a / l;
+    }
+}
+
+// Splits of the key tiles: as many as bring the launch to one workgroup per CU, each with at least four tiles of keys.
+int talk_key_splits(int64_t rows, int64_t unit_blocks, int64_t max_keys) {
+    const int64_t wg = (rows + 15) / 16 * unit_blocks, tiles = max_keys / 32;
+    int64_t n = 256 / wg;
+    n = n < tiles / 4 ? n : tiles / 4;
+    return (int)(n < 1 ? 1 : (n > 16 ? 16 : n));
+}
+int talk_unit_blocks(int64_t H, int64_t vp) {               // units a launch takes: NW * U of the instance for H heads
+    const int64_t per = H <= 8 ? 16 : (H <= 16 ? 32 : 64);
+    return (int)((H * ((vp + 63) / 64) + per - 1) / per);
+}
+
 template <int NW, int NHW, bool SHARED_K, int U, int VS, int KT>
 int talk_launch(const float *q, const float *kc, const float *vc, const float *talk, float scale, int window, int keep, float out_scale, float *out,
-                int64_t out_stride, int pos, int rows, int H, int G, int dp, int vdim, int vp, int ctx, hipStream_t s) {
+                int64_t out_stride, float *part, int nz, int pos, int rows, int H, int G, int dp, int vdim, int vp, int ctx, hipStream_t s) {
     constexpr int HP = (NW * NHW + 15) / 16 * 16;
     constexpr size_t lds = (size_t)(HP * (16 * (KT + 4) + 16) + HP * (HP + 4) + 3 * HP * 16) * sizeof(float);
     if (lds > 64 * 1024) {
@@ -219,8 +267,11 @@ int talk_launch(const float *q, const float *kc, const float *vc, const float *t
         if (e) return e;
     }
     const int units = H * ((vp + 63) / 64);
-    hipLaunchKernelGGL((talk_attention_kernel<NW, NHW, SHARED_K, U, VS, KT>), dim3((rows + 15) / 16, (units + NW * U - 1) / (NW * U)), dim3(64 * NW), lds, s, q,
-                       kc, vc, talk, scale, window, keep, out_scale, out, out_stride, pos, rows, H, G, dp, vdim, vp, ctx);
+    hipLaunchKernelGGL((talk_attention_kernel<NW, NHW, SHARED_K, U, VS, KT>), dim3((rows + 15) / 16, (units + NW * U - 1) / (NW * U), nz), dim3(64 * NW), lds,
+                       s, q, kc, vc, talk, scale, window, keep, out_scale, out, out_stride, part, pos, rows, H, G, dp, vdim, vp, ctx);
+    if (nz > 1)
+        hipLaunchKernelGGL(talk_combine_kernel, dim3((unsigned)(((int64_t)rows * H + 3) / 4)), dim3(256), 0, s, (const float *)part, nz, (int64_t)rows, H, vdim, out_scale,
+                           out, out_stride);
     return (int)hipGetLastError();
 }
 
@@ -237,8 +288,8 @@ __global__ __launch_bounds__(1024) void talk_decode_kernel(const float *__restri
                                                            const int32_t *__restrict__ pos_dev, int pos0, float *__restrict__ rec, int splits) {
     extern __shared__ __attribute__((aligned(16))) float smem[];
     const int H = gq.heads, G = gk.heads, R = H / G, dp = gk.dim_pad, vdim = gv.dim, vp = gv.dim_pad, ctx = gk.ctx;
-    constexpr int SS = KD + 1, PB = 2;
-    float *qs = smem, *kn = qs + H * dp, *vn = kn + G * dp, *T = vn + G * vp, *sc = T + H * H, *mx = sc + H * SS;
+    constexpr int SS = KD + 4, PB = 2;                               // rows of scores start on 16 bytes
+    float *qs = smem, *kn = qs + H * dp, *vn = kn + G * dp, *sc = vn + G * vp, *mx = sc + H * SS, *T = mx + H * SS;
     const int tid = threadIdx.x, lane = tid & 63, wv = __builtin_amdgcn_readfirstlane(tid >> 6), sp = blockIdx.x;
     const int p = pos0 + (pos_dev ? pos_dev[0] : 0);
     const Visible vis = visible_keys(p, window, keep_first);
@@ -383,9 +434,11 @@ __global__ __launch_bounds__(1024) void talk_decode_kernel(const float *__restri
                     for (int j = 0; j < 16; j++) vv[j] = jb + j >= cnt - 1 ? x : vv[j];
                 }
 #pragma unroll
-                for (int j = 0; j < 16; j++)
+                for (int x = 0; x < 4; x++) {
+                    const f32x4 *w = reinterpret_cast<const f32x4 *>(sc + (g * R + min(r + x, R - 1)) * SS + jb);
 #pragma unroll
-                    for (int x = 0; x < 4; x++) a[x] = fmaf(sc[(g * R + min(r + x, R - 1)) * SS + jb + j], vv[j], a[x]);
+                    for (int j = 0; j < 16; j++) a[x] = fmaf(w[j >> 2][j & 3], vv[j], a[x]);
+                }
             }
 #pragma unroll
             for (int x = 0; x < 4; x++)
@@ -398,7 +451,7 @@ template <int NC, int KD>
 int talk_decode_launch(const float *row, const cq_mix_heads *g, float eps, const float *talk, float scale, int window, int keep, const int32_t *pos_dev, int pos,
                        float *rec, int splits, hipStream_t s) {
     const int H = g[0].heads, G = g[1].heads;
-    const size_t lds = (size_t)(H * (g[1].dim_pad + 2 * (KD + 1) + H) + G * (g[1].dim_pad + g[2].dim_pad)) * sizeof(float);
+    const size_t lds = (size_t)(H * (g[1].dim_pad + 2 * (KD + 4) + H) + G * (g[1].dim_pad + g[2].dim_pad)) * sizeof(float);
     if (lds > 160 * 1024) return CQ_ERR_RANGE;
     if (lds > 64 * 1024) {
         const int e = (int)hipFuncSetAttribute(reinterpret_cast<const void *>(talk_decode_kernel<NC, KD>), hipFuncAttributeMaxDynamicSharedMemorySize,
@@ -414,11 +467,17 @@ int talk_decode_launch(const float *row, const cq_mix_heads *g, float eps, const
 
 extern "C" {
 
+int64_t cq_mix_talk_attention_workspace_bytes(int64_t rows, int64_t n_head, int64_t vdim, int64_t window, int64_t keep_first, int64_t pos) {
+    if (rows <= 0 || n_head <= 0 || vdim <= 0 || window < 1 || keep_first < 0 || pos < 0) return 0;
+    const int nz = talk_key_splits(rows, talk_unit_blocks(n_head, (vdim + 15) / 16 * 16), talk_max_keys(window, keep_first, pos + rows));
+    return nz > 1 ? nz * rows * n_head * (vdim + 2) * 4 : 0;
+}
+
 int cq_mix_talk_attention(const float *q_dev, const float *k_cache_dev, const float *v_cache_dev, const float *talk_dev, float scale, int64_t window,
                           int64_t keep_first, float out_scale, float *out_dev, int64_t out_stride, int64_t pos, int64_t rows, int64_t n_head,
-                          int64_t n_kv_head, int64_t dim_pad, int64_t vdim, int64_t vdim_pad, int64_t ctx, void *stream) {
-    if (rows < 0 || pos < 0 || n_head <= 0 || n_kv_head <= 0 || n_head % n_kv_head || dim_pad <= 0 || dim_pad % 16 || vdim <= 0 || vdim_pad % 16 ||
-        vdim_pad < vdim || ctx <= 0 || window < 1 || keep_first < 0 || out_stride < n_head * vdim)
+                          int64_t n_kv_head, int64_t dim_pad, int64_t vdim, int64_t vdim_pad, int64_t ctx, void *workspace_dev, int64_t workspace_bytes, void *stream) {
+    if (rows < 0 || pos < 0 || n_head <= 0 || n_kv_head <= 0 || n_head % n_kv_head || dim_pad <= 0 || dim_pad % 16 || vdim <= 0 || 
+        vdim_pad != (vdim + 15) / 16 * 16 || ctx <= 0 || window < 1 || keep_first < 0 || out_stride < n_head * vdim)
         return CQ_ERR_SHAPE;
     if (rows == 0) return CQ_OK;
     if (!q_dev || !k_cache_dev || !v_cache_dev || !talk_dev || !out_dev) return CQ_ERR_NULL;
@@ -427,10 +486,12 @@ int cq_mix_talk_attention(const float *q_dev, const float *k_cache_dev, const fl
     if (ctx * (dim_pad > vdim_pad ? dim_pad : vdim_pad) * 4 > 0x7fffffffLL) return CQ_ERR_RANGE;      // byte offsets inside a kv head are 32-bit
     const int w = (int)(window < ctx ? window : ctx), keep = (int)(keep_first < ctx ? keep_first : ctx);
     const int H = (int)n_head, G = (int)n_kv_head, R = H / G;
+    const int nz = talk_key_splits(rows, talk_unit_blocks(n_head, vdim_pad), talk_max_keys(window, keep_first, pos + rows));
+    if (nz > 1 && (!workspace_dev || workspace_bytes < cq_mix_talk_attention_workspace_bytes(rows, n_head, vdim, window, keep_first, pos))) return CQ_ERR_WORKSPACE;
     hipStream_t s = (hipStream_t)stream;
 #define CQ_TA(NW_, NHW_, SH_, U_, VS_, KT_)                                                                                                            \
-    talk_launch<NW_, NHW_, SH_, U_, VS_, KT_>(q_dev, k_cache_dev, v_cache_dev, talk_dev, scale, w, keep, out_scale, out_dev, out_stride, (int)pos, (int)rows, \
-                                              H, G, (int)dim_pad, (int)vdim, (int)vdim_pad, (int)ctx, s)
+    talk_launch<NW_, NHW_, SH_, U_, VS_, KT_>(q_dev, k_cache_dev, v_cache_dev, talk_dev, scale, w, keep, out_scale, out_dev, out_stride,      \
+                                              (float *)workspace_dev, nz, (int)pos, (int)rows, H, G, (int)dim_pad, (int)vdim, (int)vdim_pad, (int)ctx, s)
     if (H <= 8) return R % 2 ? CQ_TA(8, 1, true, 2, 1, 32) : CQ_TA(8, 1, true, 2, 2, 32);
     if (H <= 16) return R % 2 ? CQ_TA(16, 1, true, 2, 1, 32) : CQ_TA(16, 1, true, 2, 2, 32);
     if (H <= 32) return R % 2 ? CQ_TA(16, 2, false, 4, 1, 32) : (R % 4 ? CQ_TA(16, 2, true, 4, 2, 32) : CQ_TA(16, 2, true, 4, 4, 32));

@@ -176,9 +176,12 @@ class TalkingAttention:
                        ctx=ctx)]
 
     def attend(self, q: int, kv, out: int, out_stride: int, out_scale: float, pos: int, rows: int, sp) -> None:
-        check("cq_mix_talk_attention", self.rt.L.cq_mix_talk_attention(
+        L = self.rt.L
+        need = L.cq_mix_talk_attention_workspace_bytes(rows, self.heads, self.vdim, self.window, self.keep_first, pos)
+        ws = self.rt.scratch("attention_splits", need // 4) if need else None
+        check("cq_mix_talk_attention", L.cq_mix_talk_attention(
             q, kv[0].data_ptr(), kv[1].data_ptr(), self.talk.data_ptr(), self.scale, self.window, self.keep_first, out_scale, out, out_stride, pos, rows, self.heads,
-            self.kv_heads, self.dp, self.vdim, self.vp, self.rt.ctx, sp))
+            self.kv_heads, self.dp, self.vdim, self.vp, self.rt.ctx, ws, need, sp))
 
     def records(self):
         n = self.rt.L.cq_mix_talk_decode_workspace_bytes(self.heads, self.vdim, self.window, self.keep_first, self.rt.ctx)

@@ -83,11 +83,14 @@ int cq_mix_head_norm_gate(const float *o_dev, int64_t o_stride, const float *g_d
  * score_h = sum_g talk[h, g] * scale * (q_g . k_g), key j visible to position i when j <= i and (i - j < window or j < keep_first), softmax
  * over the visible keys, out[r, h * vdim + e] = out_scale * sum_j p_h(j) v(j).  Query head h uses kv head h / (n_head / n_kv_head).
  * q [rows, n_head, dim_pad], caches [n_kv_head, ctx, dim_pad] and [n_kv_head, ctx, vdim_pad]; dim_pad and vdim_pad are multiples of 16
- * (padding zero), at most CQ_MIX_MAX_DIM; n_head <= CQ_MIX_MAX_HEADS. */
+ * (padding zero; vdim_pad the least one), at most CQ_MIX_MAX_DIM; n_head <= CQ_MIX_MAX_HEADS.  Calls with few rows split the keys over workgroups and merge
+ * through the workspace (0 bytes when not split). */
 #define CQ_MIX_MAX_HEADS 64
+int64_t cq_mix_talk_attention_workspace_bytes(int64_t rows, int64_t n_head, int64_t vdim, int64_t window, int64_t keep_first, int64_t pos);
 int cq_mix_talk_attention(const float *q_dev, const float *k_cache_dev, const float *v_cache_dev, const float *talk_dev, float scale, int64_t window,
                           int64_t keep_first, float out_scale, float *out_dev, int64_t out_stride, int64_t pos, int64_t rows, int64_t n_head,
-                          int64_t n_kv_head, int64_t dim_pad, int64_t vdim, int64_t vdim_pad, int64_t ctx, void *stream);
+                          int64_t n_kv_head, int64_t dim_pad, int64_t vdim, int64_t vdim_pad, int64_t ctx, void *workspace_dev, int64_t workspace_bytes,
+                          void *stream);
 
 /* The same for one new token straight from its projection row: the three groups (q; k and v with their caches as dst, by_position
  * set) are normalized, rotated and appended as cq_mix_pack_heads would, then attended, in one launch that leaves a record per split of
