@@ -286,7 +286,7 @@ Plan plan(int precision, int64_t m, int64_t n, int64_t k) {
 }
 
 // ---- one row --------------------------------------------------------------------------------------------------------------
-// 8 waves; a wave takes one weight row at a time and walks it in blocks of 64 lanes x 8 elements x U, one block ahead; the first
+// 8 waves; a wave takes one weight row at a time and walks it in blocks of 64 lanes x 8 elements x 4, one block ahead; the first
 // block is requested before the prologue.  Weights are read once per step: non-temporal loads (33.3 -> 27.1 us on 4096 x 14336).  At most two
 // workgroups per CU, which then walk the rows together.  The input row sits in LDS as f32, zero beyond `dim` and up to a whole block.
 __device__ __forceinline__ float block_sum_512(float v, float *red) {
@@ -297,11 +297,12 @@ __device__ __forceinline__ float block_sum_512(float v, float *red) {
     return ((red[0] + red[1]) + (red[2] + red[3])) + ((red[4] + red[5]) + (red[6] + red[7]));
 }
 
-template <int PRO, int U>
+constexpr int MV_U = 4, MV_BLOCK = 512 * MV_U;
+template <int PRO>
 __global__ __launch_bounds__(512) void dense_matvec_kernel(const uint16_t *__restrict__ w, int64_t ldw, const float *__restrict__ x,
                                                            const float *__restrict__ vec, float eps, int dim, float *dst, const float *add, int accumulate,
                                                            int n, int k) {
-    constexpr int BLOCK = 512 * U;
+    constexpr int U = MV_U, BLOCK = MV_BLOCK;
     extern __shared__ __attribute__((aligned(16))) float xs[];           // k rounded up to BLOCK
     __shared__ float red[8];
     const int tid = threadIdx.x, lane = tid & 63, wv = __builtin_amdgcn_readfirstlane(tid >> 6);
@@ -315,35 +316,49 @@ __global__ __launch_bounds__(512) void dense_matvec_kernel(const uint16_t *__res
     };
     if (r < n) load(r, 0, cur);
 
-    const int k_all = kb_n * BLOCK;
-    if (PRO == CQ_DENSE_PLAIN) {
-        for (int i = tid; i < k_all; i += 512) xs[i] = i < dim ? x[i] : 0.0f;
-    } else if (PRO == CQ_DENSE_NORM) {
-        float s = 0.0f;
-        for (int i = tid; i < k_all; i += 512) {
-            const float v = i < dim ? x[i] : 0.0f;
-            xs[i] = v;
-            s = fmaf(v, v, s);
+    // the input row into LDS, several 16-byte loads per thread in flight (it comes from another kernel's hands, far away)
+    constexpr int PF = PRO == CQ_DENSE_POLY ? 8 : 4;
+    const int n4 = kb_n * BLOCK / 4;
+    f32x4 *xs4 = reinterpret_cast<f32x4 *>(xs);
+    float s2 = 0.0f, s4 = 0.0f, s6 = 0.0f;
+    for (int i0 = tid; i0 < n4; i0 += 512 * PF) {
+        f32x4 v[PF];
+#pragma unroll
+        for (int j = 0; j < PF; j++) v[j] = *reinterpret_cast<const f32x4 *>(x + min(4 * (i0 + 512 * j), k - 4));
+#pragma unroll
+        for (int j = 0; j < PF; j++) {
+            const int i = i0 + 512 * j;
+            if (i >= n4) break;
+#pragma unroll
+            for (int e = 0; e < 4; e++) {
+                const float z = 4 * i + e < dim ? v[j][e] : 0.0f, q = z * z;
+                v[j][e] = z;
+                if (PRO != CQ_DENSE_PLAIN) s2 += q;
+                if (PRO == CQ_DENSE_POLY) {
+                    s4 = fmaf(q, q, s4);
+                    s6 = fmaf(q * q, q, s6);
+                }
+            }
+            xs4[i] = v[j];
         }
-        const float m = sqrtf(block_sum_512(s, red) / (float)dim + eps);
+    }
+    if (PRO == CQ_DENSE_NORM) {
+        const float m = sqrtf(block_sum_512(s2, red) / (float)dim + eps);
         for (int i = tid; i < dim; i += 512) xs[i] = xs[i] / m * vec[i];
-    } else {
-        float s2 = 0.0f, s4 = 0.0f, s6 = 0.0f;
-        for (int i = tid; i < k_all; i += 512) {
-            const float v = i < dim ? x[i] : 0.0f, q = v * v;
-            xs[i] = v;
-            s2 += q;
-            s4 = fmaf(q, q, s4);
-            s6 = fmaf(q * q, q, s6);
-        }
+    } else if (PRO == CQ_DENSE_POLY) {
         const float inv = 1.0f / (float)dim;
         const float i1 = vec[0] / sqrtf(block_sum_512(s2, red) * inv + eps);
         const float i2 = vec[1] / sqrtf(block_sum_512(s4, red) * inv + eps);
         const float i3 = vec[2] / sqrtf(block_sum_512(s6, red) * inv + eps);
         const float e = vec[3];
-        for (int i = tid; i < dim; i += 512) {
-            const float v = xs[i], q = v * v;
-            xs[i] = fmaf(i1, v, fmaf(i2, q, fmaf(i3, q * v, e)));
+        for (int i = tid; i < n4; i += 512) {
+            f32x4 v = xs4[i];
+#pragma unroll
+            for (int j = 0; j < 4; j++) {
+                const float q = v[j] * v[j];
+                v[j] = 4 * i + j < dim ? fmaf(i1, v[j], fmaf(i2, q, fmaf(i3, q * v[j], e))) : 0.0f;
+            }
+            xs4[i] = v;
         }
     }
     __syncthreads();
@@ -379,20 +394,13 @@ __global__ __launch_bounds__(512) void dense_matvec_kernel(const uint16_t *__res
 template <int PRO>
 int matvec_launch(const uint16_t *w, int64_t ldw, const float *x, const float *vec, float eps, int dim, float *dst, const float *add, int accumulate, int n,
                   int k, hipStream_t s) {
-    const int u = k <= 2048 ? 4 : 8, block = 512 * u;
-    const size_t lds = (size_t)((k + block - 1) / block) * block * sizeof(float);
+    const size_t lds = (size_t)((k + MV_BLOCK - 1) / MV_BLOCK) * MV_BLOCK * sizeof(float);
     const int blocks = (n + 7) / 8 < 512 ? (n + 7) / 8 : 512;
-#define CQ_MV(U_)                                                                                                                                    \
-    do {                                                                                                                                              \
-        if (lds > 64 * 1024) {                                                                                                                        \
-            const int e = (int)hipFuncSetAttribute(reinterpret_cast<const void *>(dense_matvec_kernel<PRO, U_>), hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024 - 64); \
-            if (e) return e;                                                                                                                          \
-        }                                                                                                                                             \
-        hipLaunchKernelGGL((dense_matvec_kernel<PRO, U_>), dim3(blocks), dim3(512), lds, s, w, ldw, x, vec, eps, dim, dst, add, accumulate, n, k);    \
-    } while (0)
-    if (u == 4) CQ_MV(4);
-    else CQ_MV(8);
-#undef CQ_MV
+    if (lds > 64 * 1024) {
+        const int e = (int)hipFuncSetAttribute(reinterpret_cast<const void *>(dense_matvec_kernel<PRO>), hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024 - 64);
+        if (e) return e;
+    }
+    hipLaunchKernelGGL(dense_matvec_kernel<PRO>, dim3(blocks), dim3(512), lds, s, w, ldw, x, vec, eps, dim, dst, add, accumulate, n, k);
     return (int)hipGetLastError();
 }
 
@@ -445,7 +453,7 @@ int cq_dense_matvec(const void *w_dev, int64_t ldw, const float *x_dev, int prol
     if (prologue < CQ_DENSE_PLAIN || prologue > CQ_DENSE_POLY) return CQ_ERR_DTYPE;
     if (n == 0) return CQ_OK;
     if (!w_dev || !x_dev || !dst_dev || (prologue != CQ_DENSE_PLAIN && !vec_dev)) return CQ_ERR_NULL;
-    if (misaligned(w_dev, 16) || misaligned(x_dev, 4) || misaligned(vec_dev, 4) || misaligned(dst_dev, 4) || misaligned(add_dev, 4)) return CQ_ERR_ALIGN;
+    if (misaligned(w_dev, 16) || misaligned(x_dev, 16) || misaligned(vec_dev, 4) || misaligned(dst_dev, 4) || misaligned(add_dev, 4)) return CQ_ERR_ALIGN;
     if (k > CQ_DENSE_MATVEC_MAX_K || n > (1 << 24)) return CQ_ERR_RANGE;
     const uint16_t *w = (const uint16_t *)w_dev;
     hipStream_t s = (hipStream_t)stream;

@@ -39,7 +39,7 @@ int cq_dense_matmul(int precision, const void *w_dev, int64_t ldw, const float *
  *   CQ_DENSE_PLAIN   f(x) = x
  *   CQ_DENSE_NORM    f(x) = x / sqrt(mean(x^2) + eps) * vec                     (vec [dim])
  *   CQ_DENSE_POLY    f(x) = vec[0] N(x) + vec[1] N(x^2) + vec[2] N(x^3) + vec[3], N(z) = z / sqrt(mean(z^2) + eps)
- * dim <= k values of x count, f is zero beyond.  k <= CQ_DENSE_MATVEC_MAX_K. */
+ * dim <= k values of x count, f is zero beyond (x is readable up to k, 16-byte aligned).  k <= CQ_DENSE_MATVEC_MAX_K. */
 enum cq_dense_prologue { CQ_DENSE_PLAIN = 0, CQ_DENSE_NORM = 1, CQ_DENSE_POLY = 2 };
 #define CQ_DENSE_MATVEC_MAX_K 32768
 int cq_dense_matvec(const void *w_dev, int64_t ldw, const float *x_dev, int prologue, const float *vec_dev, float eps, int64_t dim, float *dst_dev,
