@@ -265,7 +265,7 @@ Plan plan(int precision, int64_t m, int64_t n, int64_t k) {
     auto tiles = [&](int bm, int bn) { return ((m + bm - 1) / bm) * ((n + bn - 1) / bn); };
     if (precision == CQ_DENSE_F32) {
         p.bm = p.bn = 64;
-    } else if (m > 64 && tiles(128, 128) >= 192) {
+    } else if (m > 64 && tiles(128, 128) * (k / 512) >= 256) {      // the large tile where splitting k can still fill the chip
         p.bm = p.bn = 128;
     } else if (m > 32) {
         p.bm = p.bn = 64;
