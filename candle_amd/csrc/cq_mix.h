@@ -16,30 +16,61 @@ __device__ __forceinline__ float head_inv_rms(const float *src, int dim, float e
     return 1.0f / sqrtf(wave_sum(s) / (float)dim + eps);
 }
 
-// One head of a group in the registers of a wave (lane: dimensions lane + 64 e): everything it needs is requested by load(), so
-// that the norm's reduction is not followed by a second trip to memory.
+// Element `other` (0 .. 64 NE - 1, lane's own choice) of a vector that a wave holds as lane + 64 e.
 template <int NE>
-struct HeadRegs {
-    float v[NE], o[NE], wv[NE], wo[NE], c[NE], s[NE];
+__device__ __forceinline__ float wave_gather(const float (&x)[NE], int other) {
+    float r = 0.0f;
+#pragma unroll
+    for (int e = 0; e < NE; e++) {
+        const float v = __shfl(x[e], other & 63, 64);
+        r = (other >> 6) == e ? v : r;
+    }
+    return r;
+}
 
-    __device__ __forceinline__ void load(const cq_mix_heads &g, const float *src, int64_t p, int lane) {
+// Heads of a group in the registers of a wave (lane: dimensions lane + 64 e).  HeadShared is what all heads of the group need at position p;
+// a head itself is one load per 64 dimensions.  The vector memory pipeline takes an instruction per 16 cycles whatever it loads, so
+// rotation partners come from other lanes, not from memory.
+template <int NE>
+struct HeadShared {
+    float w[NE], wo[NE], c[NE], s[NE];           // norm weight, that of the rotation partner, cos, sin
+    __device__ __forceinline__ void load(const cq_mix_heads &g, int64_t p, int lane) {
         const int half = g.rot_dims >> 1;
 #pragma unroll
         for (int e = 0; e < NE; e++) {
-            const int d = lane + 64 * e;
-            const bool ok = d < g.dim, rot = d < g.rot_dims;
-            const int i = d < half ? d : d - half, other = d < half ? d + half : d - half;
-            v[e] = ok ? src[d] : 0.0f;
-            wv[e] = ok && g.norm_dev ? g.norm_dev[d] : 1.0f;
-            o[e] = rot ? src[other] : 0.0f;
-            wo[e] = rot && g.norm_dev ? g.norm_dev[other] : 1.0f;
+            const int d = lane + 64 * e, i = d < half ? d : d - half;
+            const bool rot = d < g.rot_dims;
+            w[e] = d < g.dim && g.norm_dev ? g.norm_dev[d] : 1.0f;
             c[e] = rot ? g.cos_dev[p * half + i] : 1.0f;
             s[e] = rot ? g.sin_dev[p * half + i] : 0.0f;
         }
     }
-    // the values after norm, rotation and factor, in place of v (zero beyond dim)
-    __device__ __forceinline__ void finish(const cq_mix_heads &g, float eps, int lane) {
-        float inv = 1.0f;
+    // after all loads have been asked for
+    __device__ __forceinline__ void ready(const cq_mix_heads &g, int lane) {
+        if (!g.norm_dev || !g.rot_dims) {
+#pragma unroll
+            for (int e = 0; e < NE; e++) wo[e] = w[e];
+            return;
+        }
+#pragma unroll
+        for (int e = 0; e < NE; e++) wo[e] = wave_gather(w, partner(g, lane + 64 * e));
+    }
+    static __device__ __forceinline__ int partner(const cq_mix_heads &g, int d) {
+        const int half = g.rot_dims >> 1;
+        return d < half ? d + half : (d < g.rot_dims ? d - half : d);
+    }
+};
+
+template <int NE>
+struct HeadRegs {
+    float v[NE];
+    __device__ __forceinline__ void load(const cq_mix_heads &g, const float *src, int lane) {
+#pragma unroll
+        for (int e = 0; e < NE; e++) v[e] = lane + 64 * e < g.dim ? src[lane + 64 * e] : 0.0f;
+    }
+    // norm, rotation and factor in place (zero beyond dim)
+    __device__ __forceinline__ void finish(const cq_mix_heads &g, const HeadShared<NE> &sh, float eps, int lane) {
+        float inv = 1.0f, o[NE];
         if (g.norm_dev) {
             float q = 0.0f;
 #pragma unroll
@@ -47,11 +78,16 @@ struct HeadRegs {
             inv = 1.0f / sqrtf(wave_sum(q) / (float)g.dim + eps);
         }
         const int half = g.rot_dims >> 1;
+        if (half)
+#pragma unroll
+            for (int e = 0; e < NE; e++) o[e] = wave_gather(v, HeadShared<NE>::partner(g, lane + 64 * e));
+        else
+#pragma unroll
+            for (int e = 0; e < NE; e++) o[e] = 0.0f;
 #pragma unroll
         for (int e = 0; e < NE; e++) {
-            const int d = lane + 64 * e;
-            const float a = v[e] * inv * wv[e], b = o[e] * inv * wo[e];
-            v[e] = (d < half ? a * c[e] - b * s[e] : a * c[e] + b * s[e]) * g.factor;
+            const float a = v[e] * inv * sh.w[e], b = o[e] * inv * sh.wo[e];
+            v[e] = (lane + 64 * e < half ? a * sh.c[e] - b * sh.s[e] : a * sh.c[e] + b * sh.s[e]) * g.factor;
         }
     }
 };
@@ -97,5 +133,12 @@ __device__ __forceinline__ float row16_max(float v) {
     CQ_MX(CQ_DPP_ROW_HALF_MIRROR);
     CQ_MX(0x140);                                          // row_mirror
 #undef CQ_MX
+    return v;
+}
+
+// sum over each aligned group of 4 lanes, in every lane
+__device__ __forceinline__ float quad_sum_f(float v) {
+    v += __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, v), CQ_DPP_QUAD_XOR1, 0xf, 0xf, true));
+    v += __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, v), CQ_DPP_QUAD_XOR2, 0xf, 0xf, true));
     return v;
 }

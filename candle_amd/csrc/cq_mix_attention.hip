@@ -281,7 +281,7 @@ int talk_launch(const float *q, const float *kc, const float *vc, const float *t
 // the same for k and v, appends them to the caches and uses its own copies.
 //   scores  16 lanes per (kv head, key), each key row read once for the heads that share it
 //   mixing  one thread per (head, key)
-//   values  one thread per (kv head, column), four heads at a time
+//   values  four lanes per (kv head, four columns), each on a quarter of the keys, four heads at a time
 template <int NC, int KD>
 __global__ __launch_bounds__(1024) void talk_decode_kernel(const float *__restrict__ row, cq_mix_heads gq, cq_mix_heads gk, cq_mix_heads gv, float eps,
                                                            const float *__restrict__ talk, float scale, int window, int keep_first,
@@ -300,9 +300,9 @@ __global__ __launch_bounds__(1024) void talk_decode_kernel(const float *__restri
         const int s = s0 + min(j, cnt - 1);
         return s < vis.keep ? s : vis.lo + s - vis.keep;
     };
-    const int sub = lane & 15, grp = wv * 4 + (lane >> 4), pairs = G * KD, items = G * vdim;
-    f32x4 kd[PB][NC];
-    float vv[16];
+    const int sub = lane & 15, grp = wv * 4 + (lane >> 4), pairs = G * KD, items = G * vp / 4;
+    const int quarter = tid & 3;                                     // of every 16 keys
+    f32x4 kd[PB][NC], vv[4];
     auto load_k = [&](int b) {
 #pragma unroll
         for (int i = 0; i < PB; i++) {
@@ -315,42 +315,61 @@ __global__ __launch_bounds__(1024) void talk_decode_kernel(const float *__restri
             }
         }
     };
-    auto load_v = [&](int i, int jb) {
-        const int g = i / vdim;
-        const float *vb = gv.dst_dev + g * gv.dst_head_stride + (i - g * vdim);
+    auto load_v = [&](int i, int jb) {                               // i: four columns of a kv head
+        const int g = i / (vp / 4);
+        const float *vb = gv.dst_dev + g * gv.dst_head_stride + 4 * (i - g * (vp / 4));
 #pragma unroll
-        for (int j = 0; j < 16; j++) vv[j] = vb[(int64_t)key_of(jb + j) * gv.dst_row_stride];
+        for (int j = 0; j < 4; j++) vv[j] = *reinterpret_cast<const f32x4 *>(vb + (int64_t)key_of(jb + 4 * quarter + j) * gv.dst_row_stride);
     };
+    // Loads complete in the order they are asked for: first what the preparation needs (two query heads per wave, and for the new token
+    // one head of k or v), then the mixing matrix, K and V.
+    const int h2 = min(wv + 16, H - 1), xn = min(wv, 2 * G - 1);
+    const cq_mix_heads &gn = xn < G ? gk : gv;
+    HeadShared<NC> qsh, nsh;
+    HeadRegs<NC> qa, qb, nw;
+    qsh.load(gq, p, lane);
+    qa.load(gq, row + gq.src_off + (int64_t)min(wv, H - 1) * gq.dim, lane);
+    if (H > 16) qb.load(gq, row + gq.src_off + (int64_t)h2 * gq.dim, lane);
+    if (owner) {
+        nsh.load(gn, p, lane);
+        nw.load(gn, row + gn.src_off + (int64_t)(xn < G ? xn : xn - G) * gn.dim, lane);
+    }
+    const float tv = talk[min(tid, H * H - 1)];
     load_k(grp);
-    load_v(min(tid, items - 1), 0);
-    for (int i = tid; i < H * H; i += 1024) T[i] = talk[i] * scale;
-    for (int h = wv; h < H; h += 32) {                                // two heads at a time
-        HeadRegs<NC> a, b;
-        const int h2 = min(h + 16, H - 1);
-        a.load(gq, row + gq.src_off + (int64_t)h * gq.dim, p, lane);
-        b.load(gq, row + gq.src_off + (int64_t)h2 * gq.dim, p, lane);
-        a.finish(gq, eps, lane);
-        b.finish(gq, eps, lane);
+    load_v(min(tid >> 2, items - 1), 0);
+    qsh.ready(gq, lane);
+    auto keep_q = [&](HeadRegs<NC> &x, int h) {
+        x.finish(gq, qsh, eps, lane);
 #pragma unroll
         for (int e = 0; e < NC; e++)
-            if (lane + 64 * e < dp) {
-                qs[h * dp + lane + 64 * e] = a.v[e];
-                if (h + 16 < H) qs[(h + 16) * dp + lane + 64 * e] = b.v[e];
-            }
-    }
-    if (owner) {
-        for (int x = wv; x < 2 * G; x += 16) {
-            const cq_mix_heads &gr = x < G ? gk : gv;
-            const int hh = x < G ? x : x - G;
-            float *dst = gr.dst_dev + hh * gr.dst_head_stride + (int64_t)p * gr.dst_row_stride, *own = (x < G ? kn : vn) + hh * gr.dim_pad;
-            HeadRegs<NC> a;
-            a.load(gr, row + gr.src_off + (int64_t)hh * gr.dim, p, lane);
-            a.finish(gr, eps, lane);
+            if (h < H && lane + 64 * e < dp) qs[h * dp + lane + 64 * e] = x.v[e];
+    };
+    auto keep_new = [&](HeadRegs<NC> &x, int i) {
+        const cq_mix_heads &gr = i < G ? gk : gv;
+        const int hh = i < G ? i : i - G;
+        float *dst = gr.dst_dev + hh * gr.dst_head_stride + (int64_t)p * gr.dst_row_stride, *own = (i < G ? kn : vn) + hh * gr.dim_pad;
+        nsh.ready(gr, lane);
+        x.finish(gr, nsh, eps, lane);
 #pragma unroll
-            for (int e = 0; e < NC; e++)
-                if (lane + 64 * e < gr.dim_pad) dst[lane + 64 * e] = own[lane + 64 * e] = a.v[e];
-        }
+        for (int e = 0; e < NC; e++)
+            if (i < 2 * G && lane + 64 * e < gr.dim_pad) dst[lane + 64 * e] = own[lane + 64 * e] = x.v[e];
+    };
+    keep_q(qa, wv);
+    if (H > 16) keep_q(qb, wv + 16);
+    if (owner && wv < 2 * G) keep_new(nw, wv);
+    for (int h = wv + 32; h < H; h += 16) {
+        qa.load(gq, row + gq.src_off + (int64_t)h * gq.dim, lane);
+        keep_q(qa, h);
     }
+    if (owner)
+        for (int x = wv + 16; x < 2 * G; x += 16) {
+            const cq_mix_heads &gr = x < G ? gk : gv;
+            nsh.load(gr, p, lane);
+            nw.load(gr, row + gr.src_off + (int64_t)(x < G ? x : x - G) * gr.dim, lane);
+            keep_new(nw, x);
+        }
+    if (tid < H * H) T[tid] = tv * scale;
+    for (int i = tid + 1024; i < H * H; i += 1024) T[i] = talk[i] * scale;
     __syncthreads();
 
     // ---- scores ----
@@ -364,20 +383,23 @@ __global__ __launch_bounds__(1024) void talk_decode_kernel(const float *__restri
                 for (int c = 0; c < NC; c++)
                     if (64 * c + 4 * sub < dp) kd[i][c] = *reinterpret_cast<const f32x4 *>(kn + g * dp + 64 * c + 4 * sub);
             }
-            for (int r = 0; r < R; r++) {
-                const float *qh = qs + (g * R + r) * dp;
-                float a = 0.0f;
+            for (int r = 0; r < R; r += 4) {                         // four heads side by side (the last one repeated)
+                float a[4] = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
                 for (int c = 0; c < NC; c++) {
-                    const int d = 64 * c + 4 * sub;
-                    const f32x4 qv = d < dp ? *reinterpret_cast<const f32x4 *>(qh + d) : f32x4{0.f, 0.f, 0.f, 0.f};
-                    a = fmaf(qv.x, kd[i][c].x, a);
-                    a = fmaf(qv.y, kd[i][c].y, a);
-                    a = fmaf(qv.z, kd[i][c].z, a);
-                    a = fmaf(qv.w, kd[i][c].w, a);
+                    const int d = min(64 * c + 4 * sub, dp - 4);     // where dp ends, kd is zero
+#pragma unroll
+                    for (int x = 0; x < 4; x++) {
+                        const f32x4 qv = *reinterpret_cast<const f32x4 *>(qs + (g * R + min(r + x, R - 1)) * dp + d);
+                        a[x] = fmaf(qv.x, kd[i][c].x, a[x]);
+                        a[x] = fmaf(qv.y, kd[i][c].y, a[x]);
+                        a[x] = fmaf(qv.z, kd[i][c].z, a[x]);
+                        a[x] = fmaf(qv.w, kd[i][c].w, a[x]);
+                    }
                 }
-                a = row16_sum(a);
-                if (sub == 0) sc[(g * R + r) * SS + j] = a;
+#pragma unroll
+                for (int x = 0; x < 4; x++) a[x] = row16_sum(a[x]);
+                if (sub < 4 && r + sub < R) sc[(g * R + r + sub) * SS + j] = sub == 0 ? a[0] : (sub == 1 ? a[1] : (sub == 2 ? a[2] : a[3]));
             }
         }
     }
@@ -388,12 +410,21 @@ __global__ __launch_bounds__(1024) void talk_decode_kernel(const float *__restri
         const float *t = T + h * H;
         float a0 = 0.0f, a1 = 0.0f;
         int g = 0;
-#pragma unroll 4
-        for (; g + 2 <= H; g += 2) {
-            a0 = fmaf(t[g], sc[g * SS + j], a0);
-            a1 = fmaf(t[g + 1], sc[(g + 1) * SS + j], a1);
+#pragma unroll 2
+        for (; g + 8 <= H; g += 8) {
+            float tv8[8], sv[8];
+#pragma unroll
+            for (int x = 0; x < 8; x++) {
+                tv8[x] = t[g + x];
+                sv[x] = sc[(g + x) * SS + j];
+            }
+#pragma unroll
+            for (int x = 0; x < 8; x += 2) {
+                a0 = fmaf(tv8[x], sv[x], a0);
+                a1 = fmaf(tv8[x + 1], sv[x + 1], a1);
+            }
         }
-        if (g < H) a0 = fmaf(t[g], sc[g * SS + j], a0);
+        for (; g < H; g++) a0 = fmaf(t[g], sc[g * SS + j], a0);
         mx[h * SS + j] = j < cnt ? a0 + a1 : -INFINITY;
     }
     __syncthreads();
@@ -422,27 +453,41 @@ __global__ __launch_bounds__(1024) void talk_decode_kernel(const float *__restri
     }
     __syncthreads();
     // ---- values ----
-    for (int i = tid; i < items; i += 1024) {
-        const int g = i / vdim, e = i - g * vdim;
+    const int v4 = (vdim + 3) / 4;
+    for (int i = tid >> 2; i < items; i += 256) {
+        const int g = i / (vp / 4), e4 = i - g * (vp / 4);
         for (int r = 0; r < R; r += 4) {
-            float a[4] = {0.f, 0.f, 0.f, 0.f};
-            for (int jb = 0; jb < KD; jb += 16) {
-                if (i != tid || jb > 0 || (KD > 16 && r > 0)) load_v(i, jb);
-                if (owner) {
-                    const float x = vn[g * vp + e];
+            f32x4 a[4];
 #pragma unroll
-                    for (int j = 0; j < 16; j++) vv[j] = jb + j >= cnt - 1 ? x : vv[j];
+            for (int x = 0; x < 4; x++) a[x] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll 1
+            for (int jb = 0; jb < KD; jb += 16) {
+                if (i != (tid >> 2) || jb > 0 || (KD > 16 && r > 0)) load_v(i, jb);
+                if (owner) {
+                    const f32x4 x = *reinterpret_cast<const f32x4 *>(vn + g * vp + 4 * e4);
+#pragma unroll
+                    for (int j = 0; j < 4; j++)
+                        if (jb + 4 * quarter + j >= cnt - 1) vv[j] = x;
                 }
 #pragma unroll
                 for (int x = 0; x < 4; x++) {
-                    const f32x4 *w = reinterpret_cast<const f32x4 *>(sc + (g * R + min(r + x, R - 1)) * SS + jb);
+                    const f32x4 w = *reinterpret_cast<const f32x4 *>(sc + (g * R + min(r + x, R - 1)) * SS + jb + 4 * quarter);
 #pragma unroll
-                    for (int j = 0; j < 16; j++) a[x] = fmaf(w[j >> 2][j & 3], vv[j], a[x]);
+                    for (int j = 0; j < 4; j++)
+#pragma unroll
+                        for (int e = 0; e < 4; e++) a[x][e] = fmaf(w[j], vv[j][e], a[x][e]);
                 }
             }
+            // the sum of the four quarters in every lane; lane `quarter` stores head r + quarter
+            f32x4 mine = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
             for (int x = 0; x < 4; x++)
-                if (r + x < R) rec[((int64_t)(g * R + r + x) * splits + sp) * stride + e] = a[x];
+#pragma unroll
+                for (int e = 0; e < 4; e++) {
+                    const float s = quad_sum_f(a[x][e]);
+                    mine[e] = quarter == x ? s : mine[e];
+                }
+            if (e4 < v4 && r + quarter < R) *reinterpret_cast<f32x4 *>(rec + ((int64_t)(g * R + r + quarter) * splits + sp) * stride + 4 * e4) = mine;
         }
     }
 }
@@ -513,9 +558,10 @@ int cq_mix_talk_decode(const float *row_dev, const cq_mix_heads *qkv, float eps,
         if (e) return e;
     }
     if (q.heads % k.heads || v.heads != k.heads || q.dim != k.dim || !k.by_position || !v.by_position || k.ctx != v.ctx || k.dim_pad % 16 || v.dim_pad % 16 ||
-        window < 1 || keep_first < 0 || pos < 0 || k.dst_row_stride % 4 || k.dst_head_stride % 4)
+        window < 1 || keep_first < 0 || pos < 0 || k.dst_row_stride % 4 || k.dst_head_stride % 4 ||
+        v.dst_row_stride % 4 || v.dst_head_stride % 4)
         return CQ_ERR_SHAPE;
-    if (mix_misaligned(k.dst_dev, 16)) return CQ_ERR_ALIGN;
+    if (mix_misaligned(k.dst_dev, 16) || mix_misaligned(v.dst_dev, 16) || mix_misaligned(workspace_dev, 16)) return CQ_ERR_ALIGN;
     if (q.heads > CQ_MIX_MAX_HEADS || k.dim_pad > CQ_MIX_MAX_DIM || v.dim_pad > CQ_MIX_MAX_DIM || k.ctx > (1 << 28) || (!pos_dev && pos >= k.ctx)) return CQ_ERR_RANGE;
     const int64_t n_max = talk_max_keys(window, keep_first, k.ctx);
     if (workspace_bytes < cq_mix_talk_decode_workspace_bytes(q.heads, v.dim, window, keep_first, k.ctx)) return CQ_ERR_WORKSPACE;

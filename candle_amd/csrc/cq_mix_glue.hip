@@ -116,9 +116,12 @@ __global__ __launch_bounds__(256) void pack_heads_kernel(const float *__restrict
     if (g.ctx > 0 && p >= g.ctx) return;
     const float *s = src + r * src_stride + g.src_off + (int64_t)h * g.dim;
     float *d = g.dst_dev + h * g.dst_head_stride + (g.by_position ? p : r) * g.dst_row_stride;
+    HeadShared<NE> sh;
     HeadRegs<NE> x;
-    x.load(g, s, p, lane);
-    x.finish(g, eps, lane);
+    sh.load(g, p, lane);
+    x.load(g, s, lane);
+    sh.ready(g, lane);
+    x.finish(g, sh, eps, lane);
 #pragma unroll
     for (int e = 0; e < NE; e++)
         if (lane + 64 * e < g.dim_pad) d[lane + 64 * e] = x.v[e];

@@ -240,9 +240,12 @@ __device__ __forceinline__ void retention_step(const StepArgs &a, int h, int p, 
     load(4 * wv);
     if (wv < 2) {
         const cq_mix_heads &g = wv == 0 ? a.gq : a.gk;
+        HeadShared<NR> sh;
         HeadRegs<NR> x;
-        x.load(g, a.row + g.src_off + (int64_t)h * g.dim, p, lane);
-        x.finish(g, a.eps, lane);
+        sh.load(g, p, lane);
+        x.load(g, a.row + g.src_off + (int64_t)h * g.dim, lane);
+        sh.ready(g, lane);
+        x.finish(g, sh, a.eps, lane);
 #pragma unroll
         for (int e = 0; e < NR; e++) sm[wv * SP + lane + 64 * e] = x.v[e];
     }
