@@ -225,15 +225,14 @@ __global__ __launch_bounds__(64 * NW) void talk_attention_kernel(const float *__
 // one wave per (row, head)
 __global__ __launch_bounds__(256) void talk_combine_kernel(const float *__restrict__ part, int nz, int64_t rows, int H, int vdim, float out_scale,
                                                            float *__restrict__ out, int64_t out_stride) {
-    const int lane = threadIdx.x & 63;
-    const int64_t id = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6), n = rows * H;
-    if (id >= n) return;
+    const int lane = threadIdx.x & 63, h = blockIdx.y * 4 + (threadIdx.x >> 6);
+    if (h >= H) return;
+    const int64_t r = blockIdx.x, id = r * H + h, n = rows * H;
     const float *ml = part + nz * n * vdim + 2 * id;
     float m = -INFINITY, l = 0.0f;
     for (int z = 0; z < nz; z++) m = fmaxf(m, ml[2 * n * z]);
     for (int z = 0; z < nz; z++) l = fmaf(ml[2 * n * z] > -INFINITY ? __expf(ml[2 * n * z] - m) : 0.0f, ml[2 * n * z + 1], l);
-    const int64_t r = id / H;
-    float *o = out + r * out_stride + (id - r * H) * vdim;
+    float *o = out + r * out_stride + (int64_t)h * vdim;
     for (int e = lane; e < vdim; e += 64) {
         float a = 0.0f;
         for (int z = 0; z < nz; z++) {
@@ -270,7 +269,7 @@ int talk_launch(const float *q, const float *kc, const float *vc, const float *t
     hipLaunchKernelGGL((talk_attention_kernel<NW, NHW, SHARED_K, U, VS, KT>), dim3((rows + 15) / 16, (units + NW * U - 1) / (NW * U), nz), dim3(64 * NW), lds,
                        s, q, kc, vc, talk, scale, window, keep, out_scale, out, out_stride, part, pos, rows, H, G, dp, vdim, vp, ctx);
     if (nz > 1)
-        hipLaunchKernelGGL(talk_combine_kernel, dim3((unsigned)(((int64_t)rows * H + 3) / 4)), dim3(256), 0, s, (const float *)part, nz, (int64_t)rows, H, vdim, out_scale,
+        hipLaunchKernelGGL(talk_combine_kernel, dim3((unsigned)rows, (unsigned)((H + 3) / 4)), dim3(256), 0, s, (const float *)part, nz, (int64_t)rows, H, vdim, out_scale,
                            out, out_stride);
     return (int)hipGetLastError();
 }

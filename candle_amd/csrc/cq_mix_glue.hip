@@ -101,50 +101,88 @@ struct Groups {
     cq_mix_heads g[CQ_MIX_MAX_GROUPS];
 };
 
-// one wave per (row, head); heads of all groups numbered through
+// One wave per (row, up to PACK_HEADS heads of a group): what depends on the position is loaded once for them, and all their values are
+// requested before the first is worked on.  blockIdx.x: row, blockIdx.y: four waves.
+constexpr int PACK_HEADS = 8;
 template <int NE>
-__global__ __launch_bounds__(256) void pack_heads_kernel(const float *__restrict__ src, int64_t src_stride, Groups gs, int n_groups, int total_heads, float eps,
-                                                         const int32_t *__restrict__ pos_dev, int64_t pos, int64_t rows) {
+__global__ __launch_bounds__(256) void pack_heads_kernel(const float *__restrict__ src, int64_t src_stride, Groups gs, int n_groups, float eps,
+                                                         const int32_t *__restrict__ pos_dev, int64_t pos) {
     const int lane = threadIdx.x & 63;
-    const int64_t id = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
-    if (id >= rows * total_heads) return;
-    const int64_t r = id / total_heads;
-    int h = (int)(id - r * total_heads), gi = 0;
-    while (gi + 1 < n_groups && h >= gs.g[gi].heads) h -= gs.g[gi++].heads;
+    int c = blockIdx.y * 4 + __builtin_amdgcn_readfirstlane((int)(threadIdx.x >> 6)), gi = 0;
+    while (gi < n_groups && c >= (gs.g[gi].heads + PACK_HEADS - 1) / PACK_HEADS) c -= (gs.g[gi++].heads + PACK_HEADS - 1) / PACK_HEADS;
+    if (gi == n_groups) return;
     const cq_mix_heads g = gs.g[gi];
-    const int64_t p = pos + (pos_dev ? pos_dev[0] : 0) + r;
+    const int64_t r = blockIdx.x, p = pos + (pos_dev ? pos_dev[0] : 0) + r;
     if (g.ctx > 0 && p >= g.ctx) return;
-    const float *s = src + r * src_stride + g.src_off + (int64_t)h * g.dim;
-    float *d = g.dst_dev + h * g.dst_head_stride + (g.by_position ? p : r) * g.dst_row_stride;
+    const int h0 = c * PACK_HEADS;
+    const float *s = src + r * src_stride + g.src_off;
+    float *d = g.dst_dev + (g.by_position ? p : r) * g.dst_row_stride;
     HeadShared<NE> sh;
-    HeadRegs<NE> x;
+    HeadRegs<NE> x[PACK_HEADS];
     sh.load(g, p, lane);
-    x.load(g, s, lane);
-    sh.ready(g, lane);
-    x.finish(g, sh, eps, lane);
 #pragma unroll
-    for (int e = 0; e < NE; e++)
-        if (lane + 64 * e < g.dim_pad) d[lane + 64 * e] = x.v[e];
+    for (int i = 0; i < PACK_HEADS; i++) x[i].load(g, s + (int64_t)min(h0 + i, g.heads - 1) * g.dim, lane);
+    sh.ready(g, lane);
+#pragma unroll
+    for (int i = 0; i < PACK_HEADS; i++) {
+        x[i].finish(g, sh, eps, lane);
+        if (h0 + i < g.heads)
+#pragma unroll
+            for (int e = 0; e < NE; e++)
+                if (lane + 64 * e < g.dim_pad) d[(h0 + i) * g.dst_head_stride + lane + 64 * e] = x[i].v[e];
+    }
 }
 
-// one wave per (row, head)
+__device__ __forceinline__ float gated(float v, float g, int kind) {
+    const float sg = mix_sigmoid(g);
+    return v * (kind == CQ_GATE_SILU ? g * sg : sg);
+}
+
+// One wave per (row, NH heads) of up to 64 NE dimensions, everything requested before the first sum.
+template <int NE, int NH>
 __global__ __launch_bounds__(256) void head_norm_gate_kernel(const float *__restrict__ o, int64_t o_stride, const float *__restrict__ gate, int64_t g_stride,
                                                              const float *__restrict__ w, int kind, float scale, float *__restrict__ out, int64_t out_stride,
-                                                             int64_t rows, int heads, int dim, float eps) {
+                                                             int heads, int dim, float eps) {
     const int lane = threadIdx.x & 63;
-    const int64_t id = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
-    if (id >= rows * heads) return;
-    const int64_t r = id / heads;
-    const int h = (int)(id - r * heads);
-    const float *s = o + r * o_stride + (int64_t)h * dim;
-    const float inv = head_inv_rms(s, dim, eps, lane);
-    for (int i = lane; i < dim; i += 64) {
-        const float g = gate[r * g_stride + (int64_t)h * dim + i];
-        const float sg = mix_sigmoid(g);
-        float v = s[i] * inv;
-        if (w) v *= w[h * dim + i];
-        out[r * out_stride + (int64_t)h * dim + i] = scale * v * (kind == CQ_GATE_SILU ? g * sg : sg);
+    const int h0 = (blockIdx.y * 4 + __builtin_amdgcn_readfirstlane((int)(threadIdx.x >> 6))) * NH;
+    if (h0 >= heads) return;
+    const int64_t r = blockIdx.x;
+    const float *orow = o + r * o_stride, *grow = gate + r * g_stride;
+    float *dst = out + r * out_stride;
+    float v[NH][NE], g[NH][NE];
+#pragma unroll
+    for (int i = 0; i < NH; i++)
+#pragma unroll
+        for (int e = 0; e < NE; e++) {
+            const int d = lane + 64 * e, at = min(h0 + i, heads - 1) * dim + d;
+            v[i][e] = d < dim ? orow[at] : 0.0f;
+            g[i][e] = d < dim ? grow[at] : 0.0f;
+        }
+#pragma unroll
+    for (int i = 0; i < NH; i++) {
+        float q = 0.0f;
+#pragma unroll
+        for (int e = 0; e < NE; e++) q = fmaf(v[i][e], v[i][e], q);
+        const float inv = 1.0f / sqrtf(wave_sum(q) / (float)dim + eps);
+#pragma unroll
+        for (int e = 0; e < NE; e++) {
+            const int d = lane + 64 * e, at = (h0 + i) * dim + d;
+            if (h0 + i < heads && d < dim) dst[at] = scale * gated(v[i][e] * inv * (w ? w[at] : 1.0f), g[i][e], kind);
+        }
     }
+}
+
+// heads of any size
+__global__ __launch_bounds__(256) void head_norm_gate_long_kernel(const float *__restrict__ o, int64_t o_stride, const float *__restrict__ gate, int64_t g_stride,
+                                                                  const float *__restrict__ w, int kind, float scale, float *__restrict__ out,
+                                                                  int64_t out_stride, int heads, int dim, float eps) {
+    const int lane = threadIdx.x & 63;
+    const int h = blockIdx.y * 4 + (threadIdx.x >> 6);
+    if (h >= heads) return;
+    const int64_t r = blockIdx.x, hd = (int64_t)h * dim;
+    const float *s = o + r * o_stride + hd;
+    const float inv = head_inv_rms(s, dim, eps, lane);
+    for (int i = lane; i < dim; i += 64) out[r * out_stride + hd + i] = scale * gated(s[i] * inv * (w ? w[hd + i] : 1.0f), gate[r * g_stride + hd + i], kind);
 }
 
 }  // namespace
@@ -195,7 +233,7 @@ int cq_mix_pack_heads(const float *src_dev, int64_t src_stride, const cq_mix_hea
     if (rows == 0) return CQ_OK;
     if (!src_dev || !groups) return CQ_ERR_NULL;
     Groups gs;
-    int64_t total = 0;
+    int64_t chunks = 0;
     int widest = 0;
     for (int i = 0; i < n_groups; i++) {
         const int e = mix_check_group(groups[i], false);
@@ -203,13 +241,13 @@ int cq_mix_pack_heads(const float *src_dev, int64_t src_stride, const cq_mix_hea
         if (groups[i].src_off + (int64_t)groups[i].heads * groups[i].dim > src_stride) return CQ_ERR_SHAPE;
         if (groups[i].ctx > 0 && !pos_dev && pos + rows > groups[i].ctx) return CQ_ERR_RANGE;
         gs.g[i] = groups[i];
-        total += groups[i].heads;
+        chunks += (groups[i].heads + PACK_HEADS - 1) / PACK_HEADS;
         widest = groups[i].dim_pad > widest ? groups[i].dim_pad : widest;
     }
-    if (total > (1 << 20) || (rows * total + 3) / 4 > 0x7fffffffLL) return CQ_ERR_RANGE;
-    const dim3 grid((unsigned)((rows * total + 3) / 4));
+    if (rows > 0x7fffffffLL || chunks > 4 * 65535) return CQ_ERR_RANGE;
+    const dim3 grid((unsigned)rows, (unsigned)((chunks + 3) / 4));
     hipStream_t s = (hipStream_t)stream;
-#define CQ_PH(NE_) hipLaunchKernelGGL(pack_heads_kernel<NE_>, grid, dim3(256), 0, s, src_dev, src_stride, gs, n_groups, (int)total, eps, pos_dev, pos, rows)
+#define CQ_PH(NE_) hipLaunchKernelGGL(pack_heads_kernel<NE_>, grid, dim3(256), 0, s, src_dev, src_stride, gs, n_groups, eps, pos_dev, pos)
     if (widest <= 64) CQ_PH(1);
     else if (widest <= 128) CQ_PH(2);
     else CQ_PH(4);
@@ -223,9 +261,16 @@ int cq_mix_head_norm_gate(const float *o_dev, int64_t o_stride, const float *g_d
     if (gate != CQ_GATE_SILU && gate != CQ_GATE_SIGMOID) return CQ_ERR_DTYPE;
     if (rows == 0) return CQ_OK;
     if (!o_dev || !g_dev || !out_dev) return CQ_ERR_NULL;
-    if (heads * dim > (1 << 24) || (rows * heads + 3) / 4 > 0x7fffffffLL) return CQ_ERR_RANGE;
-    hipLaunchKernelGGL(head_norm_gate_kernel, dim3((unsigned)((rows * heads + 3) / 4)), dim3(256), 0, (hipStream_t)stream, o_dev, o_stride, g_dev, g_stride,
-                       weight_dev, gate, scale, out_dev, out_stride, rows, (int)heads, (int)dim, eps);
+    if (heads * dim > (1 << 24) || heads > 4 * 65535 || rows > 0x7fffffffLL) return CQ_ERR_RANGE;
+    hipStream_t s = (hipStream_t)stream;
+#define CQ_HG(K_, NH_)                                                                                                                                 \
+    hipLaunchKernelGGL(K_, dim3((unsigned)rows, (unsigned)((heads + 4 * NH_ - 1) / (4 * NH_))), dim3(256), 0, s, o_dev, o_stride, g_dev, g_stride, weight_dev, gate, \
+                       scale, out_dev, out_stride, (int)heads, (int)dim, eps)
+    if (dim <= 64) CQ_HG((head_norm_gate_kernel<1, 8>), 8);
+    else if (dim <= 128) CQ_HG((head_norm_gate_kernel<2, 4>), 4);
+    else if (dim <= 256) CQ_HG((head_norm_gate_kernel<4, 2>), 2);
+    else CQ_HG(head_norm_gate_long_kernel, 1);
+#undef CQ_HG
     return (int)hipGetLastError();
 }
 

@@ -369,11 +369,9 @@ __device__ __forceinline__ void delta_pack(const float *r, const float *k, const
 __global__ __launch_bounds__(256) void delta_prep_kernel(const float *__restrict__ row, int64_t row_stride, int64_t r_off, int64_t k_off, int64_t a_off,
                                                          const float *__restrict__ wl, int64_t wl_stride, const float *__restrict__ w0,
                                                          const float *__restrict__ ab, float *__restrict__ packed, int64_t rows, int heads, int dim, int sp) {
-    const int lane = threadIdx.x & 63;
-    const int64_t id = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
-    if (id >= rows * heads) return;
-    const int64_t t = id / heads;
-    const int64_t hd = (id - t * heads) * dim;
+    const int lane = threadIdx.x & 63, h = blockIdx.y * 4 + (threadIdx.x >> 6);
+    if (h >= heads) return;
+    const int64_t t = blockIdx.x, id = t * heads + h, hd = (int64_t)h * dim;
     const float *s = row + t * row_stride + hd, *w = wl + t * wl_stride + hd;
     delta_pack(s + r_off, s + k_off, s + a_off, [&](int d) { return w[d]; }, w0 + hd, ab + hd, packed + id * 4 * sp, packed + rows * heads * 4 * sp + id, dim, sp, lane);
 }
@@ -674,8 +672,8 @@ int cq_mix_delta_prep(const float *row_dev, int64_t row_stride, int64_t r_off, i
     if (row_stride < top + heads * dim) return CQ_ERR_SHAPE;
     if (rows == 0) return CQ_OK;
     if (!row_dev || !wl_dev || !w0_dev || !a_bias_dev || !packed_dev) return CQ_ERR_NULL;
-    if (dim > CQ_MIX_MAX_DIM || heads > (1 << 20) || (rows * heads + 3) / 4 > 0x7fffffffLL) return CQ_ERR_RANGE;
-    hipLaunchKernelGGL(delta_prep_kernel, dim3((unsigned)((rows * heads + 3) / 4)), dim3(256), 0, (hipStream_t)stream, row_dev, row_stride, r_off, k_off, a_off,
+    if (dim > CQ_MIX_MAX_DIM || heads > 4 * 65535 || rows > 0x7fffffffLL) return CQ_ERR_RANGE;
+    hipLaunchKernelGGL(delta_prep_kernel, dim3((unsigned)rows, (unsigned)((heads + 3) / 4)), dim3(256), 0, (hipStream_t)stream, row_dev, row_stride, r_off, k_off, a_off,
                        wl_dev, wl_stride, w0_dev, a_bias_dev, packed_dev, rows, (int)heads, (int)dim, (int)cq_mix_state_pad(dim));
     return (int)hipGetLastError();
 }
