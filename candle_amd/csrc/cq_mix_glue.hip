@@ -67,7 +67,7 @@ __global__ __launch_bounds__(256) void rms_norm_rows_kernel(float *x, int64_t x_
     }
 }
 
-// a N(z) + b N(z^2) + c N(z^3) + e: one workgroup per row, the row re-read after its three sums
+// sum over n = 1..3 of coef[n-1] z^n / rms(z^n), plus coef[3]: one workgroup per row, the row re-read after its three sums
 __global__ __launch_bounds__(256) void poly_norm_kernel(const float *z, int64_t z_stride, const float *__restrict__ coef, float *out, int64_t out_stride,
                                                         int dim, float eps) {
     __shared__ float red[4];

@@ -119,7 +119,7 @@ int cq_mix_talk_merge_retention_step(const void *workspace_dev, int64_t n_head, 
                                      float *ret_out_dev, const int32_t *pos_dev, int64_t pos, void *stream);
 
 /* ---- generalized delta rule -----------------------------------------------------------------------------------------
- * S <- diag(w) S - (a u)(u^T S) + k v^T (both terms read the old S), o = S^T r, u = k / sqrt(sum(k^2) + 1e-6),
+ * S <- (diag(w) - (a u) u^T) S + k v^T, o = S^T r, u = k / sqrt(sum(k^2) + 1e-6),
  * w = exp(-exp(-1/2) sigmoid(wl + w0)), a = sigmoid(al + a_bias).  States [heads, dim, state_pad], column-major as above.
  * row_dev: projection rows with r, k, v, al at the given offsets (each heads * dim); wl [rows, heads * dim].
  * cq_mix_delta_prep packs w | a u | u | r per (row, head), state_pad floats each, and behind them the |k| = sqrt(sum(k^2) + 1e-6) of every

@@ -52,9 +52,8 @@ def rotate_half(z, base, dims):
 
 
 def poly_norm(z, coef, eps):
-    """a N(z) + b N(z^2) + c N(z^3) + e with N = division by the row's root mean square."""
-    a, b, c, e = coef
-    return a * over_rms(z, eps) + b * over_rms(z * z, eps) + c * over_rms(z * z * z, eps) + e
+    """Cubic without a constant, each power divided by the row's root mean square of that power, plus the last coefficient."""
+    return sum(coef[n - 1] * over_rms(z ** n, eps) for n in (1, 2, 3)) + coef[3]
 
 
 # ------------------------------------------------------------------------------------------------- attention
@@ -112,7 +111,7 @@ def retention_mixer(h, t, pre, m, eps):
 
 # ------------------------------------------------------------------------------------------------- generalized delta rule
 def general_delta(r, k, v, w, a):
-    """All [T, H, d]: S <- diag(w) S - (a u)(u^T S) + k v^T with u the unit key, o = S^T r, token by token."""
+    """All [T, H, d]: S <- (diag(w) - (a u) u^T) S + k v^T with u the unit key, o = S^T r, token by token."""
     T, H, d = r.shape
     u = k / np.sqrt(np.sum(k * k, axis=-1, keepdims=True) + 1e-6)
     S = np.zeros((H, d, d))
