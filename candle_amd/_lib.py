@@ -88,12 +88,37 @@ class MixHeads(ctypes.Structure):
 
 _heads = ctypes.POINTER(MixHeads)
 
+
+class DenseArgs(ctypes.Structure):
+    """cq_dense_args of include/candle_hip_mixer.h."""
+    _fields_ = [(n, _vp) for n in ("w_dev", "x_dev", "dst_dev", "add_dev", "row_scale_dev", "src_rows_dev", "dst_rows_dev", "n_tiles_dev", "tiles_dev")] + \
+               [(n, _i64) for n in ("ldw", "ldx", "ldd", "ld_add", "m", "n", "k", "batch", "w_batch", "x_batch", "dst_batch", "max_tiles", "tile_rows")] + \
+               [(n, ctypes.c_int32) for n in ("x_bf16", "dst_bf16", "accumulate", "act")]
+
+
+class Latent(ctypes.Structure):
+    """cq_latent of include/candle_hip_mixer.h."""
+    _fields_ = [(n, _vp) for n in ("norm_dev", "cos_dev", "sin_dev")] + \
+               [(n, ctypes.c_int32) for n in ("heads", "dim", "rot_dim", "vdim", "rank", "rank_pad", "rot_pad", "ctx", "bf16")] + \
+               [("scale", _f32), ("eps", _f32), ("reserved", ctypes.c_int32)]
+
+
+class Moe(ctypes.Structure):
+    """cq_moe of include/candle_hip_mixer.h."""
+    _fields_ = [(n, _vp) for n in ("up_dev", "down_dev", "shared_up_dev", "shared_down_dev")] + [("up_stride", _i64), ("down_stride", _i64)] + \
+               [(n, ctypes.c_int32) for n in ("experts", "top", "kp", "ff", "ffp", "shared_ff", "shared_ffp", "reserved")]
+
+
+_dense, _latent, _moe = ctypes.POINTER(DenseArgs), ctypes.POINTER(Latent), ctypes.POINTER(Moe)
+
 # include/candle_hip_mixer.h
 MIXER_SIGNATURES = {
     "cq_dense_matmul_workspace_bytes": (_i64, [_int, _i64, _i64, _i64]),
     "cq_dense_matmul": (_int, [_int, _vp, _i64, _vp, _i64, _vp, _i64, _vp, _i64, _int, _i64, _i64, _i64, _vp, _i64, _vp]),
+    "cq_dense_product": (_int, [_int, _dense, _vp, _i64, _vp]),
     "cq_dense_matvec": (_int, [_vp, _i64, _vp, _int, _vp, _f32, _i64, _vp, _vp, _int, _i64, _i64, _vp]),
     "cq_mix_rms_norm_rows": (_int, [_vp, _i64, _vp, _vp, _i64, _vp, _vp, _i64, _i64, _i64, _f32, _vp]),
+    "cq_mix_layer_norm_rows": (_int, [_vp, _i64, _vp, _vp, _vp, _i64, _i64, _i64, _f32, _vp]),
     "cq_mix_poly_norm": (_int, [_vp, _i64, _vp, _vp, _i64, _i64, _i64, _f32, _vp]),
     "cq_mix_tanh": (_int, [_vp, _i64, _vp, _i64, _i64, _i64, _vp]),
     "cq_mix_pack_heads": (_int, [_vp, _i64, _heads, _int, _f32, _vp, _i64, _i64, _vp]),
@@ -111,6 +136,19 @@ MIXER_SIGNATURES = {
     "cq_mix_delta_scan": (_int, [_vp, _vp, _i64, _vp, _vp, _i64, _i64, _i64, _i64, _vp]),
     "cq_mix_delta_step": (_int, [_vp, _i64, _i64, _i64, _i64, _i64, _i64, _vp, _i64, _i64, _vp, _vp, _vp, _vp, _vp, _i64, _i64, _f32, _vp]),
 }
+MIXER_SIGNATURES.update({
+    "cq_mix_latent_pack": (_int, [_latent, _vp, _i64, _i64, _vp, _vp, _i64, _vp, _i64, _i64, _i64, _i64, _vp]),
+    "cq_mix_latent_expanded": (_int, [_latent, _vp, _i64, _vp, _i64, _i64, _i64, _vp, _vp, _i64, _vp, _i64, _i64, _i64, _vp]),
+    "cq_mix_latent_absorbed_workspace_bytes": (_i64, [_latent, _i64, _i64, _int]),
+    "cq_mix_latent_absorbed": (_int, [_latent, _vp, _vp, _vp, _i64, _vp, _i64, _i64, _vp, _i64, _vp]),
+    "cq_mix_latent_step": (_int, [_latent, _vp, _i64, _vp, _vp, _i64, _vp, _i64, _i64, _vp, _vp, _vp, _i64, _vp, _i64, _vp]),
+    "cq_mix_moe_select": (_int, [_vp, _i64, _i64, _i64, _i64, _vp, _vp, _vp, _vp]),
+    "cq_mix_moe_max_tiles": (_i64, [_i64, _i64, _i64, _i64]),
+    "cq_mix_moe_plan": (_int, [_vp, _vp, _i64, _i64, _i64, _i64, _vp, _vp, _vp, _vp, _vp, _vp]),
+    "cq_mix_moe_add": (_int, [_vp, _i64, _i64, _vp, _i64, _i64, _i64, _vp]),
+    "cq_mix_moe_step_fits": (_int, [_moe]),
+    "cq_mix_moe_step": (_int, [_moe, _vp, _int, _vp, _f32, _i64, _vp, _vp, _vp, _vp, _vp]),
+})
 # glue that the mixer library carries as well
 _MIXER_GLUE = ("cq_status_string", "cq_nn_embedding", "cq_nn_argmax")
 

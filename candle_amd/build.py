@@ -29,8 +29,8 @@ LIB_BENCH = os.path.join(HERE, "libcq_bench.so")
 SOURCES = ["cq_api.hip", "cq_dequant.hip", "cq_actquant.hip", "cq_matvec.hip", "cq_matmul.hip", "cq_moe.hip", "cq_quantize.hip", "cq_nn.hip", "cq_layer.hip", "cq_matvec_batch.hip", "cq_status.hip"]
 # models with bfloat16 weights: dense products and sequence mixers, with the glue of cq_nn.hip; complete without the library above, so
 # that such a model can run without compiling the quantized kernels
-MIXER_SOURCES = ["cq_nn.hip", "cq_status.hip", "cq_dense.hip", "cq_mix_glue.hip", "cq_mix_attention.hip", "cq_mix_state.hip"]
-MIXER_HEADERS = ("candle_hip_mixer.h", "cq_mix.h")
+MIXER_SOURCES = ["cq_nn.hip", "cq_status.hip", "cq_dense.hip", "cq_mix_glue.hip", "cq_mix_attention.hip", "cq_mix_state.hip", "cq_mix_latent.hip", "cq_mix_moe.hip"]
+MIXER_HEADERS = ("candle_hip_mixer.h", "cq_mix.h", "cq_dense.h")
 # the benchmark's plain-read yardstick kernel: a library of its own, not part of the C ABI
 BENCH_SOURCES = ["cq_bench.hip"]
 

@@ -1,4 +1,4 @@
-"""What a decoder keeps of one sequence: preallocated key/value caches and recurrent states, one per layer run."""
+"""What a decoder keeps of one sequence: preallocated key/value caches, latent rows and recurrent states, per layer run."""
 from __future__ import annotations
 
 from typing import List, Tuple
@@ -7,13 +7,14 @@ import torch
 
 
 class SequenceCache:
-    """Key/value caches are written at absolute positions and need no clearing; recurrent states start at zero and only move
+    """Key/value caches and latent rows are written at absolute positions and need no clearing; recurrent states start at zero and only move
     forward, so a model with states continues where the last call ended (``begin``) or starts over at position 0."""
 
     def __init__(self, device):
         self.device = torch.device(device)
         self.length = 0                              # positions held
         self.kv: List[Tuple[torch.Tensor, torch.Tensor]] = []
+        self.rows: List[torch.Tensor] = []
         self.states: List[torch.Tensor] = []
 
     def add_kv(self, heads: int, ctx: int, k_dim: int, v_dim: int) -> Tuple[torch.Tensor, torch.Tensor]:
@@ -21,6 +22,12 @@ class SequenceCache:
         pair = (torch.zeros((heads, ctx, k_dim), **f32), torch.zeros((heads, ctx, v_dim), **f32))
         self.kv.append(pair)
         return pair
+
+    def add_rows(self, ctx: int, width: int, dtype: torch.dtype) -> torch.Tensor:
+        """One row per position that all heads share (latents); layers may attend to another layer's rows."""
+        t = torch.zeros((ctx, width), dtype=dtype, device=self.device)
+        self.rows.append(t)
+        return t
 
     def add_state(self, *shape: int) -> torch.Tensor:
         s = torch.zeros(shape, dtype=torch.float32, device=self.device)
@@ -41,4 +48,4 @@ class SequenceCache:
             raise ValueError(f"position {pos} does not continue a sequence of {self.length} tokens (recurrent states cannot move back)")
 
     def nbytes(self) -> int:
-        return sum(t.numel() * t.element_size() for t in [x for p in self.kv for x in p] + self.states)
+        return sum(t.numel() * t.element_size() for t in [x for p in self.kv for x in p] + self.rows + self.states)

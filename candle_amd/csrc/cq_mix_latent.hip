@@ -1,0 +1,776 @@
+// Attention over latents: what a position leaves in the cache is one row shared by all heads, a normed latent c and a rotated key part.
+// A head's unrotated key is W_uk c and its value W_uv c.  Two ways to the same result:
+//   expanded   keys and values of all heads are computed (a dense product over the cache rows) and attended to head by head: many query rows
+//   absorbed   W_uk is applied to the query instead and W_uv to the attended latent: every head attends to the cache rows themselves, few query rows
+// T is the type that the products read: bfloat16, or float for products in f32.  Scores, weights, sums and outputs are f32.
+#include "cq_dense.h"
+#include "cq_mix.h"
+
+namespace {
+
+// ---- operands in 16-byte chunks: four chunks side by side (one per lane group) are one step of a product ------------------------------
+template <typename T> struct Chunk {
+    static constexpr int N = 16 / sizeof(T);               // elements
+    static constexpr int STEP = 4 * N;
+    static constexpr int KEYS = 128 / sizeof(T);           // keys per tile: a row of transposed values is eight chunks
+};
+template <typename T> __device__ __forceinline__ f32x4 mma(const u32x4 &a, const u32x4 &b, f32x4 c);
+template <> __device__ __forceinline__ f32x4 mma<__bf16>(const u32x4 &a, const u32x4 &b, f32x4 c) {
+    return __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, a), __builtin_bit_cast(bf16x8, b), c, 0, 0, 0);
+}
+template <> __device__ __forceinline__ f32x4 mma<float>(const u32x4 &a, const u32x4 &b, f32x4 c) {
+    const f32x4 x = __builtin_bit_cast(f32x4, a), y = __builtin_bit_cast(f32x4, b);
+#pragma unroll
+    for (int e = 0; e < 4; e++) c = mfma4(x[e], y[e], c);
+    return c;
+}
+
+// LDS chunk of 16 bytes `c` of key row r (rows of a multiple of eight chunks) and of value column r (eight chunks of keys)
+__device__ __forceinline__ int key_slot(int r, int c) { return c ^ (r & 7); }
+__device__ __forceinline__ int value_slot(int r, int c) { return c ^ ((r ^ (r >> 3)) & 7); }
+
+// Values of keys 4 a .. 4 a + 3, columns of chunk cg, transposed into LDS: [column][key].  The keys of a row are ordered so that the chunk that a lane reads
+// holds the keys whose scores it has: for bf16 4 lk .. 4 lk + 3 of two neighbouring tiles of 16.
+template <typename T> __device__ __forceinline__ void store_values(u32x4 *vs, int a, int cg, const u32x4 (&v)[4]);
+template <> __device__ __forceinline__ void store_values<__bf16>(u32x4 *vs, int a, int cg, const u32x4 (&v)[4]) {
+    const int chunk = (a >> 3) * 4 + (a & 3), half = (a >> 2) & 1;
+#pragma unroll
+    for (int j = 0; j < 8; j++) {
+        const int r = cg * 8 + j, w = j >> 1;
+        u32x2 x;
+        if (j & 1) {
+            x.x = (v[0][w] >> 16) | (v[1][w] & 0xffff0000u);
+            x.y = (v[2][w] >> 16) | (v[3][w] & 0xffff0000u);
+        } else {
+            x.x = (v[0][w] & 0xffffu) | (v[1][w] << 16);
+            x.y = (v[2][w] & 0xffffu) | (v[3][w] << 16);
+        }
+        reinterpret_cast<u32x2 *>(vs + r * 8 + value_slot(r, chunk))[half] = x;
+    }
+}
+template <> __device__ __forceinline__ void store_values<float>(u32x4 *vs, int a, int cg, const u32x4 (&v)[4]) {
+#pragma unroll
+    for (int j = 0; j < 4; j++) {
+        const int r = cg * 4 + j;
+        vs[r * 8 + value_slot(r, a)] = u32x4{v[0][j], v[1][j], v[2][j], v[3][j]};
+    }
+}
+
+// weights of a lane's keys (tiles of 16 in order, four keys each) as operand chunk s
+template <typename T> __device__ __forceinline__ u32x4 weight_chunk(const f32x4 *p, int s);
+template <> __device__ __forceinline__ u32x4 weight_chunk<__bf16>(const f32x4 *p, int s) {
+    bf16x8 r;
+#pragma unroll
+    for (int i = 0; i < 4; i++) {
+        r[i] = (__bf16)p[2 * s][i];
+        r[4 + i] = (__bf16)p[2 * s + 1][i];
+    }
+    return __builtin_bit_cast(u32x4, r);
+}
+template <> __device__ __forceinline__ u32x4 weight_chunk<float>(const f32x4 *p, int s) { return __builtin_bit_cast(u32x4, p[s]); }
+
+// over the four lanes that share lane & 15
+__device__ __forceinline__ float group_max(float v) {
+    v = fmaxf(v, __shfl_xor(v, 16, 64));
+    return fmaxf(v, __shfl_xor(v, 32, 64));
+}
+__device__ __forceinline__ float group_sum(float v) {
+    v += __shfl_xor(v, 16, 64);
+    return v + __shfl_xor(v, 32, 64);
+}
+
+// ---- expanded: causal attention head by head ---------------------------------------------------------------------------------------------
+// Workgroup: four waves of 16 NQ query rows of one head; tiles of keys through LDS, the next one on its way in registers.  Scores come out
+// transposed (key x query), so a lane holds one query's keys and its weights are the operand of the value product as they are; the outputs
+// come out as value column x query.
+struct Expanded {
+    const void *q, *k, *kr, *v;                            // [row][head], [key][head], [key], [key][head]
+    int64_t q_row, k_row, kr_row, v_row;
+    int q_head, k_head, v_head, d1, d2, vdim, v_pad;       // d1: unrotated dimensions (padded), d2: rotated
+    const float *gate;
+    int64_t gate_row;
+    float *out;
+    int64_t out_row;
+    int pos, rows, heads;
+    float scale_log2;
+};
+
+template <typename T, int DK, int DV, int NQ>
+__global__ __launch_bounds__(256) void latent_expanded_kernel(Expanded p) {
+    constexpr int CH = Chunk<T>::N, KT = Chunk<T>::KEYS, NT = KT / 16, NKF = DK / Chunk<T>::STEP, KC = DK / CH, NVF = DV / 16, BM = 64 * NQ;
+    constexpr int KL = KT * KC / 256, VT = (KT / 4) * (DV / CH), VL = (VT + 255) / 256;
+    __shared__ u32x4 ks[KT * KC], vs[DV * 8];
+    const int tid = threadIdx.x, lane = tid & 63, wv = __builtin_amdgcn_readfirstlane(tid >> 6), lr = lane & 15, lk = lane >> 4;
+    const int blocks = (p.rows + BM - 1) / BM, id = xcd_tile(blockIdx.x, blocks * p.heads), h = id / blocks;
+    const int m0 = (blocks - 1 - id % blocks) * BM, mw = m0 + wv * 16 * NQ;             // the longest rows first
+    const int last = p.pos + min(m0 + BM, p.rows) - 1, n_tiles = last / KT + 1, dk = p.d1 + p.d2;
+    const T *kb = (const T *)p.k + (int64_t)h * p.k_head, *krb = (const T *)p.kr, *vb = (const T *)p.v + (int64_t)h * p.v_head;
+
+    u32x4 qf[NQ][NKF];
+    int pq[NQ];
+#pragma unroll
+    for (int i = 0; i < NQ; i++) {
+        const int r = min(mw + 16 * i + lr, p.rows - 1);
+        pq[i] = p.pos + r;
+        const T *qr = (const T *)p.q + r * p.q_row + (int64_t)h * p.q_head;
+#pragma unroll
+        for (int s = 0; s < NKF; s++) {
+            const int c = (4 * s + lk) * CH;
+            qf[i][s] = c < dk ? *reinterpret_cast<const u32x4 *>(qr + c) : u32x4{0, 0, 0, 0};
+        }
+    }
+    u32x4 rk[KL], rv[VL][4];
+    auto fetch = [&](int j0) {
+#pragma unroll
+        for (int i = 0; i < KL; i++) {
+            const int idx = tid + 256 * i, c = (idx % KC) * CH;
+            const int64_t key = min(j0 + idx / KC, last);
+            rk[i] = u32x4{0, 0, 0, 0};
+            if (c < p.d1) rk[i] = *reinterpret_cast<const u32x4 *>(kb + key * p.k_row + c);
+            else if (c < dk) rk[i] = *reinterpret_cast<const u32x4 *>(krb + key * p.kr_row + c - p.d1);
+        }
+#pragma unroll
+        for (int i = 0; i < VL; i++) {
+            const int idx = tid + 256 * i, a = idx % (KT / 4), c = idx / (KT / 4) * CH;
+            if (c < p.v_pad)
+#pragma unroll
+                for (int j = 0; j < 4; j++) rv[i][j] = *reinterpret_cast<const u32x4 *>(vb + (int64_t)min(j0 + 4 * a + j, last) * p.v_row + c);
+        }
+    };
+    auto stage = [&]() {
+#pragma unroll
+        for (int i = 0; i < KL; i++) {
+            const int idx = tid + 256 * i, r = idx / KC;
+            ks[r * KC + key_slot(r, idx % KC)] = rk[i];
+        }
+#pragma unroll
+        for (int i = 0; i < VL; i++) {
+            const int idx = tid + 256 * i, a = idx % (KT / 4), cg = idx / (KT / 4);
+            if (cg * CH < p.v_pad) store_values<T>(vs, a, cg, rv[i]);
+        }
+    };
+
+    f32x4 o[NQ][NVF];
+    float m_run[NQ], l_run[NQ];
+#pragma unroll
+    for (int i = 0; i < NQ; i++) {
+        m_run[i] = -INFINITY;
+        l_run[i] = 0.0f;
+#pragma unroll
+        for (int n = 0; n < NVF; n++) o[i][n] = f32x4{0.f, 0.f, 0.f, 0.f};
+    }
+    fetch(0);
+    for (int it = 0; it < n_tiles; it++) {
+        const int j0 = it * KT;
+        __syncthreads();
+        stage();
+        __syncthreads();
+        if (it + 1 < n_tiles) fetch(j0 + KT);
+        if (j0 > p.pos + mw + 16 * NQ - 1) continue;       // wave-uniform: nothing visible to this wave's rows
+        f32x4 s[NQ][NT];
+#pragma unroll
+        for (int i = 0; i < NQ; i++)
+#pragma unroll
+            for (int t = 0; t < NT; t++) s[i][t] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int k = 0; k < NKF; k++)
+#pragma unroll
+            for (int t = 0; t < NT; t++) {
+                const int r = 16 * t + lr;
+                const u32x4 a = ks[r * KC + key_slot(r, 4 * k + lk)];
+#pragma unroll
+                for (int i = 0; i < NQ; i++) s[i][t] = mma<T>(a, qf[i][k], s[i][t]);
+            }
+        const bool edge = j0 + KT - 1 > p.pos + mw;        // some key of the tile lies after some row
+#pragma unroll
+        for (int i = 0; i < NQ; i++) {
+            float mx = -INFINITY;
+#pragma unroll
+            for (int t = 0; t < NT; t++)
+#pragma unroll
+                for (int e = 0; e < 4; e++) {
+                    float z = s[i][t][e] * p.scale_log2;
+                    if (edge && j0 + 16 * t + 4 * lk + e > pq[i]) z = -INFINITY;
+                    s[i][t][e] = z;
+                    mx = fmaxf(mx, z);
+                }
+            const float m = fmaxf(m_run[i], group_max(mx));                            // finite from the first tile on: key 0 is visible to every row
+            const float al = __builtin_amdgcn_exp2f(m_run[i] - m);
+            float sum = 0.0f;
+#pragma unroll
+            for (int t = 0; t < NT; t++)
+#pragma unroll
+                for (int e = 0; e < 4; e++) {
+                    s[i][t][e] = __builtin_amdgcn_exp2f(s[i][t][e] - m);
+                    sum += s[i][t][e];
+                }
+            if (__any(m > m_run[i])) {
+#pragma unroll
+                for (int n = 0; n < NVF; n++) o[i][n] *= al;
+            }
+            l_run[i] = l_run[i] * al + sum;
+            m_run[i] = m;
+        }
+#pragma unroll
+        for (int sp = 0; sp < 2; sp++) {
+            u32x4 w[NQ];
+#pragma unroll
+            for (int i = 0; i < NQ; i++) w[i] = weight_chunk<T>(s[i], sp);
+#pragma unroll
+            for (int n = 0; n < NVF; n++) {
+                const int r = 16 * n + lr;
+                const u32x4 a = vs[r * 8 + value_slot(r, 4 * sp + lk)];
+#pragma unroll
+                for (int i = 0; i < NQ; i++) o[i][n] = mma<T>(a, w[i], o[i][n]);
+            }
+        }
+    }
+    const bool vec = p.vdim % 4 == 0 && p.out_row % 4 == 0;
+#pragma unroll
+    for (int i = 0; i < NQ; i++) {
+        const int r = mw + 16 * i + lr;
+        const float l = group_sum(l_run[i]);
+        if (r >= p.rows) continue;
+        const float f = mix_sigmoid(p.gate[r * p.gate_row + h]) / l;
+        float *dst = p.out + r * p.out_row + (int64_t)h * p.vdim;
+#pragma unroll
+        for (int n = 0; n < NVF; n++) {
+            const int c = 16 * n + 4 * lk;
+            if (vec) {
+                if (c < p.vdim) *reinterpret_cast<f32x4 *>(dst + c) = o[i][n] * f;
+            } else {
+#pragma unroll
+                for (int e = 0; e < 4; e++)
+                    if (c + e < p.vdim) dst[c + e] = o[i][n][e] * f;
+            }
+        }
+    }
+}
+
+// ---- absorbed: every (row, head) attends to the cache rows themselves ------------------------------------------------------------------------
+// Workgroup: 16 NQ of the rows * heads queries, all on the same keys.  Per tile: wave t takes 16 keys of the scores, every wave does the softmax
+// of all queries from LDS, and takes every fourth 16 columns of the latent in the value product.  A cache row is read once for both products.
+// blockIdx.z: split of the key tiles.
+struct Absorbed {
+    const void *q, *cache;                                 // [row][head][ld], [key][ld]: rank_pad latent columns, then the rotated part
+    int ld, rank_pad, heads, rows, pos, ctx;
+    const int32_t *pos_dev;
+    float scale_log2;
+    const float *gate;
+    int64_t gate_row;
+    float *out;                                            // [row][head][rank_pad], gated
+    float *part;                                           // records instead: [split][query][rank_pad] unnormalized, then [split][query] of (maximum, sum)
+};
+
+template <typename T, int DK, int DV, int NQ>
+__global__ __launch_bounds__(256, 1) void latent_absorbed_kernel(Absorbed p) {
+    constexpr int CH = Chunk<T>::N, KT = Chunk<T>::KEYS, NT = KT / 16, NKF = DK / Chunk<T>::STEP, KC = DK / CH, NVW = DV / 64, BM = 16 * NQ;
+    constexpr int TASKS = (KT / 4) * KC, TL = (TASKS + 255) / 256, SS = KT + 4;
+    extern __shared__ __attribute__((aligned(16))) u32x4 lds[];
+    u32x4 *ks = lds, *vs = ks + KT * KC;
+    float *ss = reinterpret_cast<float *>(vs + DV * 8);    // scores [query][key]
+    const int tid = threadIdx.x, lane = tid & 63, wv = __builtin_amdgcn_readfirstlane(tid >> 6), lr = lane & 15, lk = lane >> 4;
+    const int M = p.rows * p.heads, m0 = blockIdx.x * BM, nz = gridDim.z, z = blockIdx.z;
+    const int pos = p.pos + (p.pos_dev ? p.pos_dev[0] : 0);
+    if (pos + p.rows > p.ctx) return;
+    const int last = pos + (min(m0 + BM, M) - 1) / p.heads, n_tiles = last / KT + 1;
+    const int lo = (int)((int64_t)n_tiles * z / nz), hi = (int)((int64_t)n_tiles * (z + 1) / nz);
+    const T *cache = (const T *)p.cache;
+
+    u32x4 qf[NQ][NKF];
+    int pq[NQ];
+#pragma unroll
+    for (int i = 0; i < NQ; i++) {
+        const int m = min(m0 + 16 * i + lr, M - 1);
+        pq[i] = pos + m / p.heads;
+#pragma unroll
+        for (int s = 0; s < NKF; s++) {
+            const int c = (4 * s + lk) * CH;
+            qf[i][s] = c < p.ld ? *reinterpret_cast<const u32x4 *>((const T *)p.q + (int64_t)m * p.ld + c) : u32x4{0, 0, 0, 0};
+        }
+    }
+    u32x4 rg[TL][4];
+    auto fetch = [&](int j0) {
+#pragma unroll
+        for (int i = 0; i < TL; i++) {
+            const int idx = tid + 256 * i, a = idx / KC, c = (idx % KC) * CH;
+#pragma unroll
+            for (int j = 0; j < 4; j++) {
+                rg[i][j] = u32x4{0, 0, 0, 0};
+                if (c < p.ld) rg[i][j] = *reinterpret_cast<const u32x4 *>(cache + (int64_t)min(j0 + 4 * a + j, last) * p.ld + c);
+            }
+        }
+    };
+    auto stage = [&]() {
+#pragma unroll
+        for (int i = 0; i < TL; i++) {
+            const int idx = tid + 256 * i, a = idx / KC, c = idx % KC;
+            if (TASKS % 256 && idx >= TASKS) break;
+#pragma unroll
+            for (int j = 0; j < 4; j++) ks[(4 * a + j) * KC + key_slot(4 * a + j, c)] = rg[i][j];
+            if (c * CH < p.rank_pad) store_values<T>(vs, a, c, rg[i]);
+        }
+    };
+
+    f32x4 o[NQ][NVW];
+    float m_run[NQ], l_run[NQ];
+#pragma unroll
+    for (int i = 0; i < NQ; i++) {
+        m_run[i] = -INFINITY;
+        l_run[i] = 0.0f;
+#pragma unroll
+        for (int n = 0; n < NVW; n++) o[i][n] = f32x4{0.f, 0.f, 0.f, 0.f};
+    }
+    if (lo < hi) fetch(lo * KT);
+    for (int it = lo; it < hi; it++) {
+        const int j0 = it * KT;
+        __syncthreads();
+        stage();
+        __syncthreads();
+        if (it + 1 < hi) fetch(j0 + KT);
+        if (wv < NT) {
+            const int r = 16 * wv + lr;
+            f32x4 s[NQ][2];
+#pragma unroll
+            for (int i = 0; i < NQ; i++) s[i][0] = s[i][1] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+            for (int k = 0; k < NKF; k++) {
+                const u32x4 a = ks[r * KC + key_slot(r, 4 * k + lk)];
+#pragma unroll
+                for (int i = 0; i < NQ; i++) s[i][k & 1] = mma<T>(a, qf[i][k], s[i][k & 1]);
+            }
+#pragma unroll
+            for (int i = 0; i < NQ; i++) *reinterpret_cast<f32x4 *>(ss + (16 * i + lr) * SS + 16 * wv + 4 * lk) = s[i][0] + s[i][1];
+        }
+        __syncthreads();
+        u32x4 w[NQ][2];
+#pragma unroll
+        for (int i = 0; i < NQ; i++) {
+            f32x4 s[NT];
+            float mx = -INFINITY, sum = 0.0f;
+#pragma unroll
+            for (int t = 0; t < NT; t++) {
+                s[t] = *reinterpret_cast<const f32x4 *>(ss + (16 * i + lr) * SS + 16 * t + 4 * lk);
+#pragma unroll
+                for (int e = 0; e < 4; e++) {
+                    s[t][e] = j0 + 16 * t + 4 * lk + e > pq[i] ? -INFINITY : s[t][e] * p.scale_log2;
+                    mx = fmaxf(mx, s[t][e]);
+                }
+            }
+            const float m = fmaxf(m_run[i], group_max(mx));
+            const float base = m > -INFINITY ? m : 0.0f;                               // a row before all keys of the split: weights of zero
+            const float al = __builtin_amdgcn_exp2f(m_run[i] - base);
+#pragma unroll
+            for (int t = 0; t < NT; t++)
+#pragma unroll
+                for (int e = 0; e < 4; e++) {
+                    s[t][e] = __builtin_amdgcn_exp2f(s[t][e] - base);
+                    sum += s[t][e];
+                }
+            if (__any(m > m_run[i])) {
+#pragma unroll
+                for (int n = 0; n < NVW; n++) o[i][n] *= al;
+            }
+            l_run[i] = l_run[i] * al + sum;
+            m_run[i] = m;
+#pragma unroll
+            for (int sp = 0; sp < 2; sp++) w[i][sp] = weight_chunk<T>(s, sp);
+        }
+#pragma unroll
+        for (int n = 0; n < NVW; n++)
+            if (64 * n + 16 * wv < p.rank_pad) {
+                const int r = 64 * n + 16 * wv + lr;
+#pragma unroll
+                for (int sp = 0; sp < 2; sp++) {
+                    const u32x4 a = vs[r * 8 + value_slot(r, 4 * sp + lk)];
+#pragma unroll
+                    for (int i = 0; i < NQ; i++) o[i][n] = mma<T>(a, w[i][sp], o[i][n]);
+                }
+            }
+    }
+#pragma unroll
+    for (int i = 0; i < NQ; i++) {
+        const int m = m0 + 16 * i + lr;
+        const float l = group_sum(l_run[i]);
+        if (m >= M) continue;
+        float f = 1.0f;
+        float *dst;
+        if (p.part) {
+            dst = p.part + ((int64_t)z * M + m) * p.rank_pad;
+            if (wv == 0 && lk == 0) {
+                float *ml = p.part + (int64_t)nz * M * p.rank_pad + 2 * ((int64_t)z * M + m);
+                ml[0] = m_run[i];
+                ml[1] = l;
+            }
+            if (lo >= hi) continue;                        // nothing but the (empty) sum
+        } else {
+            dst = p.out + (int64_t)m * p.rank_pad;
+            f = mix_sigmoid(p.gate[(m / p.heads) * p.gate_row + m % p.heads]) / l;
+        }
+#pragma unroll
+        for (int n = 0; n < NVW; n++) {
+            const int c = 64 * n + 16 * wv + 4 * lk;
+            if (c < p.rank_pad) *reinterpret_cast<f32x4 *>(dst + c) = o[i][n] * f;
+        }
+    }
+}
+
+// weights of the splits of one query into LDS: exp2(m - max) / sum (zero for empty splits).  One wave.
+__device__ __forceinline__ void split_weights(const float *__restrict__ ml, int64_t stride, int nz, float *wz, int lane) {
+    float m = -INFINITY, l = 0.0f;
+    for (int z = lane; z < nz; z += 64) m = fmaxf(m, ml[z * stride]);
+    m = wave_max(m);
+    for (int z = lane; z < nz; z += 64) {
+        const float e = __builtin_amdgcn_exp2f(ml[z * stride] - m);
+        wz[z] = e;
+        l = fmaf(e, ml[z * stride + 1], l);
+    }
+    l = wave_sum(l);
+    for (int z = lane; z < nz; z += 64) wz[z] /= l;
+}
+
+constexpr int MAX_SPLITS = 256;
+__device__ __forceinline__ void merge_latent(const float *__restrict__ part, int64_t stride, int nz, const float *wz, float f, float *dst, int n4, int tid, int threads) {
+    for (int c = tid; c < n4; c += threads) {
+        f32x4 a = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll 8
+        for (int z = 0; z < nz; z++) {
+            const float w = wz[z];
+            const f32x4 v = *reinterpret_cast<const f32x4 *>(part + z * stride + 4 * c);
+            a += w > 0.0f ? w * v : f32x4{0.f, 0.f, 0.f, 0.f};                         // an empty split has not written its record
+        }
+        *reinterpret_cast<f32x4 *>(dst + 4 * c) = a * f;
+    }
+}
+
+// one workgroup per query: the records of its splits into the gated latent
+__global__ __launch_bounds__(128) void latent_combine_kernel(const float *__restrict__ part, int nz, int M, int heads, int rank_pad, const float *__restrict__ gate,
+                                                             int64_t gate_row, float *__restrict__ out) {
+    __shared__ float wz[MAX_SPLITS];
+    const int m = blockIdx.x;
+    if (threadIdx.x < 64) split_weights(part + (int64_t)nz * M * rank_pad + 2 * m, 2 * (int64_t)M, nz, wz, threadIdx.x);
+    __syncthreads();
+    const float f = mix_sigmoid(gate[(m / heads) * gate_row + m % heads]);
+    merge_latent(part + (int64_t)m * rank_pad, (int64_t)M * rank_pad, nz, wz, f, out + (int64_t)m * rank_pad, rank_pad >> 2, threadIdx.x, 128);
+}
+
+// ---- projection rows into queries and cache rows -----------------------------------------------------------------------------------------------
+template <typename T> __device__ __forceinline__ float turned(const cq_latent &g, const float *src, int64_t p, int d) {
+    const int half = g.rot_dim >> 1;
+    const float c = g.cos_dev[p * half + (d >> 1)], s = g.sin_dev[p * half + (d >> 1)], v = src[d], w = src[d ^ 1];
+    return d & 1 ? v * c + w * s : v * c - w * s;
+}
+
+// latent (normed) and rotated key part of one projection row into the cache row of position p; all threads of the workgroup
+template <typename T, int THREADS> __device__ __forceinline__ void append_row(const cq_latent &g, const float *src, T *dst, int64_t p, float *red) {
+    const int tid = threadIdx.x, lane = tid & 63;
+    float q = 0.0f;
+    for (int i = tid; i < g.rank; i += THREADS) q = fmaf(src[i], src[i], q);
+    q = wave_sum(q);
+    if (lane == 0) red[tid >> 6] = q;
+    __syncthreads();
+    q = 0.0f;
+#pragma unroll
+    for (int i = 0; i < THREADS / 64; i++) q += red[i];
+    const float m = sqrtf(q / (float)g.rank + g.eps);
+    for (int i = tid; i < g.rank; i += THREADS) dst[i] = (T)(src[i] / m * g.norm_dev[i]);
+    for (int d = tid; d < g.rot_dim; d += THREADS) dst[g.rank_pad + d] = (T)turned<T>(g, src + g.rank, p, d);
+}
+
+// One workgroup per row.  plain != nullptr: unrotated query dimensions go there as f32, [row][head][plain_head]; else to the front of the head in q.
+template <typename T>
+__global__ __launch_bounds__(256) void latent_pack_kernel(cq_latent g, const float *__restrict__ row, int64_t row_stride, int64_t kv_off, T *cache, float *plain,
+                                                          int plain_head, T *q, int q_head, int rot_off, int64_t pos) {
+    __shared__ float red[4];
+    const int64_t r = blockIdx.x, p = pos + r;
+    const float *src = row + r * row_stride;
+    const int lane = threadIdx.x & 63, dq = g.dim + g.rot_dim;
+    for (int h = threadIdx.x >> 6; h < g.heads; h += 4) {
+        const float *s = src + (int64_t)h * dq;
+        T *d = q + (r * g.heads + h) * q_head;
+        float *f = plain ? plain + (r * g.heads + h) * plain_head : nullptr;
+        for (int i = lane; i < g.dim; i += 64) {
+            if (f) f[i] = s[i];
+            else d[i] = (T)s[i];
+        }
+        if (!f)
+            for (int i = g.dim + lane; i < rot_off; i += 64) d[i] = (T)0.0f;
+        for (int i = lane; i < q_head - rot_off; i += 64) d[rot_off + i] = i < g.rot_dim ? (T)turned<T>(g, s + g.dim, p, i) : (T)0.0f;
+    }
+    if (kv_off >= 0) append_row<T, 256>(g, src + kv_off, cache + p * (g.rank_pad + g.rot_pad), p, red);
+}
+
+// One token: workgroup (head, 64 latent columns) takes W_uk of its head to the query; those of the first columns rotate the rest of it.  The last workgroup
+// appends the cache row.  w_ukt [head][rank][ldw]: row j is column j of W_uk.
+template <typename T>
+__global__ __launch_bounds__(256) void latent_absorb_step_kernel(cq_latent g, const float *__restrict__ row, int64_t kv_off, T *cache, const uint16_t *__restrict__ w_ukt,
+                                                                 int ldw, T *__restrict__ q, const int32_t *__restrict__ pos_dev, int pos0) {
+    __shared__ float red[4];
+    const int lane = threadIdx.x & 63, wv = threadIdx.x >> 6, sub = lane & 15, dq = g.dim + g.rot_dim, ld = g.rank_pad + g.rot_pad;
+    const int pieces = (g.rank + 63) / 64, h = blockIdx.x / pieces, piece = blockIdx.x % pieces;
+    const int64_t p = pos0 + (pos_dev ? pos_dev[0] : 0);
+    if (p >= g.ctx) return;
+    if (h == g.heads) {
+        if (kv_off >= 0) append_row<T, 256>(g, row + kv_off, cache + p * ld, p, red);
+        return;
+    }
+    const float *s = row + (int64_t)h * dq;
+    T *d = q + (int64_t)h * ld;
+    const int j0 = piece * 64 + wv * 16 + (lane >> 4);
+    const uint16_t *w = w_ukt + (int64_t)h * g.rank * ldw;
+    float acc[4][2] = {};
+    for (int c0 = 0; c0 < g.dim; c0 += 128) {
+        const int c = c0 + 8 * sub;
+        u32x4 wr[4];
+#pragma unroll
+        for (int i = 0; i < 4; i++) wr[i] = c < ldw ? *reinterpret_cast<const u32x4 *>(w + (int64_t)min(j0 + 4 * i, g.rank - 1) * ldw + c) : u32x4{0, 0, 0, 0};
+        f32x4 a, b;
+#pragma unroll
+        for (int e = 0; e < 4; e++) {
+            a[e] = c + e < g.dim ? s[c + e] : 0.0f;
+            b[e] = c + 4 + e < g.dim ? s[c + 4 + e] : 0.0f;
+        }
+#pragma unroll
+        for (int i = 0; i < 4; i++) dot8(wr[i], a, b, acc[i]);
+    }
+#pragma unroll
+    for (int i = 0; i < 4; i++) {
+        const float v = row16_sum(acc[i][0] + acc[i][1]);
+        if (sub == 0 && j0 + 4 * i < g.rank) d[j0 + 4 * i] = (T)v;
+    }
+    if (piece == 0)
+        for (int i = threadIdx.x; i < g.rot_pad; i += 256) d[g.rank_pad + i] = i < g.rot_dim ? (T)turned<T>(g, s + g.dim, p, i) : (T)0.0f;
+}
+
+// One token: workgroup (head, 16 value rows) merges the records of the head's splits and takes W_uv to the gated latent.
+__global__ __launch_bounds__(256) void latent_merge_step_kernel(const float *__restrict__ part, int nz, int heads, int rank_pad, const uint16_t *__restrict__ w_uv, int ldw,
+                                                                const float *__restrict__ gate, float *__restrict__ out, int vdim) {
+    extern __shared__ __attribute__((aligned(16))) float o[];              // rank_pad floats
+    __shared__ float wz[MAX_SPLITS];
+    const int lane = threadIdx.x & 63, wv = threadIdx.x >> 6, h = blockIdx.x, e0 = blockIdx.y * 16 + 4 * wv;
+    const uint16_t *w[4];
+    u32x4 wr[4];
+#pragma unroll
+    for (int i = 0; i < 4; i++) {
+        w[i] = w_uv + ((int64_t)h * vdim + min(e0 + i, vdim - 1)) * ldw;
+        wr[i] = *reinterpret_cast<const u32x4 *>(w[i] + min(8 * lane, ldw - 8));
+    }
+    const float g = gate[h];
+    if (wv == 0) split_weights(part + (int64_t)nz * heads * rank_pad + 2 * h, 2 * (int64_t)heads, nz, wz, lane);
+    __syncthreads();
+    merge_latent(part + (int64_t)h * rank_pad, (int64_t)heads * rank_pad, nz, wz, 1.0f, o, rank_pad >> 2, threadIdx.x, 256);
+    __syncthreads();
+    float acc[4][2] = {};
+    for (int c = 8 * lane; c < rank_pad; c += 512) {
+        const f32x4 a = *reinterpret_cast<const f32x4 *>(o + c), b = *reinterpret_cast<const f32x4 *>(o + c + 4);
+#pragma unroll
+        for (int i = 0; i < 4; i++) dot8(c < 512 ? wr[i] : *reinterpret_cast<const u32x4 *>(w[i] + c), a, b, acc[i]);
+    }
+#pragma unroll
+    for (int i = 0; i < 4; i++) {
+        const float v = wave_sum(acc[i][0] + acc[i][1]);
+        if (lane == 0 && e0 + i < vdim) out[h * vdim + e0 + i] = v * mix_sigmoid(g);
+    }
+}
+
+int check_latent(const cq_latent *g) {
+    if (!g) return CQ_ERR_NULL;
+    if (g->heads <= 0 || g->dim <= 0 || g->vdim <= 0 || g->rank <= 0 || g->rot_dim < 0 || g->rot_dim % 2 || g->ctx <= 0 || g->rank_pad < g->rank || g->rank_pad % 64 ||
+        g->rot_pad < g->rot_dim || g->rot_pad % 8)
+        return CQ_ERR_SHAPE;
+    if (g->rot_dim && (!g->cos_dev || !g->sin_dev)) return CQ_ERR_NULL;
+    if (g->rank_pad > CQ_LATENT_MAX_RANK || g->rank_pad + g->rot_pad > CQ_LATENT_MAX_ROW || g->heads > 4096 || g->dim > 4096 || g->vdim > 4096 || g->ctx > (1 << 24))
+        return CQ_ERR_RANGE;
+    return CQ_OK;
+}
+
+// queries per workgroup / 16, and splits of the keys
+int absorbed_nq(int bf16, int64_t m) { return bf16 && m > 16 ? 2 : 1; }
+int absorbed_splits(int bf16, int64_t m, int64_t keys) {
+    const int64_t blocks = (m + 16 * absorbed_nq(bf16, m) - 1) / (16 * absorbed_nq(bf16, m)), kt = bf16 ? 64 : 32, tiles = (keys + kt - 1) / kt;
+    int64_t n = blocks >= 256 ? 1 : 256 / blocks;
+    n = n < tiles ? n : tiles;
+    return (int)(n < MAX_SPLITS ? n : MAX_SPLITS);
+}
+
+template <typename T, int DK, int DV, int NQ> int absorbed_launch(const Absorbed &a, int nz, hipStream_t s) {
+    constexpr size_t lds = (size_t)Chunk<T>::KEYS * DK * sizeof(T) + (size_t)DV * 128 + (size_t)16 * NQ * (Chunk<T>::KEYS + 4) * sizeof(float);
+    static_assert(lds <= 160 * 1024, "LDS");
+    if (lds > 64 * 1024) {
+        const int e = (int)hipFuncSetAttribute(reinterpret_cast<const void *>(latent_absorbed_kernel<T, DK, DV, NQ>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+        if (e) return e;
+    }
+    hipLaunchKernelGGL((latent_absorbed_kernel<T, DK, DV, NQ>), dim3((unsigned)((a.rows * a.heads + 16 * NQ - 1) / (16 * NQ)), 1, nz), dim3(256), lds, s, a);
+    return (int)hipGetLastError();
+}
+template <typename T> int absorbed_dispatch(const Absorbed &a, int nz, hipStream_t s) {
+#define CQ_AB(DK_, DV_)                                                                                                                              \
+    do {                                                                                                                                             \
+        if constexpr (sizeof(T) == 2) {                                                                                                              \
+            if (absorbed_nq(1, (int64_t)a.rows * a.heads) == 2) return absorbed_launch<T, DK_, DV_, 2>(a, nz, s);                                      \
+        }                                                                                                                                            \
+        return absorbed_launch<T, DK_, DV_, 1>(a, nz, s);                                                                                            \
+    } while (0)
+    if (a.ld <= 192 && a.rank_pad <= 128) CQ_AB(192, 128);
+    if (a.ld <= 320 && a.rank_pad <= 256) CQ_AB(320, 256);
+    CQ_AB(576, 512);
+#undef CQ_AB
+}
+
+template <typename T, int DK, int DV, int NQ> int expanded_launch(const Expanded &a, hipStream_t s) {
+    const int64_t blocks = (int64_t)((a.rows + 64 * NQ - 1) / (64 * NQ)) * a.heads;
+    if (blocks > 0x7fffffffLL) return CQ_ERR_RANGE;
+    hipLaunchKernelGGL((latent_expanded_kernel<T, DK, DV, NQ>), dim3((unsigned)blocks), dim3(256), 0, s, a);
+    return (int)hipGetLastError();
+}
+
+}  // namespace
+
+extern "C" {
+
+int cq_mix_latent_pack(const cq_latent *g, const float *row_dev, int64_t row_stride, int64_t kv_off, void *cache_dev, float *plain_dev, int64_t plain_head, void *q_dev,
+                       int64_t q_head, int64_t rot_off, int64_t pos, int64_t rows, void *stream) {
+    const int e = check_latent(g);
+    if (e) return e;
+    const int64_t dq = g->dim + g->rot_dim;
+    if (rows < 0 || pos < 0 || row_stride < g->heads * dq || (kv_off >= 0 && kv_off + g->rank + g->rot_dim > row_stride) || q_head < rot_off + g->rot_dim ||
+        (plain_dev ? plain_head < g->dim : rot_off < g->dim))
+        return CQ_ERR_SHAPE;
+    if (rows == 0) return CQ_OK;
+    if (!row_dev || !q_dev || (kv_off >= 0 && (!cache_dev || !g->norm_dev))) return CQ_ERR_NULL;
+    if (pos + rows > g->ctx || q_head > (1 << 20)) return CQ_ERR_RANGE;
+#define CQ_LP(T_) hipLaunchKernelGGL(latent_pack_kernel<T_>, dim3((unsigned)rows), dim3(256), 0, (hipStream_t)stream, *g, row_dev, row_stride, kv_off, (T_ *)cache_dev, \
+                                     plain_dev, (int)plain_head, (T_ *)q_dev, (int)q_head, (int)rot_off, pos)
+    if (g->bf16) CQ_LP(__bf16);
+    else CQ_LP(float);
+#undef CQ_LP
+    return (int)hipGetLastError();
+}
+
+int cq_mix_latent_expanded(const cq_latent *g, const void *q_dev, int64_t dim_pad, const void *kv_dev, int64_t kv_row, int64_t v_off, int64_t v_pad, const void *cache_dev,
+                           const float *gate_dev, int64_t gate_row, float *out_dev, int64_t out_row, int64_t pos, int64_t rows, void *stream) {
+    const int e = check_latent(g);
+    if (e) return e;
+    if (rows < 0 || pos < 0 || dim_pad < g->dim || dim_pad % 8 || v_pad < g->vdim || v_pad % 8 || v_off % 8 || kv_row % 8 || v_off < g->heads * dim_pad ||
+        kv_row < v_off + g->heads * v_pad || gate_row < g->heads || out_row < g->heads * g->vdim)
+        return CQ_ERR_SHAPE;
+    if (rows == 0) return CQ_OK;
+    if (!q_dev || !kv_dev || !cache_dev || !gate_dev || !out_dev) return CQ_ERR_NULL;
+    if (misaligned(q_dev, 16) || misaligned(kv_dev, 16) || misaligned(cache_dev, 16) || misaligned(out_dev, 16)) return CQ_ERR_ALIGN;
+    if (pos + rows > g->ctx || dim_pad + g->rot_pad > CQ_LATENT_MAX_HEAD || v_pad > CQ_LATENT_MAX_VALUE) return CQ_ERR_RANGE;
+    Expanded a;
+    const size_t el = g->bf16 ? 2 : 4;
+    a.q = q_dev;
+    a.k = kv_dev;
+    a.kr = (const char *)cache_dev + el * g->rank_pad;
+    a.v = (const char *)kv_dev + el * v_off;
+    a.q_head = (int)(dim_pad + g->rot_pad);
+    a.q_row = (int64_t)g->heads * a.q_head;
+    a.k_row = a.v_row = kv_row;
+    a.kr_row = g->rank_pad + g->rot_pad;
+    a.k_head = a.d1 = (int)dim_pad;
+    a.d2 = g->rot_pad;
+    a.v_head = a.v_pad = (int)v_pad;
+    a.vdim = g->vdim;
+    a.gate = gate_dev;
+    a.gate_row = gate_row;
+    a.out = out_dev;
+    a.out_row = out_row;
+    a.pos = (int)pos;
+    a.rows = (int)rows;
+    a.heads = g->heads;
+    a.scale_log2 = g->scale * 1.44269504088896341f;
+    hipStream_t s = (hipStream_t)stream;
+    const int dk = a.q_head;
+    // 32 query rows per wave where that leaves two workgroups per CU
+    const bool wide = (rows + 127) / 128 * g->heads >= 512;
+#define CQ_EX(DK_, DV_)                                                                                                     \
+    do {                                                                                                                    \
+        if (!g->bf16) return expanded_launch<float, DK_, DV_, 1>(a, s);                                                     \
+        return wide ? expanded_launch<__bf16, DK_, DV_, 2>(a, s) : expanded_launch<__bf16, DK_, DV_, 1>(a, s);              \
+    } while (0)
+    if (dk <= 128 && v_pad <= 128) CQ_EX(128, 128);
+    if (dk <= 192 && v_pad <= 128) CQ_EX(192, 128);
+    return g->bf16 ? expanded_launch<__bf16, 320, 256, 1>(a, s) : expanded_launch<float, 320, 256, 1>(a, s);
+#undef CQ_EX
+}
+
+int64_t cq_mix_latent_absorbed_workspace_bytes(const cq_latent *g, int64_t rows, int64_t pos, int step) {
+    if (check_latent(g) || rows <= 0) return -1;
+    const int64_t m = rows * g->heads;
+    const int nz = absorbed_splits(g->bf16, m, step ? g->ctx : pos + rows);
+    return nz > 1 || step ? nz * m * (g->rank_pad + 2) * 4 : 0;
+}
+
+int cq_mix_latent_absorbed(const cq_latent *g, const void *q_dev, const void *cache_dev, const float *gate_dev, int64_t gate_row, float *out_dev, int64_t pos, int64_t rows,
+                           void *workspace_dev, int64_t workspace_bytes, void *stream) {
+    const int e = check_latent(g);
+    if (e) return e;
+    if (rows < 0 || pos < 0 || gate_row < g->heads) return CQ_ERR_SHAPE;
+    if (rows == 0) return CQ_OK;
+    if (!q_dev || !cache_dev || !gate_dev || !out_dev) return CQ_ERR_NULL;
+    if (misaligned(q_dev, 16) || misaligned(cache_dev, 16) || misaligned(out_dev, 16) || misaligned(workspace_dev, 16)) return CQ_ERR_ALIGN;
+    if (pos + rows > g->ctx || rows * g->heads > (1 << 24)) return CQ_ERR_RANGE;
+    const int64_t m = rows * g->heads, need = cq_mix_latent_absorbed_workspace_bytes(g, rows, pos, 0);
+    const int nz = absorbed_splits(g->bf16, m, pos + rows);
+    if (need && (!workspace_dev || workspace_bytes < need)) return CQ_ERR_WORKSPACE;
+    Absorbed a;
+    a.q = q_dev;
+    a.cache = cache_dev;
+    a.ld = g->rank_pad + g->rot_pad;
+    a.rank_pad = g->rank_pad;
+    a.heads = g->heads;
+    a.rows = (int)rows;
+    a.pos = (int)pos;
+    a.ctx = g->ctx;
+    a.pos_dev = nullptr;
+    a.scale_log2 = g->scale * 1.44269504088896341f;
+    a.gate = gate_dev;
+    a.gate_row = gate_row;
+    a.out = out_dev;
+    a.part = nz > 1 ? (float *)workspace_dev : nullptr;
+    hipStream_t s = (hipStream_t)stream;
+    const int r = g->bf16 ? absorbed_dispatch<__bf16>(a, nz, s) : absorbed_dispatch<float>(a, nz, s);
+    if (r || nz == 1) return r;
+    hipLaunchKernelGGL(latent_combine_kernel, dim3((unsigned)m), dim3(128), 0, s, (const float *)workspace_dev, nz, (int)m, g->heads, g->rank_pad, gate_dev, gate_row, out_dev);
+    return (int)hipGetLastError();
+}
+
+int cq_mix_latent_step(const cq_latent *g, const float *row_dev, int64_t kv_off, void *cache_dev, const void *w_ukt_dev, int64_t ld_ukt, const void *w_uv_dev, int64_t ld_uv,
+                       int64_t gate_off, void *q_dev, float *out_dev, const int32_t *pos_dev, int64_t pos, void *workspace_dev, int64_t workspace_bytes, void *stream) {
+    const int e = check_latent(g);
+    if (e) return e;
+    if (pos < 0 || ld_ukt < g->dim || ld_ukt % 8 || ld_uv < g->rank_pad || ld_uv % 8 || gate_off < 0) return CQ_ERR_SHAPE;
+    if (!row_dev || !cache_dev || !w_ukt_dev || !w_uv_dev || !q_dev || !out_dev || !workspace_dev || (kv_off >= 0 && !g->norm_dev)) return CQ_ERR_NULL;
+    if (misaligned(cache_dev, 16) || misaligned(w_ukt_dev, 16) || misaligned(w_uv_dev, 16) || misaligned(q_dev, 16) || misaligned(workspace_dev, 16)) return CQ_ERR_ALIGN;
+    if (pos >= g->ctx) return CQ_ERR_RANGE;
+    if (workspace_bytes < cq_mix_latent_absorbed_workspace_bytes(g, 1, 0, 1)) return CQ_ERR_WORKSPACE;
+    const int nz = absorbed_splits(g->bf16, g->heads, g->ctx);
+    hipStream_t s = (hipStream_t)stream;
+    const dim3 grid((unsigned)(g->heads * ((g->rank + 63) / 64) + 1));
+    if (g->bf16)
+        hipLaunchKernelGGL(latent_absorb_step_kernel<__bf16>, grid, dim3(256), 0, s, *g, row_dev, kv_off, (__bf16 *)cache_dev, (const uint16_t *)w_ukt_dev, (int)ld_ukt,
+                           (__bf16 *)q_dev, pos_dev, (int)pos);
+    else
+        hipLaunchKernelGGL(latent_absorb_step_kernel<float>, grid, dim3(256), 0, s, *g, row_dev, kv_off, (float *)cache_dev, (const uint16_t *)w_ukt_dev, (int)ld_ukt,
+                           (float *)q_dev, pos_dev, (int)pos);
+    Absorbed a = {};
+    a.q = q_dev;
+    a.cache = cache_dev;
+    a.ld = g->rank_pad + g->rot_pad;
+    a.rank_pad = g->rank_pad;
+    a.heads = g->heads;
+    a.rows = 1;
+    a.pos = (int)pos;
+    a.ctx = g->ctx;
+    a.pos_dev = pos_dev;
+    a.scale_log2 = g->scale * 1.44269504088896341f;
+    a.part = (float *)workspace_dev;
+    const int r = g->bf16 ? absorbed_dispatch<__bf16>(a, nz, s) : absorbed_dispatch<float>(a, nz, s);
+    if (r) return r;
+    hipLaunchKernelGGL(latent_merge_step_kernel, dim3((unsigned)g->heads, (unsigned)((g->vdim + 15) / 16)), dim3(256), g->rank_pad * sizeof(float), s,
+                       (const float *)workspace_dev, nz, g->heads, g->rank_pad, (const uint16_t *)w_uv_dev, (int)ld_uv, row_dev + gate_off, out_dev, g->vdim);
+    return (int)hipGetLastError();
+}
+
+}  // extern "C"

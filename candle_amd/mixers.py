@@ -17,11 +17,12 @@ import numpy as np
 import torch
 
 from . import _lib
-from ._lib import MixHeads
+from ._lib import DenseArgs, Latent, MixHeads, Moe
 from .cache import SequenceCache
 
 BF16, F32 = 0, 1                                     # enum cq_dense_precision
-PLAIN, NORM, POLY = 0, 1, 2                          # enum cq_dense_prologue
+PLAIN, NORM, POLY, LAYER_NORM, RELU2 = 0, 1, 2, 3, 4  # enum cq_dense_prologue
+ACT_NONE, ACT_RELU2, ACT_SWIGLU = 0, 1, 2            # enum cq_dense_act
 SILU, SIGMOID = 0, 1                                 # enum cq_gate
 MATVEC_MAX_K = 32768                                 # CQ_DENSE_MATVEC_MAX_K
 
@@ -30,6 +31,22 @@ check = _lib.check
 
 def pad_to(n: int, m: int) -> int:
     return (n + m - 1) // m * m
+
+
+def frequencies(base: float, dims: int, scaling: Optional[dict] = None) -> tuple:
+    """Angle per position of each pair of dimensions, base^(-2 i / dims), and a factor on cos and sin (1 without scaling).
+
+    YaRN scaling: pairs that turn more than ``fast`` times over ``original`` positions keep their frequency, those that turn less than ``slow``
+    times are slowed down by ``factor``, those between are blended linearly in i; cos and sin grow by 0.1 ln(factor) + 1."""
+    i = np.arange(dims // 2, dtype=np.float64)
+    freq = np.float64(base) ** (-2.0 * i / dims)
+    if not scaling:
+        return freq, 1.0
+    factor, original = float(scaling["factor"]), float(scaling["original"])
+    pair = lambda turns: dims * math.log(original / (2.0 * math.pi * turns)) / (2.0 * math.log(base))
+    lo, hi = max(math.floor(pair(float(scaling["fast"]))), 0), min(math.ceil(pair(float(scaling["slow"]))), dims - 1)
+    slowed = np.clip((i - lo) / max(hi - lo, 0.001), 0.0, 1.0)
+    return freq * (1.0 - slowed) + freq / factor * slowed, 0.1 * math.log(factor) + 1.0
 
 
 class Runtime:
@@ -60,12 +77,23 @@ class Runtime:
             self.generation += 1
         return t.data_ptr()
 
-    def rotation(self, base: float, dims: int) -> tuple:
-        """cos / sin [ctx, dims / 2] of t * base^(-2 i / dims), evaluated in double and rounded once."""
-        key = (float(base), int(dims))
+    @property
+    def t_bf16(self) -> bool:
+        """Whether intermediate values that only feed matrix products are kept in bfloat16."""
+        return self.precision == BF16
+
+    def typed(self, name: str, count: int) -> int:
+        """Scratch for ``count`` values of the products' input type.  A name is used either for these or for f32 (one read as the other
+        need not be finite)."""
+        return self.scratch(name, (count + 1) // 2 if self.t_bf16 else count)
+
+    def rotation(self, base: float, dims: int, scaling: Optional[dict] = None) -> tuple:
+        """cos / sin [ctx, dims / 2] of t * frequency, evaluated in double and rounded once (see ``frequencies``)."""
+        key = (float(base), int(dims), tuple(sorted(scaling.items())) if scaling else None)
         if key not in self._tables:
-            ang = np.arange(self.ctx, dtype=np.float64)[:, None] * np.float64(base) ** (-2.0 * np.arange(dims // 2, dtype=np.float64) / dims)
-            self._tables[key] = tuple(torch.from_numpy(f(ang).astype(np.float32)).to(self.device) for f in (np.cos, np.sin))
+            freq, factor = frequencies(base, dims, scaling)
+            ang = np.arange(self.ctx, dtype=np.float64)[:, None] * freq
+            self._tables[key] = tuple(torch.from_numpy((factor * f(ang)).astype(np.float32)).to(self.device) for f in (np.cos, np.sin))
         return self._tables[key]
 
     def vector(self, t: torch.Tensor) -> torch.Tensor:
@@ -101,17 +129,58 @@ class Dense:
     def nbytes(self) -> int:
         return self.w.numel() * 2
 
-    def rows(self, x: int, ldx: int, dst: int, ldd: int, rows: int, sp, accumulate: bool = False) -> None:
+    def rows(self, x: int, ldx: int, dst: int, ldd: int, rows: int, sp, accumulate: bool = False, precision: Optional[int] = None, **options) -> None:
+        """Several rows; `options` are further fields of cq_dense_args."""
         rt = self.rt
-        need = rt.L.cq_dense_matmul_workspace_bytes(rt.precision, rows, self.n, self.kp)
-        ws = rt.scratch("dense_planes", need // 4) if need else None
-        check("cq_dense_matmul", rt.L.cq_dense_matmul(rt.precision, self.w.data_ptr(), self.kp, x, ldx, dst, ldd, None, 0, int(accumulate), rows, self.n, self.kp,
-                                                      ws, need, sp))
+        precision = rt.precision if precision is None else precision
+        need = rt.L.cq_dense_matmul_workspace_bytes(precision, rows, self.n, self.kp)
+        dense_product(rt, precision, sp, rt.scratch("dense_planes", need // 4) if need else None, need, w_dev=self.w.data_ptr(), ldw=self.kp, x_dev=x, ldx=ldx, dst_dev=dst,
+                      ldd=ldd, m=rows, n=self.n, k=self.kp, batch=1, accumulate=int(accumulate), **options)
 
     def row(self, x: int, dst: int, sp, prologue: int = PLAIN, vec: Optional[torch.Tensor] = None, eps: float = 0.0, accumulate: bool = False,
             add: Optional[int] = None) -> None:
         check("cq_dense_matvec", self.rt.L.cq_dense_matvec(self.w.data_ptr(), self.kp, x, prologue, vec.data_ptr() if vec is not None else None, eps, self.k, dst,
                                                           add, int(accumulate), self.n, self.kp, sp))
+
+
+def dense_product(rt: Runtime, precision: int, sp, workspace=None, workspace_bytes: int = 0, **fields) -> None:
+    check("cq_dense_product", rt.L.cq_dense_product(precision, DenseArgs(**fields), workspace, workspace_bytes, sp))
+
+
+def alternate(gate: torch.Tensor, up: torch.Tensor) -> torch.Tensor:
+    """Rows gate 0, up 0, gate 1, up 1, ...: what the gated activation of a product takes."""
+    return torch.stack([gate, up], dim=1).reshape(2 * gate.shape[0], gate.shape[1])
+
+
+class RmsNorm:
+    """x / rms(x) * weight, over rows or as the prologue of a single-row product."""
+
+    prologue = NORM
+
+    def __init__(self, rt: Runtime, get: Callable[[str], torch.Tensor], name: str, eps: float):
+        self.rt, self.eps = rt, eps
+        self.vec = rt.vector(get(name))
+        self.dim = self.vec.numel()
+
+    def rows(self, x: int, ldx: int, out: int, ldo: int, rows: int, sp, index: Optional[int] = None, delta: Optional[int] = None) -> None:
+        """Rows of x (those that `index` names) into out; `delta` [rows, ldx] is added to x first."""
+        check("cq_mix_rms_norm_rows", self.rt.L.cq_mix_rms_norm_rows(x, ldx, index, delta, ldx, self.vec.data_ptr(), out, ldo, rows, self.dim, self.eps, sp))
+
+
+class LayerNorm:
+    """(x - mean) / standard deviation * weight + bias; the bias is the tensor of the same name with '.b' added."""
+
+    prologue = LAYER_NORM
+
+    def __init__(self, rt: Runtime, get: Callable[[str], torch.Tensor], name: str, eps: float):
+        self.rt, self.eps = rt, eps
+        self.vec = torch.cat([rt.vector(get(name)), rt.vector(get(name + ".b"))])
+        self.dim = self.vec.numel() // 2
+
+    def rows(self, x: int, ldx: int, out: int, ldo: int, rows: int, sp, index: Optional[int] = None, delta: Optional[int] = None) -> None:
+        if delta is not None:
+            raise ValueError("this norm adds nothing to its input")
+        check("cq_mix_layer_norm_rows", self.rt.L.cq_mix_layer_norm_rows(x, ldx, index, self.vec.data_ptr(), out, ldo, rows, self.dim, self.eps, sp))
 
 
 def _heads(src_off: int, heads: int, dim: int, *, dim_pad: int = 0, dst: Optional[int] = None, row_stride: int = 0, head_stride: int = 0,
@@ -128,7 +197,7 @@ def _group_array(groups: List[MixHeads]):
 class Rotation:
     def __init__(self, rt: Runtime, cfg: Optional[dict]):
         self.dims = int(cfg["dims"]) if cfg else 0
-        self.tables = rt.rotation(cfg["base"], self.dims) if self.dims else None
+        self.tables = rt.rotation(cfg["base"], self.dims, cfg.get("scaling")) if self.dims else None
 
     def args(self) -> dict:
         return dict(tables=self.tables, rot_dims=self.dims)
@@ -239,6 +308,8 @@ class Retention:
 class Mixer:
     """A layer's first sublayer: x <- x + mixer(norm(x)).  ``norm_rows`` has left norm(x) in `h` for ``prefill``; ``step`` applies it itself."""
 
+    kv_from: Optional[int] = None                    # a layer whose cache this one attends to instead of having its own
+
     def denses(self) -> List[Dense]:
         raise NotImplementedError
 
@@ -248,7 +319,7 @@ class Mixer:
     def prefill(self, h: int, ldh: int, x: int, ldx: int, kept, pos: int, rows: int, sp) -> None:
         raise NotImplementedError
 
-    def step(self, x: int, norm: torch.Tensor, kept, pos_dev: Optional[int], pos: int, add: Optional[int], sp) -> None:
+    def step(self, x: int, norm, kept, pos_dev: Optional[int], pos: int, add: Optional[int], sp) -> None:
         raise NotImplementedError
 
 
@@ -294,7 +365,7 @@ class Parallel(Mixer):
         kv, state = kept
         row, out = rt.scratch("projection", self.w_in.n), rt.scratch("mixer_out", self.w_out.kp)
         rec, rec_bytes = lt.records()
-        self.w_in.row(x, row, sp, NORM, norm, self.eps)
+        self.w_in.row(x, row, sp, norm.prologue, norm.vec, norm.eps)
         check("cq_mix_talk_decode", rt.L.cq_mix_talk_decode(row, _group_array(lt.groups(kv, 0, None)), self.eps, lt.talk.data_ptr(), lt.scale, lt.window,
                                                             lt.keep_first, pos_dev, pos, rec, rec_bytes, sp))
         v_off, g_off = rg.offsets(self.off)
@@ -347,7 +418,7 @@ class GeneralDelta(Mixer):
     def step(self, x, norm, kept, pos_dev, pos, add, sp):
         rt = self.rt
         row, out = rt.scratch("projection", self.w_in.n), rt.scratch("mixer_out", self.w_out.kp)
-        self.w_in.row(x, row, sp, NORM, norm, self.eps)
+        self.w_in.row(x, row, sp, norm.prologue, norm.vec, norm.eps)
         check("cq_mix_delta_step", rt.L.cq_mix_delta_step(row, self.r_off, self.k_off, self.v_off, self.g_off, self.a_off, self.low_off, self.w2.w.data_ptr(), self.w2.kp,
                                                           self.rank, self.w0.data_ptr(), self.a_bias.data_ptr(), self.norm.data_ptr(), kept.data_ptr(), out,
                                                           self.heads, self.dim, self.eps, sp))
@@ -377,9 +448,206 @@ class PolyFeedForward:
 
     def step(self, x, norm, add, sp):
         z = self.rt.scratch("feed_forward", self.down.kp)
-        self.up.row(x, z, sp, NORM, norm, self.eps)
+        self.up.row(x, z, sp, norm.prologue, norm.vec, norm.eps)
         self.down.row(z, x, sp, POLY, self.coef, self.eps, accumulate=True, add=add)
 
 
-MIXERS = {"parallel": Parallel, "general_delta": GeneralDelta}
-FEED_FORWARDS = {"dense": PolyFeedForward}
+class LatentAttention(Mixer):
+    """Causal softmax attention whose keys and values are linear in a cached latent: per position one normed latent and one rotated key part for all
+    heads.  Heads are gated by a sigmoid of their own.  With ``kv_from`` the layer has no latent of its own and attends to another layer's cache.
+
+    Many rows: keys and values of all heads are computed from the cache rows, then attended to head by head.  Few rows and single tokens: the key matrix is
+    applied to the query and the value matrix to the attended latent, so that the heads attend to the cache rows themselves."""
+
+    MAX_RANK, MAX_ROW, MAX_HEAD, MAX_VALUE = 512, 576, 320, 256      # CQ_LATENT_MAX_*
+
+    def __init__(self, rt: Runtime, cfg: dict, get: Callable[[str], torch.Tensor], eps: float):
+        self.rt, self.eps = rt, eps
+        self.heads, self.dim, self.rot_dim, self.vdim, self.rank = (int(cfg[k]) for k in ("heads", "dim", "rot_dim", "vdim", "kv_rank"))
+        self.kv_from = None if cfg.get("kv_from") is None else int(cfg["kv_from"])
+        H, r = self.heads, self.rank
+        self.rank_pad, self.rot_pad, self.dim_pad, self.v_pad = pad_to(r, 64), pad_to(self.rot_dim, 8), pad_to(self.dim, 8), pad_to(self.vdim, 8)
+        self.ld = self.rank_pad + self.rot_pad
+        if self.rank_pad > self.MAX_RANK or self.ld > self.MAX_ROW:
+            raise ValueError(f"latents of {r} + {self.rot_dim} are longer than {self.MAX_RANK} + {self.MAX_ROW - self.MAX_RANK}")
+        rot = Rotation(rt, cfg.get("rot"))
+        if rot.dims != self.rot_dim:
+            raise ValueError("the rotated part of a head is rotated as a whole")
+        own = self.kv_from is None
+        self.w_in = Dense(rt, [get("q")] + ([get("dkv")] if own else []) + [get("g")])
+        self.kv_off = H * (self.dim + self.rot_dim) if own else -1
+        self.g_off = self.w_in.n - H
+        if self.w_in.n != H * (self.dim + self.rot_dim + 1) + (r + self.rot_dim if own else 0):
+            raise ValueError("projection sizes do not match the mixer's configuration")
+        uk, uv = get("uk").to(rt.device), get("uv").to(rt.device)
+        if uk.shape != (H * self.dim, r) or uv.shape != (H * self.vdim, r):
+            raise ValueError("key and value sizes do not match the mixer's configuration")
+        self.ukt = torch.zeros((H, r, pad_to(self.dim, 64)), dtype=torch.bfloat16, device=rt.device)
+        self.ukt[..., :self.dim] = uk.view(H, self.dim, r).transpose(1, 2)
+        self.uv = Dense(rt, [uv])
+        self.w_out = Dense(rt, [get("o")])
+        self.expand = None
+        if self.dim_pad + self.rot_pad <= self.MAX_HEAD and self.v_pad <= self.MAX_VALUE:
+            padded = lambda w, d, dp: torch.nn.functional.pad(w.view(H, d, r), (0, 0, 0, dp - d)).reshape(H * dp, r)
+            self.expand = Dense(rt, [padded(uk, self.dim, self.dim_pad), padded(uv, self.vdim, self.v_pad)])
+        norm = rt.vector(get("dkv.norm")) if own else None
+        self.norm, self.tables = norm, rot.tables
+        self.shape = Latent(norm.data_ptr() if own else None, rot.tables[0].data_ptr() if rot.dims else None, rot.tables[1].data_ptr() if rot.dims else None, H, self.dim,
+                            self.rot_dim, self.vdim, r, self.rank_pad, self.rot_pad, rt.ctx, int(rt.t_bf16), float(cfg["scale"]), eps, 0)
+
+    def denses(self) -> List[Dense]:
+        return [self.w_in, self.uv, self.w_out]
+
+    def token_bytes(self) -> int:
+        """Weight bytes of a single-token step."""
+        return sum(d.nbytes() for d in self.denses()) + self.ukt.numel() * 2
+
+    def new_cache(self, cache: SequenceCache) -> torch.Tensor:
+        return cache.add_rows(self.rt.ctx, self.ld, torch.bfloat16 if self.rt.t_bf16 else torch.float32)
+
+    def expands(self, rows: int) -> bool:
+        """Whether computing keys and values per head costs less than attending to latents with `rows` queries."""
+        d = self.dim + self.vdim
+        return self.expand is not None and rows * (2 * self.rank - d) > self.rank * d
+
+    def prefill(self, h, ldh, x, ldx, kept, pos, rows, sp):
+        rt, L, H = self.rt, self.rt.L, self.heads
+        ldp, ldo, bf = pad_to(self.w_in.n, 4), self.w_out.kp, int(rt.t_bf16)
+        row, out = rt.scratch("projection", rows * ldp), rt.scratch("mixer_out", rows * ldo)
+        gate = row + 4 * self.g_off
+        self.w_in.rows(h, ldh, row, ldp, rows, sp)
+        if self.expands(rows):
+            head, ldkv, keys = self.dim_pad + self.rot_pad, self.expand.n, pos + rows
+            q, kv = rt.typed("latent_q", rows * H * head), rt.typed("latent_kv", keys * ldkv)
+            check("cq_mix_latent_pack", L.cq_mix_latent_pack(self.shape, row, ldp, self.kv_off, kept.data_ptr(), None, 0, q, head, self.dim_pad, pos, rows, sp))
+            self.expand.rows(kept.data_ptr(), self.ld, kv, ldkv, keys, sp, x_bf16=bf, dst_bf16=bf)
+            check("cq_mix_latent_expanded", L.cq_mix_latent_expanded(self.shape, q, self.dim_pad, kv, ldkv, H * self.dim_pad, self.v_pad, kept.data_ptr(), gate, ldp, out, ldo,
+                                                                     pos, rows, sp))
+        else:
+            kp = self.ukt.shape[2]
+            plain, q, lat = rt.scratch("latent_plain", rows * H * kp), rt.typed("latent_q", rows * H * self.ld), rt.scratch("latent_out", rows * H * self.rank_pad)
+            check("cq_mix_latent_pack", L.cq_mix_latent_pack(self.shape, row, ldp, self.kv_off, kept.data_ptr(), plain, kp, q, self.ld, self.rank_pad, pos, rows, sp))
+            dense_product(rt, rt.precision, sp, w_dev=self.ukt.data_ptr(), ldw=kp, w_batch=self.rank * kp, x_dev=plain, ldx=H * kp, x_batch=kp, dst_dev=q, ldd=H * self.ld,
+                          dst_batch=self.ld, dst_bf16=bf, m=rows, n=self.rank, k=kp, batch=H)
+            need = L.cq_mix_latent_absorbed_workspace_bytes(self.shape, rows, pos, 0)
+            ws = rt.scratch("attention_splits", need // 4) if need else None
+            check("cq_mix_latent_absorbed", L.cq_mix_latent_absorbed(self.shape, q, kept.data_ptr(), gate, ldp, lat, pos, rows, ws, need, sp))
+            dense_product(rt, rt.precision, sp, w_dev=self.uv.w.data_ptr(), ldw=self.uv.kp, w_batch=self.vdim * self.uv.kp, x_dev=lat, ldx=H * self.rank_pad,
+                          x_batch=self.rank_pad, dst_dev=out, ldd=ldo, dst_batch=self.vdim, m=rows, n=self.vdim, k=self.uv.kp, batch=H)
+        self.w_out.rows(out, ldo, x, ldx, rows, sp, accumulate=True)
+
+    def step(self, x, norm, kept, pos_dev, pos, add, sp):
+        rt, L = self.rt, self.rt.L
+        row, out, q = rt.scratch("projection", self.w_in.n), rt.scratch("mixer_out", self.w_out.kp), rt.typed("latent_q", self.heads * self.ld)
+        need = L.cq_mix_latent_absorbed_workspace_bytes(self.shape, 1, 0, 1)
+        ws = rt.scratch("attention_records", need // 4)
+        self.w_in.row(x, row, sp, norm.prologue, norm.vec, norm.eps)
+        check("cq_mix_latent_step", L.cq_mix_latent_step(self.shape, row, self.kv_off, kept.data_ptr(), self.ukt.data_ptr(), self.ukt.shape[2], self.uv.w.data_ptr(), self.uv.kp,
+                                                         self.g_off, q, out, pos_dev, pos, ws, need, sp))
+        self.w_out.row(out, x, sp, accumulate=True, add=add)
+
+
+class ReluSquaredFeedForward:
+    """down(relu(up(norm(x)))^2)."""
+
+    def __init__(self, rt: Runtime, cfg: dict, get: Callable[[str], torch.Tensor], eps: float):
+        self.rt = rt
+        self.up, self.down = Dense(rt, [get("up")]), Dense(rt, [get("down")])
+        if self.up.n != int(cfg["ff"]) or self.down.k != int(cfg["ff"]):
+            raise ValueError("feed-forward sizes do not match the configuration")
+
+    def denses(self) -> List[Dense]:
+        return [self.up, self.down]
+
+    def prefill(self, h, ldh, x, ldx, rows, sp):
+        rt, ld, bf = self.rt, self.down.kp, int(self.rt.t_bf16)
+        z = rt.typed("activation", rows * ld)
+        self.up.rows(h, ldh, z, ld, rows, sp, act=ACT_RELU2, dst_bf16=bf)
+        self.down.rows(z, ld, x, ldx, rows, sp, accumulate=True, x_bf16=bf)
+
+    def step(self, x, norm, add, sp):
+        z = self.rt.scratch("feed_forward", self.down.kp)
+        self.up.row(x, z, sp, norm.prologue, norm.vec, norm.eps)
+        self.down.row(z, x, sp, RELU2, accumulate=True, add=add)
+
+
+class GatedExperts:
+    """A mixture of small feed-forwards down(silu(gate(h)) * up(h)), weighted by the softmax over the chosen router logits, and optionally one that every token
+    takes, weighted by a sigmoid.  The choice and everything after it stay on the device."""
+
+    def __init__(self, rt: Runtime, cfg: dict, get: Callable[[str], torch.Tensor], eps: float):
+        self.rt = rt
+        self.experts, self.top, self.ff = int(cfg["router"]["experts"]), int(cfg["router"]["top"]), int(cfg["expert"]["ff"])
+        router = get("router")
+        self.width = router.shape[1]
+        if not 1 <= self.top <= self.experts or router.shape[0] != self.experts:
+            raise ValueError("router sizes do not match the configuration")
+        shared = cfg.get("shared")
+        self.shared_ff = int(shared["ff"]) if shared else 0
+        self.router = Dense(rt, [router] + ([get("shared.sg")] if shared else []))
+        self.kp, self.ffp = pad_to(self.width, 64), pad_to(self.ff, 64)
+        self.up = torch.zeros((self.experts, 2 * self.ff, self.kp), dtype=torch.bfloat16, device=rt.device)
+        self.down = torch.zeros((self.experts, self.width, self.ffp), dtype=torch.bfloat16, device=rt.device)
+        for e in range(self.experts):
+            gate, up, down = (get(f"e{e}.{n}").to(rt.device) for n in ("gate", "up", "down"))
+            if gate.shape != (self.ff, self.width) or up.shape != gate.shape or down.shape != (self.width, self.ff):
+                raise ValueError("expert sizes do not match the configuration")
+            self.up[e, :, :self.width] = alternate(gate, up)
+            self.down[e, :, :self.ff] = down
+        self.shared_up = self.shared_down = None
+        if shared:
+            self.shared_up, self.shared_down = Dense(rt, [alternate(get("shared.gate"), get("shared.up"))]), Dense(rt, [get("shared.down")])
+            if self.shared_up.n != 2 * self.shared_ff or self.shared_down.k != self.shared_ff:
+                raise ValueError("shared expert sizes do not match the configuration")
+        self.sizes = Moe(self.up.data_ptr(), self.down.data_ptr(), self.shared_up.w.data_ptr() if shared else None, self.shared_down.w.data_ptr() if shared else None,
+                         self.up[0].numel(), self.down[0].numel(), self.experts, self.top, self.kp, self.ff, self.ffp, self.shared_ff, self.shared_down.kp if shared else 0, 0)
+        self.fused = bool(rt.L.cq_mix_moe_step_fits(self.sizes))
+
+    def denses(self) -> List[Dense]:
+        return [self.router]
+
+    def token_bytes(self) -> int:
+        """Weight bytes of a single-token step."""
+        shared = self.shared_up.nbytes() + self.shared_down.nbytes() if self.shared_ff else 0
+        return self.router.nbytes() + shared + 2 * self.top * (self.up[0].numel() + self.down[0].numel())
+
+    def prefill(self, h, ldh, x, ldx, rows, sp):
+        rt, L, E, top, bf = self.rt, self.rt.L, self.experts, self.top, int(self.rt.t_bf16)
+        ldl, pairs = pad_to(self.router.n, 4), rows * top
+        logits = rt.scratch("router_logits", rows * ldl)
+        ids, weights, shared = rt.scratch("expert_ids", pairs), rt.scratch("expert_weights", pairs), rt.scratch("shared_weights", rows)
+        self.router.rows(h, ldh, logits, ldl, rows, sp, precision=F32)
+        check("cq_mix_moe_select", L.cq_mix_moe_select(logits, ldl, rows, E, top, ids, weights, shared if self.shared_ff else None, sp))
+        if self.shared_ff:
+            ld = self.shared_down.kp
+            z = rt.typed("shared_activation", rows * ld)
+            self.shared_up.rows(h, ldh, z, ld, rows, sp, act=ACT_SWIGLU, row_scale_dev=shared, dst_bf16=bf)
+            self.shared_down.rows(z, ld, x, ldx, rows, sp, accumulate=True, x_bf16=bf)
+        per_expert = pairs / E
+        tile = 64 if not bf else (128 if per_expert >= 96 else (64 if per_expert >= 24 else 32))
+        max_tiles = L.cq_mix_moe_max_tiles(rows, E, top, tile)
+        src, dst, scale = (rt.scratch("pair_" + n, pairs) for n in ("src", "dst", "scale"))
+        tiles, n_tiles = rt.scratch("pair_tiles", 4 * max_tiles), rt.scratch("pair_n_tiles", 1)
+        check("cq_mix_moe_plan", L.cq_mix_moe_plan(ids, weights, rows, E, top, tile, src, dst, scale, tiles, n_tiles, sp))
+        z, ldy = rt.typed("expert_activation", pairs * self.ffp), pad_to(self.width, 4)
+        y = rt.scratch("expert_out", pairs * ldy)
+        grouped = dict(tiles_dev=tiles, n_tiles_dev=n_tiles, max_tiles=max_tiles, tile_rows=tile, m=pairs, batch=1)
+        dense_product(rt, rt.precision, sp, w_dev=self.up.data_ptr(), ldw=self.kp, w_batch=self.up[0].numel(), x_dev=h, ldx=ldh, dst_dev=z, ldd=self.ffp, n=2 * self.ff,
+                      k=self.kp, src_rows_dev=src, row_scale_dev=scale, act=ACT_SWIGLU, dst_bf16=bf, **grouped)
+        dense_product(rt, rt.precision, sp, w_dev=self.down.data_ptr(), ldw=self.ffp, w_batch=self.down[0].numel(), x_dev=z, ldx=self.ffp, dst_dev=y, ldd=ldy, n=self.width,
+                      k=self.ffp, dst_rows_dev=dst, x_bf16=bf, **grouped)
+        check("cq_mix_moe_add", L.cq_mix_moe_add(y, ldy, top, x, ldx, rows, self.width, sp))
+
+    def step(self, x, norm, add, sp):
+        rt = self.rt
+        if not self.fused:                           # sizes beyond the two launches: the several-row path with one row
+            if add is not None:
+                raise ValueError("no addend on this path")
+            h = rt.scratch("h", self.kp)
+            norm.rows(x, self.kp, h, self.kp, 1, sp)
+            self.prefill(h, self.kp, x, self.kp, 1, sp)
+            return
+        logits, ids = rt.scratch("router_logits", pad_to(self.router.n, 4)), rt.scratch("expert_ids", self.top)
+        act = rt.scratch("feed_forward", self.top * self.ffp + (self.shared_down.kp if self.shared_ff else 0))
+        self.router.row(x, logits, sp, norm.prologue, norm.vec, norm.eps)
+        check("cq_mix_moe_step", rt.L.cq_mix_moe_step(self.sizes, x, norm.prologue, norm.vec.data_ptr(), norm.eps, self.width, logits, act, ids, add, sp))

@@ -10,8 +10,13 @@ def _venizen():
     return Model
 
 
+def _kudurax():
+    from .kudurax import Model
+    return Model
+
+
 # config.json "architecture" -> class with from_pretrained(path, device, dtype, ctx)
-ARCHITECTURES = {"Venizen": _venizen}
+ARCHITECTURES = {"Venizen": _venizen, "Kudurax": _kudurax}
 
 
 def load_model(path: str, device="cuda:0", dtype: str = "bfloat16", ctx: int = 4096):
