@@ -43,6 +43,8 @@ The JSON line carries, besides the driver contract fields:
     python bench.py --workload venizen [--steps 128] [--prompt 2048]
                                    Venizen decoders at two sizes (random bf16 weights): prompt and decode tok/s, each beside
                                    the Q4_K_M llama decoder of the same width, depth and feed-forward
+    python bench.py --workload kudurax [--steps 128] [--prompt 2048]
+                                   the same for Kudurax decoders, beside the Venizen decoder of the same width, depth and feed-forward
 """
 import argparse
 import json
@@ -350,10 +352,39 @@ def venizen_config(width, vocab, ctx):
             "loop": {"start": 2, "stop": 4, "times": 2}}
 
 
-def venizen(args):
-    """Prompt and decode throughput of Venizen decoders at two widths, and of the Q4_K_M llama decoder of equal size."""
+def kudurax_config(width, vocab, ctx):
+    """Eight layers, heads of 128 + 64 over latents of 512, half of the layers attending to another one's latents; dense feed-forwards and mixtures of 64
+    experts, of which a token takes 6 and the shared one, in turn."""
+    heads, ff = width // 128, width * 7 // 2
+    mixer = {"heads": heads, "dim": 128, "rot_dim": 64, "vdim": 128, "kv_rank": 512, "scale": 192 ** -0.5,
+             "rot": {"base": 10000.0, "dims": 64, "scaling": {"factor": 40.0, "fast": 32.0, "slow": 1.0, "original": 4096}}}
+    dense = {"kind": "dense", "ff": ff}
+    mixture = {"kind": "moe", "router": {"experts": 64, "top": 6}, "expert": {"ff": width * 11 // 16}, "shared": {"ff": width * 11 // 8}}
+    layer = lambda mlp, source=None: {"type": "latent_attention", "mixer": dict(mixer, kv_from=source) if source is not None else mixer, "mlp": mlp}
+    half = lambda at: [layer(dense), layer(mixture), layer(dense, at + 1), layer(mixture, at + 1)]
+    return {"vocab": vocab, "width": width, "norm": {"eps": 1e-5}, "embedding": {"scale": 1.0}, "layers": half(0) + half(4)}
+
+
+def timed_generation(model, prompt, n_new, ctx):
+    """Prompt and decode throughput: the best of three generations after a warm one."""
+    model.generate_greedy(prompt, 8)
+    best = None
+    for _ in range(3):
+        r = model.generate_greedy(prompt, n_new, max_kv=ctx)
+        best = r if best is None or r["decode_seconds"] < best["decode_seconds"] else best
+        best["prompt_seconds"] = min(best["prompt_seconds"], r["prompt_seconds"])
+    tok_s, wbytes = best["decode_steps"] / best["decode_seconds"], model.weight_bytes_per_token()
+    return {"prompt_tok_s": round(len(prompt) / best["prompt_seconds"], 1), "decode_tok_s": round(tok_s, 1), "weight_bytes_per_token": wbytes,
+            "decode_frac_of_weight_roofline": round(tok_s * wbytes / 1e9 / HBM_PEAK_GBPS, 4),
+            "prompt_weight_matmul_TFLOPs": round((wbytes - model.head.nbytes()) * len(prompt) / best["prompt_seconds"] / 1e12, 1) if hasattr(model, "head") else None}
+
+
+def bf16_decoder(args):
+    """Prompt and decode throughput of the decoders with bfloat16 weights at two widths, each beside the closest other decoder of equal size: Venizen beside the
+    Q4_K_M llama decoder, Kudurax beside Venizen."""
     import torch
 
+    from candle_amd import kudurax as kd
     from candle_amd import quantized_llama as ql
     from candle_amd import venizen as vz
 
@@ -362,31 +393,21 @@ def venizen(args):
     gen.manual_seed(99)
     ctx, vocab, records = args.prompt + n_new + 8, 32768, []
     for width in (2048, 4096):
-        d = venizen_config(width, vocab, ctx)
-        cfg = vz.Config.from_dict(d, ctx)
+        vcfg, kcfg = vz.Config.from_dict(venizen_config(width, vocab, ctx), ctx), kd.Config.from_dict(kudurax_config(width, vocab, ctx), ctx)
+        lcfg = ql.Config(n_layer=len(vcfg.order), hidden=width, n_head=width // 128, n_kv_head=max(1, width // 512), head_dim=128, ffn=width * 7 // 2, vocab=vocab, ctx=ctx)
         prompt = torch.randint(0, vocab, (args.prompt,), generator=gen).tolist()
-        lcfg = ql.Config(n_layer=len(cfg.order), hidden=width, n_head=width // 128, n_kv_head=max(1, width // 512), head_dim=128, ffn=width * 7 // 2, vocab=vocab, ctx=ctx)
-        rec = {"width": width, "layer_runs": len(cfg.order), "ff": width * 7 // 2, "prompt": args.prompt}
-        for name, make in (("venizen_bf16", lambda: vz.Model.random_init(cfg, seed=7)), ("llama_q4_k_m", lambda: ql.ModelWeights.random_init(lcfg, seed=7))):
-            model = make()
-            model.generate_greedy(prompt, 8)
-            best = None
-            for _ in range(3):
-                r = model.generate_greedy(prompt, n_new, max_kv=ctx)
-                best = r if best is None or r["decode_seconds"] < best["decode_seconds"] else best
-                best["prompt_seconds"] = min(best["prompt_seconds"], r["prompt_seconds"])
-            tok_s, wbytes = best["decode_steps"] / best["decode_seconds"], model.weight_bytes_per_token()
-            rec[name] = {"prompt_tok_s": round(args.prompt / best["prompt_seconds"], 1), "decode_tok_s": round(tok_s, 1), "weight_bytes_per_token": wbytes,
-                         "decode_frac_of_weight_roofline": round(tok_s * wbytes / 1e9 / HBM_PEAK_GBPS, 4)}
-            if name == "venizen_bf16":
-                flop = 2.0 * sum(w.numel() for la in [model.layers[i] for i, _ in cfg.order]
-                                 for w in [x.w for x in la.mixer.denses() + (la.mlp.denses() if la.mlp else [])])
-                rec[name]["prompt_matmul_TFLOPs"] = round(flop * args.prompt / best["prompt_seconds"] / 1e12, 1)
+        makes = {"venizen_bf16": lambda: vz.Model.random_init(vcfg, seed=7), "llama_q4_k_m": lambda: ql.ModelWeights.random_init(lcfg, seed=7),
+                 "kudurax_bf16": lambda: kd.Model.random_init(kcfg, seed=7)}
+        rec = {"width": width, "layer_runs": len(vcfg.order), "ff": width * 7 // 2, "prompt": args.prompt}
+        for name in ("venizen_bf16", "llama_q4_k_m") if args.workload == "venizen" else ("kudurax_bf16", "venizen_bf16"):
+            model = makes[name]()
+            rec[name] = timed_generation(model, prompt, n_new, ctx)
             del model
             torch.cuda.empty_cache()
         records.append(rec)
-    big = records[-1]["venizen_bf16"]
-    return {"metric": "Venizen decode tok/s (batch 1, greedy, width 4096)", "value": big["decode_tok_s"], "unit": "tok/s", "n_gpus": 1, "steps": n_new - 1, "warmup": 8,
+    design = args.workload.capitalize()
+    big = records[-1][args.workload + "_bf16"]
+    return {"metric": "%s decode tok/s (batch 1, greedy, width 4096)" % design, "value": big["decode_tok_s"], "unit": "tok/s", "n_gpus": 1, "steps": n_new - 1, "warmup": 8,
             "ms_per_step": round(1e3 / big["decode_tok_s"], 4), "higher_is_better": True, "scaling": "weak", "vs_baseline": None, "dtype": "bf16", "data": "synthetic",
             "config": {"workload": "random-init weights, 8 layer runs, vocab %d, %d prompt tokens, then %d greedy steps from one HIP graph" % (vocab, args.prompt, n_new - 1)},
             "results": records}
@@ -552,9 +573,9 @@ def main():
     ap.add_argument("--gpus", type=int, default=1)
     ap.add_argument("--steps", type=int, default=None)
     ap.add_argument("--warmup", type=int, default=None)
-    ap.add_argument("--workload", choices=["decode", "prefill", "decode8b", "moe", "venizen"], default="decode")
+    ap.add_argument("--workload", choices=["decode", "prefill", "decode8b", "moe", "venizen", "kudurax"], default="decode")
     ap.add_argument("--layers", type=int, default=32, help="--workload decode8b: number of decoder layers")
-    ap.add_argument("--prompt", type=int, default=512, help="--workload decode8b / venizen: prompt tokens")
+    ap.add_argument("--prompt", type=int, default=512, help="--workload decode8b / venizen / kudurax: prompt tokens")
     ap.add_argument("--moe-tokens", default="1,16,256", help="--workload moe: token counts, comma separated")
     ap.add_argument("--moe-layers", type=int, default=48, help="--workload moe: layers, each with its own expert weights (340 MB per layer)")
     ap.add_argument("--wdtype", choices=sorted(WDTYPES), default="q4k",
@@ -576,8 +597,8 @@ def main():
     if args.workload == "moe":
         print(json.dumps(moe(args)))
         return
-    if args.workload == "venizen":
-        print(json.dumps(venizen(args)))
+    if args.workload in ("venizen", "kudurax"):
+        print(json.dumps(bf16_decoder(args)))
         return
     if args.steps is None:
         args.steps = 4000 if args.workload == "decode" else 50
