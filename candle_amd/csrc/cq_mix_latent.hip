@@ -2,7 +2,8 @@
 // A head's unrotated key is W_uk c and its value W_uv c.  Two ways to the same result:
 //   expanded   keys and values of all heads are computed (a dense product over the cache rows) and attended to head by head: many query rows
 //   absorbed   W_uk is applied to the query instead and W_uv to the attended latent: every head attends to the cache rows themselves, few query rows
-// T is the type that the products read: bfloat16, or float for products in f32.  Scores, weights, sums and outputs are f32.
+// T is the type that the products read: bfloat16, or float for products in f32.  Scores, weights, sums and outputs are f32.  Queries are packed with the scale and
+// log2(e) multiplied in, so that a weight is a power of two.
 #include "cq_dense.h"
 #include "cq_mix.h"
 
@@ -24,6 +25,10 @@ template <> __device__ __forceinline__ f32x4 mma<float>(const u32x4 &a, const u3
     for (int e = 0; e < 4; e++) c = mfma4(x[e], y[e], c);
     return c;
 }
+
+// Weights are taken relative to a reference that follows the running maximum only when that is more than this far ahead (in powers of two): sums and outputs
+// are rarely rescaled, and no weight exceeds 2^8.
+constexpr float LAG = 8.0f;
 
 // LDS chunk of 16 bytes `c` of key row r (rows of a multiple of eight chunks) and of value column r (eight chunks of keys)
 __device__ __forceinline__ int key_slot(int r, int c) { return c ^ (r & 7); }
@@ -92,7 +97,6 @@ struct Expanded {
     float *out;
     int64_t out_row;
     int pos, rows, heads;
-    float scale_log2;
 };
 
 template <typename T, int DK, int DV, int NQ>
@@ -101,8 +105,11 @@ __global__ __launch_bounds__(256) void latent_expanded_kernel(Expanded p) {
     constexpr int KL = KT * KC / 256, VT = (KT / 4) * (DV / CH), VL = (VT + 255) / 256;
     __shared__ u32x4 ks[KT * KC], vs[DV * 8];
     const int tid = threadIdx.x, lane = tid & 63, wv = __builtin_amdgcn_readfirstlane(tid >> 6), lr = lane & 15, lk = lane >> 4;
-    const int blocks = (p.rows + BM - 1) / BM, id = xcd_tile(blockIdx.x, blocks * p.heads), h = id / blocks;
-    const int m0 = (blocks - 1 - id % blocks) * BM, mw = m0 + wv * 16 * NQ;             // the longest rows first
+    // the longest rows first; with heads in eighths a head stays on one XCD, whose L2 then holds its keys and values
+    const int blocks = (p.rows + BM - 1) / BM, id = blockIdx.x, per = p.heads >> 3;
+    const bool split = (p.heads & 7) == 0;
+    const int h = split ? (id & 7) * per + (id >> 3) % per : id % p.heads, block = blocks - 1 - (split ? (id >> 3) / per : id / p.heads);
+    const int m0 = block * BM, mw = m0 + wv * 16 * NQ;
     const int last = p.pos + min(m0 + BM, p.rows) - 1, n_tiles = last / KT + 1, dk = p.d1 + p.d2;
     const T *kb = (const T *)p.k + (int64_t)h * p.k_head, *krb = (const T *)p.kr, *vb = (const T *)p.v + (int64_t)h * p.v_head;
 
@@ -119,23 +126,29 @@ __global__ __launch_bounds__(256) void latent_expanded_kernel(Expanded p) {
             qf[i][s] = c < dk ? *reinterpret_cast<const u32x4 *>(qr + c) : u32x4{0, 0, 0, 0};
         }
     }
+    // where a thread's pieces of a tile come from: key row of the tile, address of the column, bytes from key to key.  Columns beyond the head meet zeros of
+    // the query: any finite values will do.
     u32x4 rk[KL], rv[VL][4];
+    const char *k_at[KL], *v_at[VL];
+    uint32_t k_step[KL];
+    const uint32_t v_step = (uint32_t)p.v_row * sizeof(T);
+#pragma unroll
+    for (int i = 0; i < KL; i++) {
+        const int c = ((tid + 256 * i) % KC) * CH;
+        const bool rotated = c >= p.d1 && c < dk;
+        k_at[i] = (const char *)(rotated ? krb + (c - p.d1) : kb + (c < p.d1 ? c : 0));
+        k_step[i] = (uint32_t)(rotated ? p.kr_row : p.k_row) * sizeof(T);
+    }
+#pragma unroll
+    for (int i = 0; i < VL; i++) v_at[i] = (const char *)(vb + min((tid + 256 * i) / (KT / 4) * CH, p.v_pad - CH));
     auto fetch = [&](int j0) {
 #pragma unroll
-        for (int i = 0; i < KL; i++) {
-            const int idx = tid + 256 * i, c = (idx % KC) * CH;
-            const int64_t key = min(j0 + idx / KC, last);
-            rk[i] = u32x4{0, 0, 0, 0};
-            if (c < p.d1) rk[i] = *reinterpret_cast<const u32x4 *>(kb + key * p.k_row + c);
-            else if (c < dk) rk[i] = *reinterpret_cast<const u32x4 *>(krb + key * p.kr_row + c - p.d1);
-        }
+        for (int i = 0; i < KL; i++) rk[i] = *reinterpret_cast<const u32x4 *>(k_at[i] + (uint64_t)(uint32_t)min(j0 + (tid + 256 * i) / KC, last) * k_step[i]);
 #pragma unroll
-        for (int i = 0; i < VL; i++) {
-            const int idx = tid + 256 * i, a = idx % (KT / 4), c = idx / (KT / 4) * CH;
-            if (c < p.v_pad)
+        for (int i = 0; i < VL; i++)
 #pragma unroll
-                for (int j = 0; j < 4; j++) rv[i][j] = *reinterpret_cast<const u32x4 *>(vb + (int64_t)min(j0 + 4 * a + j, last) * p.v_row + c);
-        }
+            for (int j = 0; j < 4; j++)
+                rv[i][j] = *reinterpret_cast<const u32x4 *>(v_at[i] + (uint64_t)(uint32_t)min(j0 + 4 * ((tid + 256 * i) % (KT / 4)) + j, last) * v_step);
     };
     auto stage = [&]() {
 #pragma unroll
@@ -159,6 +172,9 @@ __global__ __launch_bounds__(256) void latent_expanded_kernel(Expanded p) {
 #pragma unroll
         for (int n = 0; n < NVF; n++) o[i][n] = f32x4{0.f, 0.f, 0.f, 0.f};
     }
+    // LDS slots of a lane: key chunks 4 k + lk of row lr by parity of k, value chunks 4 sp + lk of column lr by (n & 3) ^ 2 sp
+    const int ka[2] = {lr * KC + (lk ^ (lr & 7)), lr * KC + ((4 + lk) ^ (lr & 7))}, vx = lk ^ (lr & 7) ^ (lr >> 3);
+    const int va[4] = {lr * 8 + vx, lr * 8 + (vx ^ 2), lr * 8 + (vx ^ 4), lr * 8 + (vx ^ 6)};
     fetch(0);
     for (int it = 0; it < n_tiles; it++) {
         const int j0 = it * KT;
@@ -176,40 +192,41 @@ __global__ __launch_bounds__(256) void latent_expanded_kernel(Expanded p) {
         for (int k = 0; k < NKF; k++)
 #pragma unroll
             for (int t = 0; t < NT; t++) {
-                const int r = 16 * t + lr;
-                const u32x4 a = ks[r * KC + key_slot(r, 4 * k + lk)];
+                const u32x4 a = ks[ka[k & 1] + 8 * (k >> 1) + 16 * t * KC];
 #pragma unroll
                 for (int i = 0; i < NQ; i++) s[i][t] = mma<T>(a, qf[i][k], s[i][t]);
             }
-        const bool edge = j0 + KT - 1 > p.pos + mw;        // some key of the tile lies after some row
+        if (j0 + KT - 1 > p.pos + mw) {                    // some key of the tile lies after some row
+#pragma unroll
+            for (int i = 0; i < NQ; i++)
+#pragma unroll
+                for (int t = 0; t < NT; t++)
+#pragma unroll
+                    for (int e = 0; e < 4; e++) s[i][t][e] = j0 + 16 * t + 4 * lk + e > pq[i] ? -INFINITY : s[i][t][e];
+        }
 #pragma unroll
         for (int i = 0; i < NQ; i++) {
-            float mx = -INFINITY;
+            float mx = s[i][0][0];
 #pragma unroll
             for (int t = 0; t < NT; t++)
 #pragma unroll
-                for (int e = 0; e < 4; e++) {
-                    float z = s[i][t][e] * p.scale_log2;
-                    if (edge && j0 + 16 * t + 4 * lk + e > pq[i]) z = -INFINITY;
-                    s[i][t][e] = z;
-                    mx = fmaxf(mx, z);
-                }
-            const float m = fmaxf(m_run[i], group_max(mx));                            // finite from the first tile on: key 0 is visible to every row
-            const float al = __builtin_amdgcn_exp2f(m_run[i] - m);
-            float sum = 0.0f;
-#pragma unroll
-            for (int t = 0; t < NT; t++)
-#pragma unroll
-                for (int e = 0; e < 4; e++) {
-                    s[i][t][e] = __builtin_amdgcn_exp2f(s[i][t][e] - m);
-                    sum += s[i][t][e];
-                }
-            if (__any(m > m_run[i])) {
+                for (int e = 0; e < 4; e++) mx = fmaxf(mx, s[i][t][e]);
+            if (__any(mx > m_run[i] + LAG)) {              // in the first tile for every row: it sees key 0
+                const float m = fmaxf(m_run[i], group_max(mx)), al = __builtin_amdgcn_exp2f(m_run[i] - m);
 #pragma unroll
                 for (int n = 0; n < NVF; n++) o[i][n] *= al;
+                l_run[i] *= al;
+                m_run[i] = m;
             }
-            l_run[i] = l_run[i] * al + sum;
-            m_run[i] = m;
+            float sum[2] = {0.0f, 0.0f};
+#pragma unroll
+            for (int t = 0; t < NT; t++)
+#pragma unroll
+                for (int e = 0; e < 4; e++) {
+                    s[i][t][e] = __builtin_amdgcn_exp2f(s[i][t][e] - m_run[i]);
+                    sum[e & 1] += s[i][t][e];
+                }
+            l_run[i] += sum[0] + sum[1];
         }
 #pragma unroll
         for (int sp = 0; sp < 2; sp++) {
@@ -218,8 +235,7 @@ __global__ __launch_bounds__(256) void latent_expanded_kernel(Expanded p) {
             for (int i = 0; i < NQ; i++) w[i] = weight_chunk<T>(s[i], sp);
 #pragma unroll
             for (int n = 0; n < NVF; n++) {
-                const int r = 16 * n + lr;
-                const u32x4 a = vs[r * 8 + value_slot(r, 4 * sp + lk)];
+                const u32x4 a = vs[va[(n & 3) ^ (2 * sp)] + 128 * n];
 #pragma unroll
                 for (int i = 0; i < NQ; i++) o[i][n] = mma<T>(a, w[i], o[i][n]);
             }
@@ -255,7 +271,6 @@ struct Absorbed {
     const void *q, *cache;                                 // [row][head][ld], [key][ld]: rank_pad latent columns, then the rotated part
     int ld, rank_pad, heads, rows, pos, ctx;
     const int32_t *pos_dev;
-    float scale_log2;
     const float *gate;
     int64_t gate_row;
     float *out;                                            // [row][head][rank_pad], gated
@@ -353,13 +368,18 @@ __global__ __launch_bounds__(256, 1) void latent_absorbed_kernel(Absorbed p) {
                 s[t] = *reinterpret_cast<const f32x4 *>(ss + (16 * i + lr) * SS + 16 * t + 4 * lk);
 #pragma unroll
                 for (int e = 0; e < 4; e++) {
-                    s[t][e] = j0 + 16 * t + 4 * lk + e > pq[i] ? -INFINITY : s[t][e] * p.scale_log2;
+                    s[t][e] = j0 + 16 * t + 4 * lk + e > pq[i] ? -INFINITY : s[t][e];
                     mx = fmaxf(mx, s[t][e]);
                 }
             }
-            const float m = fmaxf(m_run[i], group_max(mx));
-            const float base = m > -INFINITY ? m : 0.0f;                               // a row before all keys of the split: weights of zero
-            const float al = __builtin_amdgcn_exp2f(m_run[i] - base);
+            if (__any(mx > m_run[i] + LAG)) {
+                const float m = fmaxf(m_run[i], group_max(mx)), al = m > -INFINITY ? __builtin_amdgcn_exp2f(m_run[i] - m) : 1.0f;
+#pragma unroll
+                for (int n = 0; n < NVW; n++) o[i][n] *= al;
+                l_run[i] *= al;
+                m_run[i] = m;
+            }
+            const float base = m_run[i] > -INFINITY ? m_run[i] : 0.0f;                 // a row before all keys of the split: weights of zero
 #pragma unroll
             for (int t = 0; t < NT; t++)
 #pragma unroll
@@ -367,12 +387,7 @@ __global__ __launch_bounds__(256, 1) void latent_absorbed_kernel(Absorbed p) {
                     s[t][e] = __builtin_amdgcn_exp2f(s[t][e] - base);
                     sum += s[t][e];
                 }
-            if (__any(m > m_run[i])) {
-#pragma unroll
-                for (int n = 0; n < NVW; n++) o[i][n] *= al;
-            }
-            l_run[i] = l_run[i] * al + sum;
-            m_run[i] = m;
+            l_run[i] += sum;
 #pragma unroll
             for (int sp = 0; sp < 2; sp++) w[i][sp] = weight_chunk<T>(s, sp);
         }
@@ -429,32 +444,56 @@ __device__ __forceinline__ void split_weights(const float *__restrict__ ml, int6
     for (int z = lane; z < nz; z += 64) wz[z] /= l;
 }
 
+// The records of one query, merged: 256 threads as groups of n4 (float4 columns of the latent), group g on splits g, g + groups, ...  The first splits are on
+// their way before the weights are known.  Leaves the sum in o (LDS, n4 float4; acc: groups * n4 float4).
 constexpr int MAX_SPLITS = 256;
-__device__ __forceinline__ void merge_latent(const float *__restrict__ part, int64_t stride, int nz, const float *wz, float f, float *dst, int n4, int tid, int threads) {
-    for (int c = tid; c < n4; c += threads) {
-        f32x4 a = {0.f, 0.f, 0.f, 0.f};
-#pragma unroll 8
-        for (int z = 0; z < nz; z++) {
-            const float w = wz[z];
-            const f32x4 v = *reinterpret_cast<const f32x4 *>(part + z * stride + 4 * c);
-            a += w > 0.0f ? w * v : f32x4{0.f, 0.f, 0.f, 0.f};                         // an empty split has not written its record
+__device__ __forceinline__ void merge_latent(const float *__restrict__ part, int64_t stride, const float *__restrict__ ml, int64_t ml_stride, int nz, int n4, f32x4 *acc,
+                                             f32x4 *o, float *wz) {
+    const int tid = threadIdx.x, groups = 256 / n4, g = tid / n4, c = tid - g * n4;
+    constexpr int U = 16;
+    f32x4 v[U], a = {0.f, 0.f, 0.f, 0.f};
+    const float *src = part + 4 * c;
+#pragma unroll
+    for (int i = 0; i < U; i++) v[i] = *reinterpret_cast<const f32x4 *>(src + min(g + i * groups, nz - 1) * stride);
+    if (tid < 64) split_weights(ml, ml_stride, nz, wz, tid);
+    __syncthreads();
+    if (g < groups)
+        for (int z0 = g; z0 < nz; z0 += U * groups) {
+            if (z0 != g) {
+#pragma unroll
+                for (int i = 0; i < U; i++) v[i] = *reinterpret_cast<const f32x4 *>(src + min(z0 + i * groups, nz - 1) * stride);
+            }
+#pragma unroll
+            for (int i = 0; i < U; i++) {
+                const int z = z0 + i * groups;
+                const float w = z < nz ? wz[z] : 0.0f;
+#pragma unroll
+                for (int e = 0; e < 4; e++) a[e] = w > 0.0f ? fmaf(w, v[i][e], a[e]) : a[e];       // an empty split has not written its record
+            }
         }
-        *reinterpret_cast<f32x4 *>(dst + 4 * c) = a * f;
+    if (g < groups) acc[tid] = a;
+    __syncthreads();
+    if (tid < n4) {
+        for (int i = 1; i < groups; i++) a += acc[tid + i * n4];
+        o[tid] = a;
     }
+    __syncthreads();
 }
 
 // one workgroup per query: the records of its splits into the gated latent
-__global__ __launch_bounds__(128) void latent_combine_kernel(const float *__restrict__ part, int nz, int M, int heads, int rank_pad, const float *__restrict__ gate,
+__global__ __launch_bounds__(256) void latent_combine_kernel(const float *__restrict__ part, int nz, int M, int heads, int rank_pad, const float *__restrict__ gate,
                                                              int64_t gate_row, float *__restrict__ out) {
     __shared__ float wz[MAX_SPLITS];
+    __shared__ f32x4 acc[256], o[CQ_LATENT_MAX_RANK / 4];
     const int m = blockIdx.x;
-    if (threadIdx.x < 64) split_weights(part + (int64_t)nz * M * rank_pad + 2 * m, 2 * (int64_t)M, nz, wz, threadIdx.x);
-    __syncthreads();
     const float f = mix_sigmoid(gate[(m / heads) * gate_row + m % heads]);
-    merge_latent(part + (int64_t)m * rank_pad, (int64_t)M * rank_pad, nz, wz, f, out + (int64_t)m * rank_pad, rank_pad >> 2, threadIdx.x, 128);
+    merge_latent(part + (int64_t)m * rank_pad, (int64_t)M * rank_pad, part + (int64_t)nz * M * rank_pad + 2 * m, 2 * (int64_t)M, nz, rank_pad >> 2, acc, o, wz);
+    if ((int)threadIdx.x < rank_pad >> 2) *reinterpret_cast<f32x4 *>(out + (int64_t)m * rank_pad + 4 * threadIdx.x) = o[threadIdx.x] * f;
 }
 
 // ---- projection rows into queries and cache rows -----------------------------------------------------------------------------------------------
+__device__ __forceinline__ float query_factor(const cq_latent &g) { return g.scale * 1.44269504088896341f; }
+
 template <typename T> __device__ __forceinline__ float turned(const cq_latent &g, const float *src, int64_t p, int d) {
     const int half = g.rot_dim >> 1;
     const float c = g.cos_dev[p * half + (d >> 1)], s = g.sin_dev[p * half + (d >> 1)], v = src[d], w = src[d ^ 1];
@@ -485,17 +524,18 @@ __global__ __launch_bounds__(256) void latent_pack_kernel(cq_latent g, const flo
     const int64_t r = blockIdx.x, p = pos + r;
     const float *src = row + r * row_stride;
     const int lane = threadIdx.x & 63, dq = g.dim + g.rot_dim;
+    const float fq = query_factor(g);
     for (int h = threadIdx.x >> 6; h < g.heads; h += 4) {
         const float *s = src + (int64_t)h * dq;
         T *d = q + (r * g.heads + h) * q_head;
         float *f = plain ? plain + (r * g.heads + h) * plain_head : nullptr;
         for (int i = lane; i < g.dim; i += 64) {
-            if (f) f[i] = s[i];
-            else d[i] = (T)s[i];
+            if (f) f[i] = fq * s[i];
+            else d[i] = (T)(fq * s[i]);
         }
         if (!f)
             for (int i = g.dim + lane; i < rot_off; i += 64) d[i] = (T)0.0f;
-        for (int i = lane; i < q_head - rot_off; i += 64) d[rot_off + i] = i < g.rot_dim ? (T)turned<T>(g, s + g.dim, p, i) : (T)0.0f;
+        for (int i = lane; i < q_head - rot_off; i += 64) d[rot_off + i] = i < g.rot_dim ? (T)(fq * turned<T>(g, s + g.dim, p, i)) : (T)0.0f;
     }
     if (kv_off >= 0) append_row<T, 256>(g, src + kv_off, cache + p * (g.rank_pad + g.rot_pad), p, red);
 }
@@ -536,39 +576,32 @@ __global__ __launch_bounds__(256) void latent_absorb_step_kernel(cq_latent g, co
 #pragma unroll
     for (int i = 0; i < 4; i++) {
         const float v = row16_sum(acc[i][0] + acc[i][1]);
-        if (sub == 0 && j0 + 4 * i < g.rank) d[j0 + 4 * i] = (T)v;
+        if (sub == 0 && j0 + 4 * i < g.rank) d[j0 + 4 * i] = (T)(query_factor(g) * v);
     }
     if (piece == 0)
-        for (int i = threadIdx.x; i < g.rot_pad; i += 256) d[g.rank_pad + i] = i < g.rot_dim ? (T)turned<T>(g, s + g.dim, p, i) : (T)0.0f;
+        for (int i = threadIdx.x; i < g.rot_pad; i += 256) d[g.rank_pad + i] = i < g.rot_dim ? (T)(query_factor(g) * turned<T>(g, s + g.dim, p, i)) : (T)0.0f;
 }
 
-// One token: workgroup (head, 16 value rows) merges the records of the head's splits and takes W_uv to the gated latent.
+// One token: workgroup (head, 16 value rows) merges the records of the head's splits and takes W_uv to the latent.
 __global__ __launch_bounds__(256) void latent_merge_step_kernel(const float *__restrict__ part, int nz, int heads, int rank_pad, const uint16_t *__restrict__ w_uv, int ldw,
                                                                 const float *__restrict__ gate, float *__restrict__ out, int vdim) {
-    extern __shared__ __attribute__((aligned(16))) float o[];              // rank_pad floats
     __shared__ float wz[MAX_SPLITS];
+    __shared__ f32x4 acc[256], o[CQ_LATENT_MAX_RANK / 4];
     const int lane = threadIdx.x & 63, wv = threadIdx.x >> 6, h = blockIdx.x, e0 = blockIdx.y * 16 + 4 * wv;
-    const uint16_t *w[4];
     u32x4 wr[4];
 #pragma unroll
-    for (int i = 0; i < 4; i++) {
-        w[i] = w_uv + ((int64_t)h * vdim + min(e0 + i, vdim - 1)) * ldw;
-        wr[i] = *reinterpret_cast<const u32x4 *>(w[i] + min(8 * lane, ldw - 8));
-    }
+    for (int i = 0; i < 4; i++) wr[i] = *reinterpret_cast<const u32x4 *>(w_uv + ((int64_t)h * vdim + min(e0 + i, vdim - 1)) * ldw + min(8 * lane, ldw - 8));
     const float g = gate[h];
-    if (wv == 0) split_weights(part + (int64_t)nz * heads * rank_pad + 2 * h, 2 * (int64_t)heads, nz, wz, lane);
-    __syncthreads();
-    merge_latent(part + (int64_t)h * rank_pad, (int64_t)heads * rank_pad, nz, wz, 1.0f, o, rank_pad >> 2, threadIdx.x, 256);
-    __syncthreads();
-    float acc[4][2] = {};
-    for (int c = 8 * lane; c < rank_pad; c += 512) {
-        const f32x4 a = *reinterpret_cast<const f32x4 *>(o + c), b = *reinterpret_cast<const f32x4 *>(o + c + 4);
+    merge_latent(part + (int64_t)h * rank_pad, (int64_t)heads * rank_pad, part + (int64_t)nz * heads * rank_pad + 2 * h, 2 * (int64_t)heads, nz, rank_pad >> 2, acc, o, wz);
+    float s[4][2] = {};
+    if (8 * lane < rank_pad) {                             // rank_pad <= 512: one piece per lane
+        const f32x4 a = o[2 * lane], b = o[2 * lane + 1];
 #pragma unroll
-        for (int i = 0; i < 4; i++) dot8(c < 512 ? wr[i] : *reinterpret_cast<const u32x4 *>(w[i] + c), a, b, acc[i]);
+        for (int i = 0; i < 4; i++) dot8(wr[i], a, b, s[i]);
     }
 #pragma unroll
     for (int i = 0; i < 4; i++) {
-        const float v = wave_sum(acc[i][0] + acc[i][1]);
+        const float v = wave_sum(s[i][0] + s[i][1]);
         if (lane == 0 && e0 + i < vdim) out[h * vdim + e0 + i] = v * mix_sigmoid(g);
     }
 }
@@ -595,7 +628,7 @@ int absorbed_splits(int bf16, int64_t m, int64_t keys) {
 
 template <typename T, int DK, int DV, int NQ> int absorbed_launch(const Absorbed &a, int nz, hipStream_t s) {
     constexpr size_t lds = (size_t)Chunk<T>::KEYS * DK * sizeof(T) + (size_t)DV * 128 + (size_t)16 * NQ * (Chunk<T>::KEYS + 4) * sizeof(float);
-    static_assert(lds <= 160 * 1024, "LDS");
+    static_assert(lds <= (size_t)160 * 1024, "LDS");
     if (lds > 64 * 1024) {
         const int e = (int)hipFuncSetAttribute(reinterpret_cast<const void *>(latent_absorbed_kernel<T, DK, DV, NQ>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
         if (e) return e;
@@ -679,7 +712,6 @@ int cq_mix_latent_expanded(const cq_latent *g, const void *q_dev, int64_t dim_pa
     a.pos = (int)pos;
     a.rows = (int)rows;
     a.heads = g->heads;
-    a.scale_log2 = g->scale * 1.44269504088896341f;
     hipStream_t s = (hipStream_t)stream;
     const int dk = a.q_head;
     // 32 query rows per wave where that leaves two workgroups per CU
@@ -724,7 +756,6 @@ int cq_mix_latent_absorbed(const cq_latent *g, const void *q_dev, const void *ca
     a.pos = (int)pos;
     a.ctx = g->ctx;
     a.pos_dev = nullptr;
-    a.scale_log2 = g->scale * 1.44269504088896341f;
     a.gate = gate_dev;
     a.gate_row = gate_row;
     a.out = out_dev;
@@ -732,7 +763,7 @@ int cq_mix_latent_absorbed(const cq_latent *g, const void *q_dev, const void *ca
     hipStream_t s = (hipStream_t)stream;
     const int r = g->bf16 ? absorbed_dispatch<__bf16>(a, nz, s) : absorbed_dispatch<float>(a, nz, s);
     if (r || nz == 1) return r;
-    hipLaunchKernelGGL(latent_combine_kernel, dim3((unsigned)m), dim3(128), 0, s, (const float *)workspace_dev, nz, (int)m, g->heads, g->rank_pad, gate_dev, gate_row, out_dev);
+    hipLaunchKernelGGL(latent_combine_kernel, dim3((unsigned)m), dim3(256), 0, s, (const float *)workspace_dev, nz, (int)m, g->heads, g->rank_pad, gate_dev, gate_row, out_dev);
     return (int)hipGetLastError();
 }
 
@@ -764,11 +795,10 @@ int cq_mix_latent_step(const cq_latent *g, const float *row_dev, int64_t kv_off,
     a.pos = (int)pos;
     a.ctx = g->ctx;
     a.pos_dev = pos_dev;
-    a.scale_log2 = g->scale * 1.44269504088896341f;
     a.part = (float *)workspace_dev;
     const int r = g->bf16 ? absorbed_dispatch<__bf16>(a, nz, s) : absorbed_dispatch<float>(a, nz, s);
     if (r) return r;
-    hipLaunchKernelGGL(latent_merge_step_kernel, dim3((unsigned)g->heads, (unsigned)((g->vdim + 15) / 16)), dim3(256), g->rank_pad * sizeof(float), s,
+    hipLaunchKernelGGL(latent_merge_step_kernel, dim3((unsigned)g->heads, (unsigned)((g->vdim + 15) / 16)), dim3(256), 0, s,
                        (const float *)workspace_dev, nz, g->heads, g->rank_pad, (const uint16_t *)w_uv_dev, (int)ld_uv, row_dev + gate_off, out_dev, g->vdim);
     return (int)hipGetLastError();
 }

@@ -517,7 +517,8 @@ class LatentAttention(Mixer):
         gate = row + 4 * self.g_off
         self.w_in.rows(h, ldh, row, ldp, rows, sp)
         if self.expands(rows):
-            head, ldkv, keys = self.dim_pad + self.rot_pad, self.expand.n, pos + rows
+            head, keys = self.dim_pad + self.rot_pad, pos + rows
+            ldkv = self.expand.n + (0 if self.expand.n // 128 % 2 else 128)     # rows an odd number of 256 bytes apart fall on all memory channels
             q, kv = rt.typed("latent_q", rows * H * head), rt.typed("latent_kv", keys * ldkv)
             check("cq_mix_latent_pack", L.cq_mix_latent_pack(self.shape, row, ldp, self.kv_off, kept.data_ptr(), None, 0, q, head, self.dim_pad, pos, rows, sp))
             self.expand.rows(kept.data_ptr(), self.ld, kv, ldkv, keys, sp, x_bf16=bf, dst_bf16=bf)

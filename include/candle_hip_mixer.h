@@ -181,7 +181,7 @@ typedef struct cq_latent {
 #define CQ_LATENT_MAX_VALUE 256
 /* Projection rows into packed queries and, with kv_off >= 0, the cache rows of positions pos ...  Query (r, h) is q[(r * heads + h) * q_head ..] of type T:
  * the rotated part at rot_off, zero up to q_head; the unrotated part in front of it (zero up to rot_off) or, with plain_dev, as f32 at
- * plain[(r * heads + h) * plain_head ..] instead. */
+ * plain[(r * heads + h) * plain_head ..] instead.  Queries come out multiplied by scale * log2(e), which is how the calls below take them. */
 int cq_mix_latent_pack(const cq_latent *g, const float *row_dev, int64_t row_stride, int64_t kv_off, void *cache_dev, float *plain_dev, int64_t plain_head, void *q_dev,
                        int64_t q_head, int64_t rot_off, int64_t pos, int64_t rows, void *stream);
 /* Attention of rows pos .. pos + rows over keys and values of all heads: kv [pos + rows][kv_row] of type T, head h's unrotated key at h * dim_pad, its value
