@@ -277,10 +277,13 @@ struct Absorbed {
     float *part;                                           // records instead: [split][query][rank_pad] unnormalized, then [split][query] of (maximum, sum)
 };
 
-template <typename T, int DK, int DV, int NQ>
+// A key row in LDS: DV latent columns, then DR rotated ones, zero where the cache row has none.
+template <typename T, int DV, int DR, int NQ>
 __global__ __launch_bounds__(256, 1) void latent_absorbed_kernel(Absorbed p) {
-    constexpr int CH = Chunk<T>::N, KT = Chunk<T>::KEYS, NT = KT / 16, NKF = DK / Chunk<T>::STEP, KC = DK / CH, NVW = DV / 64, BM = 16 * NQ;
-    constexpr int TASKS = (KT / 4) * KC, TL = (TASKS + 255) / 256, SS = KT + 4;
+    constexpr int CH = Chunk<T>::N, KT = Chunk<T>::KEYS, NT = KT / 16, NKF = (DV + DR) / Chunk<T>::STEP, KC = (DV + DR) / CH, NVW = DV / 64, BM = 16 * NQ, SS = KT + 4;
+    // a thread's pieces: four keys x one chunk, latent ones (AL groups of keys apart) and rotated ones
+    constexpr int NC = DV / CH, AL = 256 / NC, TL = KT / 4 / AL, NR = DR / CH, RT = (KT / 4) * NR, RL = (RT + 255) / 256;
+    static_assert(256 % NC == 0 && (KT / 4) % AL == 0, "pieces");
     extern __shared__ __attribute__((aligned(16))) u32x4 lds[];
     u32x4 *ks = lds, *vs = ks + KT * KC;
     float *ss = reinterpret_cast<float *>(vs + DV * 8);    // scores [query][key]
@@ -289,43 +292,60 @@ __global__ __launch_bounds__(256, 1) void latent_absorbed_kernel(Absorbed p) {
     const int pos = p.pos + (p.pos_dev ? p.pos_dev[0] : 0);
     if (pos + p.rows > p.ctx) return;
     const int last = pos + (min(m0 + BM, M) - 1) / p.heads, n_tiles = last / KT + 1;
-    const int lo = (int)((int64_t)n_tiles * z / nz), hi = (int)((int64_t)n_tiles * (z + 1) / nz);
+    const int lo = (int)((uint32_t)n_tiles * z / (uint32_t)nz), hi = (int)((uint32_t)n_tiles * (z + 1) / (uint32_t)nz);
     const T *cache = (const T *)p.cache;
 
-    u32x4 qf[NQ][NKF];
-    int pq[NQ];
-#pragma unroll
-    for (int i = 0; i < NQ; i++) {
-        const int m = min(m0 + 16 * i + lr, M - 1);
-        pq[i] = pos + m / p.heads;
-#pragma unroll
-        for (int s = 0; s < NKF; s++) {
-            const int c = (4 * s + lk) * CH;
-            qf[i][s] = c < p.ld ? *reinterpret_cast<const u32x4 *>((const T *)p.q + (int64_t)m * p.ld + c) : u32x4{0, 0, 0, 0};
-        }
-    }
-    u32x4 rg[TL][4];
+    // cache pieces first, then the queries (where the cache row has no column, the query's value does not matter)
+    u32x4 rg[TL][4], rr[RL][4];
+    const int ca = (tid % NC) * CH, a0 = tid / NC;
     auto fetch = [&](int j0) {
 #pragma unroll
-        for (int i = 0; i < TL; i++) {
-            const int idx = tid + 256 * i, a = idx / KC, c = (idx % KC) * CH;
+        for (int i = 0; i < TL; i++)
 #pragma unroll
             for (int j = 0; j < 4; j++) {
                 rg[i][j] = u32x4{0, 0, 0, 0};
-                if (c < p.ld) rg[i][j] = *reinterpret_cast<const u32x4 *>(cache + (int64_t)min(j0 + 4 * a + j, last) * p.ld + c);
+                if (ca < p.rank_pad) rg[i][j] = *reinterpret_cast<const u32x4 *>(cache + (int64_t)min(j0 + 4 * (a0 + AL * i) + j, last) * p.ld + ca);
+            }
+#pragma unroll
+        for (int i = 0; i < RL; i++) {
+            const int idx = tid + 256 * i, a = idx / NR, c = (idx % NR) * CH;
+#pragma unroll
+            for (int j = 0; j < 4; j++) {
+                rr[i][j] = u32x4{0, 0, 0, 0};
+                if (c < p.ld - p.rank_pad && idx < RT) rr[i][j] = *reinterpret_cast<const u32x4 *>(cache + (int64_t)min(j0 + 4 * a + j, last) * p.ld + p.rank_pad + c);
             }
         }
     };
     auto stage = [&]() {
 #pragma unroll
         for (int i = 0; i < TL; i++) {
-            const int idx = tid + 256 * i, a = idx / KC, c = idx % KC;
-            if (TASKS % 256 && idx >= TASKS) break;
+            const int a = a0 + AL * i, c = tid % NC;
 #pragma unroll
             for (int j = 0; j < 4; j++) ks[(4 * a + j) * KC + key_slot(4 * a + j, c)] = rg[i][j];
-            if (c * CH < p.rank_pad) store_values<T>(vs, a, c, rg[i]);
+            store_values<T>(vs, a, c, rg[i]);
+        }
+#pragma unroll
+        for (int i = 0; i < RL; i++) {
+            const int idx = tid + 256 * i, a = idx / NR, c = NC + idx % NR;
+            if (idx < RT)
+#pragma unroll
+                for (int j = 0; j < 4; j++) ks[(4 * a + j) * KC + key_slot(4 * a + j, c)] = rr[i][j];
         }
     };
+    if (lo < hi) fetch(lo * KT);
+    u32x4 qf[NQ][NKF];
+    int pq[NQ];
+#pragma unroll
+    for (int i = 0; i < NQ; i++) {
+        const int m = min(m0 + 16 * i + lr, M - 1);
+        pq[i] = pos + m / p.heads;
+        const T *qr = (const T *)p.q + (int64_t)m * p.ld;
+#pragma unroll
+        for (int s = 0; s < NKF; s++) {
+            const int c = (4 * s + lk) * CH;               // a step lies in one of the two parts
+            qf[i][s] = *reinterpret_cast<const u32x4 *>(qr + min(4 * s < NC ? min(c, p.rank_pad - CH) : p.rank_pad + c - DV, p.ld - CH));
+        }
+    }
 
     f32x4 o[NQ][NVW];
     float m_run[NQ], l_run[NQ];
@@ -336,7 +356,6 @@ __global__ __launch_bounds__(256, 1) void latent_absorbed_kernel(Absorbed p) {
 #pragma unroll
         for (int n = 0; n < NVW; n++) o[i][n] = f32x4{0.f, 0.f, 0.f, 0.f};
     }
-    if (lo < hi) fetch(lo * KT);
     for (int it = lo; it < hi; it++) {
         const int j0 = it * KT;
         __syncthreads();
@@ -612,41 +631,49 @@ int check_latent(const cq_latent *g) {
         g->rot_pad < g->rot_dim || g->rot_pad % 8)
         return CQ_ERR_SHAPE;
     if (g->rot_dim && (!g->cos_dev || !g->sin_dev)) return CQ_ERR_NULL;
-    if (g->rank_pad > CQ_LATENT_MAX_RANK || g->rank_pad + g->rot_pad > CQ_LATENT_MAX_ROW || g->heads > 4096 || g->dim > 4096 || g->vdim > 4096 || g->ctx > (1 << 24))
+    if (g->rot_pad > 192 || g->rank_pad > (g->rot_pad > 64 ? 256 : CQ_LATENT_MAX_RANK) || g->heads > 4096 || g->dim > 4096 || g->vdim > 4096 || g->ctx > (1 << 24))
         return CQ_ERR_RANGE;
     return CQ_OK;
 }
 
-// queries per workgroup / 16, and splits of the keys
-int absorbed_nq(int bf16, int64_t m) { return bf16 && m > 16 ? 2 : 1; }
-int absorbed_splits(int bf16, int64_t m, int64_t keys) {
-    const int64_t blocks = (m + 16 * absorbed_nq(bf16, m) - 1) / (16 * absorbed_nq(bf16, m)), kt = bf16 ? 64 : 32, tiles = (keys + kt - 1) / kt;
+// Queries per workgroup (in 16s) and splits of the keys: 16 while all (block of queries, tile of keys) pairs can run side by side.
+struct AbsorbedPlan {
+    int nq, splits;
+};
+AbsorbedPlan absorbed_plan(int bf16, int64_t m, int64_t keys) {
+    const int64_t kt = bf16 ? 64 : 32, tiles = (keys + kt - 1) / kt, fine = (m + 15) / 16;
+    AbsorbedPlan p;
+    p.nq = bf16 && fine > 1 && fine * tiles > 256 ? 2 : 1;
+    const int64_t blocks = (m + 16 * p.nq - 1) / (16 * p.nq);
     int64_t n = blocks >= 256 ? 1 : 256 / blocks;
     n = n < tiles ? n : tiles;
-    return (int)(n < MAX_SPLITS ? n : MAX_SPLITS);
+    p.splits = (int)(n < MAX_SPLITS ? n : MAX_SPLITS);
+    return p;
 }
 
-template <typename T, int DK, int DV, int NQ> int absorbed_launch(const Absorbed &a, int nz, hipStream_t s) {
-    constexpr size_t lds = (size_t)Chunk<T>::KEYS * DK * sizeof(T) + (size_t)DV * 128 + (size_t)16 * NQ * (Chunk<T>::KEYS + 4) * sizeof(float);
+template <typename T, int DV, int DR, int NQ> int absorbed_launch(const Absorbed &a, int nz, hipStream_t s) {
+    constexpr size_t lds = (size_t)Chunk<T>::KEYS * (DV + DR) * sizeof(T) + (size_t)DV * 128 + (size_t)16 * NQ * (Chunk<T>::KEYS + 4) * sizeof(float);
     static_assert(lds <= (size_t)160 * 1024, "LDS");
     if (lds > 64 * 1024) {
-        const int e = (int)hipFuncSetAttribute(reinterpret_cast<const void *>(latent_absorbed_kernel<T, DK, DV, NQ>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+        const int e = (int)hipFuncSetAttribute(reinterpret_cast<const void *>(latent_absorbed_kernel<T, DV, DR, NQ>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
         if (e) return e;
     }
-    hipLaunchKernelGGL((latent_absorbed_kernel<T, DK, DV, NQ>), dim3((unsigned)((a.rows * a.heads + 16 * NQ - 1) / (16 * NQ)), 1, nz), dim3(256), lds, s, a);
+    hipLaunchKernelGGL((latent_absorbed_kernel<T, DV, DR, NQ>), dim3((unsigned)((a.rows * a.heads + 16 * NQ - 1) / (16 * NQ)), 1, nz), dim3(256), lds, s, a);
     return (int)hipGetLastError();
 }
-template <typename T> int absorbed_dispatch(const Absorbed &a, int nz, hipStream_t s) {
-#define CQ_AB(DK_, DV_)                                                                                                                              \
+template <typename T> int absorbed_dispatch(const Absorbed &a, const AbsorbedPlan &plan, hipStream_t s) {
+    const int nz = plan.splits;
+#define CQ_AB(DV_, DR_)                                                                                                                              \
     do {                                                                                                                                             \
         if constexpr (sizeof(T) == 2) {                                                                                                              \
-            if (absorbed_nq(1, (int64_t)a.rows * a.heads) == 2) return absorbed_launch<T, DK_, DV_, 2>(a, nz, s);                                      \
+            if (plan.nq == 2) return absorbed_launch<T, DV_, DR_, 2>(a, nz, s);                                      \
         }                                                                                                                                            \
-        return absorbed_launch<T, DK_, DV_, 1>(a, nz, s);                                                                                            \
+        return absorbed_launch<T, DV_, DR_, 1>(a, nz, s);                                                                                            \
     } while (0)
-    if (a.ld <= 192 && a.rank_pad <= 128) CQ_AB(192, 128);
-    if (a.ld <= 320 && a.rank_pad <= 256) CQ_AB(320, 256);
-    CQ_AB(576, 512);
+    if (a.ld - a.rank_pad > 64) CQ_AB(256, 192);
+    if (a.rank_pad <= 128) CQ_AB(128, 64);
+    if (a.rank_pad <= 256) CQ_AB(256, 64);
+    CQ_AB(512, 64);
 #undef CQ_AB
 }
 
@@ -730,7 +757,7 @@ int cq_mix_latent_expanded(const cq_latent *g, const void *q_dev, int64_t dim_pa
 int64_t cq_mix_latent_absorbed_workspace_bytes(const cq_latent *g, int64_t rows, int64_t pos, int step) {
     if (check_latent(g) || rows <= 0) return -1;
     const int64_t m = rows * g->heads;
-    const int nz = absorbed_splits(g->bf16, m, step ? g->ctx : pos + rows);
+    const int nz = absorbed_plan(g->bf16, m, step ? g->ctx : pos + rows).splits;
     return nz > 1 || step ? nz * m * (g->rank_pad + 2) * 4 : 0;
 }
 
@@ -744,7 +771,8 @@ int cq_mix_latent_absorbed(const cq_latent *g, const void *q_dev, const void *ca
     if (misaligned(q_dev, 16) || misaligned(cache_dev, 16) || misaligned(out_dev, 16) || misaligned(workspace_dev, 16)) return CQ_ERR_ALIGN;
     if (pos + rows > g->ctx || rows * g->heads > (1 << 24)) return CQ_ERR_RANGE;
     const int64_t m = rows * g->heads, need = cq_mix_latent_absorbed_workspace_bytes(g, rows, pos, 0);
-    const int nz = absorbed_splits(g->bf16, m, pos + rows);
+    const AbsorbedPlan plan = absorbed_plan(g->bf16, m, pos + rows);
+    const int nz = plan.splits;
     if (need && (!workspace_dev || workspace_bytes < need)) return CQ_ERR_WORKSPACE;
     Absorbed a;
     a.q = q_dev;
@@ -761,7 +789,7 @@ int cq_mix_latent_absorbed(const cq_latent *g, const void *q_dev, const void *ca
     a.out = out_dev;
     a.part = nz > 1 ? (float *)workspace_dev : nullptr;
     hipStream_t s = (hipStream_t)stream;
-    const int r = g->bf16 ? absorbed_dispatch<__bf16>(a, nz, s) : absorbed_dispatch<float>(a, nz, s);
+    const int r = g->bf16 ? absorbed_dispatch<__bf16>(a, plan, s) : absorbed_dispatch<float>(a, plan, s);
     if (r || nz == 1) return r;
     hipLaunchKernelGGL(latent_combine_kernel, dim3((unsigned)m), dim3(256), 0, s, (const float *)workspace_dev, nz, (int)m, g->heads, g->rank_pad, gate_dev, gate_row, out_dev);
     return (int)hipGetLastError();
@@ -776,7 +804,8 @@ int cq_mix_latent_step(const cq_latent *g, const float *row_dev, int64_t kv_off,
     if (misaligned(cache_dev, 16) || misaligned(w_ukt_dev, 16) || misaligned(w_uv_dev, 16) || misaligned(q_dev, 16) || misaligned(workspace_dev, 16)) return CQ_ERR_ALIGN;
     if (pos >= g->ctx) return CQ_ERR_RANGE;
     if (workspace_bytes < cq_mix_latent_absorbed_workspace_bytes(g, 1, 0, 1)) return CQ_ERR_WORKSPACE;
-    const int nz = absorbed_splits(g->bf16, g->heads, g->ctx);
+    const AbsorbedPlan plan = absorbed_plan(g->bf16, g->heads, g->ctx);
+    const int nz = plan.splits;
     hipStream_t s = (hipStream_t)stream;
     const dim3 grid((unsigned)(g->heads * ((g->rank + 63) / 64) + 1));
     if (g->bf16)
@@ -796,7 +825,7 @@ int cq_mix_latent_step(const cq_latent *g, const float *row_dev, int64_t kv_off,
     a.ctx = g->ctx;
     a.pos_dev = pos_dev;
     a.part = (float *)workspace_dev;
-    const int r = g->bf16 ? absorbed_dispatch<__bf16>(a, nz, s) : absorbed_dispatch<float>(a, nz, s);
+    const int r = g->bf16 ? absorbed_dispatch<__bf16>(a, plan, s) : absorbed_dispatch<float>(a, plan, s);
     if (r) return r;
     hipLaunchKernelGGL(latent_merge_step_kernel, dim3((unsigned)g->heads, (unsigned)((g->vdim + 15) / 16)), dim3(256), 0, s,
                        (const float *)workspace_dev, nz, g->heads, g->rank_pad, (const uint16_t *)w_uv_dev, (int)ld_uv, row_dev + gate_off, out_dev, g->vdim);

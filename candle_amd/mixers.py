@@ -459,7 +459,7 @@ class LatentAttention(Mixer):
     Many rows: keys and values of all heads are computed from the cache rows, then attended to head by head.  Few rows and single tokens: the key matrix is
     applied to the query and the value matrix to the attended latent, so that the heads attend to the cache rows themselves."""
 
-    MAX_RANK, MAX_ROW, MAX_HEAD, MAX_VALUE = 512, 576, 320, 256      # CQ_LATENT_MAX_*
+    MAX_RANK, MAX_HEAD, MAX_VALUE = 512, 320, 256    # CQ_LATENT_MAX_*; rotated parts of more than 64 (up to 192) with latents up to 256
 
     def __init__(self, rt: Runtime, cfg: dict, get: Callable[[str], torch.Tensor], eps: float):
         self.rt, self.eps = rt, eps
@@ -468,8 +468,8 @@ class LatentAttention(Mixer):
         H, r = self.heads, self.rank
         self.rank_pad, self.rot_pad, self.dim_pad, self.v_pad = pad_to(r, 64), pad_to(self.rot_dim, 8), pad_to(self.dim, 8), pad_to(self.vdim, 8)
         self.ld = self.rank_pad + self.rot_pad
-        if self.rank_pad > self.MAX_RANK or self.ld > self.MAX_ROW:
-            raise ValueError(f"latents of {r} + {self.rot_dim} are longer than {self.MAX_RANK} + {self.MAX_ROW - self.MAX_RANK}")
+        if self.rot_pad > 192 or self.rank_pad > (256 if self.rot_pad > 64 else self.MAX_RANK):
+            raise ValueError(f"latents of {r} + {self.rot_dim} values: at most {self.MAX_RANK} + 64 or 256 + 192")
         rot = Rotation(rt, cfg.get("rot"))
         if rot.dims != self.rot_dim:
             raise ValueError("the rotated part of a head is rotated as a whole")

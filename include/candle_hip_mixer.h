@@ -175,8 +175,7 @@ typedef struct cq_latent {
     float scale, eps;
     int32_t reserved;
 } cq_latent;
-#define CQ_LATENT_MAX_RANK 512       /* rank_pad */
-#define CQ_LATENT_MAX_ROW 576        /* rank_pad + rot_pad */
+#define CQ_LATENT_MAX_RANK 512       /* rank_pad; 256 with rot_pad > 64, which is at most 192 */
 #define CQ_LATENT_MAX_HEAD 320       /* dim_pad + rot_pad of the expanded form */
 #define CQ_LATENT_MAX_VALUE 256
 /* Projection rows into packed queries and, with kv_off >= 0, the cache rows of positions pos ...  Query (r, h) is q[(r * heads + h) * q_head ..] of type T:
