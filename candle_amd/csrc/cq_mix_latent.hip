@@ -34,11 +34,12 @@ constexpr float LAG = 8.0f;
 __device__ __forceinline__ int key_slot(int r, int c) { return c ^ (r & 7); }
 __device__ __forceinline__ int value_slot(int r, int c) { return c ^ ((r ^ (r >> 3)) & 7); }
 
+// In columns of every other block of 64 the two halves of a bf16 chunk change places, so that the lanes of a store fall on all banks; so do the weights for them.
 // Values of keys 4 a .. 4 a + 3, columns of chunk cg, transposed into LDS: [column][key].  The keys of a row are ordered so that the chunk that a lane reads
 // holds the keys whose scores it has: for bf16 4 lk .. 4 lk + 3 of two neighbouring tiles of 16.
 template <typename T> __device__ __forceinline__ void store_values(u32x4 *vs, int a, int cg, const u32x4 (&v)[4]);
 template <> __device__ __forceinline__ void store_values<__bf16>(u32x4 *vs, int a, int cg, const u32x4 (&v)[4]) {
-    const int chunk = (a >> 3) * 4 + (a & 3), half = (a >> 2) & 1;
+    const int chunk = (a >> 3) * 4 + (a & 3), half = ((a >> 2) ^ (cg >> 3)) & 1;
 #pragma unroll
     for (int j = 0; j < 8; j++) {
         const int r = cg * 8 + j, w = j >> 1;
@@ -73,6 +74,8 @@ template <> __device__ __forceinline__ u32x4 weight_chunk<__bf16>(const f32x4 *p
     return __builtin_bit_cast(u32x4, r);
 }
 template <> __device__ __forceinline__ u32x4 weight_chunk<float>(const f32x4 *p, int s) { return __builtin_bit_cast(u32x4, p[s]); }
+// ... for the columns of block b of 64
+template <typename T> __device__ __forceinline__ u32x4 for_block(const u32x4 &w, int b) { return sizeof(T) == 2 && (b & 1) ? u32x4{w.z, w.w, w.x, w.y} : w; }
 
 // over the four lanes that share lane & 15
 __device__ __forceinline__ float group_max(float v) {
@@ -237,7 +240,7 @@ __global__ __launch_bounds__(256) void latent_expanded_kernel(Expanded p) {
             for (int n = 0; n < NVF; n++) {
                 const u32x4 a = vs[va[(n & 3) ^ (2 * sp)] + 128 * n];
 #pragma unroll
-                for (int i = 0; i < NQ; i++) o[i][n] = mma<T>(a, w[i], o[i][n]);
+                for (int i = 0; i < NQ; i++) o[i][n] = mma<T>(a, for_block<T>(w[i], n >> 2), o[i][n]);
             }
         }
     }
@@ -264,8 +267,9 @@ __global__ __launch_bounds__(256) void latent_expanded_kernel(Expanded p) {
 }
 
 // ---- absorbed: every (row, head) attends to the cache rows themselves ------------------------------------------------------------------------
-// Workgroup: 16 NQ of the rows * heads queries, all on the same keys.  Per tile: wave t takes 16 keys of the scores, every wave does the softmax
-// of all queries from LDS, and takes every fourth 16 columns of the latent in the value product.  A cache row is read once for both products.
+// Workgroup: 16 NQ of the rows * heads queries, all on the same keys.  Per tile: a wave takes half of the keys and half of the columns of the scores (a quarter of
+// the query registers), every wave does the softmax of all queries from the sums in LDS, and takes every fourth 16 columns of the latent in the value
+// product.  A cache row is read once for both products.
 // blockIdx.z: split of the key tiles.
 struct Absorbed {
     const void *q, *cache;                                 // [row][head][ld], [key][ld]: rank_pad latent columns, then the rotated part
@@ -283,10 +287,11 @@ __global__ __launch_bounds__(256, 1) void latent_absorbed_kernel(Absorbed p) {
     constexpr int CH = Chunk<T>::N, KT = Chunk<T>::KEYS, NT = KT / 16, NKF = (DV + DR) / Chunk<T>::STEP, KC = (DV + DR) / CH, NVW = DV / 64, BM = 16 * NQ, SS = KT + 4;
     // a thread's pieces: four keys x one chunk, latent ones (AL groups of keys apart) and rotated ones
     constexpr int NC = DV / CH, AL = 256 / NC, TL = KT / 4 / AL, NR = DR / CH, RT = (KT / 4) * NR, RL = (RT + 255) / 256;
-    static_assert(256 % NC == 0 && (KT / 4) % AL == 0, "pieces");
+    constexpr int NKH = NKF / 2, NTH = NT / 2;             // steps and tiles of keys of a wave's scores
+    static_assert(256 % NC == 0 && (KT / 4) % AL == 0 && NKF % 2 == 0, "pieces");
     extern __shared__ __attribute__((aligned(16))) u32x4 lds[];
     u32x4 *ks = lds, *vs = ks + KT * KC;
-    float *ss = reinterpret_cast<float *>(vs + DV * 8);    // scores [query][key]
+    float *ss = reinterpret_cast<float *>(vs + DV * 8);    // scores [half of the columns][query][key]
     const int tid = threadIdx.x, lane = tid & 63, wv = __builtin_amdgcn_readfirstlane(tid >> 6), lr = lane & 15, lk = lane >> 4;
     const int M = p.rows * p.heads, m0 = blockIdx.x * BM, nz = gridDim.z, z = blockIdx.z;
     const int pos = p.pos + (p.pos_dev ? p.pos_dev[0] : 0);
@@ -333,19 +338,20 @@ __global__ __launch_bounds__(256, 1) void latent_absorbed_kernel(Absorbed p) {
         }
     };
     if (lo < hi) fetch(lo * KT);
-    u32x4 qf[NQ][NKF];
-    int pq[NQ];
+    const int k0 = (wv & 1) * NKH, t0 = (wv >> 1) * NTH;
+    u32x4 qf[NQ][NKH];
 #pragma unroll
     for (int i = 0; i < NQ; i++) {
-        const int m = min(m0 + 16 * i + lr, M - 1);
-        pq[i] = pos + m / p.heads;
-        const T *qr = (const T *)p.q + (int64_t)m * p.ld;
+        const T *qr = (const T *)p.q + (int64_t)min(m0 + 16 * i + lr, M - 1) * p.ld;
 #pragma unroll
-        for (int s = 0; s < NKF; s++) {
-            const int c = (4 * s + lk) * CH;               // a step lies in one of the two parts
-            qf[i][s] = *reinterpret_cast<const u32x4 *>(qr + min(4 * s < NC ? min(c, p.rank_pad - CH) : p.rank_pad + c - DV, p.ld - CH));
+        for (int s = 0; s < NKH; s++) {
+            const int k = k0 + s, c = (4 * k + lk) * CH;   // a step lies in one of the two parts
+            qf[i][s] = *reinterpret_cast<const u32x4 *>(qr + min(4 * k < NC ? min(c, p.rank_pad - CH) : p.rank_pad + c - DV, p.ld - CH));
         }
     }
+    int pq[NQ];
+#pragma unroll
+    for (int i = 0; i < NQ; i++) pq[i] = pos + min(m0 + 16 * i + lr, M - 1) / p.heads;
 
     f32x4 o[NQ][NVW];
     float m_run[NQ], l_run[NQ];
@@ -362,19 +368,24 @@ __global__ __launch_bounds__(256, 1) void latent_absorbed_kernel(Absorbed p) {
         stage();
         __syncthreads();
         if (it + 1 < hi) fetch(j0 + KT);
-        if (wv < NT) {
-            const int r = 16 * wv + lr;
-            f32x4 s[NQ][2];
+        {
+            f32x4 s[NQ][NTH];
 #pragma unroll
-            for (int i = 0; i < NQ; i++) s[i][0] = s[i][1] = f32x4{0.f, 0.f, 0.f, 0.f};
+            for (int i = 0; i < NQ; i++)
 #pragma unroll
-            for (int k = 0; k < NKF; k++) {
-                const u32x4 a = ks[r * KC + key_slot(r, 4 * k + lk)];
+                for (int t = 0; t < NTH; t++) s[i][t] = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-                for (int i = 0; i < NQ; i++) s[i][k & 1] = mma<T>(a, qf[i][k], s[i][k & 1]);
-            }
+            for (int k = 0; k < NKH; k++)
 #pragma unroll
-            for (int i = 0; i < NQ; i++) *reinterpret_cast<f32x4 *>(ss + (16 * i + lr) * SS + 16 * wv + 4 * lk) = s[i][0] + s[i][1];
+                for (int t = 0; t < NTH; t++) {
+                    const u32x4 a = ks[(16 * (t0 + t) + lr) * KC + key_slot(lr, 4 * (k0 + k) + lk)];
+#pragma unroll
+                    for (int i = 0; i < NQ; i++) s[i][t] = mma<T>(a, qf[i][k], s[i][t]);
+                }
+#pragma unroll
+            for (int i = 0; i < NQ; i++)
+#pragma unroll
+                for (int t = 0; t < NTH; t++) *reinterpret_cast<f32x4 *>(ss + ((wv & 1) * BM + 16 * i + lr) * SS + 16 * (t0 + t) + 4 * lk) = s[i][t];
         }
         __syncthreads();
         u32x4 w[NQ][2];
@@ -384,7 +395,8 @@ __global__ __launch_bounds__(256, 1) void latent_absorbed_kernel(Absorbed p) {
             float mx = -INFINITY, sum = 0.0f;
 #pragma unroll
             for (int t = 0; t < NT; t++) {
-                s[t] = *reinterpret_cast<const f32x4 *>(ss + (16 * i + lr) * SS + 16 * t + 4 * lk);
+                const float *sum_of = ss + (16 * i + lr) * SS + 16 * t + 4 * lk;
+                s[t] = *reinterpret_cast<const f32x4 *>(sum_of) + *reinterpret_cast<const f32x4 *>(sum_of + BM * SS);
 #pragma unroll
                 for (int e = 0; e < 4; e++) {
                     s[t][e] = j0 + 16 * t + 4 * lk + e > pq[i] ? -INFINITY : s[t][e];
@@ -411,16 +423,15 @@ __global__ __launch_bounds__(256, 1) void latent_absorbed_kernel(Absorbed p) {
             for (int sp = 0; sp < 2; sp++) w[i][sp] = weight_chunk<T>(s, sp);
         }
 #pragma unroll
-        for (int n = 0; n < NVW; n++)
-            if (64 * n + 16 * wv < p.rank_pad) {
-                const int r = 64 * n + 16 * wv + lr;
+        for (int n = 0; n < NVW; n++) {                    // columns beyond the latent are zero
+            const int r = 64 * n + 16 * wv + lr;
 #pragma unroll
-                for (int sp = 0; sp < 2; sp++) {
-                    const u32x4 a = vs[r * 8 + value_slot(r, 4 * sp + lk)];
+            for (int sp = 0; sp < 2; sp++) {
+                const u32x4 a = vs[r * 8 + value_slot(r, 4 * sp + lk)];
 #pragma unroll
-                    for (int i = 0; i < NQ; i++) o[i][n] = mma<T>(a, w[i][sp], o[i][n]);
-                }
+                for (int i = 0; i < NQ; i++) o[i][n] = mma<T>(a, for_block<T>(w[i][sp], n), o[i][n]);
             }
+        }
     }
 #pragma unroll
     for (int i = 0; i < NQ; i++) {
@@ -652,7 +663,7 @@ AbsorbedPlan absorbed_plan(int bf16, int64_t m, int64_t keys) {
 }
 
 template <typename T, int DV, int DR, int NQ> int absorbed_launch(const Absorbed &a, int nz, hipStream_t s) {
-    constexpr size_t lds = (size_t)Chunk<T>::KEYS * (DV + DR) * sizeof(T) + (size_t)DV * 128 + (size_t)16 * NQ * (Chunk<T>::KEYS + 4) * sizeof(float);
+    constexpr size_t lds = (size_t)Chunk<T>::KEYS * (DV + DR) * sizeof(T) + (size_t)DV * 128 + (size_t)2 * 16 * NQ * (Chunk<T>::KEYS + 4) * sizeof(float);
     static_assert(lds <= (size_t)160 * 1024, "LDS");
     if (lds > 64 * 1024) {
         const int e = (int)hipFuncSetAttribute(reinterpret_cast<const void *>(latent_absorbed_kernel<T, DV, DR, NQ>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
