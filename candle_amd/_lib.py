@@ -118,7 +118,7 @@ MIXER_SIGNATURES = {
     "cq_dense_product": (_int, [_int, _dense, _vp, _i64, _vp]),
     "cq_dense_matvec": (_int, [_vp, _i64, _vp, _int, _vp, _f32, _i64, _vp, _vp, _int, _i64, _i64, _vp]),
     "cq_mix_rms_norm_rows": (_int, [_vp, _i64, _vp, _vp, _i64, _vp, _vp, _i64, _i64, _i64, _f32, _vp]),
-    "cq_mix_layer_norm_rows": (_int, [_vp, _i64, _vp, _vp, _vp, _i64, _i64, _i64, _f32, _vp]),
+    "cq_mix_layer_norm_rows": (_int, [_vp, _i64, _vp, _vp, _vp, _vp, _i64, _i64, _i64, _f32, _vp]),
     "cq_mix_poly_norm": (_int, [_vp, _i64, _vp, _vp, _i64, _i64, _i64, _f32, _vp]),
     "cq_mix_tanh": (_int, [_vp, _i64, _vp, _i64, _i64, _i64, _vp]),
     "cq_mix_pack_heads": (_int, [_vp, _i64, _heads, _int, _f32, _vp, _i64, _i64, _vp]),

@@ -69,12 +69,13 @@ __global__ __launch_bounds__(256) void rms_norm_rows_kernel(float *x, int64_t x_
 
 // One workgroup per row; the first KEEP * 256 values stay in registers between the mean, the variance and the result.
 __global__ __launch_bounds__(256) void layer_norm_rows_kernel(const float *__restrict__ x, int64_t x_stride, const int32_t *__restrict__ index,
-                                                              const float *__restrict__ vec, float *__restrict__ out, int64_t out_stride, int dim, float eps) {
+                                                              const float *__restrict__ vec, float *__restrict__ out, __bf16 *__restrict__ out16, int64_t out_stride, int dim,
+                                                              float eps) {
     __shared__ float red[4];
     constexpr int KEEP = 16;
     const int64_t r = blockIdx.x;
     const float *xr = x + (index ? (int64_t)index[r] : r) * x_stride;
-    float *o = out + r * out_stride, keep[KEEP], sum = 0.0f, q = 0.0f;
+    float keep[KEEP], sum = 0.0f, q = 0.0f;
 #pragma unroll
     for (int c = 0; c < KEEP; c++) {
         const int i = threadIdx.x + 256 * c;
@@ -90,12 +91,17 @@ __global__ __launch_bounds__(256) void layer_norm_rows_kernel(const float *__res
     }
     for (int i = threadIdx.x + 256 * KEEP; i < dim; i += 256) q = fmaf(xr[i] - mean, xr[i] - mean, q);
     const float m = sqrtf(block_sum(q, red) / (float)dim + eps);
+    auto emit = [&](int i, float v) {
+        v = (v - mean) / m * vec[i] + vec[dim + i];
+        if (out) out[r * out_stride + i] = v;
+        if (out16) out16[r * out_stride + i] = (__bf16)v;
+    };
 #pragma unroll
     for (int c = 0; c < KEEP; c++) {
         const int i = threadIdx.x + 256 * c;
-        if (i < dim) o[i] = (keep[c] - mean) / m * vec[i] + vec[dim + i];
+        if (i < dim) emit(i, keep[c]);
     }
-    for (int i = threadIdx.x + 256 * KEEP; i < dim; i += 256) o[i] = (xr[i] - mean) / m * vec[i] + vec[dim + i];
+    for (int i = threadIdx.x + 256 * KEEP; i < dim; i += 256) emit(i, xr[i]);
 }
 
 // sum over n = 1..3 of coef[n-1] z^n / rms(z^n), plus coef[3]: one workgroup per row, the row re-read after its three sums
@@ -239,14 +245,14 @@ int cq_mix_rms_norm_rows(float *x_dev, int64_t x_stride, const int32_t *index_de
     return (int)hipGetLastError();
 }
 
-int cq_mix_layer_norm_rows(const float *x_dev, int64_t x_stride, const int32_t *index_dev, const float *vec_dev, float *out_dev, int64_t out_stride,
-                           int64_t rows, int64_t dim, float eps, void *stream) {
+int cq_mix_layer_norm_rows(const float *x_dev, int64_t x_stride, const int32_t *index_dev, const float *vec_dev, float *out_dev, void *out_bf16_dev,
+                           int64_t out_stride, int64_t rows, int64_t dim, float eps, void *stream) {
     if (rows < 0 || dim <= 0 || x_stride < dim || out_stride < dim) return CQ_ERR_SHAPE;
     if (rows == 0) return CQ_OK;
-    if (!x_dev || !vec_dev || !out_dev) return CQ_ERR_NULL;
+    if (!x_dev || !vec_dev || (!out_dev && !out_bf16_dev)) return CQ_ERR_NULL;
     if (rows > 0x7fffffffLL || dim > (1 << 24)) return CQ_ERR_RANGE;
-    hipLaunchKernelGGL(layer_norm_rows_kernel, dim3((unsigned)rows), dim3(256), 0, (hipStream_t)stream, x_dev, x_stride, index_dev, vec_dev, out_dev, out_stride,
-                       (int)dim, eps);
+    hipLaunchKernelGGL(layer_norm_rows_kernel, dim3((unsigned)rows), dim3(256), 0, (hipStream_t)stream, x_dev, x_stride, index_dev, vec_dev, out_dev,
+                       (__bf16 *)out_bf16_dev, out_stride, (int)dim, eps);
     return (int)hipGetLastError();
 }
 

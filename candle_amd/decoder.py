@@ -160,16 +160,18 @@ class Decoder(GreedyDecoder):
     def _enqueue_rows(self, ids: int, rows: int, pos: int, sp) -> int:
         """`rows` new tokens through all layers; returns the residual stream."""
         rt, ld = self.rt, self.ld
-        x, h = rt.scratch("x", rows * ld), rt.scratch("h", rows * ld)
+        x = rt.scratch("x", rows * ld)
         emb = rt.scratch("embedding", rows * ld) if self.loops else None
         self._embed(ids, x, rows, sp)
         if self.loops:
             self._embed(ids, emb, rows, sp)
         for run, (i, again) in enumerate(self.cfg.order):
             layer = self.layers[i]
+            h = rt.normed(layer.mixer.INPUT, rows * ld)
             layer.norm1.rows(x, ld, h, ld, rows, sp, delta=emb if again else None)
             layer.mixer.prefill(h, ld, x, ld, self.kept[run], pos, rows, sp)
             if layer.mlp:
+                h = rt.normed(layer.mlp.INPUT, rows * ld)
                 layer.norm2.rows(x, ld, h, ld, rows, sp)
                 layer.mlp.prefill(h, ld, x, ld, rows, sp)
             if self.tap:
@@ -226,11 +228,11 @@ class Decoder(GreedyDecoder):
                 x = self._enqueue_rows(ids.data_ptr() + 4 * lo, rows, pos + lo, sp)
                 if at:
                     index = torch.tensor([want[j] - lo for j in at], dtype=torch.int32).to(self.device)
-                    h = rt.scratch("h", len(at) * self.ld)
+                    h = rt.normed(mixers.AS_F32, len(at) * self.ld)
                     ldl = pad_to(cfg.vocab, 4)
                     logits = rt.scratch("logits", len(at) * ldl)
                     self.final_norm.rows(x, self.ld, h, self.ld, len(at), sp, index=index.data_ptr())
-                    self.head.rows(h, self.ld, logits, ldl, len(at), sp)
+                    self.head.rows(h.f32, self.ld, logits, ldl, len(at), sp)
                     out[at] = rt._scratch["logits"][:len(at) * ldl].view(len(at), ldl)[:, :cfg.vocab]
         self.cache.length = pos + n
         return out

@@ -11,7 +11,7 @@ from __future__ import annotations
 
 import ctypes
 import math
-from typing import Callable, Dict, List, Optional
+from typing import Callable, Dict, List, NamedTuple, Optional
 
 import numpy as np
 import torch
@@ -87,6 +87,14 @@ class Runtime:
         need not be finite)."""
         return self.scratch(name, (count + 1) // 2 if self.t_bf16 else count)
 
+    def normed(self, kinds: tuple, count: int) -> Normed:
+        """Scratch for normed rows.  Without reduced precision both kinds are one buffer."""
+        f32, typed = kinds
+        if not self.t_bf16:
+            p = self.scratch("h", count)
+            return Normed(p, p)
+        return Normed(self.scratch("h", count) if f32 else None, self.typed("h_typed", count) if typed else None)
+
     def rotation(self, base: float, dims: int, scaling: Optional[dict] = None) -> tuple:
         """cos / sin [ctx, dims / 2] of t * frequency, evaluated in double and rounded once (see ``frequencies``)."""
         key = (float(base), int(dims), tuple(sorted(scaling.items())) if scaling else None)
@@ -152,6 +160,16 @@ def alternate(gate: torch.Tensor, up: torch.Tensor) -> torch.Tensor:
     return torch.stack([gate, up], dim=1).reshape(2 * gate.shape[0], gate.shape[1])
 
 
+class Normed(NamedTuple):
+    """Normed rows as a block asks for them (``INPUT``): f32, the type of the products' inputs, or both.  Row strides are the same in elements."""
+
+    f32: Optional[int] = None
+    typed: Optional[int] = None
+
+
+AS_F32, AS_TYPED, AS_BOTH = (True, False), (False, True), (True, True)
+
+
 class RmsNorm:
     """x / rms(x) * weight, over rows or as the prologue of a single-row product."""
 
@@ -162,9 +180,11 @@ class RmsNorm:
         self.vec = rt.vector(get(name))
         self.dim = self.vec.numel()
 
-    def rows(self, x: int, ldx: int, out: int, ldo: int, rows: int, sp, index: Optional[int] = None, delta: Optional[int] = None) -> None:
+    def rows(self, x: int, ldx: int, out: Normed, ldo: int, rows: int, sp, index: Optional[int] = None, delta: Optional[int] = None) -> None:
         """Rows of x (those that `index` names) into out; `delta` [rows, ldx] is added to x first."""
-        check("cq_mix_rms_norm_rows", self.rt.L.cq_mix_rms_norm_rows(x, ldx, index, delta, ldx, self.vec.data_ptr(), out, ldo, rows, self.dim, self.eps, sp))
+        if out.f32 is None or (out.typed is not None and out.typed != out.f32):
+            raise ValueError("this norm writes f32 only")
+        check("cq_mix_rms_norm_rows", self.rt.L.cq_mix_rms_norm_rows(x, ldx, index, delta, ldx, self.vec.data_ptr(), out.f32, ldo, rows, self.dim, self.eps, sp))
 
 
 class LayerNorm:
@@ -177,10 +197,11 @@ class LayerNorm:
         self.vec = torch.cat([rt.vector(get(name)), rt.vector(get(name + ".b"))])
         self.dim = self.vec.numel() // 2
 
-    def rows(self, x: int, ldx: int, out: int, ldo: int, rows: int, sp, index: Optional[int] = None, delta: Optional[int] = None) -> None:
+    def rows(self, x: int, ldx: int, out: Normed, ldo: int, rows: int, sp, index: Optional[int] = None, delta: Optional[int] = None) -> None:
         if delta is not None:
             raise ValueError("this norm adds nothing to its input")
-        check("cq_mix_layer_norm_rows", self.rt.L.cq_mix_layer_norm_rows(x, ldx, index, self.vec.data_ptr(), out, ldo, rows, self.dim, self.eps, sp))
+        f32, bf16 = (out.f32, out.typed) if self.rt.t_bf16 else (out.f32 or out.typed, None)
+        check("cq_mix_layer_norm_rows", self.rt.L.cq_mix_layer_norm_rows(x, ldx, index, self.vec.data_ptr(), f32, bf16, ldo, rows, self.dim, self.eps, sp))
 
 
 def _heads(src_off: int, heads: int, dim: int, *, dim_pad: int = 0, dst: Optional[int] = None, row_stride: int = 0, head_stride: int = 0,
@@ -306,8 +327,9 @@ class Retention:
 
 
 class Mixer:
-    """A layer's first sublayer: x <- x + mixer(norm(x)).  ``norm_rows`` has left norm(x) in `h` for ``prefill``; ``step`` applies it itself."""
+    """A layer's first sublayer: x <- x + mixer(norm(x)).  ``prefill`` finds norm(x) in `h`; ``step`` applies the norm itself."""
 
+    INPUT = AS_F32                                   # how `prefill` wants its normed rows
     kv_from: Optional[int] = None                    # a layer whose cache this one attends to instead of having its own
 
     def denses(self) -> List[Dense]:
@@ -316,7 +338,7 @@ class Mixer:
     def new_cache(self, cache: SequenceCache):
         raise NotImplementedError
 
-    def prefill(self, h: int, ldh: int, x: int, ldx: int, kept, pos: int, rows: int, sp) -> None:
+    def prefill(self, h: Normed, ldh: int, x: int, ldx: int, kept, pos: int, rows: int, sp) -> None:
         raise NotImplementedError
 
     def step(self, x: int, norm, kept, pos_dev: Optional[int], pos: int, add: Optional[int], sp) -> None:
@@ -353,7 +375,7 @@ class Parallel(Mixer):
         q = rt.scratch("attention_q", rows * lt.heads * lt.dp)
         rq, rk = rt.scratch("retention_q", rows * rg.heads * rg.dp), rt.scratch("retention_k", rows * rg.heads * rg.dp)
         out = rt.scratch("mixer_out", rows * ldo)
-        self.w_in.rows(h, ldh, row, ldp, rows, sp)
+        self.w_in.rows(h.f32, ldh, row, ldp, rows, sp)
         groups = _group_array(lt.groups(kv, 0, q) + rg.groups(self.off, rq, rk))
         check("cq_mix_pack_heads", rt.L.cq_mix_pack_heads(row, ldp, groups, len(groups), self.eps, None, pos, rows, sp))
         lt.attend(q, kv, out, ldo, self.left_scale, pos, rows, sp)
@@ -405,7 +427,7 @@ class GeneralDelta(Mixer):
         low, wl = rt.scratch("delta_low", rows * self.w2.kp), rt.scratch("delta_decay", rows * ldw)
         packed = rt.scratch("delta_packed", rows * self.heads * (4 * L.cq_mix_state_pad(self.dim) + 1))
         raw, out = rt.scratch("mixer_raw", rows * w), rt.scratch("mixer_out", rows * ldo)
-        self.w_in.rows(h, ldh, row, ldp, rows, sp)
+        self.w_in.rows(h.f32, ldh, row, ldp, rows, sp)
         check("cq_mix_tanh", L.cq_mix_tanh(row + 4 * self.low_off, ldp, low, self.w2.kp, rows, self.rank, sp))
         self.w2.rows(low, self.w2.kp, wl, ldw, rows, sp)
         check("cq_mix_delta_prep", L.cq_mix_delta_prep(row, ldp, self.r_off, self.k_off, self.a_off, wl, ldw, self.w0.data_ptr(), self.a_bias.data_ptr(), packed, rows,
@@ -425,7 +447,22 @@ class GeneralDelta(Mixer):
         self.w_out.row(out, x, sp, accumulate=True, add=add)
 
 
-class PolyFeedForward:
+class FeedForward:
+    """A layer's second sublayer, like ``Mixer`` without anything kept."""
+
+    INPUT = AS_F32
+
+    def denses(self) -> List[Dense]:
+        raise NotImplementedError
+
+    def prefill(self, h: Normed, ldh: int, x: int, ldx: int, rows: int, sp) -> None:
+        raise NotImplementedError
+
+    def step(self, x: int, norm, add: Optional[int], sp) -> None:
+        raise NotImplementedError
+
+
+class PolyFeedForward(FeedForward):
     """down(PolyNorm(up(norm(x)))): the activation is a polynomial whose powers are each divided by the row's root mean square."""
 
     def __init__(self, rt: Runtime, cfg: dict, get: Callable[[str], torch.Tensor], eps: float):
@@ -442,7 +479,7 @@ class PolyFeedForward:
     def prefill(self, h, ldh, x, ldx, rows, sp):
         rt, ld = self.rt, self.down.kp
         z = rt.scratch("feed_forward", rows * ld)
-        self.up.rows(h, ldh, z, ld, rows, sp)
+        self.up.rows(h.f32, ldh, z, ld, rows, sp)
         check("cq_mix_poly_norm", rt.L.cq_mix_poly_norm(z, ld, self.coef.data_ptr(), z, ld, rows, self.ff, self.eps, sp))
         self.down.rows(z, ld, x, ldx, rows, sp, accumulate=True)
 
@@ -459,6 +496,7 @@ class LatentAttention(Mixer):
     Many rows: keys and values of all heads are computed from the cache rows, then attended to head by head.  Few rows and single tokens: the key matrix is
     applied to the query and the value matrix to the attended latent, so that the heads attend to the cache rows themselves."""
 
+    INPUT = AS_TYPED
     MAX_RANK, MAX_HEAD, MAX_VALUE = 512, 320, 256    # CQ_LATENT_MAX_*; rotated parts of more than 64 (up to 192) with latents up to 256
 
     def __init__(self, rt: Runtime, cfg: dict, get: Callable[[str], torch.Tensor], eps: float):
@@ -515,7 +553,7 @@ class LatentAttention(Mixer):
         ldp, ldo, bf = pad_to(self.w_in.n, 4), self.w_out.kp, int(rt.t_bf16)
         row, out = rt.scratch("projection", rows * ldp), rt.scratch("mixer_out", rows * ldo)
         gate = row + 4 * self.g_off
-        self.w_in.rows(h, ldh, row, ldp, rows, sp)
+        self.w_in.rows(h.typed, ldh, row, ldp, rows, sp, x_bf16=bf)
         if self.expands(rows):
             head, keys = self.dim_pad + self.rot_pad, pos + rows
             ldkv = self.expand.n + (0 if self.expand.n // 128 % 2 else 128)     # rows an odd number of 256 bytes apart fall on all memory channels
@@ -548,8 +586,10 @@ class LatentAttention(Mixer):
         self.w_out.row(out, x, sp, accumulate=True, add=add)
 
 
-class ReluSquaredFeedForward:
+class ReluSquaredFeedForward(FeedForward):
     """down(relu(up(norm(x)))^2)."""
+
+    INPUT = AS_TYPED
 
     def __init__(self, rt: Runtime, cfg: dict, get: Callable[[str], torch.Tensor], eps: float):
         self.rt = rt
@@ -563,7 +603,7 @@ class ReluSquaredFeedForward:
     def prefill(self, h, ldh, x, ldx, rows, sp):
         rt, ld, bf = self.rt, self.down.kp, int(self.rt.t_bf16)
         z = rt.typed("activation", rows * ld)
-        self.up.rows(h, ldh, z, ld, rows, sp, act=ACT_RELU2, dst_bf16=bf)
+        self.up.rows(h.typed, ldh, z, ld, rows, sp, act=ACT_RELU2, x_bf16=bf, dst_bf16=bf)
         self.down.rows(z, ld, x, ldx, rows, sp, accumulate=True, x_bf16=bf)
 
     def step(self, x, norm, add, sp):
@@ -572,9 +612,11 @@ class ReluSquaredFeedForward:
         self.down.row(z, x, sp, RELU2, accumulate=True, add=add)
 
 
-class GatedExperts:
+class GatedExperts(FeedForward):
     """A mixture of small feed-forwards down(silu(gate(h)) * up(h)), weighted by the softmax over the chosen router logits, and optionally one that every token
     takes, weighted by a sigmoid.  The choice and everything after it stay on the device."""
+
+    INPUT = AS_BOTH                                  # the router reads f32
 
     def __init__(self, rt: Runtime, cfg: dict, get: Callable[[str], torch.Tensor], eps: float):
         self.rt = rt
@@ -617,12 +659,12 @@ class GatedExperts:
         ldl, pairs = pad_to(self.router.n, 4), rows * top
         logits = rt.scratch("router_logits", rows * ldl)
         ids, weights, shared = rt.scratch("expert_ids", pairs), rt.scratch("expert_weights", pairs), rt.scratch("shared_weights", rows)
-        self.router.rows(h, ldh, logits, ldl, rows, sp, precision=F32)
+        self.router.rows(h.f32, ldh, logits, ldl, rows, sp, precision=F32)
         check("cq_mix_moe_select", L.cq_mix_moe_select(logits, ldl, rows, E, top, ids, weights, shared if self.shared_ff else None, sp))
         if self.shared_ff:
             ld = self.shared_down.kp
             z = rt.typed("shared_activation", rows * ld)
-            self.shared_up.rows(h, ldh, z, ld, rows, sp, act=ACT_SWIGLU, row_scale_dev=shared, dst_bf16=bf)
+            self.shared_up.rows(h.typed, ldh, z, ld, rows, sp, act=ACT_SWIGLU, row_scale_dev=shared, x_bf16=bf, dst_bf16=bf)
             self.shared_down.rows(z, ld, x, ldx, rows, sp, accumulate=True, x_bf16=bf)
         per_expert = pairs / E
         tile = 64 if not bf else (128 if per_expert >= 96 else (64 if per_expert >= 24 else 32))
@@ -633,8 +675,8 @@ class GatedExperts:
         z, ldy = rt.typed("expert_activation", pairs * self.ffp), pad_to(self.width, 4)
         y = rt.scratch("expert_out", pairs * ldy)
         grouped = dict(tiles_dev=tiles, n_tiles_dev=n_tiles, max_tiles=max_tiles, tile_rows=tile, m=pairs, batch=1)
-        dense_product(rt, rt.precision, sp, w_dev=self.up.data_ptr(), ldw=self.kp, w_batch=self.up[0].numel(), x_dev=h, ldx=ldh, dst_dev=z, ldd=self.ffp, n=2 * self.ff,
-                      k=self.kp, src_rows_dev=src, row_scale_dev=scale, act=ACT_SWIGLU, dst_bf16=bf, **grouped)
+        dense_product(rt, rt.precision, sp, w_dev=self.up.data_ptr(), ldw=self.kp, w_batch=self.up[0].numel(), x_dev=h.typed, ldx=ldh, dst_dev=z, ldd=self.ffp,
+                      n=2 * self.ff, k=self.kp, src_rows_dev=src, row_scale_dev=scale, act=ACT_SWIGLU, x_bf16=bf, dst_bf16=bf, **grouped)
         dense_product(rt, rt.precision, sp, w_dev=self.down.data_ptr(), ldw=self.ffp, w_batch=self.down[0].numel(), x_dev=z, ldx=self.ffp, dst_dev=y, ldd=ldy, n=self.width,
                       k=self.ffp, dst_rows_dev=dst, x_bf16=bf, **grouped)
         check("cq_mix_moe_add", L.cq_mix_moe_add(y, ldy, top, x, ldx, rows, self.width, sp))
@@ -644,7 +686,7 @@ class GatedExperts:
         if not self.fused:                           # sizes beyond the two launches: the several-row path with one row
             if add is not None:
                 raise ValueError("no addend on this path")
-            h = rt.scratch("h", self.kp)
+            h = rt.normed(self.INPUT, self.kp)
             norm.rows(x, self.kp, h, self.kp, 1, sp)
             self.prefill(h, self.kp, x, self.kp, 1, sp)
             return

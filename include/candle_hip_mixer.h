@@ -75,9 +75,10 @@ int cq_dense_matvec(const void *w_dev, int64_t ldw, const float *x_dev, int prol
  * delta, s also replaces the row of x.  Any dim; strides in floats. */
 int cq_mix_rms_norm_rows(float *x_dev, int64_t x_stride, const int32_t *index_dev, const float *delta_dev, int64_t delta_stride, const float *weight_dev,
                          float *out_dev, int64_t out_stride, int64_t rows, int64_t dim, float eps, void *stream);
-/* Layer norm of (selected) rows: out[r] = (s - mean(s)) / sqrt(var(s) + eps) * vec[0..dim) + vec[dim..2 dim), s = x[index ? index[r] : r]. */
-int cq_mix_layer_norm_rows(const float *x_dev, int64_t x_stride, const int32_t *index_dev, const float *vec_dev, float *out_dev, int64_t out_stride,
-                           int64_t rows, int64_t dim, float eps, void *stream);
+/* Layer norm of (selected) rows: out[r] = (s - mean(s)) / sqrt(var(s) + eps) * vec[0..dim) + vec[dim..2 dim), s = x[index ? index[r] : r], as f32,
+ * as bfloat16 or both (out_dev, out_bf16_dev: one may be NULL). */
+int cq_mix_layer_norm_rows(const float *x_dev, int64_t x_stride, const int32_t *index_dev, const float *vec_dev, float *out_dev, void *out_bf16_dev,
+                           int64_t out_stride, int64_t rows, int64_t dim, float eps, void *stream);
 /* out = coef[0] N(z) + coef[1] N(z^2) + coef[2] N(z^3) + coef[3], N(z) = z / sqrt(mean(z^2) + eps), row by row (out may be z). */
 int cq_mix_poly_norm(const float *z_dev, int64_t z_stride, const float *coef_dev, float *out_dev, int64_t out_stride, int64_t rows, int64_t dim, float eps,
                      void *stream);

@@ -64,11 +64,15 @@ def test_layer_norm_rows(dim):
     x, w, b = rnd(1, 9, dim) + 2.0, rnd(2, dim), rnd(3, dim)
     xd, vec, out = up(padded(x, ld)), up(np.concatenate([w, b])), torch.full((9, ld), 7.0, device=DEV)
     want = ko.layer_norm(x.astype(np.float64), w, b, EPS)
-    _lib.check("n", L.cq_mix_layer_norm_rows(xd.data_ptr(), ld, None, vec.data_ptr(), out.data_ptr(), ld, 9, dim, EPS, sp()))
+    _lib.check("n", L.cq_mix_layer_norm_rows(xd.data_ptr(), ld, None, vec.data_ptr(), out.data_ptr(), None, ld, 9, dim, EPS, sp()))
     assert rel(out[:, :dim], want) < 3e-6 and bool((out[:, dim:] == 7.0).all())
     index = torch.tensor([8, 0, 3], dtype=torch.int32, device=DEV)
-    _lib.check("n", L.cq_mix_layer_norm_rows(xd.data_ptr(), ld, index.data_ptr(), vec.data_ptr(), out.data_ptr(), ld, 3, dim, EPS, sp()))
+    _lib.check("n", L.cq_mix_layer_norm_rows(xd.data_ptr(), ld, index.data_ptr(), vec.data_ptr(), out.data_ptr(), None, ld, 3, dim, EPS, sp()))
     assert rel(out[:3, :dim], want[[8, 0, 3]]) < 3e-6
+    for also in (True, False):
+        out, out16 = torch.full((9, ld), 7.0, device=DEV), torch.full((9, ld), 7.0, device=DEV, dtype=torch.bfloat16)
+        _lib.check("n", L.cq_mix_layer_norm_rows(xd.data_ptr(), ld, None, vec.data_ptr(), out.data_ptr() if also else None, out16.data_ptr(), ld, 9, dim, EPS, sp()))
+        assert rel(out16[:, :dim], want) < 5e-3 and bool((out16[:, dim:] == 7.0).all()) and (rel(out[:, :dim], want) < 3e-6 if also else bool((out == 7.0).all()))
 
 
 @pytest.mark.parametrize("n,k", [(1, 8), (37, 72), (530, 2100), (21, 14336)])
@@ -175,8 +179,10 @@ class Feed:
         self.rt = mixers.Runtime(DEV, precision, 8)
         self.m = mixers.GatedExperts(self.rt, mlp, lambda n: up(ts[n], torch.bfloat16), EPS)
         vec = {"n": 1.0 + rnd(7, width, scale=0.2), "n.b": rnd(8, width, scale=0.2)}
-        self.norms = [mixers.LayerNorm(self.rt, lambda n: torch.from_numpy(vec[n]), "n", EPS), mixers.RmsNorm(self.rt, lambda n: torch.from_numpy(vec[n]), "n", EPS)]
-        self.normed = [lambda x: ko.layer_norm(x, vec["n"], vec["n.b"], EPS), lambda x: ko.rms_norm(x, vec["n"], EPS)]
+        self.norm = mixers.LayerNorm(self.rt, lambda n: torch.from_numpy(vec[n]), "n", EPS)
+        self.rms = mixers.RmsNorm(self.rt, lambda n: torch.from_numpy(vec[n]), "n", EPS)
+        self.normed = lambda x: ko.layer_norm(x, vec["n"], vec["n.b"], EPS)
+        self.rms_normed = lambda x: ko.rms_norm(x, vec["n"], EPS)
 
 
 @pytest.mark.parametrize("width,mlp", [(40, kc.moe(1, 1, 8)), (72, kc.moe(6, 2, 24, 40)), (2100, kc.moe(9, 3, 70, 10)), (136, kc.moe(130, 9, 65)), (64, kc.moe(5, 4, 520, 1030))])
@@ -184,19 +190,23 @@ def test_experts_single_token_and_rows(width, mlp):
     for precision, tol in ((mixers.F32, 2e-5), (mixers.BF16, 2e-2)):
         f = Feed(width, mlp, precision)
         ld = mixers.pad_to(width, 64)
-        for norm, normed in zip(f.norms, f.normed):
-            x = rnd(2, 40, width)
-            want = x + ko.mixture(normed(x.astype(np.float64)), f.ts, "", mlp)
-            assert f.rt.L.cq_mix_moe_step_fits(f.m.sizes)
-            for fused in (True, False):
-                f.m.fused = fused
-                xd = up(padded(x[:1], ld))
-                f.m.step(xd.data_ptr(), norm, None, sp())
-                assert rel(xd[:, :width], want[:1]) < (2e-5 if fused else tol), fused
-            xd, h = up(padded(x, ld)), torch.zeros((40, ld), device=DEV)
-            norm.rows(xd.data_ptr(), ld, h.data_ptr(), ld, 40, sp())
-            f.m.prefill(h.data_ptr(), ld, xd.data_ptr(), ld, 40, sp())
-            assert rel(xd[:, :width], want) < tol and not xd[:, width:].any()
+        x = rnd(2, 40, width)
+        x64 = x.astype(np.float64)
+        want = x + ko.mixture(f.normed(x64), f.ts, "", mlp)
+        assert f.rt.L.cq_mix_moe_step_fits(f.m.sizes)
+        for fused in (True, False):
+            f.m.fused = fused
+            xd = up(padded(x[:1], ld))
+            f.m.step(xd.data_ptr(), f.norm, None, sp())
+            assert rel(xd[:, :width], want[:1]) < (2e-5 if fused else tol), fused
+        f.m.fused = True
+        xd = up(padded(x[:1], ld))
+        f.m.step(xd.data_ptr(), f.rms, ptr(np.full((1, width), 0.25, np.float32)), sp())
+        assert rel(xd[:, :width], x[:1] + ko.mixture(f.rms_normed(x64[:1]), f.ts, "", mlp) + 0.25) < 2e-5
+        xd, h = up(padded(x, ld)), f.rt.normed(f.m.INPUT, 40 * ld)
+        f.norm.rows(xd.data_ptr(), ld, h, ld, 40, sp())
+        f.m.prefill(h, ld, xd.data_ptr(), ld, 40, sp())
+        assert rel(xd[:, :width], want) < tol and not xd[:, width:].any()
 
 
 # ---------------------------------------------------------------------------------------------- latent attention
