@@ -2,7 +2,7 @@
 // A head's unrotated key is W_uk c and its value W_uv c.  Two ways to the same result:
 //   expanded   keys and values of all heads are computed (a dense product over the cache rows) and attended to head by head: many query rows
 //   absorbed   W_uk is applied to the query instead and W_uv to the attended latent: every head attends to the cache rows themselves, few query rows
-// T is the type that the products read: bfloat16, or float for products in f32.  Scores, weights, sums and outputs are f32.  Queries are packed with the scale and
+// T is the type that the products read: bfloat16, or float for products in f32.  Scores, weights and sums are f32.  Queries are packed with the scale and
 // log2(e) multiplied in, so that a weight is a power of two.
 #include "cq_dense.h"
 #include "cq_mix.h"
@@ -43,14 +43,10 @@ template <> __device__ __forceinline__ void store_values<__bf16>(u32x4 *vs, int 
 #pragma unroll
     for (int j = 0; j < 8; j++) {
         const int r = cg * 8 + j, w = j >> 1;
+        const uint32_t pick = j & 1 ? 0x07060302u : 0x05040100u;           // the high or low halves of two registers
         u32x2 x;
-        if (j & 1) {
-            x.x = (v[0][w] >> 16) | (v[1][w] & 0xffff0000u);
-            x.y = (v[2][w] >> 16) | (v[3][w] & 0xffff0000u);
-        } else {
-            x.x = (v[0][w] & 0xffffu) | (v[1][w] << 16);
-            x.y = (v[2][w] & 0xffffu) | (v[3][w] << 16);
-        }
+        x.x = __builtin_amdgcn_perm(v[1][w], v[0][w], pick);
+        x.y = __builtin_amdgcn_perm(v[3][w], v[2][w], pick);
         reinterpret_cast<u32x2 *>(vs + r * 8 + value_slot(r, chunk))[half] = x;
     }
 }
@@ -97,7 +93,7 @@ struct Expanded {
     int q_head, k_head, v_head, d1, d2, vdim, v_pad;       // d1: unrotated dimensions (padded), d2: rotated
     const float *gate;
     int64_t gate_row;
-    float *out;
+    void *out;                                             // of type T, like everything that only feeds a product
     int64_t out_row;
     int pos, rows, heads;
 };
@@ -251,16 +247,22 @@ __global__ __launch_bounds__(256) void latent_expanded_kernel(Expanded p) {
         const float l = group_sum(l_run[i]);
         if (r >= p.rows) continue;
         const float f = mix_sigmoid(p.gate[r * p.gate_row + h]) / l;
-        float *dst = p.out + r * p.out_row + (int64_t)h * p.vdim;
+        T *dst = (T *)p.out + r * p.out_row + (int64_t)h * p.vdim;
 #pragma unroll
         for (int n = 0; n < NVF; n++) {
             const int c = 16 * n + 4 * lk;
             if (vec) {
-                if (c < p.vdim) *reinterpret_cast<f32x4 *>(dst + c) = o[i][n] * f;
+                if (c < p.vdim) {
+                    typedef T T4 __attribute__((ext_vector_type(4)));
+                    T4 v;
+#pragma unroll
+                    for (int e = 0; e < 4; e++) v[e] = (T)(o[i][n][e] * f);
+                    *reinterpret_cast<T4 *>(dst + c) = v;
+                }
             } else {
 #pragma unroll
                 for (int e = 0; e < 4; e++)
-                    if (c + e < p.vdim) dst[c + e] = o[i][n][e] * f;
+                    if (c + e < p.vdim) dst[c + e] = (T)(o[i][n][e] * f);
             }
         }
     }
@@ -719,7 +721,7 @@ int cq_mix_latent_pack(const cq_latent *g, const float *row_dev, int64_t row_str
 }
 
 int cq_mix_latent_expanded(const cq_latent *g, const void *q_dev, int64_t dim_pad, const void *kv_dev, int64_t kv_row, int64_t v_off, int64_t v_pad, const void *cache_dev,
-                           const float *gate_dev, int64_t gate_row, float *out_dev, int64_t out_row, int64_t pos, int64_t rows, void *stream) {
+                           const float *gate_dev, int64_t gate_row, void *out_dev, int64_t out_row, int64_t pos, int64_t rows, void *stream) {
     const int e = check_latent(g);
     if (e) return e;
     if (rows < 0 || pos < 0 || dim_pad < g->dim || dim_pad % 8 || v_pad < g->vdim || v_pad % 8 || v_off % 8 || kv_row % 8 || v_off < g->heads * dim_pad ||

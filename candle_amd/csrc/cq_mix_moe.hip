@@ -67,7 +67,15 @@ __global__ __launch_bounds__(1024) void moe_plan_kernel(const int32_t *__restric
     const int tid = threadIdx.x, lane = tid & 63, wv = tid >> 6;
     if (tid < MAX_EXPERTS) count[tid] = 0;
     __syncthreads();
-    for (int i = tid; i < pairs; i += 1024) atomicAdd(&count[ids[i]], 1);
+    // the first PER of a thread's ids stay in registers
+    constexpr int PER = 16;
+    int id[PER];
+#pragma unroll
+    for (int j = 0; j < PER; j++) id[j] = tid + 1024 * j < pairs ? ids[tid + 1024 * j] : -1;
+#pragma unroll
+    for (int j = 0; j < PER; j++)
+        if (id[j] >= 0) atomicAdd(&count[id[j]], 1);
+    for (int i = tid + 1024 * PER; i < pairs; i += 1024) atomicAdd(&count[ids[i]], 1);
     __syncthreads();
     // exclusive sums of rows and tiles over the experts: within the wave, then over the waves
     const int n = tid < experts ? count[tid] : 0, nt = (n + tile_rows - 1) / tile_rows;
@@ -106,12 +114,19 @@ __global__ __launch_bounds__(1024) void moe_plan_kernel(const int32_t *__restric
         if (tid == experts - 1) n_tiles[0] = b + nt;
     }
     __syncthreads();
-    for (int i = tid; i < pairs; i += 1024) {
-        const int at = atomicAdd(&start[ids[i]], 1);
+    auto place = [&](int i, int e, float w) {
+        const int at = atomicAdd(&start[e], 1);
         src_rows[at] = i / top;
         dst_rows[at] = i;
-        scale[at] = weights[i];
-    }
+        scale[at] = w;
+    };
+    float w[PER];
+#pragma unroll
+    for (int j = 0; j < PER; j++) w[j] = id[j] >= 0 ? weights[tid + 1024 * j] : 0.0f;
+#pragma unroll
+    for (int j = 0; j < PER; j++)
+        if (id[j] >= 0) place(tid + 1024 * j, id[j], w[j]);
+    for (int i = tid + 1024 * PER; i < pairs; i += 1024) place(i, ids[i], weights[i]);
 }
 
 // x[r] += sum over the choices of y[r * top + j], in order

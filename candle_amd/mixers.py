@@ -544,14 +544,15 @@ class LatentAttention(Mixer):
         return cache.add_rows(self.rt.ctx, self.ld, torch.bfloat16 if self.rt.t_bf16 else torch.float32)
 
     def expands(self, rows: int) -> bool:
-        """Whether computing keys and values per head costs less than attending to latents with `rows` queries."""
+        """Whether computing keys and values per head costs less than attending to latents with `rows` queries (whose longer products run at about half the
+        rate)."""
         d = self.dim + self.vdim
-        return self.expand is not None and rows * (2 * self.rank - d) > self.rank * d
+        return self.expand is not None and 2 * rows * (2 * self.rank - d) > self.rank * d
 
     def prefill(self, h, ldh, x, ldx, kept, pos, rows, sp):
         rt, L, H = self.rt, self.rt.L, self.heads
         ldp, ldo, bf = pad_to(self.w_in.n, 4), self.w_out.kp, int(rt.t_bf16)
-        row, out = rt.scratch("projection", rows * ldp), rt.scratch("mixer_out", rows * ldo)
+        row, out = rt.scratch("projection", rows * ldp), rt.typed("mixer_out_typed", rows * ldo)
         gate = row + 4 * self.g_off
         self.w_in.rows(h.typed, ldh, row, ldp, rows, sp, x_bf16=bf)
         if self.expands(rows):
@@ -572,8 +573,8 @@ class LatentAttention(Mixer):
             ws = rt.scratch("attention_splits", need // 4) if need else None
             check("cq_mix_latent_absorbed", L.cq_mix_latent_absorbed(self.shape, q, kept.data_ptr(), gate, ldp, lat, pos, rows, ws, need, sp))
             dense_product(rt, rt.precision, sp, w_dev=self.uv.w.data_ptr(), ldw=self.uv.kp, w_batch=self.vdim * self.uv.kp, x_dev=lat, ldx=H * self.rank_pad,
-                          x_batch=self.rank_pad, dst_dev=out, ldd=ldo, dst_batch=self.vdim, m=rows, n=self.vdim, k=self.uv.kp, batch=H)
-        self.w_out.rows(out, ldo, x, ldx, rows, sp, accumulate=True)
+                          x_batch=self.rank_pad, dst_dev=out, ldd=ldo, dst_batch=self.vdim, dst_bf16=bf, m=rows, n=self.vdim, k=self.uv.kp, batch=H)
+        self.w_out.rows(out, ldo, x, ldx, rows, sp, accumulate=True, x_bf16=bf)
 
     def step(self, x, norm, kept, pos_dev, pos, add, sp):
         rt, L = self.rt, self.rt.L

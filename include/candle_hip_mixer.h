@@ -186,9 +186,9 @@ int cq_mix_latent_pack(const cq_latent *g, const float *row_dev, int64_t row_str
                        int64_t q_head, int64_t rot_off, int64_t pos, int64_t rows, void *stream);
 /* Attention of rows pos .. pos + rows over keys and values of all heads: kv [pos + rows][kv_row] of type T, head h's unrotated key at h * dim_pad, its value
  * at v_off + h * v_pad (padding of keys zero).  q as packed with rot_off = dim_pad, q_head = dim_pad + rot_pad.  gate row r at gate + r * gate_row, [heads] raw.
- * out[r, h * vdim + e] f32. */
+ * out[r, h * vdim + e] of type T. */
 int cq_mix_latent_expanded(const cq_latent *g, const void *q_dev, int64_t dim_pad, const void *kv_dev, int64_t kv_row, int64_t v_off, int64_t v_pad, const void *cache_dev,
-                           const float *gate_dev, int64_t gate_row, float *out_dev, int64_t out_row, int64_t pos, int64_t rows, void *stream);
+                           const float *gate_dev, int64_t gate_row, void *out_dev, int64_t out_row, int64_t pos, int64_t rows, void *stream);
 /* The same over the cache rows themselves: q [rows][heads][rank_pad + rot_pad] holds W_uk^T q beside the rotated part; out [rows][heads][rank_pad] f32 is the
  * attended latent times the gate, which W_uv takes to the head's output.  Few queries split the keys and merge through the workspace (0 bytes
  * when not split).  step: the workspace of cq_mix_latent_step. */

@@ -121,7 +121,7 @@ def test_product_batches(precision, tol):
     assert rel(y[..., :n], want) < tol and not y[..., n:].any()
 
 
-@pytest.mark.parametrize("rows,experts,top,tile", [(1, 5, 2, 64), (40, 3, 3, 64), (300, 7, 2, 32), (300, 7, 2, 128), (130, 300, 4, 64), (4096, 2, 1, 128)])
+@pytest.mark.parametrize("rows,experts,top,tile", [(1, 5, 2, 64), (40, 3, 3, 64), (300, 7, 2, 32), (300, 7, 2, 128), (130, 300, 4, 64), (4096, 2, 1, 128), (4096, 40, 5, 64)])
 @pytest.mark.parametrize("precision", [mixers.F32, mixers.BF16])
 def test_grouped_product_over_a_plan(rows, experts, top, tile, precision):
     if precision == mixers.F32 and tile != 64:
@@ -262,6 +262,7 @@ class Attention:
                                                      self.g_off, q.data_ptr(), o.data_ptr(), pos_dev.data_ptr(), at - int(pos_dev), ws.data_ptr(), need, sp()))
             elif form == "expanded":
                 head = la.dim_pad + la.rot_pad
+                o = o.to(kind)
                 q, kv = torch.full((n, H, head), float("nan"), device=DEV, dtype=kind), torch.full((at + n, la.expand.n), float("nan"), device=DEV, dtype=kind)
                 _lib.check("p", L.cq_mix_latent_pack(la.shape, row, ldp, la.kv_off, self.kept.data_ptr(), None, 0, q.data_ptr(), head, la.dim_pad, at, n, sp()))
                 # the product reads whole steps of 64 columns of finite values; copy the rows that exist
@@ -282,7 +283,7 @@ class Attention:
                 _lib.check("a", L.cq_mix_latent_absorbed(la.shape, q.data_ptr(), self.kept.data_ptr(), gate, ldp, lat.data_ptr(), at, n, ws.data_ptr(), need, sp()))
                 uv = torch.from_numpy(self.ts["uv"].reshape(H, self.e, self.rank)).to(DEV)
                 o = torch.einsum("nhr,her->nhe", lat[..., :self.rank].float(), uv).reshape(n, H * self.e)
-            out.append(o)
+            out.append(o.float())
             at += n
         assert bool(self.kept[at:, :la.rank].isnan().all())                      # nothing written beyond
         return torch.cat(out)
@@ -388,7 +389,7 @@ def test_large_prompts_expand_and_small_portions_absorb():
     """Full-size latents: a prompt that is long enough for keys and values per head, then portions and tokens over the latents themselves."""
     cfg, ts, m = model_of("large", "float32")
     ids = kc.token_ids(cfg, 300, 4)
-    assert m.layers[0].mixer.expands(280) and not m.layers[0].mixer.expands(100)
+    assert m.layers[0].mixer.expands(200) and not m.layers[0].mixer.expands(60)
     want = ko.forward(cfg, ts, ids)
     for cuts in ([280, 5, 1], [3, 270, 2], [300]):
         m.reset()
