@@ -365,7 +365,7 @@ def kudurax_config(width, vocab, ctx):
     return {"vocab": vocab, "width": width, "norm": {"eps": 1e-5}, "embedding": {"scale": 1.0}, "layers": half(0) + half(4)}
 
 
-def timed_generation(model, prompt, n_new, ctx):
+def timed_generation(model, prompt, n_new, ctx, bf16):
     """Prompt and decode throughput: the best of three generations after a warm one."""
     model.generate_greedy(prompt, 8)
     best = None
@@ -376,7 +376,7 @@ def timed_generation(model, prompt, n_new, ctx):
     tok_s, wbytes = best["decode_steps"] / best["decode_seconds"], model.weight_bytes_per_token()
     return {"prompt_tok_s": round(len(prompt) / best["prompt_seconds"], 1), "decode_tok_s": round(tok_s, 1), "weight_bytes_per_token": wbytes,
             "decode_frac_of_weight_roofline": round(tok_s * wbytes / 1e9 / HBM_PEAK_GBPS, 4),
-            "prompt_weight_matmul_TFLOPs": round((wbytes - model.head.nbytes()) * len(prompt) / best["prompt_seconds"] / 1e12, 1) if hasattr(model, "head") else None}
+            "prompt_weight_matmul_TFLOPs": round((wbytes - model.head.nbytes()) * len(prompt) / best["prompt_seconds"] / 1e12, 1) if bf16 else None}
 
 
 def bf16_decoder(args):
@@ -401,7 +401,7 @@ def bf16_decoder(args):
         rec = {"width": width, "layer_runs": len(vcfg.order), "ff": width * 7 // 2, "prompt": args.prompt}
         for name in ("venizen_bf16", "llama_q4_k_m") if args.workload == "venizen" else ("kudurax_bf16", "venizen_bf16"):
             model = makes[name]()
-            rec[name] = timed_generation(model, prompt, n_new, ctx)
+            rec[name] = timed_generation(model, prompt, n_new, ctx, name.endswith("bf16"))
             del model
             torch.cuda.empty_cache()
         records.append(rec)

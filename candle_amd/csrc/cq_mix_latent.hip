@@ -104,10 +104,13 @@ __global__ __launch_bounds__(256) void latent_expanded_kernel(Expanded p) {
     constexpr int KL = KT * KC / 256, VT = (KT / 4) * (DV / CH), VL = (VT + 255) / 256;
     __shared__ u32x4 ks[KT * KC], vs[DV * 8];
     const int tid = threadIdx.x, lane = tid & 63, wv = __builtin_amdgcn_readfirstlane(tid >> 6), lr = lane & 15, lk = lane >> 4;
-    // the longest rows first; with heads in eighths a head stays on one XCD, whose L2 then holds its keys and values
-    const int blocks = (p.rows + BM - 1) / BM, id = blockIdx.x, per = p.heads >> 3;
+    // The longest rows first; where two workgroups per CU hold them all, the shortest join the longest.  With heads in eighths a head stays on one XCD, whose L2
+    // then holds its keys and values.
+    const int blocks = (p.rows + BM - 1) / BM, per = p.heads >> 3, total = blocks * p.heads;
     const bool split = (p.heads & 7) == 0;
-    const int h = split ? (id & 7) * per + (id >> 3) % per : id % p.heads, block = blocks - 1 - (split ? (id >> 3) / per : id / p.heads);
+    const int n = split ? total >> 3 : total, half = (n + 1) / 2, turn = split ? blockIdx.x >> 3 : blockIdx.x;
+    const int rank = NQ == 1 && total <= 512 && turn >= half ? n - 1 - (turn - half) : turn, heads = split ? per : p.heads;
+    const int h = (split ? (blockIdx.x & 7) * per : 0) + rank % heads, block = blocks - 1 - rank / heads;
     const int m0 = block * BM, mw = m0 + wv * 16 * NQ;
     const int last = p.pos + min(m0 + BM, p.rows) - 1, n_tiles = last / KT + 1, dk = p.d1 + p.d2;
     const T *kb = (const T *)p.k + (int64_t)h * p.k_head, *krb = (const T *)p.kr, *vb = (const T *)p.v + (int64_t)h * p.v_head;
