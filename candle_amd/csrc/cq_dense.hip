@@ -483,7 +483,7 @@ int cq_dense_product(int precision, const cq_dense_args *args, void *workspace_d
     if (m < 0 || n < 0 || k <= 0 || k % 64 || a.ldw % 64 || a.ldw < k || a.ldx % (a.x_bf16 ? 8 : 4) || a.ldx < k || a.ldd < cols || (a.add_dev && a.ld_add < cols) ||
         a.batch < 1)
         return CQ_ERR_SHAPE;
-    if ((a.act == CQ_DENSE_ACT_SWIGLU && n % 2) || ((a.act || a.dst_bf16 || a.row_scale_dev) && (a.accumulate || a.add_dev) && (a.act || a.dst_bf16))) return CQ_ERR_SHAPE;
+    if ((a.act == CQ_DENSE_ACT_SWIGLU && n % 2) || ((a.act || a.dst_bf16) && (a.accumulate || a.add_dev))) return CQ_ERR_SHAPE;
     if (a.batch > 1 && (a.accumulate || a.add_dev || a.row_scale_dev || a.tiles_dev || a.w_batch % 8 || a.x_batch % (a.x_bf16 ? 8 : 4))) return CQ_ERR_SHAPE;
     if (a.tiles_dev && (a.max_tiles < 1 || a.accumulate || a.add_dev || a.w_batch % 8 || (a.tile_rows != 32 && a.tile_rows != 64 && a.tile_rows != 128) ||
                         (precision == CQ_DENSE_F32 && a.tile_rows != 64)))
